@@ -23,35 +23,13 @@
 #include <cmath>
 
 #include "../include/inference.h"
+#include "read.h"
 
 namespace tinyinfer {
 
-namespace {
-const Json& need(const Json& d, const char* key, const std::string& where) {
-  const Json* v = d.type() == Json::Object ? d.find(key) : nullptr;
-  if (!v || v->is_null()) throw ConfigError("config.json: " + where + "'" + key + "' is missing");
-  return *v;
-}
-int64_t need_int(const Json& d, const char* key, const std::string& where, int64_t least = 1) {
-  const Json& v = need(d, key, where);
-  const bool whole = v.type() == Json::Int || (v.type() == Json::Float && v.as_double() == std::floor(v.as_double()));
-  if (!whole) throw ConfigError("config.json: " + where + "'" + key + "' must be an integer, got " + v.dump());
-  if (v.as_int() < least)
-    throw ConfigError("config.json: " + where + "'" + key + "' must be at least " + std::to_string(least) + ", got " + v.dump());
-  return v.as_int();
-}
-double need_float(const Json& d, const char* key, const std::string& where) {
-  const Json& v = need(d, key, where);
-  if (!v.is_number()) throw ConfigError("config.json: " + where + "'" + key + "' must be a number, got " + v.dump());
-  return v.as_double();
-}
-double need_positive(const Json& d, const char* key, const std::string& where) {
-  const double v = need_float(d, key, where);
-  if (!(v > 0.0)) throw ConfigError("config.json: " + where + "'" + key + "' must be positive");
-  return v;
-}
-bool given(const Json& d, const char* key) { return d.type() == Json::Object && d.has(key); }
+using namespace config_read;
 
+namespace {
 // "rot": {"base", "dims"} or absent; `most`: the entries a head has to turn
 Json read_rot(const Json& m, const std::string& mw, int64_t most) {
   if (!given(m, "rot")) return Json();

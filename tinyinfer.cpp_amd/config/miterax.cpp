@@ -16,30 +16,11 @@
 #include <cmath>
 
 #include "../include/inference.h"
+#include "read.h"
 
 namespace tinyinfer {
 
-namespace {
-const Json& need(const Json& d, const char* key, const std::string& where) {
-  const Json* v = d.find(key);
-  if (!v || v->is_null()) throw ConfigError("config.json: " + where + "'" + key + "' is missing");
-  return *v;
-}
-int64_t need_int(const Json& d, const char* key, const std::string& where, int64_t least = 1) {
-  const Json& v = need(d, key, where);
-  const bool whole = v.type() == Json::Int || (v.type() == Json::Float && v.as_double() == std::floor(v.as_double()));
-  if (!whole) throw ConfigError("config.json: " + where + "'" + key + "' must be an integer, got " + v.dump());
-  if (v.as_int() < least)
-    throw ConfigError("config.json: " + where + "'" + key + "' must be at least " + std::to_string(least) + ", got " + v.dump());
-  return v.as_int();
-}
-double need_float(const Json& d, const char* key, const std::string& where) {
-  const Json& v = need(d, key, where);
-  if (!v.is_number()) throw ConfigError("config.json: " + where + "'" + key + "' must be a number, got " + v.dump());
-  return v.as_double();
-}
-bool given(const Json& d, const char* key) { return d.has(key); }
-}  // namespace
+using namespace config_read;
 
 // config.json with every default filled in; ConfigError names the key that is wrong
 Json miterax_typed_config(const Json& d) {

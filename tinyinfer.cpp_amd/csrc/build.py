@@ -53,12 +53,13 @@ ON_DEMAND = ("measure",)
 
 # libraries that only some architectures call into (by the name config.json gives the architecture); every other
 # library serves them all
-ONLY_FOR = {"pointwise": ("Miterax", "Nazorax", "Dubozen"), "recurrent": ("Miterax",), "residual": ("Mumasun",), "diff_attention": ("Mumasun",),
-            "diff_attention_bf16": ("Mumasun",), "moe": ("Mumasun", "Nazorax", "Dubozen"), "moe_bf16": ("Mumasun", "Nazorax", "Dubozen"),
-            "latent_attention": ("Nazorax",), "latent_attention_bf16": ("Nazorax",), "hyper": ("Dubozen",),
-            "gated_attention": ("Dubozen",), "linear_attention": ("Dubozen",)}
+ONLY_FOR = {"pointwise": ("Miterax", "Nazorax", "Dubozen"), "recurrent": ("Miterax",), "residual": ("Mumasun", "Lupolorn"), "diff_attention": ("Mumasun",),
+            "diff_attention_bf16": ("Mumasun",), "moe": ("Mumasun", "Nazorax", "Dubozen", "Lupolorn"),
+            "moe_bf16": ("Mumasun", "Nazorax", "Dubozen", "Lupolorn"), "latent_attention": ("Nazorax", "Lupolorn"),
+            "latent_attention_bf16": ("Nazorax", "Lupolorn"), "hyper": ("Dubozen",), "gated_attention": ("Dubozen", "Lupolorn"),
+            "linear_attention": ("Dubozen",), "mingru": ("Lupolorn",)}
 # ... and libraries that a named architecture never calls into
-NOT_FOR = {"attention_generic": ("Mumasun", "Dubozen"), "attention_bf16": ("Mumasun",)}
+NOT_FOR = {"attention_generic": ("Mumasun", "Dubozen", "Lupolorn"), "attention_bf16": ("Mumasun",)}
 
 
 def libraries_for(dtype: str, architecture: str = None) -> List[str]:
@@ -92,10 +93,11 @@ def architecture_of(model_dir: str):
 # the host library (configuration, weights, parts, cache manager, step function, scheduler, sampler
 # and the C interface the Python package binds): C++17, no device code
 PKG = os.path.dirname(HERE)
-HOST_SOURCES = ["config/json.cpp", "config/config.cpp", "config/miterax.cpp", "config/mumasun.cpp", "config/nazorax.cpp", "config/dubozen.cpp", "ops/ops.cpp", "parts/parts.cpp", "weights/weights.cpp",
+HOST_SOURCES = ["config/json.cpp", "config/config.cpp", "config/miterax.cpp", "config/mumasun.cpp", "config/nazorax.cpp", "config/dubozen.cpp",
+                "config/lupolorn.cpp", "ops/ops.cpp", "parts/parts.cpp", "weights/weights.cpp",
                 "models/model.cpp", "cache/cache_manager.cpp", "engine/engine.cpp", "engine/scheduler.cpp",
                 "sampling/sampler.cpp", "engine/c_api.cpp"]
-HOST_HEADERS = ["include/inference.h", "weights/weights.h", "csrc/tinyinfer_kernels.h"]
+HOST_HEADERS = ["include/inference.h", "config/read.h", "weights/weights.h", "csrc/tinyinfer_kernels.h"]
 HOST_FLAGS = ["-std=c++17", "-O2", "-fPIC", "-D__HIP_PLATFORM_AMD__", "-Wall", "-Wno-unused-function"]
 ROCM = os.environ.get("ROCM_PATH", "/opt/rocm")
 

@@ -20,6 +20,15 @@ typedef uint16_t bf16_t;   // bfloat16 bits; arithmetic always happens in float
 #define TI_EPI_STORE_ACT 2   // out T   [M,N] = A W^T
 #define TI_EPI_SWIGLU 3      // W = [gate; up] ([2F,K]); out T [M,F] = silu(g) * u
 #define TI_EPI_QKV_PREP 4    // W = [q; k; v] heads: per-head norm, rotation, q out and cache write (own entry point)
+#define TI_EPI_RELU2 5       // out T   [M,N] = relu(A W^T)^2
+
+// a product's sum as the epilogues that store activations write it
+#define TI_EPI_ACT(E) ((E) == TI_EPI_STORE_ACT || (E) == TI_EPI_RELU2)
+template <int EPI> __device__ __forceinline__ float epi_act(float v) {
+  if (EPI != TI_EPI_RELU2) return v;
+  v = fmaxf(v, 0.f);
+  return v * v;
+}
 
 __device__ __forceinline__ float bf2f(bf16_t v) { return __uint_as_float(((uint32_t)v) << 16); }
 

@@ -11,10 +11,10 @@ TI_ERROR_API
 // ------------------------------------------------------------------ embedding
 // x[m, :] = float(E[t, :]) with t = tok[m], or, where tok[m] is below zero, t = fed[-1 - tok[m]]:
 // an id that an earlier kernel on the stream (the sampler) left on the device, so that the host
-// can launch a step before it has read the step before.
+// can launch a step before it has read the step before.  scale: a factor on every element, in 32-bit.
 template <typename T>
 __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict__ tok, const int* __restrict__ fed, int n_fed,
-                             float* __restrict__ x, int H, int V) {
+                             float* __restrict__ x, int H, int V, float scale) {
   const int m = blockIdx.x;
   int t = tok[m];
   if (t < 0 && fed && -1 - t < n_fed) t = fed[-1 - t];
@@ -24,21 +24,26 @@ __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict_
     return;
   }
   const T* src = table + (size_t)t * H;
-  for (int i = threadIdx.x; i < H; i += blockDim.x) row[i] = ld<T>(src + i);
+  for (int i = threadIdx.x; i < H; i += blockDim.x) row[i] = ld<T>(src + i) * scale;
 }
 
-extern "C" int ti_embed_fed(int dtype, const void* table, const int* tok, const int* fed, int n_fed, float* x, int M, int H,
-                            int V, hipStream_t stream) {
+extern "C" int ti_embed_scaled(int dtype, const void* table, const int* tok, const int* fed, int n_fed, float* x, int M, int H,
+                               int V, float scale, hipStream_t stream) {
   TI_REQUIRE(M >= 0 && H > 0 && V > 0 && n_fed >= 0, "embed: bad sizes M=%d H=%d V=%d n_fed=%d", M, H, V, n_fed);
   if (M == 0) return 0;
   if (dtype == TI_F32)
-    embed_kernel<float><<<M, 256, 0, stream>>>((const float*)table, tok, fed, n_fed, x, H, V);
+    embed_kernel<float><<<M, 256, 0, stream>>>((const float*)table, tok, fed, n_fed, x, H, V, scale);
   else if (dtype == TI_BF16)
-    embed_kernel<bf16_t><<<M, 256, 0, stream>>>((const bf16_t*)table, tok, fed, n_fed, x, H, V);
+    embed_kernel<bf16_t><<<M, 256, 0, stream>>>((const bf16_t*)table, tok, fed, n_fed, x, H, V, scale);
   else
     TI_REQUIRE(false, "embed: unknown dtype %d", dtype);
   TI_LAUNCH_CHECK();
   return 0;
+}
+
+extern "C" int ti_embed_fed(int dtype, const void* table, const int* tok, const int* fed, int n_fed, float* x, int M, int H,
+                            int V, hipStream_t stream) {
+  return ti_embed_scaled(dtype, table, tok, fed, n_fed, x, M, H, V, 1.0f, stream);
 }
 
 extern "C" int ti_embed(int dtype, const void* table, const int* tok, float* x, int M, int H, int V,

@@ -2,9 +2,10 @@
 // storage types (the float32 path of such layers, and the path of sizes the matrix-core kernels do not take).
 //
 //   preparation   from the 32-bit sums of one stacked projection [q | k | v | ...]: per-head RMS norms of q and k (a weight
-//                 of the head's size shared by all heads; before the rotation), rotation of the first rot_dims entries of
-//                 every query and key head, values that are the keys as projected (no v columns), values mixed with the
-//                 values another layer left for the same tokens, q out, k and v into the pages
+//                 of the head's size shared by all heads, before the rotation; or none, behind it), rotation of the first
+//                 rot_dims entries of every query and key head (entry i with entry i + rot_dims / 2, or neighbours in pairs),
+//                 values that are the keys as projected (no v columns), values mixed with the values another layer left for
+//                 the same tokens, q out, k and v into the pages
 //   attention     causal softmax over the pages with a learned number a head in the denominator (a sink: no key, no value,
 //                 not scaled) and a sigmoid gate on the output, one number an entry or one a head, read from the 32-bit sums
 //
@@ -30,17 +31,22 @@ __device__ __forceinline__ void ga_rotation(const float* __restrict__ inv_freq, 
   }
 }
 
-// grid (token, heads + kv heads), a wavefront each: a query head, or a key head with its value head
+// A wavefront per token and head: a query head, or a key head with its value head.  Grid (token, heads + kv heads in fours).
+// pairs: entries 2i and 2i + 1 turn together (else i and i + rot_dims / 2); unit_norm: the head divided by its root mean square
+// behind the rotation
+#define GA_PREP_WAVES 4
 template <typename T>
-__global__ void __launch_bounds__(TI_WAVE)
+__global__ void __launch_bounds__(TI_WAVE * GA_PREP_WAVES)
 gated_qkv_prep_kernel(const float* __restrict__ proj, int ld, int off_q, int off_k, int off_v, const float* __restrict__ q_w,
                       const float* __restrict__ k_w, float eps, const float* __restrict__ inv_freq,
                       const float* __restrict__ rope_table, int table_len, float mag, int rot_dims, int mix_mode,
                       const float* __restrict__ mix_lambda, float* __restrict__ v_kept, const int* __restrict__ pos,
                       const int* __restrict__ slot, const int* __restrict__ table, int table_stride, T* __restrict__ pool,
-                      T* __restrict__ q_out, int n_head, int n_kv, int dk, int dv, int dvr, int P) {
-  __shared__ float s_h[256];
-  const int m = blockIdx.x, unit = blockIdx.y, lane = threadIdx.x;
+                      T* __restrict__ q_out, int n_head, int n_kv, int dk, int dv, int dvr, int P, int pairs, int unit_norm) {
+  __shared__ float s_all[GA_PREP_WAVES][256];
+  const int m = blockIdx.x, unit = blockIdx.y * GA_PREP_WAVES + threadIdx.x / TI_WAVE, lane = threadIdx.x % TI_WAVE;
+  if (unit >= n_head + n_kv) return;      // (no barrier below: a wavefront keeps to itself)
+  float* const s_h = s_all[threadIdx.x / TI_WAVE];
   const int p = pos[m];
   const bool is_q = unit < n_head;
   const int h = is_q ? unit : unit - n_head;
@@ -76,13 +82,27 @@ gated_qkv_prep_kernel(const float* __restrict__ proj, int ld, int off_q, int off
     }
   }
   const int half = inv_freq ? rot_dims / 2 : 0;
-  if (half > 0) {
+  if (half > 0 && pairs) {
+    // neighbours lie in neighbouring lanes
+#pragma unroll
+    for (int i = 0; i < GA_MAX_DPL; ++i) {
+      const int d = lane + i * TI_WAVE;
+      if (i * TI_WAVE < 2 * half) {      // (the same in every lane)
+        const float other = __shfl_xor(v[i], 1, TI_WAVE);
+        if (d < 2 * half) {
+          float c, s;
+          ga_rotation(inv_freq, rope_table, table_len, mag, half, p, d >> 1, &c, &s);
+          v[i] = (d & 1) ? v[i] * c + other * s : v[i] * c - other * s;
+        }
+      }
+    }
+  } else if (half > 0) {
 #pragma unroll
     for (int i = 0; i < GA_MAX_DPL; ++i) {
       const int d = lane + i * TI_WAVE;
       if (d < dk) s_h[d] = v[i];
     }
-    __syncthreads();
+    __threadfence_block();      // (a wavefront's LDS accesses are served in order)
 #pragma unroll
     for (int i = 0; i < GA_MAX_DPL; ++i) {
       const int d = lane + i * TI_WAVE;
@@ -92,6 +112,14 @@ gated_qkv_prep_kernel(const float* __restrict__ proj, int ld, int off_q, int off
         v[i] = d < half ? s_h[d] * c - s_h[d + half] * s : s_h[d] * c + s_h[d - half] * s;
       }
     }
+  }
+  if (unit_norm) {
+    float sr = 0.f;
+#pragma unroll
+    for (int i = 0; i < GA_MAX_DPL; ++i) sr = fmaf(v[i], v[i], sr);      // (entries beyond the head are zero)
+    const float inv = 1.0f / sqrtf(group_sum<TI_WAVE>(sr) / (float)dk + eps);
+#pragma unroll
+    for (int i = 0; i < GA_MAX_DPL; ++i) v[i] *= inv;
   }
   if (is_q) {
     T* dst = q_out + ((size_t)m * n_head + h) * dk;
@@ -131,6 +159,16 @@ extern "C" int ti_gated_qkv_prep(int dtype, const float* proj, int ld, int off_q
                                  float mag, int rot_dims, int mix_mode, const float* mix_lambda, float* v_kept, const int* pos,
                                  const int* slot, const int* table, int table_stride, void* pool, void* q_out, int M, int n_head,
                                  int n_kv, int dk, int dv, int dv_rows, int page_size, hipStream_t stream) {
+  return ti_gated_qkv_prep_form(dtype, proj, ld, off_q, off_k, off_v, q_w, k_w, eps, inv_freq, rope_table, table_len, mag, rot_dims, mix_mode,
+                                mix_lambda, v_kept, pos, slot, table, table_stride, pool, q_out, M, n_head, n_kv, dk, dv, dv_rows, page_size,
+                                0, 0, stream);
+}
+
+extern "C" int ti_gated_qkv_prep_form(int dtype, const float* proj, int ld, int off_q, int off_k, int off_v, const float* q_w,
+                                      const float* k_w, float eps, const float* inv_freq, const float* rope_table, int table_len,
+                                      float mag, int rot_dims, int mix_mode, const float* mix_lambda, float* v_kept, const int* pos,
+                                      const int* slot, const int* table, int table_stride, void* pool, void* q_out, int M, int n_head,
+                                      int n_kv, int dk, int dv, int dv_rows, int page_size, int pairs, int unit_norm, hipStream_t stream) {
   const int dvr = dv_rows > 0 ? dv_rows : dv;
   TI_REQUIRE(n_head > 0 && n_kv > 0 && dk > 0 && dk <= 256 && dv > 0 && dv <= 256 && dvr >= dv && dvr <= 256 && page_size > 0 &&
                  table_stride > 0 && n_head + n_kv <= 65535,
@@ -143,17 +181,17 @@ extern "C" int ti_gated_qkv_prep(int dtype, const float* proj, int ld, int off_q
   TI_REQUIRE(off_q >= 0 && off_k >= 0 && off_q + n_head * dk <= ld && off_k + n_kv * dk <= ld && (off_v < 0 || off_v + n_kv * dv <= ld),
              "gated_qkv_prep: the columns do not lie inside rows of %d", ld);
   if (M == 0) return 0;
-  const dim3 grid(M, n_head + n_kv);
+  const dim3 grid(M, (n_head + n_kv + GA_PREP_WAVES - 1) / GA_PREP_WAVES);
   if (dtype == TI_F32)
-    gated_qkv_prep_kernel<float><<<grid, TI_WAVE, 0, stream>>>(proj, ld, off_q, off_k, off_v, q_w, k_w, eps, inv_freq, rope_table,
+    gated_qkv_prep_kernel<float><<<grid, TI_WAVE * GA_PREP_WAVES, 0, stream>>>(proj, ld, off_q, off_k, off_v, q_w, k_w, eps, inv_freq, rope_table,
                                                                table_len, mag, rot_dims, mix_mode, mix_lambda, v_kept, pos, slot,
                                                                table, table_stride, (float*)pool, (float*)q_out, n_head, n_kv, dk,
-                                                               dv, dvr, page_size);
+                                                               dv, dvr, page_size, pairs, unit_norm);
   else if (dtype == TI_BF16)
-    gated_qkv_prep_kernel<bf16_t><<<grid, TI_WAVE, 0, stream>>>(proj, ld, off_q, off_k, off_v, q_w, k_w, eps, inv_freq, rope_table,
+    gated_qkv_prep_kernel<bf16_t><<<grid, TI_WAVE * GA_PREP_WAVES, 0, stream>>>(proj, ld, off_q, off_k, off_v, q_w, k_w, eps, inv_freq, rope_table,
                                                                 table_len, mag, rot_dims, mix_mode, mix_lambda, v_kept, pos, slot,
                                                                 table, table_stride, (bf16_t*)pool, (bf16_t*)q_out, n_head, n_kv,
-                                                                dk, dv, dvr, page_size);
+                                                                dk, dv, dvr, page_size, pairs, unit_norm);
   else
     TI_REQUIRE(false, "gated_qkv_prep: unknown dtype %d", dtype);
   TI_LAUNCH_CHECK();
@@ -176,12 +214,50 @@ __global__ void sigmoid_gate_kernel(const T* __restrict__ src, int src_dv, T* __
   }
 }
 
+// the same, eight neighbouring entries a thread: dv a multiple of 8, 16-byte aligned rows; the same bits.  Grid (pieces of the
+// heads side by side, rows).
+__global__ void __launch_bounds__(256)
+sigmoid_gate_wide_kernel(const bf16_t* __restrict__ src, int src_dv, bf16_t* __restrict__ out, const float* __restrict__ gate, int gate_ld,
+                         int gate_mode, int n_head, int dv) {
+  const int m = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * 8;
+  const int W = n_head * dv;
+  if (c >= W) return;
+  const int h = c / dv;
+  const uint4 a = *reinterpret_cast<const uint4*>(src + (size_t)m * n_head * src_dv + (size_t)h * src_dv + (c - h * dv));
+  const unsigned w[4] = {a.x, a.y, a.z, a.w};
+  float y[8];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    y[2 * i] = __uint_as_float(w[i] << 16);
+    y[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
+  }
+  if (gate) {
+    const float* g = gate + (size_t)m * gate_ld;
+    if (gate_mode == 2) {
+      const float s = 1.0f / (1.0f + expf(-g[h]));
+#pragma unroll
+      for (int i = 0; i < 8; ++i) y[i] *= s;
+    } else {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) y[i] *= 1.0f / (1.0f + expf(-g[c + i]));
+    }
+  }
+  *reinterpret_cast<uint4*>(out + (size_t)m * W + c) = make_uint4(pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3]), pack_bf16x2(y[4], y[5]),
+                                                                  pack_bf16x2(y[6], y[7]));
+}
+
 extern "C" int ti_sigmoid_gate(int dtype, const void* src, int src_dv, void* out, const float* gate, int gate_ld, int gate_mode, int M,
                                int n_head, int dv, hipStream_t stream) {
   TI_REQUIRE(M >= 0 && n_head > 0 && dv > 0 && src_dv >= dv && (src != out || src_dv == dv) &&
                  (!gate || (gate_mode == 1 && gate_ld >= n_head * dv) || (gate_mode == 2 && gate_ld >= n_head)),
              "sigmoid_gate: bad sizes M=%d heads=%d dv=%d (from %d) gate mode %d in rows of %d", M, n_head, dv, src_dv, gate_mode, gate_ld);
   if (M == 0) return 0;
+  if (dtype == TI_BF16 && dv % 8 == 0 && src_dv % 8 == 0 && M <= 65535 && (((uintptr_t)src | (uintptr_t)out) & 15) == 0) {
+    sigmoid_gate_wide_kernel<<<dim3((n_head * dv / 8 + 255) / 256, M), 256, 0, stream>>>((const bf16_t*)src, src_dv, (bf16_t*)out, gate, gate_ld,
+                                                                                        gate_mode, n_head, dv);
+    TI_LAUNCH_CHECK();
+    return 0;
+  }
   const long n = (long)M * n_head * dv;
   const unsigned blocks = (unsigned)((n + 255) / 256 < 16384 ? (n + 255) / 256 : 16384);
   if (dtype == TI_F32)

@@ -150,7 +150,7 @@ gemm_skinny_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, v
       const size_t o = (size_t)m * N + n;
       if (EPI == TI_EPI_STORE_F32) ((float*)out_)[o] = s;
       if (EPI == TI_EPI_ADD_F32) ((float*)out_)[o] = prev[t] + s;
-      if (EPI == TI_EPI_STORE_ACT) ((bf16_t*)out_)[o] = f2bf(s);
+      if (TI_EPI_ACT(EPI)) ((bf16_t*)out_)[o] = f2bf(epi_act<EPI>(s));
     }
   }
 }
@@ -365,7 +365,7 @@ gemm_skinny_staged_kernel(Producer producer, const bf16_t* __restrict__ W, void*
     const size_t o = (size_t)tok * N + n;
     if (EPI == TI_EPI_STORE_F32) ((float*)out_)[o] = sum;
     if (EPI == TI_EPI_ADD_F32) ((float*)out_)[o] = prev + sum;
-    if (EPI == TI_EPI_STORE_ACT) ((bf16_t*)out_)[o] = f2bf(sum);
+    if (TI_EPI_ACT(EPI)) ((bf16_t*)out_)[o] = f2bf(epi_act<EPI>(sum));
   }
 }
 
@@ -521,7 +521,7 @@ gemm_skinny_pieces_kernel(const bf16_t* __restrict__ A, long lda, const bf16_t* 
     if (SPLIT) partial[(size_t)split * M * N + o] = sum;
     else if (EPI == TI_EPI_STORE_F32) ((float*)out_)[o] = sum;
     else if (EPI == TI_EPI_ADD_F32) ((float*)out_)[o] = prev + sum;
-    else if (EPI == TI_EPI_STORE_ACT) ((bf16_t*)out_)[o] = f2bf(sum);
+    else if (TI_EPI_ACT(EPI)) ((bf16_t*)out_)[o] = f2bf(epi_act<EPI>(sum));
   }
 }
 
@@ -619,7 +619,7 @@ gemv_rows_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, voi
     const size_t o = (size_t)lane * N + n;
     if (EPI == TI_EPI_STORE_F32) ((float*)out_)[o] = mine;
     if (EPI == TI_EPI_ADD_F32) ((float*)out_)[o] = prev + mine;
-    if (EPI == TI_EPI_STORE_ACT) ((bf16_t*)out_)[o] = f2bf(mine);
+    if (TI_EPI_ACT(EPI)) ((bf16_t*)out_)[o] = f2bf(epi_act<EPI>(mine));
   }
 }
 
@@ -681,7 +681,7 @@ gemv_rows_direct_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__
     const size_t o = (size_t)lane * N + n;
     if (EPI == TI_EPI_STORE_F32) ((float*)out_)[o] = mine;
     if (EPI == TI_EPI_ADD_F32) ((float*)out_)[o] = prev + mine;
-    if (EPI == TI_EPI_STORE_ACT) ((bf16_t*)out_)[o] = f2bf(mine);
+    if (TI_EPI_ACT(EPI)) ((bf16_t*)out_)[o] = f2bf(epi_act<EPI>(mine));
   }
 }
 
@@ -807,7 +807,7 @@ gemm_tiled_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, vo
           const float s = acc[a][b][i];
           if (EPI == TI_EPI_STORE_F32) ((float*)out_)[o] = s;
           if (EPI == TI_EPI_ADD_F32) ((float*)out_)[o] += s;
-          if (EPI == TI_EPI_STORE_ACT) ((bf16_t*)out_)[o] = f2bf(s);
+          if (TI_EPI_ACT(EPI)) ((bf16_t*)out_)[o] = f2bf(epi_act<EPI>(s));
         }
       }
     }
@@ -1244,7 +1244,7 @@ gemm_pipelined_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W
           const float v = acc[a][b][i];
           if (EPI == TI_EPI_STORE_F32) ((float*)out_)[o] = v;
           if constexpr (EPI == TI_EPI_ADD_F32) ((float*)out_)[o] = (PREV ? prev[a][b][i] : ((const float*)out_)[o]) + v;
-          if (EPI == TI_EPI_STORE_ACT) ((bf16_t*)out_)[o] = f2bf(v);
+          if (TI_EPI_ACT(EPI)) ((bf16_t*)out_)[o] = f2bf(epi_act<EPI>(v));
         }
       }
     }
@@ -1558,7 +1558,7 @@ static int g_row_per_wave = 1;
 // workgroups of 16 rows; 1.7B's, 2,048 x 2,048: 3.9 against 3.0).
 static bool row_per_wave_serves(int M, int N, int K, int epi) {
   return g_row_per_wave && M <= GR_MMAX && N < GR_ROWS_BELOW && (M <= 4 || N <= 4 * compute_units()) && K % 8 == 0 &&
-         K <= 64 * 8 * GR_LOADS && (epi == TI_EPI_STORE_F32 || epi == TI_EPI_ADD_F32);
+         K <= 64 * 8 * GR_LOADS && (epi == TI_EPI_STORE_F32 || epi == TI_EPI_ADD_F32 || epi == TI_EPI_RELU2);
 }
 
 static int g_rows_direct = 1;     // a hook for measurements: 0: the token rows go through LDS for every K
@@ -1632,6 +1632,10 @@ extern "C" int ti_gemm_bf16_normed(const float* x, const float* nw, float eps, c
   TI_REQUIRE(M >= 0 && N > 0 && K > 0, "gemm_bf16_normed: bad sizes M=%d N=%d K=%d", M, N, K);
   if (M > 16 || K % 64 != 0 || K > 4096 || ((uintptr_t)W & 15) || ((uintptr_t)x & 15) || ((uintptr_t)nw & 15)) {
     ti_set_error("gemm_bf16_normed: M=%d K=%d is not served (M <= 16, K %% 64 == 0, K <= 4096)", M, K);
+    return 3;
+  }
+  if (epi == TI_EPI_RELU2) {
+    ti_set_error("gemm_bf16_normed: this epilogue is left to the norm's kernel and the product's");
     return 3;
   }
   if (row_per_wave_serves(M, N, K, epi)) {
@@ -1805,7 +1809,7 @@ gemm_mblocks_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, 
     if (EPI == TI_EPI_ADD_F32 && KS > 1) partial[(size_t)split * M * N + o] = v[i];
     else if (EPI == TI_EPI_ADD_F32) ((float*)out_)[o] += v[i];
     else if (EPI == TI_EPI_STORE_F32) ((float*)out_)[o] = v[i];
-    else ((bf16_t*)out_)[o] = f2bf(v[i]);
+    else ((bf16_t*)out_)[o] = f2bf(epi_act<EPI>(v[i]));
   }
 }
 
@@ -1976,7 +1980,7 @@ static int launch_pieces(const bf16_t* a, long lda, const bf16_t* w, void* out, 
 static int g_pieces = 1;
 static bool pieces_serves(int M, int N, int K, int epi) {
   if (!g_pieces || M > 16 || K % 64 != 0 || K < 2 * SP_PIECE) return false;
-  if (epi < TI_EPI_STORE_F32 || epi > TI_EPI_SWIGLU) return false;
+  if ((epi < TI_EPI_STORE_F32 || epi > TI_EPI_SWIGLU) && epi != TI_EPI_RELU2) return false;
   // few tokens times a weight of few rows: a row per wavefront wins (and fills the compute units)
   if (row_per_wave_serves(M, N, K, epi)) return false;
   // where the kernels with the norm in front take eight wavefronts, this one would give other bits
@@ -2135,6 +2139,7 @@ extern "C" int ti_gemm_bf16_pieces_any(const void* A, const void* W, void* out, 
   switch (epi) {
     case TI_EPI_STORE_F32: rc = launch_pieces<TI_EPI_STORE_F32, false>(a, lda, w, out, nullptr, M, N, K, 1, stream); break;
     case TI_EPI_STORE_ACT: rc = launch_pieces<TI_EPI_STORE_ACT, false>(a, lda, w, out, nullptr, M, N, K, 1, stream); break;
+    case TI_EPI_RELU2: rc = launch_pieces<TI_EPI_RELU2, false>(a, lda, w, out, nullptr, M, N, K, 1, stream); break;
     case TI_EPI_SWIGLU: rc = launch_pieces<TI_EPI_SWIGLU, false>(a, lda, w, out, nullptr, M, N, K, 1, stream); break;
     case TI_EPI_ADD_F32:
       if (ks == 1) {
@@ -2207,6 +2212,7 @@ extern "C" int ti_gemm_bf16_mblocks_any(const void* A, const void* W, void* out,
   switch (epi) {
     case TI_EPI_STORE_F32: launch_mblocks<TI_EPI_STORE_F32>(a, w, out, nullptr, M, N, K, lda, 1, stream); break;
     case TI_EPI_STORE_ACT: launch_mblocks<TI_EPI_STORE_ACT>(a, w, out, nullptr, M, N, K, lda, 1, stream); break;
+    case TI_EPI_RELU2: launch_mblocks<TI_EPI_RELU2>(a, w, out, nullptr, M, N, K, lda, 1, stream); break;
     case TI_EPI_SWIGLU: launch_mblocks<TI_EPI_SWIGLU>(a, w, out, nullptr, M, N, K, lda, 1, stream); break;
     case TI_EPI_ADD_F32:
       launch_mblocks<TI_EPI_ADD_F32>(a, w, out, (float*)partial, M, N, K, lda, ks, stream);
@@ -2248,6 +2254,7 @@ extern "C" int ti_gemm_bf16(const void* A, const void* W, void* out, int M, int 
       case TI_EPI_STORE_F32: rc_ = launch_pieces<TI_EPI_STORE_F32, false>(a, lda, w, out, nullptr, M, N, K, 1, stream); break;
       case TI_EPI_ADD_F32: rc_ = launch_pieces<TI_EPI_ADD_F32, false>(a, lda, w, out, nullptr, M, N, K, 1, stream); break;
       case TI_EPI_STORE_ACT: rc_ = launch_pieces<TI_EPI_STORE_ACT, false>(a, lda, w, out, nullptr, M, N, K, 1, stream); break;
+      case TI_EPI_RELU2: rc_ = launch_pieces<TI_EPI_RELU2, false>(a, lda, w, out, nullptr, M, N, K, 1, stream); break;
       default: rc_ = launch_pieces<TI_EPI_SWIGLU, false>(a, lda, w, out, nullptr, M, N, K, 1, stream); break;
     }
     if (rc_) return rc_;
@@ -2262,6 +2269,7 @@ extern "C" int ti_gemm_bf16(const void* A, const void* W, void* out, int M, int 
   if (row_per_wave_serves(M, N, K, epi)) {
     int rc_ = 0;
     if (epi == TI_EPI_STORE_F32) rc_ = launch_rows<TI_EPI_STORE_F32>(a, w, out, M, N, K, lda, stream);
+    else if (epi == TI_EPI_RELU2) rc_ = launch_rows<TI_EPI_RELU2>(a, w, out, M, N, K, lda, stream);
     else rc_ = launch_rows<TI_EPI_ADD_F32>(a, w, out, M, N, K, lda, stream);
     if (rc_) return rc_;
     TI_LAUNCH_CHECK();
@@ -2285,6 +2293,7 @@ extern "C" int ti_gemm_bf16(const void* A, const void* W, void* out, int M, int 
     TI_GO(TI_EPI_ADD_F32)
     TI_GO(TI_EPI_STORE_ACT)
     TI_GO(TI_EPI_SWIGLU)
+    TI_GO(TI_EPI_RELU2)
     default:
       TI_REQUIRE(false, "gemm_bf16: unknown epilogue %d", epi);
   }

@@ -71,7 +71,7 @@ gemm_generic_kernel(const T* __restrict__ A, const T* __restrict__ W, void* __re
       const size_t o = (size_t)m * N + n;
       if (EPI == TI_EPI_STORE_F32) ((float*)out_)[o] = acc[i][j];
       if (EPI == TI_EPI_ADD_F32) ((float*)out_)[o] += acc[i][j];
-      if (EPI == TI_EPI_STORE_ACT) st<T>((T*)out_ + o, acc[i][j]);
+      if (TI_EPI_ACT(EPI)) st<T>((T*)out_ + o, epi_act<EPI>(acc[i][j]));
       if (EPI == TI_EPI_SWIGLU) {
         const float g = acc[i][j];
         st<T>((T*)out_ + o, g / (1.0f + expf(-g)) * accu[SW ? i : 0][j]);
@@ -96,6 +96,9 @@ static int launch(const void* A, const void* W, void* out, int M, int N, int K, 
       break;
     case TI_EPI_SWIGLU:
       gemm_generic_kernel<T, TI_EPI_SWIGLU><<<grid, 256, 0, stream>>>((const T*)A, (const T*)W, out, M, N, K, lda);
+      break;
+    case TI_EPI_RELU2:
+      gemm_generic_kernel<T, TI_EPI_RELU2><<<grid, 256, 0, stream>>>((const T*)A, (const T*)W, out, M, N, K, lda);
       break;
     default:
       ti_set_error("gemm_generic: unknown epilogue %d", epi);

@@ -32,17 +32,26 @@ __device__ __forceinline__ void latent_rotation(const float* __restrict__ inv_fr
 
 // ------------------------------------------------------------ preparation
 // proj f32 [M, ld]: the heads' queries [H][d + r] from column 0, then the latent (R) and the shared key part (r) from
-// column off_kv.  A workgroup per token.
+// column off_kv.  A workgroup per token.  cq (null: none): the queries come from a latent of their own, Rq numbers from column
+// off_q on (H = 0 then: no queries in proj); its norm (q_norm_w, eps) goes to cq T [M, Rq], for the product that makes the queries.
 template <typename T>
 __global__ void __launch_bounds__(256)
 latent_prep_kernel(float* __restrict__ proj, int ldp, int off_kv, const float* __restrict__ norm_w, float eps,
                    const float* __restrict__ inv_freq, const float* __restrict__ rope_table, int table_len, float mag, int rot_dims,
                    const int* __restrict__ pos, const int* __restrict__ slot, const int* __restrict__ table, int table_stride,
-                   T* __restrict__ pool, size_t page_elems, int H, int d, int r, int R, int P) {
+                   T* __restrict__ pool, size_t page_elems, int H, int d, int r, int R, int P, int off_q, int Rq,
+                   const float* __restrict__ q_norm_w, T* __restrict__ cq) {
   __shared__ float red[4];
   const int m = blockIdx.x;
   const int p = pos[m];
   float* row = proj + (size_t)m * ldp;
+  if (cq) {
+    const float* u = row + off_q;
+    float sq = 0.f;
+    for (int i = threadIdx.x; i < Rq; i += 256) sq = fmaf(u[i], u[i], sq);
+    const float inv = 1.0f / sqrtf(block_sum<256>(sq, red) / (float)Rq + eps);
+    for (int i = threadIdx.x; i < Rq; i += 256) st<T>(cq + (size_t)m * Rq + i, u[i] * inv * q_norm_w[i]);
+  }
   const float* c = row + off_kv;
   float ss = 0.f;
   for (int i = threadIdx.x; i < R; i += 256) ss = fmaf(c[i], c[i], ss);
@@ -88,14 +97,25 @@ extern "C" int ti_latent_prep(int dtype, float* proj, int ldp, int off_kv, const
                               const float* rope_table, int table_len, float mag, int rot_dims, const int* pos, const int* slot,
                               const int* table, int table_stride, void* pool, long page_elems, int M, int H, int d, int r, int R,
                               int page_size, hipStream_t stream) {
-  TI_REQUIRE(H > 0 && d >= 0 && r >= 0 && R > 0 && page_size > 0 && table_stride > 0 && off_kv >= H * (d + r) && ldp >= off_kv + R + r &&
+  return ti_latent_prep_queries(dtype, proj, ldp, off_kv, norm_w, eps, inv_freq, rope_table, table_len, mag, rot_dims, pos, slot, table,
+                                table_stride, pool, page_elems, M, H, d, r, R, page_size, 0, 0, nullptr, nullptr, stream);
+}
+
+extern "C" int ti_latent_prep_queries(int dtype, float* proj, int ldp, int off_kv, const float* norm_w, float eps, const float* inv_freq,
+                                      const float* rope_table, int table_len, float mag, int rot_dims, const int* pos, const int* slot,
+                                      const int* table, int table_stride, void* pool, long page_elems, int M, int H, int d, int r, int R,
+                                      int page_size, int off_q, int Rq, const float* q_norm_w, void* cq, hipStream_t stream) {
+  TI_REQUIRE(!cq || (Rq > 0 && off_q >= 0 && off_q + Rq <= ldp && q_norm_w && (off_q + Rq <= off_kv || off_q >= off_kv + R + r)),
+             "latent_prep: a query latent of %d from column %d does not fit rows of %d", Rq, off_q, ldp);
+  TI_REQUIRE((H > 0 || cq) && d >= 0 && r >= 0 && R > 0 && page_size > 0 && table_stride > 0 && off_kv >= H * (d + r) && ldp >= off_kv + R + r &&
                  page_elems >= (long)page_size * (R + r),
              "latent_prep: bad sizes heads=%d dim=%d rot=%d rank=%d ld=%d page=%ld", H, d, r, R, ldp, page_elems);
   TI_REQUIRE(!inv_freq || (rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= r), "latent_prep: %d rotated entries do not fit %d", rot_dims, r);
   if (M == 0) return 0;
 #define LATENT_PREP(T)                                                                                                              \
   latent_prep_kernel<T><<<M, 256, 0, stream>>>(proj, ldp, off_kv, norm_w, eps, inv_freq, rope_table, table_len, mag, rot_dims, pos, \
-                                               slot, table, table_stride, (T*)pool, (size_t)page_elems, H, d, r, R, page_size)
+                                               slot, table, table_stride, (T*)pool, (size_t)page_elems, H, d, r, R, page_size,      \
+                                               off_q, Rq, q_norm_w, (T*)cq)
   if (dtype == TI_F32) LATENT_PREP(float);
   else if (dtype == TI_BF16) LATENT_PREP(bf16_t);
   else TI_REQUIRE(false, "latent_prep: unknown dtype %d", dtype);

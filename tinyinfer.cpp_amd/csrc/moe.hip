@@ -64,7 +64,8 @@ template <typename T, bool VEC>
 __global__ void __launch_bounds__(256)
 moe_route_kernel(const T* __restrict__ h, const float* __restrict__ router, int* __restrict__ ids, float* __restrict__ wts,
                  int W, int E, int top, int score_kind, int renormalize, const float* __restrict__ correction = nullptr,
-                 int n_groups = 0, int keep = 0, float weight_scale = 1.f, float sum_floor = 0.f) {
+                 int n_groups = 0, int keep = 0, float weight_scale = 1.f, float sum_floor = 0.f,
+                 const float* __restrict__ gate_row = nullptr, float* __restrict__ gate_out = nullptr) {
   __shared__ float s_score[MOE_MAX_EXPERTS];
   __shared__ float s_plain[MOE_MAX_EXPERTS];      // the scores the weights are taken from, where the choice reads corrected ones
   __shared__ float s_group[MOE_MAX_EXPERTS];
@@ -76,6 +77,10 @@ moe_route_kernel(const T* __restrict__ h, const float* __restrict__ router, int*
   for (int e = wave; e < E; e += 4) {
     const float z = wave_dot<T, VEC>([&](int c) { return router[(size_t)e * W + c]; }, row, W, lane);
     if (lane == 0) s_score[e] = z;
+  }
+  if (gate_row && wave == E % 4) {      // one more row beside the router's: sigmoid(gate_row . h), a factor for another branch
+    const float z = wave_dot<T, VEC>([&](int c) { return gate_row[c]; }, row, W, lane);
+    if (lane == 0) gate_out[m] = 1.0f / (1.0f + expf(-z));
   }
   __syncthreads();
   if (score_kind == MOE_SOFTMAX) {
@@ -178,6 +183,15 @@ extern "C" int ti_moe_route(int dtype, const void* h, const float* router, int* 
 extern "C" int ti_moe_route_grouped(int dtype, const void* h, const float* router, const float* correction, int* ids, float* wts,
                                     int M, int W, int E, int top, int score_kind, int renormalize, int n_groups, int keep,
                                     float weight_scale, float sum_floor, hipStream_t stream) {
+  return ti_moe_route_gate(dtype, h, router, correction, ids, wts, M, W, E, top, score_kind, renormalize, n_groups, keep, weight_scale,
+                           sum_floor, nullptr, nullptr, stream);
+}
+
+// the same, and gate_out f32 [M] = sigmoid(gate_row . h) with gate_row f32 [W] (null: none), in 32-bit
+extern "C" int ti_moe_route_gate(int dtype, const void* h, const float* router, const float* correction, int* ids, float* wts, int M, int W,
+                                 int E, int top, int score_kind, int renormalize, int n_groups, int keep, float weight_scale,
+                                 float sum_floor, const float* gate_row, float* gate_out, hipStream_t stream) {
+  TI_REQUIRE(!gate_row || gate_out, "moe_route: a gate needs room for its numbers");
   TI_REQUIRE(n_groups <= 1 || (E % n_groups == 0 && keep >= 1 && keep <= n_groups && (long)keep * (E / n_groups) >= top),
              "moe_route: %d groups of which %d are kept do not fit %d experts and top %d", n_groups, keep, E, top);
   TI_REQUIRE((!correction && n_groups <= 1) || score_kind != MOE_SOFTMAX_CHOSEN, "moe_route: a correction or groups do not go with weights from the chosen logits");
@@ -188,7 +202,7 @@ extern "C" int ti_moe_route_grouped(int dtype, const void* h, const float* route
   if (M == 0) return 0;
   const int piece = dtype == TI_F32 ? 4 : 8;
   const bool vec = W % piece == 0 && ((uintptr_t)h & 15) == 0;
-#define MOE_ROUTE(T, V) moe_route_kernel<T, V><<<M, 256, 0, stream>>>((const T*)h, router, ids, wts, W, E, top, score_kind, renormalize, correction, n_groups, keep, weight_scale, sum_floor)
+#define MOE_ROUTE(T, V) moe_route_kernel<T, V><<<M, 256, 0, stream>>>((const T*)h, router, ids, wts, W, E, top, score_kind, renormalize, correction, n_groups, keep, weight_scale, sum_floor, gate_row, gate_out)
   if (dtype == TI_F32) {
     if (vec) MOE_ROUTE(float, true);
     else MOE_ROUTE(float, false);

@@ -66,7 +66,8 @@ moe_group_kernel(const int* __restrict__ ids, int n_pairs, int E, int* __restric
 // run a pair's place is its count in LDS.
 __global__ void __launch_bounds__(256)
 moe_place_kernel(const bf16_t* __restrict__ h, const int* __restrict__ ids, const float* __restrict__ wts, int* __restrict__ meta,
-                 int E, int top, int W, int n_pairs, int* __restrict__ where, bf16_t* __restrict__ rows) {
+                 int E, int top, int W, int n_pairs, int* __restrict__ where, bf16_t* __restrict__ rows,
+                 const float* __restrict__ out_w = nullptr, float* __restrict__ row_w = nullptr) {
   __shared__ int count[MOE_MAX_E];      // pairs of this workgroup per expert, then the first row of their run
   __shared__ int s_row[64];
   const int pair0 = blockIdx.x * 64;
@@ -84,6 +85,7 @@ moe_place_kernel(const bf16_t* __restrict__ h, const int* __restrict__ ids, cons
   if (e_mine >= 0) {
     const int r = count[e_mine] + local;
     where[pair0 + threadIdx.x] = r;
+    if (row_w) row_w[r] = out_w[pair0 + threadIdx.x];      // weights on the experts' outputs: with the row
     s_row[threadIdx.x] = r;
   }
   __syncthreads();
@@ -110,12 +112,12 @@ moe_place_kernel(const bf16_t* __restrict__ h, const int* __restrict__ ids, cons
 // wavefronts two by two, each 64 outputs (four blocks of 16) against 64 rows (four blocks of 16).  A step of 32 along k of both
 // operands is fetched once by the workgroup (thread t the 16-byte pieces t, t + 256) into one of two LDS stages while the step
 // before it is multiplied from the other; one barrier a step.  Rows of a stage are 80 bytes apart, so that the fragments'
-// reads spread over the banks.  EPI 0: relu^2, bfloat16; 1: 32-bit.
+// reads spread over the banks.  EPI 0: relu^2, bfloat16; 1: 32-bit; 2: 32-bit, times the row's weight row_w[row].
 #define MOE_LDS_ROW 40       // bfloat16 elements between rows of a stage (32 + 8)
 template <int EPI>
 __global__ void __launch_bounds__(256)
 moe_grouped_kernel(const bf16_t* __restrict__ rows, const bf16_t* __restrict__ w, const int* __restrict__ meta, int E, void* __restrict__ out,
-                   int N, int K) {
+                   int N, int K, const float* __restrict__ row_w = nullptr) {
   __shared__ __attribute__((aligned(16))) bf16_t lds[2][2][128 * MOE_LDS_ROW];      // [stage][weights | rows]
   const int n_tiles = meta[0];
   if ((int)blockIdx.x >= n_tiles) return;
@@ -176,6 +178,7 @@ moe_grouped_kernel(const bf16_t* __restrict__ rows, const bf16_t* __restrict__ w
   for (int b = 0; b < 4; ++b) {
     const int r = 64 * wx + 16 * b + r16;
     if (r >= n_rows) continue;
+    const float s = EPI == 2 ? row_w[row0 + r] : 1.f;
 #pragma unroll
     for (int a = 0; a < 4; ++a) {
       const int n = n0 + 16 * a + 4 * quad;
@@ -189,6 +192,8 @@ moe_grouped_kernel(const bf16_t* __restrict__ rows, const bf16_t* __restrict__ w
           z[i] *= z[i];
         }
         *reinterpret_cast<uint2*>((bf16_t*)out + (size_t)(row0 + r) * N + n) = make_uint2(pack_bf16x2(z[0], z[1]), pack_bf16x2(z[2], z[3]));
+      } else if (EPI == 2) {
+        *reinterpret_cast<float4*>((float*)out + (size_t)(row0 + r) * N + n) = make_float4(v[0] * s, v[1] * s, v[2] * s, v[3] * s);
       } else {
         *reinterpret_cast<float4*>((float*)out + (size_t)(row0 + r) * N + n) = make_float4(v[0], v[1], v[2], v[3]);
       }
@@ -210,22 +215,26 @@ extern "C" long ti_moe_grouped_meta_ints(int n_pairs, int E) { return 1 + (E + 1
 
 // h bf16 [M, W]; ids, wts [M top]; up [E][F][W], down [E][W][F] bf16.  Scratch: meta int32 [ti_moe_grouped_meta_ints],
 // where int32 [M top], rows bf16 [M top][W], act bf16 [M top][F], out f32 [M top][W].  y (may be null): the tokens' sums;
-// without it the caller adds the rows out[where[m top + k]] itself.  3: sizes not served (W, F multiples of 32, E <= 1024).
+// without it the caller adds the rows out[where[m top + k]] itself.  The weights multiply the experts' inputs (scale_input) or
+// their outputs (row_w: f32 scratch [M top]).  3: sizes not served (W, F multiples of 32, E <= 1024).
 extern "C" int ti_moe_experts_grouped_bf16(const void* h, const int* ids, const float* wts, const void* up, const void* down,
                                            int* meta, int* where, void* rows, void* act, float* out, float* y, int M, int W, int F,
-                                           int E, int top, int scale_input, hipStream_t stream) {
-  if (W % 32 || F % 32 || E > MOE_MAX_E || !scale_input) {
+                                           int E, int top, int scale_input, float* row_w, hipStream_t stream) {
+  if (W % 32 || F % 32 || E > MOE_MAX_E) {
     ti_set_error("moe_experts (grouped): W=%d, F=%d, %d experts are not served", W, F, E);
     return 3;
   }
-  TI_REQUIRE(M >= 0 && top > 0 && E > 0, "moe_experts (grouped): bad sizes");
+  TI_REQUIRE(M >= 0 && top > 0 && E > 0 && (scale_input || row_w), "moe_experts (grouped): bad sizes");
   if (M == 0) return 0;
   const int n_pairs = M * top;
   const int max_tiles = (n_pairs + MOE_TILE - 1) / MOE_TILE + E;
   moe_group_kernel<<<1, 1024, 0, stream>>>(ids, n_pairs, E, meta);
-  moe_place_kernel<<<(n_pairs + 63) / 64, 256, 0, stream>>>((const bf16_t*)h, ids, wts, meta, E, top, W, n_pairs, where, (bf16_t*)rows);
+  moe_place_kernel<<<(n_pairs + 63) / 64, 256, 0, stream>>>((const bf16_t*)h, ids, scale_input ? wts : nullptr, meta, E, top, W, n_pairs, where,
+                                                            (bf16_t*)rows, wts, scale_input ? nullptr : row_w);
   moe_grouped_kernel<0><<<dim3(max_tiles, (F + 127) / 128), 256, 0, stream>>>((const bf16_t*)rows, (const bf16_t*)up, meta, E, act, F, W);
-  moe_grouped_kernel<1><<<dim3(max_tiles, (W + 127) / 128), 256, 0, stream>>>((const bf16_t*)act, (const bf16_t*)down, meta, E, out, W, F);
+  const dim3 grid_down(max_tiles, (W + 127) / 128);
+  if (scale_input) moe_grouped_kernel<1><<<grid_down, 256, 0, stream>>>((const bf16_t*)act, (const bf16_t*)down, meta, E, out, W, F);
+  else moe_grouped_kernel<2><<<grid_down, 256, 0, stream>>>((const bf16_t*)act, (const bf16_t*)down, meta, E, out, W, F, row_w);
   if (y) moe_combine_kernel<<<M, 256, 0, stream>>>(out, where, y, W, top);
   TI_LAUNCH_CHECK();
   return 0;

@@ -77,6 +77,147 @@ extern "C" int ti_norm_residual(float* x, const float* y, const float* g, const 
   return 0;
 }
 
+// Layers with a norm on either side of a sublayer, both in one pass over the row:
+//   x[m] += y'[m] / sqrt(mean(y'[m]^2) + eps) * g,   then   out[m] = x[m] / sqrt(mean(x[m]^2) + next_eps) * next_g  (RT)
+// y'[m]: the rows of y as above, in ascending order, and behind them plus_gate[m] plus[m] (plus null: none; plus_gate null:
+// times one).  out null: the first line alone.  A workgroup per row; x, y' and both gains are asked for before the first
+// sum is known and stay in registers: NV pieces of four elements a thread (NV 0: any width, element by element from memory).
+template <typename RT, int NV>
+__global__ void __launch_bounds__(256)
+norm_residual_next_kernel(float* __restrict__ x, const float* __restrict__ y, const int* __restrict__ gather, int n_gather,
+                          const float* __restrict__ plus, const float* __restrict__ plus_gate, const float* __restrict__ g, float eps,
+                          const float* __restrict__ next_g, float next_eps, RT* __restrict__ out, int H) {
+  __shared__ float red[4];
+  const int m = blockIdx.x;
+  const int terms = (gather || n_gather > 1) ? n_gather : 1;
+  const float pg = plus_gate ? plus_gate[m] : 1.f;
+  float* const row = x + (size_t)m * H;
+  auto source = [&](int k) { return y + (gather ? (size_t)gather[(size_t)m * n_gather + k] : (size_t)m * terms + k) * H; };
+  if constexpr (NV > 0) {
+    float4 v[NV], xv[NV], gv[NV], nv[NV];
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int i = (j * 256 + threadIdx.x) * 4;
+      const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+      v[j] = xv[j] = gv[j] = nv[j] = zero;
+      if (i < H) {
+        xv[j] = *reinterpret_cast<const float4*>(row + i);
+        gv[j] = *reinterpret_cast<const float4*>(g + i);
+        if (out) nv[j] = *reinterpret_cast<const float4*>(next_g + i);
+      }
+    }
+    for (int k = 0; k < terms; ++k) {
+      const float* src = source(k);
+#pragma unroll
+      for (int j = 0; j < NV; ++j) {
+        const int i = (j * 256 + threadIdx.x) * 4;
+        if (i < H) {
+          const float4 a = *reinterpret_cast<const float4*>(src + i);
+          v[j] = k == 0 ? a : make_float4(v[j].x + a.x, v[j].y + a.y, v[j].z + a.z, v[j].w + a.w);
+        }
+      }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int i = (j * 256 + threadIdx.x) * 4;
+      if (plus && i < H) {
+        const float4 a = *reinterpret_cast<const float4*>(plus + (size_t)m * H + i);
+        v[j] = make_float4(fmaf(pg, a.x, v[j].x), fmaf(pg, a.y, v[j].y), fmaf(pg, a.z, v[j].z), fmaf(pg, a.w, v[j].w));
+      }
+      ss = rms_accumulate(ss, v[j]);
+    }
+    const float scale = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)H + eps);
+    float s2 = 0.f;
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int i = (j * 256 + threadIdx.x) * 4;
+      xv[j] = make_float4(xv[j].x + v[j].x * scale * gv[j].x, xv[j].y + v[j].y * scale * gv[j].y, xv[j].z + v[j].z * scale * gv[j].z,
+                          xv[j].w + v[j].w * scale * gv[j].w);
+      if (i < H) *reinterpret_cast<float4*>(row + i) = xv[j];
+      s2 = rms_accumulate(s2, xv[j]);
+    }
+    if (!out) return;
+    const float next = 1.0f / sqrtf(block_sum<256>(s2, red) / (float)H + next_eps);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int i = (j * 256 + threadIdx.x) * 4;
+      if (i >= H) continue;
+      const float4 o = make_float4(xv[j].x * next * nv[j].x, xv[j].y * next * nv[j].y, xv[j].z * next * nv[j].z, xv[j].w * next * nv[j].w);
+      RT* dst = out + (size_t)m * H + i;
+      if constexpr (sizeof(RT) == 2) {
+        *reinterpret_cast<uint2*>(dst) = make_uint2(pack_bf16x2(o.x, o.y), pack_bf16x2(o.z, o.w));
+      } else {
+        *reinterpret_cast<float4*>(dst) = o;
+      }
+    }
+  } else {
+    auto value = [&](int i) {
+      float v = 0.f;
+      for (int k = 0; k < terms; ++k) {
+        const float a = source(k)[i];
+        v = k == 0 ? a : v + a;
+      }
+      return plus ? fmaf(pg, plus[(size_t)m * H + i], v) : v;
+    };
+    float ss = 0.f, s2 = 0.f;
+    for (int i = threadIdx.x; i < H; i += 256) {
+      const float v = value(i);
+      ss = fmaf(v, v, ss);
+    }
+    const float scale = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)H + eps);
+    for (int i = threadIdx.x; i < H; i += 256) {
+      const float now = row[i] + value(i) * scale * g[i];
+      row[i] = now;
+      s2 = fmaf(now, now, s2);
+    }
+    if (!out) return;
+    const float next = 1.0f / sqrtf(block_sum<256>(s2, red) / (float)H + next_eps);
+    for (int i = threadIdx.x; i < H; i += 256) st<RT>(out + (size_t)m * H + i, row[i] * next * next_g[i]);      // (its own elements)
+  }
+}
+
+extern "C" int ti_norm_residual_next(float* x, const float* y, const int* gather, int n_gather, const float* plus, const float* plus_gate,
+                                     const float* g, float eps, const float* next_g, float next_eps, void* out, int out_dtype, int M,
+                                     int H, hipStream_t stream) {
+  TI_REQUIRE(M >= 0 && H > 0 && (!gather || n_gather > 0) && (!out || next_g), "norm_residual_next: bad sizes M=%d H=%d gather=%d", M, H, n_gather);
+  TI_REQUIRE(!out || out_dtype == TI_F32 || out_dtype == TI_BF16, "norm_residual_next: unknown dtype %d", out_dtype);
+  if (M == 0) return 0;
+  const bool v4 = H % 4 == 0 && H <= 8192 && (((uintptr_t)x | (uintptr_t)y | (uintptr_t)g | (uintptr_t)plus | (uintptr_t)next_g | (uintptr_t)out) & 15) == 0;
+#define TI_NRN(RT, NV)                                                                                                             \
+  norm_residual_next_kernel<RT, NV><<<M, 256, 0, stream>>>(x, y, gather, n_gather, plus, plus_gate, g, eps, next_g, next_eps, (RT*)out, H)
+#define TI_NRN_WIDTH(RT)               \
+  do {                                 \
+    if (!v4) TI_NRN(RT, 0);            \
+    else if (H <= 1024) TI_NRN(RT, 1); \
+    else if (H <= 2048) TI_NRN(RT, 2); \
+    else if (H <= 4096) TI_NRN(RT, 4); \
+    else TI_NRN(RT, 8);                \
+  } while (0)
+  if (out && out_dtype == TI_BF16) TI_NRN_WIDTH(bf16_t);
+  else TI_NRN_WIDTH(float);
+#undef TI_NRN_WIDTH
+#undef TI_NRN
+  TI_LAUNCH_CHECK();
+  return 0;
+}
+
+// y[m] += gate[m] plus[m]  (gate null: times one)
+__global__ void add_gated_rows_kernel(float* __restrict__ y, const float* __restrict__ plus, const float* __restrict__ gate, long n, int H) {
+  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long)gridDim.x * blockDim.x)
+    y[i] = fmaf(gate ? gate[i / H] : 1.f, plus[i], y[i]);
+}
+
+extern "C" int ti_add_gated_rows(float* y, const float* plus, const float* gate, int M, int H, hipStream_t stream) {
+  TI_REQUIRE(M >= 0 && H > 0, "add_gated_rows: bad sizes M=%d H=%d", M, H);
+  if (M == 0) return 0;
+  const long n = (long)M * H;
+  const unsigned blocks = (unsigned)((n + 255) / 256 < 8192 ? (n + 255) / 256 : 8192);
+  add_gated_rows_kernel<<<blocks, 256, 0, stream>>>(y, plus, gate, n, H);
+  TI_LAUNCH_CHECK();
+  return 0;
+}
+
 // out = x rounded to the compute dtype
 template <typename T>
 __global__ void round_rows_kernel(const float* __restrict__ x, T* __restrict__ out, long n) {

@@ -25,6 +25,9 @@ int ti_embed(int dtype, const void* table, const int* tok, float* x, int M, int 
 // the same; a token below zero stands for fed[-1 - token], an id an earlier kernel on the stream left (fed may be null)
 int ti_embed_fed(int dtype, const void* table, const int* tok, const int* fed, int n_fed, float* x, int M, int H, int V,
                  hipStream_t stream);
+// the same with a factor on every element (in 32-bit)
+int ti_embed_scaled(int dtype, const void* table, const int* tok, const int* fed, int n_fed, float* x, int M, int H, int V, float scale,
+                    hipStream_t stream);
 // out[r] = rmsnorm(x[rows ? rows[r] : r]) * w, in `out_dtype`
 int ti_rmsnorm(int out_dtype, const float* x, const float* w, const int* rows, void* out, int n_rows, int H, float eps,
                hipStream_t stream);
@@ -141,6 +144,12 @@ int ti_latent_prep(int dtype, float* proj, int ld, int off_kv, const float* norm
                    const float* rope_table, int table_len, float mag, int rot_dims, const int* pos, const int* slot,
                    const int* table, int table_stride, void* pool, long page_elems, int M, int H, int d, int r, int R, int page_size,
                    hipStream_t stream);
+// the same for queries that come from a latent of their own: Rq numbers of proj from column off_q on, RMS-normed (q_norm_w [Rq],
+// eps) into cq [M, Rq] of `dtype` (null: none); H may be 0 then (proj holds no queries)
+int ti_latent_prep_queries(int dtype, float* proj, int ld, int off_kv, const float* norm_w, float eps, const float* inv_freq,
+                           const float* rope_table, int table_len, float mag, int rot_dims, const int* pos, const int* slot,
+                           const int* table, int table_stride, void* pool, long page_elems, int M, int H, int d, int r, int R,
+                           int page_size, int off_q, int Rq, const float* q_norm_w, void* cq, hipStream_t stream);
 // qa f32 [M, H, R + r] = [W_uk_h^T q_h[:d] | q_h[d:]] with w_uk [H d][R] in `dtype`
 int ti_latent_absorb(int dtype, const float* proj, int ld, const void* w_uk, float* qa, int M, int H, int d, int r, int R,
                      hipStream_t stream);
@@ -223,6 +232,13 @@ int ti_gated_qkv_prep(int dtype, const float* proj, int ld, int off_q, int off_k
                       int mix_mode, const float* mix_lambda, float* v_kept, const int* pos, const int* slot, const int* table,
                       int table_stride, void* pool, void* q_out, int M, int n_head, int n_kv, int dk, int dv, int dv_rows,
                       int page_size, hipStream_t stream);
+// the same with another form of rotation and norm: pairs 1: entries 2i and 2i + 1 of a head turn together (0: i and
+// i + rot_dims / 2); unit_norm 1: q and k heads are divided by sqrt(mean of their squares + eps) behind the rotation
+int ti_gated_qkv_prep_form(int dtype, const float* proj, int ld, int off_q, int off_k, int off_v, const float* q_w, const float* k_w,
+                           float eps, const float* inv_freq, const float* rope_table, int table_len, float mag, int rot_dims,
+                           int mix_mode, const float* mix_lambda, float* v_kept, const int* pos, const int* slot, const int* table,
+                           int table_stride, void* pool, void* q_out, int M, int n_head, int n_kv, int dk, int dv, int dv_rows,
+                           int page_size, int pairs, int unit_norm, hipStream_t stream);
 // out (T [M, n_head dv]) = src (T [M, n_head src_dv], the first dv of every head) times sigmoid(gate), gate f32 rows of gate_ld
 // floats: entry h dv + d (gate_mode 1) or h (gate_mode 2); gate null: times one; src may be out where src_dv = dv
 int ti_sigmoid_gate(int dtype, const void* src, int src_dv, void* out, const float* gate, int gate_ld, int gate_mode, int M,
@@ -248,12 +264,30 @@ int ti_decay_scan_chunked(const float* proj, int ld, int off_q, int off_k, int o
 int ti_gated_row_norm(int out_dtype, const float* o, const float* gate, int ld, int off_g, const float* w, void* out, int M, int W,
                       float eps, hipStream_t stream);
 
+// ---- libti_mingru: S <- (1 - s) S + s c element by element, s = sigmoid(z + bias_z), c = u + 1/2 (u >= 0) or sigmoid(u) with
+// u = x + bias_x; out = S g sigmoid(g).  proj f32 [M, ld] with W columns of z, x and g from off_z, off_x, off_g on; state f32
+// [slots][slot_stride >= W]; entry_meta [n_entries][4] = (row0, tokens, start, slot); out [M, W] of out_dtype
+int ti_mingru_scan(int out_dtype, const float* proj, int ld, int off_z, int off_x, int off_g, const float* bias_z, const float* bias_x,
+                   float* state, long slot_stride, const int* entry_meta, int n_entries, void* out, int W, hipStream_t stream);
+// the same with the entries' tokens in chunks that run side by side (lists as ti_decay_scan_chunked's; scratch float
+// [n_chunks][2][W] and behind it [n_entries][W])
+int ti_mingru_scan_chunked(int out_dtype, const float* proj, int ld, int off_z, int off_x, int off_g, const float* bias_z,
+                           const float* bias_x, float* state, long slot_stride, const int* entry_meta, int n_entries, const int* chunks,
+                           int n_chunks, const int* spans, float* scratch, void* out, int W, hipStream_t stream);
+
 // ---- libti_residual: layers that norm what a sublayer returns
 // x[m] (+)= y'[m] / sqrt(mean(y'[m]^2) + eps) * g; y'[m] = y[m], or with `gather` (int32 [M][n_gather]) the sum of
 // the rows y[gather[m][k]] in ascending k (gather null and n_gather > 1: of the rows y[m n_gather + k]).  accumulate 0: x is overwritten (y may be x itself).  rounded (may be null):
 // [M][H] of rounded_dtype, the new x rounded for the product that reads it next
 int ti_norm_residual(float* x, const float* y, const float* g, const int* gather, int n_gather, int M, int H, float eps,
                      int accumulate, void* rounded, int rounded_dtype, hipStream_t stream);
+// x[m] += y'[m] / sqrt(mean(y'[m]^2) + eps) * g, y' as above plus plus_gate[m] plus[m] (plus f32 [M][H], null: none; plus_gate
+// f32 [M], null: times one); then out[m] = x[m] / sqrt(mean(x[m]^2) + next_eps) * next_g in out_dtype (out null: not written)
+int ti_norm_residual_next(float* x, const float* y, const int* gather, int n_gather, const float* plus, const float* plus_gate,
+                          const float* g, float eps, const float* next_g, float next_eps, void* out, int out_dtype, int M, int H,
+                          hipStream_t stream);
+// y[m] += gate[m] plus[m] (gate null: times one)
+int ti_add_gated_rows(float* y, const float* plus, const float* gate, int M, int H, hipStream_t stream);
 // out = x rounded to out_dtype
 int ti_round_rows(int out_dtype, const float* x, void* out, long n, hipStream_t stream);
 // x *= s
@@ -312,6 +346,10 @@ int ti_moe_route(int dtype, const void* h, const float* router, int* ids, float*
 int ti_moe_route_grouped(int dtype, const void* h, const float* router, const float* correction, int* ids, float* wts, int M,
                          int W, int E, int top, int score_kind, int renormalize, int n_groups, int keep, float weight_scale,
                          float sum_floor, hipStream_t stream);
+// the same, and gate_out f32 [M] = sigmoid(gate_row . h), gate_row f32 [W] (null: none), in 32-bit
+int ti_moe_route_gate(int dtype, const void* h, const float* router, const float* correction, int* ids, float* wts, int M, int W, int E,
+                      int top, int score_kind, int renormalize, int n_groups, int keep, float weight_scale, float sum_floor,
+                      const float* gate_row, float* gate_out, hipStream_t stream);
 // y f32 [M, W] = sum_k down[e_k] relu(up[e_k] (s_k h))^2 (scale_input) or sum_k s_k down[e_k] relu(up[e_k] h)^2;
 // up [E][F][W], down [E][W][F] in the dtype of h; act: scratch of that dtype, [M top][F]; part: f32 [M top][W].  A workgroup
 // per expert and 16 outputs walks its weights once for all the pairs that chose the expert: steps of few tokens, and float32.
@@ -329,11 +367,12 @@ int ti_moe_experts_rows_gated(int dtype, const void* h, const int* ids, const fl
 // ---- libti_moe_bf16: the experts for steps of many tokens, on the matrix cores: the (token, expert) pairs are laid out expert
 // by expert in tiles of 128 rows and both products run over the tiles.  Scratch: meta int32 [ti_moe_grouped_meta_ints(M top, E)],
 // where int32 [M top] (the row of every pair), rows bf16 [M top][W], act bf16 [M top][F], out f32 [M top][W].  y (may be
-// null): the tokens' sums; without it the caller adds the rows out[where[m top + k]] in ascending k.  3: sizes not served
+// null): the tokens' sums; without it the caller adds the rows out[where[m top + k]] in ascending k.  The weights multiply the
+// experts' inputs (scale_input) or their outputs (row_w: f32 scratch [M top]).  3: sizes not served
 long ti_moe_grouped_meta_ints(int n_pairs, int E);
 int ti_moe_experts_grouped_bf16(const void* h, const int* ids, const float* wts, const void* up, const void* down, int* meta,
                                 int* where, void* rows, void* act, float* out, float* y, int M, int W, int F, int E, int top,
-                                int scale_input, hipStream_t stream);
+                                int scale_input, float* row_w, hipStream_t stream);
 
 // the gated experts of ti_moe_experts_rows_gated over such tiles; z: f32 scratch [M top][2F]; y is written (the tokens' weighted sums)
 int ti_moe_experts_grouped_gated_bf16(const void* h, const int* ids, const float* wts, const void* gate_up, const void* down,

@@ -1154,7 +1154,7 @@ int ti_ops_call(void* ops_, const char* op_, const ti_tensor* t, int n_t, const 
     }
   };
   if (op == "embed") {
-    ops.embed(arg(0), iptr(1), arg(1).numel(), arg(2));
+    ops.embed(arg(0), iptr(1), arg(1).numel(), arg(2), nullptr, 0, n_s > 0 ? (float)num(0) : 1.f);
   } else if (op == "rmsnorm") {
     const bool rows = n_t > 3 && arg(3).defined();
     ops.rmsnorm(arg(0), arg(1), (float)num(0), arg(2), rows ? iptr(3) : nullptr, rows ? arg(3).numel() : 0);
@@ -1272,9 +1272,10 @@ int ti_ops_call(void* ops_, const char* op_, const ti_tensor* t, int n_t, const 
                     n_t > 5 ? arg(5) : Tensor(), n_t > 6 ? arg(6) : Tensor(), n_s > 2 ? (float)num(2) : 0.f, n_t > 7 ? arg(7) : Tensor());
   } else if (op == "gated_qkv_prep") {
     // proj, q_w, k_w, inv_freq, rope_table, positions, slots, table, pool, q_out, lambda, kept; eps, heads, kv_heads, dk, dv,
-    // columns of q, k, v (v < 0: the values are the keys), rotated entries, mix mode
+    // columns of q, k, v (v < 0: the values are the keys), rotated entries, mix mode, [neighbours in pairs, unit norm behind]
     Ops::Rotation r = rotation(3, 4);
     r.dims = (int)num(8);
+    r.pairs = n_s > 10 && num(10) != 0;
     Ops::QkvColumns c;
     c.q = (int)num(5);
     c.k = (int)num(6);
@@ -1286,7 +1287,7 @@ int ti_ops_call(void* ops_, const char* op_, const ti_tensor* t, int n_t, const 
       mix.kept = arg(11);
     }
     ops.gated_qkv_prep(arg(0), c, arg(1), arg(2), (float)num(0), r, mix, iptr(5), iptr(6), view_of(7, arg(8)), arg(8), arg(9), (int)num(1),
-                       (int)num(2), (int)num(3), (int)num(4));
+                       (int)num(2), (int)num(3), (int)num(4), n_s > 11 && num(11) != 0);
   } else if (op == "gated_attention") {
     // q, pool, table, positions, slots, sink, gate proj, out; heads, kv_heads, dk, dv, scale, window, gate column, gate mode
     Ops::AttentionGate g;
@@ -1310,9 +1311,13 @@ int ti_ops_call(void* ops_, const char* op_, const ti_tensor* t, int n_t, const 
     // o, proj, w, out; gate column, eps
     ops.gated_row_norm(arg(0), arg(1), (int)num(0), arg(2), (float)num(1), arg(3));
   } else if (op == "moe_route_grouped") {
-    // h, router, ids, wts, correction (may be absent); top, score, renormalize, groups, keep, weight scale, sum floor
+    // h, router, ids, wts, correction (may be absent), [gate row, gate out]; top, score, renormalize, groups, keep, weight scale, sum floor
     Ops::RouterGroups g;
     if (n_t > 4) g.correction = arg(4);
+    if (n_t > 6) {
+      g.gate_row = arg(5);
+      g.gate_out = arg(6);
+    }
     g.groups = (int)num(3);
     g.keep = (int)num(4);
     g.weight_scale = (float)num(5);
@@ -1325,6 +1330,31 @@ int ti_ops_call(void* ops_, const char* op_, const ti_tensor* t, int n_t, const 
     r.mag = (float)num(7);
     ops.latent_prep(arg(0), (int)num(0), arg(1), (float)num(1), r, iptr(4), iptr(5), view_of(6, arg(7)), arg(7), (int)num(2), (int)num(3),
                     (int)num(4), (int)num(5));
+  } else if (op == "latent_prep_queries") {
+    // proj, norm_w, q_norm_w, positions, slots, table, pool, cq; off_kv, eps, off_q, q_rank, rank
+    Ops::QueryLatent ql;
+    ql.col = (int)num(2);
+    ql.rank = (int)num(3);
+    ql.norm_w = arg(2);
+    ql.out = arg(7);
+    ops.latent_prep(arg(0), (int)num(0), arg(1), (float)num(1), ql, iptr(3), iptr(4), view_of(5, arg(6)), arg(6), (int)num(4));
+  } else if (op == "mingru_scan") {
+    // proj, bias_z, bias_x, state, entries [R, 4], out, [chunks, spans]; width, columns of z, x, g
+    Ops::GruColumns c;
+    c.z = (int)num(1);
+    c.x = (int)num(2);
+    c.g = (int)num(3);
+    const bool chunked = n_t > 7 && arg(6).defined();
+    ops.mingru_scan(arg(0), c, arg(1), arg(2), arg(3), iptr(4), (int)arg(4).shape[0], arg(5), (int)num(0), chunked ? iptr(6) : nullptr,
+                    chunked ? (int)arg(6).shape[0] : 0, chunked ? iptr(7) : nullptr, chunked ? &workspace_of(&ops) : nullptr);
+  } else if (op == "norm_residual_next") {
+    // x, y, gain, gather [M, n] (may be absent), plus, plus_gate, next_gain, next_out (each may be absent); eps, next_eps,
+    // rows of y a row of x sums where no list names them
+    const bool g = arg(3).defined();
+    ops.norm_residual_next(arg(0), arg(1), g ? iptr(3) : nullptr, g ? (int)arg(3).shape[1] : (int)num(2), arg(4), arg(5), arg(2), (float)num(0),
+                           arg(6), (float)num(1), arg(7));
+  } else if (op == "add_gated_rows") {
+    ops.add_gated_rows(arg(0), arg(1), n_t > 2 ? arg(2) : Tensor());
   } else if (op == "latent_attention") {
     // proj, w_uk, w_uv, sink (may be absent), pool, table, positions, slots, out, [w_uk_t, tiles [n, 3], rows [n], entries [R, 4]];
     // heads, dim, rot_dim, rank, v_dim, scale, window, [rows of single tokens where no list names them, their longest context]

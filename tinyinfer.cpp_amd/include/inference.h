@@ -172,6 +172,9 @@ ModelSpec nazorax_spec(const Json& config);
 // the Dubozen decoder (config/dubozen.cpp)
 Json dubozen_typed_config(const Json& config);
 ModelSpec dubozen_spec(const Json& config);
+// the Lupolorn decoder (config/lupolorn.cpp)
+Json lupolorn_typed_config(const Json& config);
+ModelSpec lupolorn_spec(const Json& config);
 // {"architecture": the registered name that matched, "config": the typed configuration (the input itself if
 // the architecture registered no reader)}; ConfigError as spec_from_config
 Json typed_config(const Json& config);
@@ -295,21 +298,24 @@ class Ops {
   int compute_units();
 
   // a token below zero stands for fed[-1 - token] (device memory, n_fed ids; may be null)
-  void embed(const Tensor& table, const int* tokens, int64_t M, const Tensor& x, const int* fed = nullptr, int n_fed = 0);
+  // scale: a factor on every element, in 32-bit
+  void embed(const Tensor& table, const int* tokens, int64_t M, const Tensor& x, const int* fed = nullptr, int n_fed = 0, float scale = 1.f);
   // out[r] = rmsnorm(x[rows ? rows[r] : r]) * w
   void rmsnorm(const Tensor& x, const Tensor& w, float eps, const Tensor& out, const int* rows = nullptr, int64_t n_rows = 0);
   void rope_neox(const Tensor& x, const int* positions, const Tensor& inv_freq);      // in place on f32 [M, heads, hd]
   void rope_table(const Tensor& inv_freq, const Tensor& table);                       // f32 [n_pos, hd/2, 2]
   // dims: how many leading entries of a head are turned (0: all of them); mag: a factor on cosine and sine (the table holds it already)
-  struct Rotation { const float* inv_freq = nullptr; const float* table = nullptr; int table_len = 0; int dims = 0; float mag = 1.f; };
+  // pairs: entries 2i and 2i + 1 of a head turn together, not i and i + dims / 2 (Ops::gated_qkv_prep; other calls refuse it)
+  struct Rotation { const float* inv_freq = nullptr; const float* table = nullptr; int table_len = 0; int dims = 0; float mag = 1.f; bool pairs = false; };
   struct CacheView { const int* table = nullptr; int table_width = 0; int page_size = 0; };
   void qk_norm_rope_kv_write(const Tensor& qkv, const float* q_w, const float* k_w, float eps, const Rotation& rot,
                              const int* positions, const int* slots, const CacheView& view, const Tensor& pool,
                              const Tensor& q_out, int heads, int kv_heads, int head_dim);
   void qk_norm_inplace(const Tensor& qkv, const float* q_w, const float* k_w, float eps, int heads, int kv_heads, int head_dim);
-  // out (op)= a w^T.  epilogue: "store" f32 = ; "add" f32 += ; "store_act" T = ; "swiglu" w = [gate; up].
+  // out (op)= a w^T.  epilogue: "store" f32 = ; "add" f32 += ; "store_act" T = ; "swiglu" w = [gate; up] ;
+  // "relu2" T = relu(.)^2.
   // may_defer (with "add"): the caller promises that `out` is read next through this object.
-  enum Epilogue { Store = 0, Add = 1, StoreAct = 2, SwiGLU = 3 };
+  enum Epilogue { Store = 0, Add = 1, StoreAct = 2, SwiGLU = 3, Relu2 = 5 };
   void linear(const Rows& a, const Tensor& w, const Tensor& out, Epilogue epi, bool may_defer = false);
   void linear(const Tensor& a, const Tensor& w, const Tensor& out, Epilogue epi, bool may_defer = false);
   bool can_fuse_norm(int64_t n_rows, DType dtype) const;
@@ -380,6 +386,11 @@ class Ops {
   // latent_prep: the latent normed (norm_w, eps) and the key part rotated into the token's row; the heads' rotated parts turned in place
   void latent_prep(const Tensor& proj, int off_kv, const Tensor& norm_w, float eps, const Rotation& rot, const int* positions,
                    const int* slots, const CacheView& view, const Tensor& pool, int heads, int dim, int rot_dim, int rank);
+  // the same for queries that come from a latent of their own (proj holds no queries): its `rank` columns from `col` on, normed
+  // (norm_w f32 [rank], the same eps), go to out [M, rank] in its own dtype, for the product that makes the queries
+  struct QueryLatent { int col = 0, rank = 0; Tensor norm_w, out; };
+  void latent_prep(const Tensor& proj, int off_kv, const Tensor& norm_w, float eps, const QueryLatent& ql, const int* positions,
+                   const int* slots, const CacheView& view, const Tensor& pool, int rank);
   // out [M, heads v_dim] = W_uv (softmax((W_uk^T q | q_rot) . [c | kr] scale; sink) c): scores and softmax in 32-bit, the
   // sink (f32 [heads], may be undefined) in the denominator only; scratch from `ws`
   // w_uk_t (w_uk's heads transposed, `latent_transpose`) and `lists` (tiles of up to 64 rows of entries of several tokens, the
@@ -414,12 +425,13 @@ class Ops {
   // holds q (heads x dk), k (kv_heads x dk) and v (kv_heads x dv) from the given columns on (off_v < 0: the values are the keys as
   // projected, before norm and rotation).  q_w / k_w (undefined: none): an RMS norm of every head with a weight of dk shared by the
   // heads, before the rotation.  mix_mode 1: this layer's values are also kept in v_kept f32 [M, kv_heads dv] for later layers; 2:
-  // v <- (1 - lambda) v + lambda v_kept, lambda f32 [1].  q to q_out, k and v into the pages (K [kv][P][dk] | V [kv][dv][P])
+  // v <- (1 - lambda) v + lambda v_kept, lambda f32 [1].  unit_norm: q and k heads are divided by their root mean square (eps)
+  // behind the rotation.  q to q_out, k and v into the pages (K [kv][P][dk] | V [kv][dv][P])
   struct QkvColumns { int q = 0, k = 0, v = -1; };
   struct ValueMix { int mode = 0; Tensor lambda, kept; };
   void gated_qkv_prep(const Tensor& proj, const QkvColumns& cols, const Tensor& q_w, const Tensor& k_w, float eps, const Rotation& rot,
                       const ValueMix& mix, const int* positions, const int* slots, const CacheView& view, const Tensor& pool,
-                      const Tensor& q_out, int heads, int kv_heads, int dk, int dv);
+                      const Tensor& q_out, int heads, int kv_heads, int dk, int dv, bool unit_norm = false);
   // causal softmax attention over such pages with a sink (f32 [heads], undefined: none) in the denominator and a sigmoid gate on
   // the output read from proj's columns from gate_col on: gate_mode 1 one number an output entry, 2 one a head (0: no gate)
   struct AttentionGate { Tensor proj; int col = 0, mode = 0; };
@@ -443,6 +455,19 @@ class Ops {
   // rounded (may be null): also receives the new x in its own dtype, for the product that reads the residual next
   void norm_residual(const Tensor& x, const Tensor& y, const Tensor& gain, float eps, bool accumulate, const int* gather = nullptr,
                      int n_gather = 0, const Tensor* rounded = nullptr);
+  // a norm on either side of a sublayer, both in one pass over the row: x += y' / rms(y') * gain, then next_out = x / rms(x) *
+  // next_gain in its own dtype (next_out undefined: the sum alone).  y': the rows of y as above, and behind them the row of
+  // `plus` (f32 [M, H], undefined: none) times plus_gate (f32 [M], undefined: one)
+  void norm_residual_next(const Tensor& x, const Tensor& y, const int* gather, int n_gather, const Tensor& plus, const Tensor& plus_gate,
+                          const Tensor& gain, float eps, const Tensor& next_gain = Tensor(), float next_eps = 0.f, const Tensor& next_out = Tensor());
+  void add_gated_rows(const Tensor& y, const Tensor& plus, const Tensor& gate);      // y[m] += gate[m] plus[m] (gate undefined: one)
+  // The minimal GRU over each entry's tokens, from and into its state slot: S <- (1 - s) S + s c with s = sigmoid(z + bias_z),
+  // c = u + 1/2 (u >= 0) or sigmoid(u), u = x + bias_x; out = S silu(g).  proj f32 [M, N]: `width` columns each of z, x and g;
+  // state f32 [slots][width]; out [M, width] in its own dtype.  chunks, spans, ws: as decay_scan's
+  struct GruColumns { int z = 0, x = 0, g = 0; };
+  void mingru_scan(const Tensor& proj, const GruColumns& cols, const Tensor& bias_z, const Tensor& bias_x, const Tensor& state,
+                   const int* entry_meta, int n_entries, const Tensor& out, int width, const int* chunks = nullptr, int n_chunks = 0,
+                   const int* spans = nullptr, Workspace* ws = nullptr);
   void round_rows(const Tensor& x, const Tensor& out);                               // out = x in out's dtype
   void scale(const Tensor& x, float s);                                              // x *= s (float32)
   // out[m, c] = sum_j taps[c, j] u(position of m - (K - 1) + j)[c] over each entry's rows, the K - 1 rows before an
@@ -475,8 +500,9 @@ class Ops {
   // a grouped router: `correction` f32 [E] (undefined: none) joins the scores for the choice only; the experts form `groups`
   // groups of neighbours (a group's score: the sum of its two largest choice scores) and only experts of the `keep` best groups
   // can be chosen (groups <= 1: none); the weights are the chosen experts' uncorrected scores, divided by their sum + sum_floor
-  // where `renormalize`, times weight_scale
-  struct RouterGroups { Tensor correction; int groups = 0, keep = 0; float weight_scale = 1.f, sum_floor = 0.f; };
+  // where `renormalize`, times weight_scale.  gate_row f32 [W] (undefined: none): one more row beside the router's, whose
+  // sigmoid(gate_row . h) goes to gate_out f32 [M]: a factor for a branch every token takes
+  struct RouterGroups { Tensor correction; int groups = 0, keep = 0; float weight_scale = 1.f, sum_floor = 0.f; Tensor gate_row, gate_out; };
   void moe_route(const Tensor& h, const Tensor& router, const Tensor& ids, const Tensor& wts, int top, RouterScore score,
                  bool renormalize, const RouterGroups& grouped);
   // y f32 [M, W] = sum over a token's experts of down_e relu(up_e h)^2, the weight on the expert's input or output;
@@ -484,7 +510,8 @@ class Ops {
   // take) y may stay unwritten: then rows->t is f32 [M top, W] and rows->gather device int32 [M][top]: row m of the result is
   // the sum of the rows rows->t[gather[m][k]], k ascending (no list: of the rows m n_gather + k), left to the norm that
   // reads it (Ops::norm_residual)
-  struct GatheredRows { Tensor t; const int* gather = nullptr; int n_gather = 0; };
+  // plus, plus_gate: a further branch of the result, f32 [M, W] times f32 [M] (undefined: none / one), for readers that say so
+  struct GatheredRows { Tensor t; const int* gather = nullptr; int n_gather = 0; Tensor plus, plus_gate; };
   void moe_experts(const Tensor& h, const Tensor& ids, const Tensor& wts, const Tensor& up, const Tensor& down, const Tensor& y,
                    int experts, bool scale_input, Workspace& ws, GatheredRows* rows = nullptr);
   // experts with a gate: y = sum_k s_k down_e act(gate_e h, up_e h); gate_up [E 2F, W] holds an expert's gate rows above its up rows
@@ -726,6 +753,8 @@ class NormPart : public Part { public: using Part::Part; const char* family() co
   // that keep the residual in several streams
   virtual bool can_mix() const { return false; }
   virtual Rows forward_mixed(StepContext& ctx, const Tensor& streams, const Tensor& coef);
+  // a plain RMS norm with a gain per channel says what it is, for kernels that take it in (false: it is something else)
+  virtual bool rms_form(Tensor& weight, float& eps) const { return false; }
   // for a writer of the streams that takes the next read in: the norm's weight, eps and the rows it would write (null: no such form)
   virtual bool mixed_form(StepContext& ctx, int64_t M, Tensor& weight, float& eps, Rows& rows) { return false; } };
 class PositionPart : public Part { public: using Part::Part; const char* family() const override { return "pos"; }
@@ -753,8 +782,9 @@ class FeedForwardPart : public Part { public: using Part::Part; const char* fami
   virtual bool can_store() const { return false; }
   virtual void forward_store(StepContext& ctx, const Rows& h, const Tensor& y);
   // as forward_store, but the part may leave the last sum to its reader: it returns rows whose sums (Ops::GatheredRows) are
-  // its output, for a norm that adds them while it reads (NormPart::forward_add).  Default: forward_store, rows.t = y
-  virtual void forward_rows(StepContext& ctx, const Rows& h, const Tensor& y, Ops::GatheredRows& rows) {
+  // its output, for a norm that adds them while it reads (NormPart::forward_add).  Default: forward_store, rows.t = y.
+  // takes_plus: the reader also adds a further branch (GatheredRows::plus); without it the part leaves none
+  virtual void forward_rows(StepContext& ctx, const Rows& h, const Tensor& y, Ops::GatheredRows& rows, bool takes_plus = false) {
     forward_store(ctx, h, y);
     rows = Ops::GatheredRows();
     rows.t = y;

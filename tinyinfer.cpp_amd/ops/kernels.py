@@ -18,7 +18,7 @@ from ..csrc import build as _build
 from ..native import KernelError  # noqa: F401
 
 F32, BF16 = 0, 1
-EPI = {"store": 0, "add": 1, "store_act": 2, "swiglu": 3}
+EPI = {"store": 0, "add": 1, "store_act": 2, "swiglu": 3, "relu2": 5}
 
 _C_TYPES = {"int": ctypes.c_int, "long": ctypes.c_long, "float": ctypes.c_float, "unsigned long": ctypes.c_ulong}
 
@@ -103,7 +103,8 @@ _LIB_OF = {"embed": "core", "rmsnorm": "core", "rope_neox": "core", "rope_table"
            "latent_attention": "latent_attention", "latent_transpose": "latent_attention", "layernorm": "hyper",
            "layernorm_mixed": "hyper", "hyper_combine": "hyper", "hyper_spread": "hyper", "hyper_write": "hyper",
            "gated_qkv_prep": "gated_attention", "gated_attention": "gated_attention", "decay_scan": "linear_attention",
-           "gated_row_norm": "linear_attention", "moe_route_grouped": "moe"}
+           "gated_row_norm": "linear_attention", "moe_route_grouped": "moe",
+           "latent_prep_queries": "latent_attention", "mingru_scan": "mingru", "norm_residual_next": "residual", "add_gated_rows": "residual"}
 
 
 class Ops:
@@ -232,8 +233,8 @@ class Ops:
         self._call("flush", libs=["core"])
 
     # --------------------------------------------------------------------- ops
-    def embed(self, table, tokens, x):
-        self._call("embed", [table, tokens, x])
+    def embed(self, table, tokens, x, scale=1.0):
+        self._call("embed", [table, tokens, x], [scale])
 
     def rmsnorm(self, x, w, eps, out, rows=None):
         self._call("rmsnorm", [x, w, out, rows], [eps])
@@ -266,7 +267,7 @@ class Ops:
     def linear(self, a, w, out, epilogue: str, may_defer: bool = False):
         """out (op)= a w^T.  a: T [M, K] (rows may be strided); w: T [N, K] contiguous.
         epilogue: "store" f32 out = ; "add" f32 out += ; "store_act" T out = ;
-        "swiglu": w is [2F, K] = [gate; up], T out [M, F] = silu(gate) * up.
+        "swiglu": w is [2F, K] = [gate; up], T out [M, F] = silu(gate) * up; "relu2": T out = relu(a w^T)^2.
         may_defer (with "add"): the caller reads `out` next through this object (see `flush`)."""
         libs = ["gemm_generic"] + (["gemm_bf16", "core"] if w.dtype == native.torch().bfloat16 and self.use_fast_gemm else [])
         if isinstance(a, NormedRows):
@@ -442,11 +443,12 @@ class Ops:
         self._call("hyper_write", [streams, mix, back, y, y2, next_coef, next_w, next_out], [f1, f2, eps])
 
     def gated_qkv_prep(self, proj, q_w, k_w, inv_freq, rope_table, positions, slots, table, pool, q_out, heads, kv_heads, dk, dv, columns,
-                       eps=1e-6, rot_dims=0, mix_mode=0, mix_lambda=None, kept=None):
+                       eps=1e-6, rot_dims=0, mix_mode=0, mix_lambda=None, kept=None, pairs=False, unit_norm=False):
         """proj f32 [M, N] with q, k, v from `columns` on (v < 0: the values are the keys as projected); per-head norms (q_w, k_w
-        or None), rotation of the first rot_dims entries, mix_mode 1: the values also go to `kept`; 2: v <- (1 - l) v + l kept."""
+        or None), rotation of the first rot_dims entries, mix_mode 1: the values also go to `kept`; 2: v <- (1 - l) v + l kept.
+        pairs: entries 2i and 2i + 1 turn together; unit_norm: q and k heads divided by their root mean square behind the rotation."""
         self._call("gated_qkv_prep", [proj, q_w, k_w, inv_freq, rope_table, positions, slots, table, pool, q_out, mix_lambda, kept],
-                   [eps, heads, kv_heads, dk, dv] + list(columns) + [rot_dims, mix_mode])
+                   [eps, heads, kv_heads, dk, dv] + list(columns) + [rot_dims, mix_mode, int(bool(pairs)), int(bool(unit_norm))])
 
     def gated_attention(self, q, pool, table, positions, slots, sink, gate_proj, out, heads, kv_heads, dk, dv, scale, window=0, gate_col=0,
                         gate_mode=0):
@@ -464,9 +466,31 @@ class Ops:
     def gated_row_norm(self, o, proj, gate_col, w, eps, out):
         self._call("gated_row_norm", [o, proj, w, out], [gate_col, eps])
 
-    def moe_route_grouped(self, h, router, ids, wts, correction, top, groups=0, keep=0, weight_scale=1.0, sum_floor=0.0, renormalize=True):
-        """Sigmoid scores; `correction` joins them for the choice only; only experts of the `keep` best of `groups` groups can be chosen."""
-        self._call("moe_route_grouped", [h, router, ids, wts, correction], [top, 0, int(bool(renormalize)), groups, keep, weight_scale, sum_floor])
+    def moe_route_grouped(self, h, router, ids, wts, correction, top, groups=0, keep=0, weight_scale=1.0, sum_floor=0.0, renormalize=True,
+                          score="sigmoid", gate_row=None, gate_out=None):
+        """`correction` joins the scores for the choice only; only experts of the `keep` best of `groups` groups can be chosen.
+        gate_row f32 [W]: gate_out f32 [M] = sigmoid(gate_row . h)."""
+        self._call("moe_route_grouped", [h, router, ids, wts, correction] + ([gate_row, gate_out] if gate_row is not None else []),
+                   [top, {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2}[score], int(bool(renormalize)), groups, keep, weight_scale, sum_floor])
+
+    # ---- norms on either side of a sublayer, the minimal GRU, queries from a latent
+    def norm_residual_next(self, x, y, gain, eps, gather=None, n_sum=0, plus=None, plus_gate=None, next_gain=None, next_eps=0.0, next_out=None):
+        """x += y' / rms(y') * gain, then next_out = x / rms(x) * next_gain (where given); y' = y, or the sum of the rows y[gather[m, k]]
+        (no list and n_sum > 1: y[m n_sum + k]), plus plus_gate[m] plus[m]."""
+        self._call("norm_residual_next", [x, y, gain, gather, plus, plus_gate, next_gain, next_out], [eps, next_eps, n_sum])
+
+    def add_gated_rows(self, y, plus, gate=None):
+        """y[m] += gate[m] plus[m]."""
+        self._call("add_gated_rows", [y, plus, gate])
+
+    def mingru_scan(self, proj, bias_z, bias_x, state, entries, out, width, columns, chunks=None, spans=None):
+        """S <- (1 - s) S + s c from and into state f32 [slots, width], s and c from the z and x columns of proj, out = S silu(g);
+        columns = (z, x, g); entries, chunks and spans as `decay_scan`'s."""
+        self._call("mingru_scan", [proj, bias_z, bias_x, state, entries, out, chunks, spans], [width] + list(columns))
+
+    def latent_prep_queries(self, proj, norm_w, q_norm_w, positions, slots, table, pool, cq, off_kv, eps, off_q, q_rank, rank):
+        """Both latents of proj normed: the keys' and values' (rank columns from off_kv) into the pages, the queries' (q_rank from off_q) to cq."""
+        self._call("latent_prep_queries", [proj, norm_w, q_norm_w, positions, slots, table, pool, cq], [off_kv, eps, off_q, q_rank, rank])
 
     def concat_round(self, a, b, out):
         self._call("concat_round", [a, b, out])

@@ -440,15 +440,15 @@ const Tensor& Rows::materialize(Ops& ops) const {
   return t;
 }
 
-void Ops::embed(const Tensor& table, const int* tokens, int64_t M, const Tensor& x, const int* fed, int n_fed) {
+void Ops::embed(const Tensor& table, const int* tokens, int64_t M, const Tensor& x, const int* fed, int n_fed, float scale) {
   TIMED("embed " + dims(x));
   require(table.ndim == 2 && x.ndim == 2, "embed: table and x must be matrices");
   const int64_t V = table.shape[0], H = table.shape[1];
   require(x.shape[0] == M && x.shape[1] == H && x.dtype == DType::F32,
           "embed: x " + x.describe() + " does not fit [" + std::to_string(M) + "," + std::to_string(H) + "] float32");
   require(table.contiguous() && x.contiguous(), "embed: table and x must be contiguous");
-  int rc = KERNEL("core", ti_embed_fed)(code(table.dtype, "embed"), table.data, tokens, fed, fed ? n_fed : 0, (float*)x.data,
-                                        (int)M, (int)H, (int)V, (hipStream_t)launch_stream());
+  int rc = KERNEL("core", ti_embed_scaled)(code(table.dtype, "embed"), table.data, tokens, fed, fed ? n_fed : 0, (float*)x.data,
+                                        (int)M, (int)H, (int)V, scale, (hipStream_t)launch_stream());
   check("core", rc, "embed");
 }
 
@@ -499,6 +499,11 @@ void Ops::rope_table(const Tensor& inv_freq, const Tensor& table) {
   check("core", rc, "rope_table");
 }
 
+// rotations of neighbours in pairs go through gated_qkv_prep alone
+static void no_pairs(const char* what, const Ops::Rotation& rot) {
+  require(!rot.pairs, std::string(what) + ": a rotation of neighbouring entries in pairs is not served here");
+}
+
 static void check_pool(const char* what, const Tensor& pool, int kv_heads, int head_dim, DType dt) {
   // a pool of one cache layer is [pages][2 * kv_heads][P][hd]: the K|V dimension is folded into
   // the second one (a tensor here has at most four dimensions)
@@ -512,6 +517,7 @@ void Ops::qk_norm_rope_kv_write(const Tensor& qkv, const float* q_w, const float
                                 const int* positions, const int* slots, const CacheView& view, const Tensor& pool,
                                 const Tensor& q_out, int heads, int kv_heads, int head_dim) {
   TIMED("qk_norm_rope_kv_write " + dims(qkv));
+  no_pairs("qk_norm_rope_kv_write", rot);
   const int64_t M = qkv.shape[0];
   const int64_t width = (int64_t)(heads + 2 * kv_heads) * head_dim;
   require(qkv.ndim == 2 && qkv.shape[1] == width && qkv.dtype == DType::F32 && qkv.contiguous(),
@@ -551,7 +557,7 @@ bool Ops::can_fuse_norm(int64_t n_rows, DType dtype) const {
 
 bool Ops::linear_with_norm(const Rows& a, const Tensor& w, const Tensor& out, Epilogue epi) {
   TunedScope tuned(*this, "gemm_bf16");
-  static const char* EPI_NAMES[] = {"store", "add", "store_act", "swiglu"};
+  static const char* EPI_NAMES[] = {"store", "add", "store_act", "swiglu", "", "relu2"};
   TIMED(std::string("norm+linear.") + EPI_NAMES[epi] + " " + dims(a.t) + " * " + dims(w));
   const int64_t M = a.t.shape[0], K = a.t.shape[1];
   if (!can_fuse_norm(M, a.t.dtype) || w.dtype != DType::BF16) return false;
@@ -586,7 +592,7 @@ void Ops::linear(const Rows& a, const Tensor& w, const Tensor& out, Epilogue epi
 
 void Ops::linear(const Tensor& a, const Tensor& w, const Tensor& out, Epilogue epi, bool may_defer) {
   TunedScope tuned(*this, "gemm_bf16");
-  static const char* EPI_NAMES[] = {"store", "add", "store_act", "swiglu"};
+  static const char* EPI_NAMES[] = {"store", "add", "store_act", "swiglu", "", "relu2"};
   TIMED(std::string("linear.") + EPI_NAMES[epi] + " " + dims(a) + " * " + dims(w));
   require(a.ndim == 2 && w.ndim == 2, "linear: a and w must be matrices");
   const int64_t M = a.shape[0], K = a.shape[1], rows = w.shape[0];
@@ -654,6 +660,7 @@ bool Ops::qkv_prepared(const Rows& a, const Tensor& w, const float* q_w, const f
                        const Tensor& q_out, int heads, int kv_heads, int head_dim) {
   TunedScope tuned(*this, "gemm_bf16");
   TIMED("qkv_prepared " + dims(a.t) + " * " + dims(w));
+  no_pairs("qkv_prepared", rot);
   if (!(use.fused_qkv_prefill && use.fast_gemm) || a.lazy) return false;
   if (a.t.dtype != DType::BF16 || w.dtype != DType::BF16 || q_out.dtype != DType::BF16) return false;
   if (!kernel_library_available("gemm_bf16")) return false;
@@ -758,6 +765,7 @@ bool Ops::attention_from_projections(const AttentionWork& work, Workspace& ws, c
   TIMED("attention.decode_prepared rows=" + std::to_string(work.M) + " context<=" + std::to_string(work.max_context));
   if (!(use.fused_qk_decode && use.fast_attention && work.decode_only && pool.dtype == DType::BF16)) return false;
   if (!kernel_library_available("attention_bf16")) return false;
+  no_pairs("attention_from_projections", rot);
   const int64_t M = qkv.shape[0];
   const int64_t width = (int64_t)(heads + (write_kv ? 2 * kv_heads : 0)) * head_dim;
   require(qkv.ndim == 2 && qkv.shape[1] >= width && qkv.dtype == DType::F32 && qkv.contiguous(),
@@ -948,6 +956,7 @@ void Ops::qkv_split_write(const Tensor& qkv, const Tensor& bias, const Rotation&
                           const CacheView& view, const Tensor& pool, const Tensor& q_out, int heads, int kv_heads, int dk, int dv,
                           float temp_coef, int temp_every) {
   TIMED("qkv_split_write " + dims(qkv) + (bias.defined() ? " bias" : "") + (rot.inv_freq ? " rotation" : ""));
+  no_pairs("qkv_split_write", rot);
   const int64_t M = qkv.shape[0];
   const int64_t width = (int64_t)heads * dk + (int64_t)kv_heads * (dk + dv);
   require(qkv.ndim == 2 && qkv.shape[1] == width && qkv.dtype == DType::F32 && qkv.contiguous(),
@@ -1014,6 +1023,7 @@ static void check_latent_pool(const char* what, const Tensor& pool, int rank, in
 void Ops::latent_prep(const Tensor& proj, int off_kv, const Tensor& norm_w, float eps, const Rotation& rot, const int* positions,
                       const int* slots, const CacheView& view, const Tensor& pool, int heads, int dim, int rot_dim, int rank) {
   TIMED("latent_prep " + dims(proj));
+  no_pairs("latent_prep", rot);
   require(proj.ndim == 2 && proj.dtype == DType::F32 && proj.contiguous() && off_kv >= (int64_t)heads * (dim + rot_dim) &&
               proj.shape[1] >= (int64_t)off_kv + rank + rot_dim,
           "latent_prep: proj " + proj.describe() + " does not hold the queries and the latent");
@@ -1027,6 +1037,25 @@ void Ops::latent_prep(const Tensor& proj, int off_kv, const Tensor& norm_w, floa
                                                       rot_dims, positions, slots, view.table, view.table_width, pool.data,
                                                       (long)(pool.shape[1] * pool.shape[2]), (int)proj.shape[0], heads, dim, rot_dim,
                                                       rank, (int)pool.shape[1], (hipStream_t)launch_stream());
+  check("latent_attention", rc, "latent_prep");
+}
+
+void Ops::latent_prep(const Tensor& proj, int off_kv, const Tensor& norm_w, float eps, const QueryLatent& ql, const int* positions,
+                      const int* slots, const CacheView& view, const Tensor& pool, int rank) {
+  TIMED("latent_prep " + dims(proj) + " queries " + std::to_string(ql.rank));
+  const int64_t M = proj.shape[0];
+  require(proj.ndim == 2 && proj.dtype == DType::F32 && proj.contiguous() && off_kv >= 0 && proj.shape[1] >= (int64_t)off_kv + rank &&
+              ql.col >= 0 && ql.rank > 0 && proj.shape[1] >= (int64_t)ql.col + ql.rank,
+          "latent_prep: proj " + proj.describe() + " does not hold the latents");
+  require(norm_w.dtype == DType::F32 && norm_w.numel() == rank && ql.norm_w.dtype == DType::F32 && ql.norm_w.numel() == ql.rank,
+          "latent_prep: the latents' norm weights " + norm_w.describe() + " / " + ql.norm_w.describe() + " do not fit");
+  check_latent_pool("latent_prep", pool, rank, 0, pool.dtype);
+  require(ql.out.ndim == 2 && ql.out.shape[0] == M && ql.out.shape[1] == ql.rank && ql.out.contiguous() && ql.out.dtype == pool.dtype,
+          "latent_prep: the query latents' rows " + ql.out.describe() + " do not fit");
+  int rc = KERNEL("latent_attention", ti_latent_prep_queries)(
+      code(pool.dtype, "latent_prep"), (float*)proj.data, (int)proj.shape[1], off_kv, (const float*)norm_w.data, eps, nullptr, nullptr, 0, 1.f,
+      0, positions, slots, view.table, view.table_width, pool.data, (long)(pool.shape[1] * pool.shape[2]), (int)M, 0, 0, 0, rank,
+      (int)pool.shape[1], ql.col, ql.rank, (const float*)ql.norm_w.data, ql.out.data, (hipStream_t)launch_stream());
   check("latent_attention", rc, "latent_prep");
 }
 
@@ -1274,8 +1303,8 @@ static int value_rows(const char* what, const Tensor& pool, int kv_heads, int dk
 
 void Ops::gated_qkv_prep(const Tensor& proj, const QkvColumns& cols, const Tensor& q_w, const Tensor& k_w, float eps, const Rotation& rot,
                          const ValueMix& mix, const int* positions, const int* slots, const CacheView& view, const Tensor& pool,
-                         const Tensor& q_out, int heads, int kv_heads, int dk, int dv) {
-  TIMED("gated_qkv_prep " + dims(proj) + (q_w.defined() ? " norm" : "") + (rot.inv_freq ? " rotation" : "") +
+                         const Tensor& q_out, int heads, int kv_heads, int dk, int dv, bool unit_norm) {
+  TIMED("gated_qkv_prep " + dims(proj) + (q_w.defined() || unit_norm ? " norm" : "") + (rot.inv_freq ? " rotation" : "") +
         (cols.v < 0 ? " v=k" : "") + (mix.mode ? " mix" + std::to_string(mix.mode) : ""));
   require(proj.ndim == 2 && proj.dtype == DType::F32 && proj.contiguous(), "gated_qkv_prep: proj must be contiguous float32 [M, N]");
   const int64_t M = proj.shape[0];
@@ -1289,12 +1318,12 @@ void Ops::gated_qkv_prep(const Tensor& proj, const QkvColumns& cols, const Tenso
   const int dvr = value_rows("gated_qkv_prep", pool, kv_heads, dk, dv);
   check_split_pool("gated_qkv_prep", pool, kv_heads, dk, dvr, q_out.dtype);
   const int rot_dims = rot.inv_freq ? (rot.dims > 0 ? rot.dims : dk) : 0;
-  int rc = KERNEL("gated_attention", ti_gated_qkv_prep)(
+  int rc = KERNEL("gated_attention", ti_gated_qkv_prep_form)(
       code(q_out.dtype, "gated_qkv_prep"), (const float*)proj.data, (int)proj.shape[1], cols.q, cols.k, cols.v,
       q_w.defined() ? (const float*)q_w.data : nullptr, k_w.defined() ? (const float*)k_w.data : nullptr, eps, rot.inv_freq, rot.table,
       rot.table_len, rot.mag, rot_dims, mix.mode, mix.mode == 2 ? (const float*)mix.lambda.data : nullptr,
       mix.mode ? (float*)mix.kept.data : nullptr, positions, slots, view.table, view.table_width, pool.data, q_out.data, (int)M, heads,
-      kv_heads, dk, dv, dvr, (int)pool.shape[2], (hipStream_t)launch_stream());
+      kv_heads, dk, dv, dvr, (int)pool.shape[2], rot.pairs ? 1 : 0, unit_norm ? 1 : 0, (hipStream_t)launch_stream());
   check("gated_attention", rc, "gated_qkv_prep");
 }
 
@@ -1399,6 +1428,68 @@ void Ops::norm_residual(const Tensor& x, const Tensor& y, const Tensor& gain, fl
   check("residual", rc, "norm_residual");
 }
 
+void Ops::norm_residual_next(const Tensor& x, const Tensor& y, const int* gather, int n_gather, const Tensor& plus, const Tensor& plus_gate,
+                             const Tensor& gain, float eps, const Tensor& next_gain, float next_eps, const Tensor& next_out) {
+  TIMED("norm_residual_next " + dims(x) + (plus.defined() ? " plus" : "") + (next_out.defined() ? " +norm" : ""));
+  const int64_t H = x.ndim == 2 ? x.shape[1] : 0;
+  require(x.ndim == 2 && x.dtype == DType::F32 && x.contiguous() && y.ndim == 2 && y.dtype == DType::F32 && y.contiguous() &&
+              y.shape[1] == H && (gather ? n_gather > 0 : y.shape[0] == x.shape[0] * std::max(1, n_gather)) &&
+              gain.dtype == DType::F32 && gain.numel() == H,
+          "norm_residual_next: x " + x.describe() + ", y " + y.describe() + " or gain " + gain.describe() + " do not fit");
+  require((!plus.defined() || (plus.dtype == DType::F32 && plus.contiguous() && plus.numel() == x.numel())) &&
+              (!plus_gate.defined() || (plus_gate.dtype == DType::F32 && plus_gate.contiguous() && plus_gate.numel() == x.shape[0])),
+          "norm_residual_next: the further branch " + plus.describe() + " or its gate do not fit");
+  require(!next_out.defined() || (next_out.contiguous() && next_out.numel() == x.numel() && next_gain.dtype == DType::F32 && next_gain.numel() == H),
+          "norm_residual_next: the next norm's rows or gain do not fit x");
+  int rc = KERNEL("residual", ti_norm_residual_next)(
+      (float*)x.data, (const float*)y.data, gather, n_gather, plus.defined() ? (const float*)plus.data : nullptr,
+      plus_gate.defined() ? (const float*)plus_gate.data : nullptr, (const float*)gain.data, eps,
+      next_out.defined() ? (const float*)next_gain.data : nullptr, next_eps, next_out.defined() ? next_out.data : nullptr,
+      next_out.defined() ? code(next_out.dtype, "norm_residual_next") : 0, (int)x.shape[0], (int)H, (hipStream_t)launch_stream());
+  check("residual", rc, "norm_residual_next");
+}
+
+void Ops::add_gated_rows(const Tensor& y, const Tensor& plus, const Tensor& gate) {
+  TIMED("add_gated_rows " + dims(y));
+  require(y.ndim == 2 && y.dtype == DType::F32 && y.contiguous() && plus.dtype == DType::F32 && plus.contiguous() && plus.numel() == y.numel() &&
+              (!gate.defined() || (gate.dtype == DType::F32 && gate.contiguous() && gate.numel() == y.shape[0])),
+          "add_gated_rows: y " + y.describe() + ", plus " + plus.describe() + " or gate " + gate.describe() + " do not fit");
+  int rc = KERNEL("residual", ti_add_gated_rows)((float*)y.data, (const float*)plus.data, gate.defined() ? (const float*)gate.data : nullptr,
+                                                 (int)y.shape[0], (int)y.shape[1], (hipStream_t)launch_stream());
+  check("residual", rc, "add_gated_rows");
+}
+
+void Ops::mingru_scan(const Tensor& proj, const GruColumns& cols, const Tensor& bias_z, const Tensor& bias_x, const Tensor& state,
+                      const int* entry_meta, int n_entries, const Tensor& out, int width, const int* chunks, int n_chunks, const int* spans,
+                      Workspace* ws) {
+  TIMED("mingru_scan " + dims(proj) + " entries=" + std::to_string(n_entries) + (chunks ? " chunks=" + std::to_string(n_chunks) : ""));
+  require(proj.ndim == 2 && proj.dtype == DType::F32 && proj.contiguous(), "mingru_scan: proj must be contiguous float32 [M, N]");
+  const int64_t W = width, N = proj.shape[1];
+  require(W > 0 && cols.z >= 0 && cols.x >= 0 && cols.g >= 0 && cols.z + W <= N && cols.x + W <= N && cols.g + W <= N,
+          "mingru_scan: the columns do not lie inside proj " + proj.describe());
+  require(bias_z.dtype == DType::F32 && bias_z.numel() == W && bias_x.dtype == DType::F32 && bias_x.numel() == W,
+          "mingru_scan: the biases must be float32 [width]");
+  require(state.dtype == DType::F32 && state.contiguous() && state.ndim >= 2 && state.numel() == state.shape[0] * W,
+          "mingru_scan: state " + state.describe() + " does not fit [slots, " + std::to_string(W) + "]");
+  require(out.ndim == 2 && out.shape[0] == proj.shape[0] && out.shape[1] == W && out.contiguous(), "mingru_scan: out " + out.describe() + " does not fit");
+  require(entry_meta != nullptr || n_entries == 0, "mingru_scan: no entry records");
+  const int dt = code(out.dtype, "mingru_scan");
+  if (chunks) {
+    require(spans && ws && n_chunks >= n_entries, "mingru_scan: chunks need spans and a workspace");
+    float* scratch = (float*)ws->get("mingru.maps", ((size_t)n_chunks * 2 + (size_t)n_entries) * W * 4);
+    int rc = KERNEL("mingru", ti_mingru_scan_chunked)(dt, (const float*)proj.data, (int)N, cols.z, cols.x, cols.g, (const float*)bias_z.data,
+                                                      (const float*)bias_x.data, (float*)state.data, (long)W, entry_meta, n_entries, chunks,
+                                                      n_chunks, spans, scratch, out.data, width, (hipStream_t)launch_stream());
+    check("mingru", rc, "mingru_scan(chunked)");
+    took("[chunked]");
+    return;
+  }
+  int rc = KERNEL("mingru", ti_mingru_scan)(dt, (const float*)proj.data, (int)N, cols.z, cols.x, cols.g, (const float*)bias_z.data,
+                                            (const float*)bias_x.data, (float*)state.data, (long)W, entry_meta, n_entries, out.data, width,
+                                            (hipStream_t)launch_stream());
+  check("mingru", rc, "mingru_scan");
+}
+
 void Ops::round_rows(const Tensor& x, const Tensor& out) {
   TIMED("round_rows " + dims(x));
   require(x.dtype == DType::F32 && x.contiguous() && out.contiguous() && out.numel() == x.numel(),
@@ -1439,6 +1530,7 @@ void Ops::diff_qk_prep(const Tensor& qkv, const float* q_w, const float* k_w, fl
                        const int* slots, const CacheView& view, const Tensor& pool, const Tensor& q_out, int heads, int kv_heads,
                        int dk, int dv, const ShortConv* conv) {
   TIMED("diff_qk_prep " + dims(qkv) + (conv ? " conv" : ""));
+  no_pairs("diff_qk_prep", rot);
   const int64_t M = qkv.shape[0];
   const int64_t width = (int64_t)heads * 2 * dk + (int64_t)kv_heads * (2 * dk + dv);
   require(qkv.ndim == 2 && qkv.shape[1] == width && qkv.dtype == DType::F32 && qkv.contiguous(),
@@ -1539,11 +1631,15 @@ void Ops::moe_route(const Tensor& h, const Tensor& router, const Tensor& ids, co
           "moe_route: ids and wts must be int32 / float32 [M, top]");
   require(!grouped.correction.defined() || (grouped.correction.dtype == DType::F32 && grouped.correction.numel() == router.shape[0]),
           "moe_route: correction " + grouped.correction.describe() + " must be float32 [experts]");
-  int rc = KERNEL("moe", ti_moe_route_grouped)(code(h.dtype, "moe_route"), h.data, (const float*)router.data,
+  require(!grouped.gate_row.defined() || (grouped.gate_row.dtype == DType::F32 && grouped.gate_row.numel() == h.shape[1] &&
+                                          grouped.gate_out.dtype == DType::F32 && grouped.gate_out.contiguous() && grouped.gate_out.numel() == M),
+          "moe_route: the gate's row " + grouped.gate_row.describe() + " or its numbers do not fit");
+  int rc = KERNEL("moe", ti_moe_route_gate)(code(h.dtype, "moe_route"), h.data, (const float*)router.data,
                                                grouped.correction.defined() ? (const float*)grouped.correction.data : nullptr,
                                                (int*)ids.data, (float*)wts.data, (int)M, (int)h.shape[1], (int)router.shape[0], top,
                                                (int)score, renormalize ? 1 : 0, grouped.groups, grouped.keep, grouped.weight_scale,
-                                               grouped.sum_floor, (hipStream_t)launch_stream());
+                                               grouped.sum_floor, grouped.gate_row.defined() ? (const float*)grouped.gate_row.data : nullptr,
+                                               grouped.gate_row.defined() ? (float*)grouped.gate_out.data : nullptr, (hipStream_t)launch_stream());
   check("moe", rc, "moe_route");
 }
 
@@ -1576,7 +1672,9 @@ void Ops::moe_experts(const Tensor& h, const Tensor& ids, const Tensor& wts, con
     int rc = KERNEL("moe_bf16", ti_moe_experts_grouped_bf16)(h.data, (const int*)ids.data, (const float*)wts.data, up.data, down.data, meta,
                                                              (int*)where.data, sorted.data, act.data, (float*)out.data,
                                                              rows ? nullptr : (float*)y.data, (int)M, (int)W, (int)F, experts, top,
-                                                             scale_input ? 1 : 0, (hipStream_t)launch_stream());
+                                                             scale_input ? 1 : 0,
+                                                             scale_input ? nullptr : (float*)ws.get("moe.row_w", (size_t)pairs * 4),
+                                                             (hipStream_t)launch_stream());
     if (rc == 0) {
       took(rows ? "[mfma, grouped, sums left]" : "[mfma, grouped]");
       if (rows) {

@@ -200,7 +200,8 @@ std::shared_ptr<Part> build_part(const std::string& family, const PartSpec& spec
 namespace {
 
 // `tensor`: the table's name in the checkpoint (default: prefix + ".weight").  `pos`: an additive position
-// encoding (a part of family "pos" with additive() true), added to every row behind the lookup.
+// encoding (a part of family "pos" with additive() true), added to every row behind the lookup.  `scale`: a factor on the
+// looked-up rows, in 32-bit (the table itself stays as it is, also for a head tied to it).
 class Embedding final : public EmbeddingPart {
  public:
   Embedding(const std::string& prefix, const Json& p, const PartChildren& children)
@@ -212,6 +213,7 @@ class Embedding final : public EmbeddingPart {
     for (const auto& c : children)
       if (c.first == "norm") norm = std::dynamic_pointer_cast<NormPart>(c.second);
     if (!norm && p.has("norm")) norm = std::dynamic_pointer_cast<NormPart>(build_part("norm", PartSpec::from_json(p.at("norm")), prefix));
+    if (p.has("scale")) scale = (float)param_float(p, "scale");
     if (norm && !norm->can_add()) throw ConfigError("embedding: the norm '" + std::string(norm->kind_name()) + "' cannot write 32-bit rows");
   }
   const char* kind_name() const override { return "table"; }
@@ -234,7 +236,7 @@ class Embedding final : public EmbeddingPart {
   }
   void load(WeightSource& src) override { weight = src.fetch(name, tensors()[0].second); }
   void forward(StepContext& ctx, const Tensor& x) override {
-    ctx.ops.embed(weight, ctx.tokens, ctx.M, x, ctx.fed_tokens, ctx.n_fed_tokens);
+    ctx.ops.embed(weight, ctx.tokens, ctx.M, x, ctx.fed_tokens, ctx.n_fed_tokens, scale);
     if (pos) pos->add(ctx, x);
     if (norm) norm->forward_add(ctx, x, x, false);
   }
@@ -242,6 +244,7 @@ class Embedding final : public EmbeddingPart {
   std::vector<std::pair<std::string, Tensor>> held() const override { return {{"weight", weight}}; }
   int64_t vocab, dim;
   std::string name;
+  float scale = 1.f;
   std::shared_ptr<PositionPart> pos;
   std::shared_ptr<NormPart> norm;      // `norm`: applied to the looked-up rows (after `pos`), in 32-bit
   Tensor weight;
@@ -328,6 +331,11 @@ class RMSNorm final : public NormPart {
     const Tensor one = src.fetch(name, tensors()[0].second);
     weight = src.alloc(DType::F32, {dim});
     spread(one, weight, src.to_host);
+  }
+  bool rms_form(Tensor& w, float& e) const override {
+    w = weight;
+    e = eps;
+    return true;
   }
   static void spread(const Tensor& one, const Tensor& all, bool on_host);     // all[:] = one[0]
   static void plus_one(const Tensor& w, const Tensor& out, bool on_host);     // out = 1 + w
@@ -528,6 +536,8 @@ class SwiGLU final : public FeedForwardPart {
   Tensor w_gate_up, w_down;
 };
 
+void put_floats(const Tensor& dst, const std::vector<float>& values, bool on_host);      // dst (device or host memory) = values
+
 const int PREFILL_TILE_Q = 128;      // query rows per work item of the tiled attention kernels
 const int PREFILL_TILE_SMALL = 64;   // and of the kernel that pairs a tile of many keys with one of few
 
@@ -548,12 +558,23 @@ class Attention final : public MixerPart {
       temp_every = (int)param_int(qt, "every");
       if (temp_every <= 0) throw ConfigError("attention: q_temp.every must be positive");
     }
-    qk_norm = p.has("qk_norm") ? p.at("qk_norm").as_bool() : true;
+    if (p.has("qk_norm") && p.at("qk_norm").type() == Json::String) {
+      if (p.at("qk_norm").as_string() != "unit_after") throw ConfigError("attention: qk_norm '" + p.at("qk_norm").as_string() + "' is not served (true, false, unit_after)");
+      qk_norm = false;
+      unit_norm = true;
+    } else {
+      qk_norm = p.has("qk_norm") ? p.at("qk_norm").as_bool() : true;
+    }
     // capped scores, a query temperature or values of another size than the keys: the kernels that serve these take
     // any sizes up to 256 and neither a per-head norm nor a rotation
     bias = p.has("bias") && p.at("bias").as_bool();
     // a sink, a gate, values from the keys or mixed with another layer's: the gated kernels (any sizes up to 256, a per-head norm too)
     has_sink = p.has("sink") && p.at("sink").as_bool();
+    if (p.has("sink_value")) {
+      if (has_sink) throw ConfigError("attention: a learned sink and a fixed one do not go together");
+      fixed_sink = true;
+      sink_value = (float)param_float(p, "sink_value");
+    }
     if (p.has("gate")) {
       const std::string g = p.at("gate").as_string();
       if (g != "entry" && g != "head") throw ConfigError("attention: gate '" + g + "' is not served (entry, head)");
@@ -565,7 +586,7 @@ class Attention final : public MixerPart {
       if (vm != "first" && vm != "mix") throw ConfigError("attention: v_mix '" + vm + "' is not served (first, mix)");
       mix_mode = vm == "first" ? 1 : 2;
     }
-    gated = has_sink || gate_mode != 0 || values_from_keys || mix_mode != 0;
+    gated = has_sink || fixed_sink || gate_mode != 0 || values_from_keys || mix_mode != 0 || unit_norm;
     if (gated) {
       if (softcap > 0.f || temp_coef != 0.f || bias || (p.has("shares_kv") && p.at("shares_kv").as_bool()))
         throw ConfigError("attention: a sink, a gate, values from the keys or mixed values go with neither capped scores, a query "
@@ -698,6 +719,10 @@ class Attention final : public MixerPart {
     if (ng) src.fill(n_gate, w_qkv.rows(nq + nk + nv, ng));
     w_o = src.alloc(src.matrix_dtype, {hidden, no});
     src.fill(n_o, w_o);
+    if (fixed_sink) {
+      sink = src.alloc(DType::F32, {(int64_t)heads});
+      put_floats(sink, std::vector<float>((size_t)heads, sink_value), src.to_host);
+    }
     if (qk_norm) {
       TensorNeed nw;
       nw.shape = {head_dim};
@@ -844,7 +869,7 @@ class Attention final : public MixerPart {
       mix.lambda = mix_lambda;
     }
     ctx.ops.gated_qkv_prep(proj, cols, q_norm_w, k_norm_w, eps, rot, mix, ctx.positions, ctx.slots, view, pool, q, heads, kv_heads,
-                           head_dim, v_dim);
+                           head_dim, v_dim, unit_norm);
     Tensor a = ctx.buf("attn.out", ctx.act_dtype, {M, no});
     Ops::AttentionGate gate;
     gate.mode = gate_mode;
@@ -926,6 +951,9 @@ class Attention final : public MixerPart {
   int heads = 0, kv_heads = 0, head_dim = 0, v_dim = 0, window = 0, temp_every = 0;
   bool qk_norm = true, shares_kv = false, general = false, bias = false;
   bool gated = false;             // any of the four below: the gated kernels run
+  bool unit_norm = false;         // `qk_norm` "unit_after": q and k heads divided by their root mean square behind the rotation
+  bool fixed_sink = false;        // `sink_value`: the same number for every head, in the place of a learned sink
+  float sink_value = 0.f;
   bool has_sink = false;          // `sink`: exp(sink_h) joins the softmax's denominator (tensor `sink_tensor`, default prefix.sink)
   int gate_mode = 0;              // `gate` "entry" (1) / "head" (2): the heads' outputs times sigmoid(W_g h) (tensor `gate_tensor`, prefix.g)
   bool values_from_keys = false;  // `values_from_keys`: no value projection; a value is its key as projected
@@ -982,17 +1010,19 @@ class PreNormBlock final : public BlockPart {
   std::shared_ptr<FeedForwardPart> ffn;
 };
 
-// down(act(up h)) with act = xIELU and its two learned numbers (p, q) in the tensor `act`:
-//   z > 0: softplus(p) z^2 + z / 2;   z <= 0: (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2.
-// The first product leaves 32-bit sums, the activation is taken in 32-bit and rounded once to the compute dtype.
+// down(act(up h)).  `activation` "xielu", with two learned numbers (p, q) in the tensor `act`:
+//   z > 0: softplus(p) z^2 + z / 2;   z <= 0: (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2;
+// "relu2": the square of relu, taken in the first product's epilogue.
+// The activation is taken in 32-bit and rounded once to the compute dtype.
 // Tensor names: prefix + ".up", ".down", ".act" unless the parameters `up`, `down`, `act` give them in full.
 class DenseFFN final : public FeedForwardPart {
  public:
   DenseFFN(const std::string& prefix, const Json& p) : FeedForwardPart(prefix) {
     hidden = param_int(p, "hidden");
     intermediate = param_int(p, "intermediate");
-    const std::string act = p.has("activation") ? p.at("activation").as_string() : "xielu";
-    if (act != "xielu") throw ConfigError("dense feed-forward: activation '" + act + "' is not served (only 'xielu')");
+    const std::string name = p.has("activation") ? p.at("activation").as_string() : "xielu";
+    if (name != "xielu" && name != "relu2") throw ConfigError("dense feed-forward: activation '" + name + "' is not served (xielu, relu2)");
+    relu2 = name == "relu2";
     if (hidden <= 0 || intermediate <= 0) throw ConfigError("dense feed-forward: sizes must be positive");
     n_up = tensor_name(p, "up", prefix, "up");
     n_down = tensor_name(p, "down", prefix, "down");
@@ -1006,6 +1036,7 @@ class DenseFFN final : public FeedForwardPart {
     TensorNeed up, down, act;
     up.shape = {intermediate, hidden};
     down.shape = {hidden, intermediate};
+    if (relu2) return {{n_up, up}, {n_down, down}};
     act.shape = {2};
     act.role = TensorNeed::Vector;
     act.a = 0.5;
@@ -1016,23 +1047,59 @@ class DenseFFN final : public FeedForwardPart {
     const auto t = tensors();
     w_up = src.fetch(n_up, t[0].second);
     w_down = src.fetch(n_down, t[1].second);
-    act = src.fetch(n_act, t[2].second);
+    if (!relu2) act = src.fetch(n_act, t[2].second);
   }
   void run(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
     const int64_t M = h.t.shape[0];
-    Tensor z = ctx.buf("ffn.z", DType::F32, {M, intermediate});
-    ctx.ops.linear(h, w_up, z, Ops::Store);
     Tensor y = ctx.buf("ffn.y", ctx.act_dtype, {M, intermediate});
-    ctx.ops.xielu(z, act, y);
+    if (relu2) {
+      ctx.ops.linear(h, w_up, y, Ops::Relu2);
+    } else {
+      Tensor z = ctx.buf("ffn.z", DType::F32, {M, intermediate});
+      ctx.ops.linear(h, w_up, z, Ops::Store);
+      ctx.ops.xielu(z, act, y);
+    }
     ctx.ops.linear(y, w_down, out, epi, epi == Ops::Add);
   }
   void forward(StepContext& ctx, const Rows& h, const Tensor& x) override { run(ctx, h, x, Ops::Add); }
   void forward_store(StepContext& ctx, const Rows& h, const Tensor& y) override { run(ctx, h, y, Ops::Store); }
   std::vector<std::pair<std::string, Tensor>> held() const override { return {{"w_up", w_up}, {"w_down", w_down}, {"act", act}}; }
   int64_t hidden = 0, intermediate = 0;
+  bool relu2 = false;
   std::string n_up, n_down, n_act;
   Tensor w_up, w_down, act;
 };
+
+// A step with a long portion for mixers with a recurrent state: every entry's tokens in chunks that run side by side, from
+// `from` tokens in one entry on.  Lists `key`.chunks [n][4] = (entry, first row, tokens, 1: the entry's first chunk + 2: its
+// last) and `key`.spans [entries][2] = (first chunk, chunks) in the step's metadata; every mixer of one key shares them, the
+// first one builds them.
+void plan_chunks(StepPlan& plan, const std::string& key, int chunk, int from) {
+  if (plan.decode_only() || plan.has(key + ".chunks")) return;
+  const auto& entries = plan.entries();
+  int longest = 0;
+  size_t n_chunks = 0;
+  for (const auto& e : entries) {
+    longest = std::max(longest, e.n_tokens);
+    n_chunks += (size_t)(e.n_tokens + chunk - 1) / chunk;
+  }
+  if (longest < from) return;
+  int* chunks = plan.ints(key + ".chunks", 4 * n_chunks);
+  int* spans = plan.ints(key + ".spans", 2 * entries.size());
+  int c = 0;
+  for (size_t i = 0; i < entries.size(); ++i) {
+    const auto& e = entries[i];
+    const int n = (e.n_tokens + chunk - 1) / chunk;
+    spans[2 * i] = c;
+    spans[2 * i + 1] = n;
+    for (int k = 0; k < n; ++k, ++c) {
+      chunks[4 * c] = (int)i;
+      chunks[4 * c + 1] = e.row0 + k * chunk;
+      chunks[4 * c + 2] = std::min(chunk, e.n_tokens - k * chunk);
+      chunks[4 * c + 3] = (k == 0 ? 1 : 0) | (k == n - 1 ? 2 : 0);
+    }
+  }
+}
 
 // The mLSTM cell.  With q = W_q h / sqrt(dk), k = W_k h (heads x dk), v = W_v h (heads x dv) and per head a log
 // input gate i = cap tanh((W_i h + b_i) / cap) and a log forget gate f = logsigmoid(cap tanh((W_f h + b_f) / cap)):
@@ -1114,32 +1181,7 @@ class MLSTM final : public MixerPart {
   // side by side and from chunk to chunk element-wise), from CHUNK_FROM tokens on, where three chunks or more make up
   // for walking the tokens twice.  The lists are the same for every mLSTM of the model; the first one builds them.
   static constexpr int CHUNK = 64, CHUNK_FROM = 192;
-  void plan(StepPlan& plan) const override {
-    if (plan.decode_only() || plan.has("mlstm.chunks")) return;
-    const auto& entries = plan.entries();
-    int longest = 0;
-    size_t n_chunks = 0;
-    for (const auto& e : entries) {
-      longest = std::max(longest, e.n_tokens);
-      n_chunks += (size_t)(e.n_tokens + CHUNK - 1) / CHUNK;
-    }
-    if (longest < CHUNK_FROM) return;
-    int* chunks = plan.ints("mlstm.chunks", 4 * n_chunks);
-    int* spans = plan.ints("mlstm.spans", 2 * entries.size());
-    int c = 0;
-    for (size_t i = 0; i < entries.size(); ++i) {
-      const auto& e = entries[i];
-      const int n = (e.n_tokens + CHUNK - 1) / CHUNK;
-      spans[2 * i] = c;
-      spans[2 * i + 1] = n;
-      for (int k = 0; k < n; ++k, ++c) {
-        chunks[4 * c] = (int)i;
-        chunks[4 * c + 1] = e.row0 + k * CHUNK;
-        chunks[4 * c + 2] = std::min(CHUNK, e.n_tokens - k * CHUNK);
-        chunks[4 * c + 3] = (k == 0 ? 1 : 0) | (k == n - 1 ? 2 : 0);
-      }
-    }
-  }
+  void plan(StepPlan& plan) const override { plan_chunks(plan, "mlstm", CHUNK, CHUNK_FROM); }
   void run(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
     const int64_t M = h.t.shape[0];
     Tensor proj = ctx.buf("mlstm.proj", DType::F32, {M, width});
@@ -1291,6 +1333,10 @@ class AddVectorBlock final : public BlockPart {
 // interpolates the frequencies as YaRN does: with dim(t) = dims ln(original / (2 pi t)) / (2 ln base),
 // lo = max(floor(dim(fast)), 0), hi = min(ceil(dim(slow)), dims - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1),
 // the frequency is f_i / factor * ramp_i + f_i (1 - ramp_i), and cosine and sine are multiplied by 0.1 ln(factor) + 1.
+// `scaling` {kind "wavelength", factor, low, high, original} stretches by wavelength: with n = original f_i / (2 pi) whole turns
+// inside the original length, f_i is kept where n > high, divided by factor where n < low, and in between, with
+// s = (n - low) / (high - low), it is (1 - s) f_i / factor + s f_i; cosine and sine are left as they are.
+// `layout` "pairs": entries 2i and 2i + 1 turn together by the angle pos * f_i (default "half", as above).
 // Frequencies and, for the positions an engine serves, cosines and sines are built on the host in double precision
 // and rounded once; a table is immutable and lives as long as the part (captured graphs hold its address).
 class RotaryPartial final : public PositionPart {
@@ -1300,7 +1346,16 @@ class RotaryPartial final : public PositionPart {
     base = param_float(p, "base");
     if (dims < 0 || dims % 2) throw ConfigError("rotary: " + std::to_string(dims) + " rotated entries: must be even and not negative");
     if (!(base > 0.0)) throw ConfigError("rotary: base must be positive");
-    if (p.has("scaling")) {
+    if (p.has("layout")) {
+      const std::string layout = p.at("layout").as_string();
+      if (layout != "half" && layout != "pairs") throw ConfigError("rotary: layout '" + layout + "' is not served (half, pairs)");
+      pairs = layout == "pairs";
+    }
+    const bool wavelength = p.has("scaling") && p.at("scaling").has("kind");
+    if (wavelength) {
+      const std::string kind = p.at("scaling").at("kind").as_string();
+      if (kind != "wavelength") throw ConfigError("rotary: scaling '" + kind + "' is not served");
+    } else if (p.has("scaling")) {
       const Json& sc = p.at("scaling");
       factor = param_float(sc, "factor");
       original = param_float(sc, "original");
@@ -1313,6 +1368,18 @@ class RotaryPartial final : public PositionPart {
     const int half = dims / 2;
     freq.resize(half);
     for (int i = 0; i < half; ++i) freq[i] = std::pow(base, -2.0 * i / dims);
+    if (wavelength) {
+      const Json& sc = p.at("scaling");
+      const double by = param_float(sc, "factor"), low = param_float(sc, "low"), high = param_float(sc, "high");
+      const double length = param_float(sc, "original"), pi = 3.14159265358979323846;
+      if (!(by > 0.0) || !(length > 0.0) || !(low > 0.0) || !(high >= low)) throw ConfigError("rotary: scaling factor, original, low and high must be positive, low at most high");
+      for (int i = 0; i < half; ++i) {
+        const double turns = length * freq[i] / (2.0 * pi);
+        if (turns > high) continue;
+        const double s = turns < low || high == low ? 0.0 : (turns - low) / (high - low);
+        freq[i] = (1.0 - s) * freq[i] / by + s * freq[i];
+      }
+    }
     if (scaled) {
       const double pi = 3.14159265358979323846;
       auto dim_of = [&](double turns) { return dims * std::log(original / (2.0 * pi * turns)) / (2.0 * std::log(base)); };
@@ -1354,6 +1421,7 @@ class RotaryPartial final : public PositionPart {
     rot.table = tables.empty() ? nullptr : (const float*)tables.back().data();
     rot.table_len = table_len;
     rot.dims = dims;
+    rot.pairs = pairs;
     rot.mag = (float)mag;
     return true;
   }
@@ -1368,7 +1436,7 @@ class RotaryPartial final : public PositionPart {
   }
   int dims = 0;
   double base = 10000.0, factor = 1.0, original = 0.0, fast = 0.0, slow = 0.0, mag = 1.0;
-  bool scaled = false;
+  bool scaled = false, pairs = false;
   std::vector<double> freq;
   DeviceBuffer inv_freq;
   std::vector<DeviceBuffer> tables;     // oldest first; the last one is read
@@ -1666,7 +1734,9 @@ class DiffAttention final : public MixerPart {
 // [intermediate, hidden], ".e<i>.down"), of which each token uses the `top` with the largest scores.  Router logits
 // W_router h and the scores (`score`: "sigmoid", or "softmax" over all experts) are 32-bit; `renormalize`: the chosen
 // scores are divided by their sum.  `scale_input` true: the score multiplies the expert's input, the output is
-// sum_e expert_e(s_e h); false: its output.  `activation`: "relu2", the square of relu.
+// sum_e expert_e(s_e h); false: its output.  `activation`: "relu2", the square of relu.  `shared_gate`: the output of the
+// `shared` feed-forward is multiplied by sigmoid(w . h), one number a token (tensor `shared_gate_tensor` [1, hidden], default
+// prefix.shared.gate); the router's kernel takes that row along.
 class MoE final : public FeedForwardPart {
  public:
   MoE(const std::string& prefix, const Json& p, const PartChildren& children = {}) : FeedForwardPart(prefix) {
@@ -1719,6 +1789,9 @@ class MoE final : public FeedForwardPart {
       const PartSpec sp = PartSpec::from_json(p.at("shared"));
       shared = std::dynamic_pointer_cast<FeedForwardPart>(build_part("ffn", sp, join(prefix, sp.name)));
     }
+    shared_gate = p.has("shared_gate") && p.at("shared_gate").as_bool();
+    n_shared_gate = tensor_name(p, "shared_gate_tensor", prefix, "shared.gate");
+    if (shared_gate && !shared) throw ConfigError("moe: a gate on the shared feed-forward needs one");
     if (shared && !shared->can_store()) throw ConfigError("moe: the shared feed-forward must be able to write its output apart from the residual");
   }
   std::vector<std::shared_ptr<Part>> children() const override {
@@ -1747,6 +1820,13 @@ class MoE final : public FeedForwardPart {
       t.emplace_back(expert_name(e, "down"), down);
     }
     t.emplace_back(n_router, router);
+    if (shared_gate) {
+      TensorNeed g;
+      g.shape = {1, hidden};
+      g.role = TensorNeed::Vector;
+      g.b = 0.1;
+      t.emplace_back(n_shared_gate, g);
+    }
     if (corrected) {
       TensorNeed c;
       c.shape = {(int64_t)experts};
@@ -1771,6 +1851,12 @@ class MoE final : public FeedForwardPart {
     router.shape = {(int64_t)experts, hidden};
     router.role = TensorNeed::Vector;
     w_router = src.fetch(n_router, router);
+    if (shared_gate) {
+      TensorNeed g;
+      g.shape = {1, hidden};
+      g.role = TensorNeed::Vector;
+      w_shared_gate = src.fetch(n_shared_gate, g);
+    }
     if (corrected) {
       TensorNeed c;
       c.shape = {(int64_t)experts};
@@ -1783,13 +1869,17 @@ class MoE final : public FeedForwardPart {
     const int64_t M = rows.shape[0];
     Tensor ids = ctx.buf("moe.ids", DType::I32, {M, (int64_t)top});
     Tensor wts = ctx.buf("moe.wts", DType::F32, {M, (int64_t)top});
-    if (corrected || groups > 1 || weight_scale != 1.f || sum_floor != 0.f) {
+    if (corrected || groups > 1 || weight_scale != 1.f || sum_floor != 0.f || shared_gate) {
       Ops::RouterGroups g;
       g.correction = correction;
       g.groups = groups;
       g.keep = keep;
       g.weight_scale = weight_scale;
       g.sum_floor = sum_floor;
+      if (shared_gate) {
+        g.gate_row = w_shared_gate;
+        g.gate_out = gate_numbers(ctx, M);
+      }
       ctx.ops.moe_route(rows, w_router, ids, wts, top, score, renormalize, g);
     } else {
       ctx.ops.moe_route(rows, w_router, ids, wts, top, score, renormalize);
@@ -1802,11 +1892,21 @@ class MoE final : public FeedForwardPart {
     if (shared) {      // the expert every token takes, added in 32-bit
       Tensor ys = ctx.buf("moe.shared", DType::F32, {y.shape[0], hidden});
       shared->forward_store(ctx, h, ys);
-      ctx.ops.scaled_add(y, ys, Tensor(), Tensor(), Tensor());
+      if (shared_gate) ctx.ops.add_gated_rows(y, ys, gate_numbers(ctx, y.shape[0]));
+      else ctx.ops.scaled_add(y, ys, Tensor(), Tensor(), Tensor());
     }
   }
-  // the sum over a token's experts may be left to the norm that reads the result
-  void forward_rows(StepContext& ctx, const Rows& h, const Tensor& y, Ops::GatheredRows& rows) override {
+  Tensor gate_numbers(StepContext& ctx, int64_t M) const { return ctx.buf("moe.shared_gate", DType::F32, {M}); }
+  // the sum over a token's experts may be left to the norm that reads the result, the shared branch beside it where it takes one
+  void forward_rows(StepContext& ctx, const Rows& h, const Tensor& y, Ops::GatheredRows& rows, bool takes_plus) override {
+    if (shared && takes_plus) {
+      run(ctx, h, y, &rows);
+      if (!rows.t.defined()) rows.t = y;
+      rows.plus = ctx.buf("moe.shared", DType::F32, {y.shape[0], hidden});
+      shared->forward_store(ctx, h, rows.plus);
+      if (shared_gate) rows.plus_gate = gate_numbers(ctx, y.shape[0]);
+      return;
+    }
     if (shared) {
       forward_store(ctx, h, y);
       rows = Ops::GatheredRows();
@@ -1821,7 +1921,9 @@ class MoE final : public FeedForwardPart {
     forward_store(ctx, h, y);
     ctx.ops.scaled_add(x, y, Tensor(), Tensor(), Tensor());
   }
-  std::vector<std::pair<std::string, Tensor>> held() const override { return {{"w_up", w_up}, {"w_down", w_down}, {"w_router", w_router}}; }
+  std::vector<std::pair<std::string, Tensor>> held() const override {
+    return {{"w_up", w_up}, {"w_down", w_down}, {"w_router", w_router}, {"w_shared_gate", w_shared_gate}};
+  }
   int64_t hidden = 0, intermediate = 0;
   int experts = 0, top = 0;
   Ops::RouterScore score = Ops::Sigmoid;
@@ -1830,11 +1932,12 @@ class MoE final : public FeedForwardPart {
   Ops::GatedAct act_kind = Ops::Silu;
   float limit = 0.f, alpha = 1.702f;       // glu_clamped: g = min(g, limit), u = clamp(u, -limit, limit), g sigmoid(alpha g) (u + 1)
   std::shared_ptr<FeedForwardPart> shared; // `shared`: a feed-forward every token takes, added to the experts' sum
-  std::string n_router, n_correction;
+  bool shared_gate = false;                // `shared_gate`: ... times sigmoid of one row against h
+  std::string n_router, n_correction, n_shared_gate;
   bool corrected = false;                  // `correction`: a vector added to the scores for the choice only (tensor prefix.correction)
   int groups = 0, keep = 0;                // `groups` {count, keep}: only experts of the best `keep` of `count` groups can be chosen
   float weight_scale = 1.f, sum_floor = 0.f;
-  Tensor w_up, w_down, w_router, correction;
+  Tensor w_up, w_down, w_router, correction, w_shared_gate;
 };
 
 // Dynamic Tanh in the place of a norm: y = tanh(alpha x) * w + b, alpha one learned number, w and b vectors; no mean and no
@@ -1968,7 +2071,9 @@ class GatedFFN final : public FeedForwardPart {
 // head's last rot_dim query entries are.  A head's unrotated key is W_uk c (head_dim rows a head), its value W_uv c
 // (v_head_dim rows a head); score = (q_plain . k_plain + q_rot . k_rot) scale; causal (`window` optional); the softmax's
 // denominator also holds exp(sink_h), a learned number a head (`sink`, optional).  Then the output projection.
-// Scores, softmax, the latent's norm and the rotation are 32-bit.  Tensor names: prefix + ".q", ".dkv", ".dkv.norm", ".uk",
+// `q_rank` (with no rotated part): the queries come from a latent of their own, W_uq c_q with c_q = W_dq h divided by its root
+// mean square and multiplied by the vector `dq.norm` (tensors ".dq", ".dq.norm", ".uq" in the place of ".q").
+// Scores, softmax, the latents' norms and the rotation are 32-bit.  Tensor names: prefix + ".q", ".dkv", ".dkv.norm", ".uk",
 // ".uv", ".sink", ".o".  Where the sizes allow (a latent of a multiple of 16 up to 512, latent and key part together a
 // multiple of 8 up to 576, an unrotated query size that is a multiple of 8, a value size that is a multiple of 16) a page holds
 // the latents a second time, transposed, and bfloat16 steps run on the matrix cores.
@@ -1989,6 +2094,8 @@ class LatentAttention final : public MixerPart {
     scale = p.has("scale") ? (float)param_float(p, "scale") : (float)(1.0 / std::sqrt((double)(dim + rot_dim)));
     window = p.has("window") ? (int)param_int(p, "window") : 0;
     has_sink = !p.has("sink") || p.at("sink").as_bool();
+    q_rank = p.has("q_rank") ? (int)param_int(p, "q_rank") : 0;
+    if (q_rank < 0 || (q_rank > 0 && rot_dim > 0)) throw ConfigError("latent_attention: queries from a latent of their own go with no rotated part");
     for (const auto& c : children)
       if (c.first == "pos") pos = std::dynamic_pointer_cast<PositionPart>(c.second);
     if (!pos && p.has("pos")) pos = std::dynamic_pointer_cast<PositionPart>(build_part("pos", PartSpec::from_json(p.at("pos")), prefix));
@@ -2024,19 +2131,32 @@ class LatentAttention final : public MixerPart {
     sk.role = TensorNeed::Vector;
     sk.b = 1.0;
     o.shape = {hidden, (int64_t)heads * v_dim};
-    std::vector<std::pair<std::string, TensorNeed>> t = {{name("q"), q}, {name("dkv"), dkv}, {name("dkv.norm"), nw}, {name("uk"), uk},
-                                                         {name("uv"), uv}};
+    std::vector<std::pair<std::string, TensorNeed>> t;
+    if (q_rank) {
+      TensorNeed dq, dqn, uq;
+      dq.shape = {(int64_t)q_rank, hidden};
+      dqn = nw;
+      dqn.shape = {(int64_t)q_rank};
+      uq.shape = {nq, (int64_t)q_rank};
+      t = {{name("dq"), dq}, {name("dq.norm"), dqn}, {name("uq"), uq}};
+    } else {
+      t = {{name("q"), q}};
+    }
+    t.insert(t.end(), {{name("dkv"), dkv}, {name("dkv.norm"), nw}, {name("uk"), uk}, {name("uv"), uv}});
     if (has_sink) t.emplace_back(name("sink"), sk);
     t.emplace_back(name("o"), o);
     return t;
   }
   void load(WeightSource& src) override {
     const auto t = tensors();
-    w_in = src.alloc(src.matrix_dtype, {nq + nkv, hidden});      // queries above the down-projection: one product
-    src.fill(name("q"), w_in.rows(0, nq));
-    src.fill(name("dkv"), w_in.rows(nq, nkv));
+    const int64_t above = q_rank ? q_rank : nq;                     // the queries (or their latent) above the down-projection: one product
+    w_in = src.alloc(src.matrix_dtype, {above + nkv, hidden});
+    src.fill(q_rank ? name("dq") : name("q"), w_in.rows(0, above));
+    src.fill(name("dkv"), w_in.rows(above, nkv));
     for (const auto& kv : t) {
       if (kv.first == name("dkv.norm")) norm_w = src.fetch(kv.first, kv.second);
+      if (kv.first == name("dq.norm")) q_norm_w = src.fetch(kv.first, kv.second);
+      if (kv.first == name("uq")) w_uq = src.fetch(kv.first, kv.second);
       if (kv.first == name("uk")) w_uk = src.fetch(kv.first, kv.second);
       if (kv.first == name("uv")) w_uv = src.fetch(kv.first, kv.second);
       if (kv.first == name("sink")) sink = src.fetch(kv.first, kv.second);
@@ -2113,15 +2233,32 @@ class LatentAttention final : public MixerPart {
   }
   void run(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
     const int64_t M = h.t.shape[0];
-    Tensor proj = ctx.buf("latent.proj", DType::F32, {M, nq + nkv});
+    const int64_t above = q_rank ? q_rank : nq;
+    Tensor proj = ctx.buf("latent.proj", DType::F32, {M, above + nkv});
     ctx.ops.linear(h, w_in, proj, Ops::Store);
     const auto bound = ctx.binding(this);
     const Tensor pool = ctx.kv_pool(bound.first, bound.second);
     const Ops::CacheView view = ctx.cache_view(bound.first);
     Ops::Rotation rot;
+    if (q_rank) {
+      // both latents normed by one kernel, then the queries from theirs
+      Ops::QueryLatent ql;
+      ql.rank = q_rank;
+      ql.norm_w = q_norm_w;
+      ql.out = ctx.buf("latent.cq", ctx.act_dtype, {M, (int64_t)q_rank});
+      ctx.ops.latent_prep(proj, (int)above, norm_w, eps, ql, ctx.positions, ctx.slots, view, pool, rank);
+      proj = ctx.buf("latent.q", DType::F32, {M, nq});
+      ctx.ops.linear(ql.out, w_uq, proj, Ops::Store);
+      attend(ctx, proj, pool, view, out, epi);
+      return;
+    }
     if (pos && !pos->fused(rot)) throw EngineError("latent_attention: the position encoding '" + std::string(pos->kind_name()) + "' has no fused form");
     ctx.ops.latent_prep(proj, (int)nq, norm_w, eps, rot, ctx.positions, ctx.slots, view, pool, heads, dim, rot_dim, rank);
-    Tensor a = ctx.buf("latent.out", ctx.act_dtype, {M, (int64_t)heads * v_dim});
+    attend(ctx, proj, pool, view, out, epi);
+  }
+  // proj: the heads' queries from column 0 on
+  void attend(StepContext& ctx, const Tensor& proj, const Tensor& pool, const Ops::CacheView& view, const Tensor& out, Ops::Epilogue epi) {
+    Tensor a = ctx.buf("latent.out", ctx.act_dtype, {proj.shape[0], (int64_t)heads * v_dim});
     const Ops::LatentLists l = lists(ctx);
     ctx.ops.latent_attention(proj, w_uk, w_uv, sink, pool, view, ctx.positions, ctx.slots, a, heads, dim, rot_dim, rank, v_dim, scale,
                              window, ctx.ws, w_uk_t, transposed && ctx.plan ? &l : nullptr);
@@ -2130,16 +2267,18 @@ class LatentAttention final : public MixerPart {
   void forward(StepContext& ctx, const Rows& h, const Tensor& x) override { run(ctx, h, x, Ops::Add); }
   void forward_store(StepContext& ctx, const Rows& h, const Tensor& y) override { run(ctx, h, y, Ops::Store); }
   std::vector<std::pair<std::string, Tensor>> held() const override {
-    return {{"w_in", w_in}, {"norm_w", norm_w}, {"w_uk", w_uk}, {"w_uv", w_uv}, {"sink", sink}, {"w_o", w_o}, {"w_uk_t", w_uk_t}};
+    return {{"w_in", w_in}, {"norm_w", norm_w}, {"w_uk", w_uk}, {"w_uv", w_uv}, {"sink", sink}, {"w_o", w_o}, {"w_uk_t", w_uk_t},
+            {"q_norm_w", q_norm_w}, {"w_uq", w_uq}};
   }
   int64_t hidden = 0, nq = 0, nkv = 0;
   int heads = 0, dim = 0, rot_dim = 0, v_dim = 0, rank = 0, window = 0;
+  int q_rank = 0;               // `q_rank` > 0: the queries come from a normed latent of this size
   bool has_sink = true;
   bool transposed = false;      // the pages hold the latents transposed as well (sizes the matrix-core kernels take)
   bool uk_transposed = false;   // w_uk_t has been filled
   float eps = 1e-6f, scale = 1.f;
   std::shared_ptr<PositionPart> pos;
-  Tensor w_in, norm_w, w_uk, w_uv, sink, w_o;
+  Tensor w_in, norm_w, w_uk, w_uv, sink, w_o, q_norm_w, w_uq;
   Tensor w_uk_t;                // bfloat16: every head's W_uk transposed, [heads][rank][dim]
 };
 
@@ -2552,7 +2691,6 @@ class DecayAttention final : public MixerPart {
     w_decay = src.alloc(DType::F32, {(int64_t)heads});
     put_floats(w_decay, decay, src.to_host);
   }
-  static void put_floats(const Tensor& dst, const std::vector<float>& values, bool on_host);
   bool has_cache() const override { return true; }
   CacheNeed cache_need() const override {
     CacheNeed n;
@@ -2564,32 +2702,7 @@ class DecayAttention final : public MixerPart {
   // to chunk element by element), from CHUNK_FROM tokens on.  The lists are the same for every such mixer of the model; the
   // first one builds them.
   static constexpr int CHUNK = 64, CHUNK_FROM = 128;
-  void plan(StepPlan& plan) const override {
-    if (plan.decode_only() || plan.has("decay.chunks")) return;
-    const auto& entries = plan.entries();
-    int longest = 0;
-    size_t n_chunks = 0;
-    for (const auto& e : entries) {
-      longest = std::max(longest, e.n_tokens);
-      n_chunks += (size_t)(e.n_tokens + CHUNK - 1) / CHUNK;
-    }
-    if (longest < CHUNK_FROM) return;
-    int* chunks = plan.ints("decay.chunks", 4 * n_chunks);
-    int* spans = plan.ints("decay.spans", 2 * entries.size());
-    int c = 0;
-    for (size_t i = 0; i < entries.size(); ++i) {
-      const auto& e = entries[i];
-      const int n = (e.n_tokens + CHUNK - 1) / CHUNK;
-      spans[2 * i] = c;
-      spans[2 * i + 1] = n;
-      for (int k = 0; k < n; ++k, ++c) {
-        chunks[4 * c] = (int)i;
-        chunks[4 * c + 1] = e.row0 + k * CHUNK;
-        chunks[4 * c + 2] = std::min(CHUNK, e.n_tokens - k * CHUNK);
-        chunks[4 * c + 3] = (k == 0 ? 1 : 0) | (k == n - 1 ? 2 : 0);
-      }
-    }
-  }
+  void plan(StepPlan& plan) const override { plan_chunks(plan, "decay", CHUNK, CHUNK_FROM); }
   void run(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
     const int64_t M = h.t.shape[0];
     Tensor proj = ctx.buf("decay.proj", DType::F32, {M, width});
@@ -2617,6 +2730,208 @@ class DecayAttention final : public MixerPart {
   float eps = 1e-6f;
   std::vector<float> decay;
   Tensor w_in, w_o, norm_w, w_decay;
+};
+
+// A minimal GRU: an element-wise recurrence over `width` channels whose gate and candidate read the current token only.
+// s = sigmoid(W_z h + b_z), u = W_x h + b_x, the candidate c = u + 1/2 where u >= 0 and sigmoid(u) elsewhere,
+// S_t = (1 - s) S_(t-1) + s c, and the output W_o (S_t silu(W_g h)).  z, x and g come from one product with the stacked weight
+// [z; x; g] (32-bit sums), the gates, the recurrence and the output's gate are 32-bit, the gated rows are rounded once.  S is
+// per-request state in 32-bit, zero at admission.  Tensor names: prefix + ".z", ".z.b", ".x", ".x.b", ".g", ".o".
+class MinGRU final : public MixerPart {
+ public:
+  MinGRU(const std::string& prefix, const Json& p) : MixerPart(prefix) {
+    hidden = param_int(p, "hidden");
+    width = param_int(p, "width");
+    if (hidden <= 0 || width <= 0) throw ConfigError("mingru: sizes must be positive");
+  }
+  const char* kind_name() const override { return "mingru"; }
+  bool takes_lazy_norm() const override { return true; }
+  bool reads_through_ops() const override { return true; }
+  bool can_store() const override { return true; }
+  std::string name(const char* t) const { return join(prefix, t); }
+  std::vector<std::pair<std::string, TensorNeed>> tensors() const override {
+    TensorNeed in, o, b;
+    in.shape = {width, hidden};
+    o.shape = {hidden, width};
+    b.shape = {width};
+    b.role = TensorNeed::Vector;
+    b.b = 0.5;
+    return {{name("z"), in}, {name("z.b"), b}, {name("x"), in}, {name("x.b"), b}, {name("g"), in}, {name("o"), o}};
+  }
+  void load(WeightSource& src) override {
+    w_in = src.alloc(src.matrix_dtype, {3 * width, hidden});
+    src.fill(name("z"), w_in.rows(0, width));
+    src.fill(name("x"), w_in.rows(width, width));
+    src.fill(name("g"), w_in.rows(2 * width, width));
+    const auto t = tensors();
+    b_z = src.fetch(t[1].first, t[1].second);
+    b_x = src.fetch(t[3].first, t[3].second);
+    w_o = src.fetch(t[5].first, t[5].second);
+  }
+  bool has_cache() const override { return true; }
+  CacheNeed cache_need() const override {
+    CacheNeed n;
+    n.kind = CacheNeed::State;
+    n.state_shape = {width};
+    return n;
+  }
+  // a chunk is a multiple of 64 tokens, no more than 64 chunks an entry: a chunk folds the maps of all chunks in front of it
+  static constexpr int CHUNK = 64, MOST_CHUNKS = 64, CHUNK_FROM = 128;
+  void plan(StepPlan& plan) const override {
+    int longest = 0;
+    for (const auto& e : plan.entries()) longest = std::max(longest, e.n_tokens);
+    const int blocks = (longest + CHUNK * MOST_CHUNKS - 1) / (CHUNK * MOST_CHUNKS);
+    plan_chunks(plan, "mingru", CHUNK * std::max(1, blocks), CHUNK_FROM);
+  }
+  void run(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
+    const int64_t M = h.t.shape[0];
+    Tensor proj = ctx.buf("mingru.proj", DType::F32, {M, 3 * width});
+    ctx.ops.linear(h, w_in, proj, Ops::Store);
+    const auto bound = ctx.binding(this);
+    Ops::GruColumns cols;
+    cols.x = (int)width;
+    cols.g = (int)(2 * width);
+    Tensor y = ctx.buf("mingru.y", ctx.act_dtype, {M, width});
+    ctx.ops.mingru_scan(proj, cols, b_z, b_x, ctx.state(bound.first, bound.second), ctx.entry_meta, (int)ctx.entries.size(), y, (int)width,
+                        ctx.planned("mingru.chunks"), (int)(ctx.planned_size("mingru.chunks") / 4), ctx.planned("mingru.spans"), &ctx.ws);
+    ctx.ops.linear(y, w_o, out, epi, epi == Ops::Add);
+  }
+  void forward(StepContext& ctx, const Rows& h, const Tensor& x) override { run(ctx, h, x, Ops::Add); }
+  void forward_store(StepContext& ctx, const Rows& h, const Tensor& y) override { run(ctx, h, y, Ops::Store); }
+  std::vector<std::pair<std::string, Tensor>> held() const override { return {{"w_in", w_in}, {"b_z", b_z}, {"b_x", b_x}, {"w_o", w_o}}; }
+  int64_t hidden = 0, width = 0;
+  Tensor w_in, b_z, b_x, w_o;
+};
+
+// A norm in front of every sublayer and another behind it: x += norm1b(mixer(norm1(x))); x += norm2b(ffn(norm2(x))).  The
+// sublayers write apart from the residual.  Where both norms at hand are plain RMS norms, the norm behind a sublayer, the
+// residual sum and the norm in front of the next sublayer are one kernel (Ops::norm_residual_next), which also adds what the
+// feed-forward left unsummed: within a layer directly, from layer to layer through a note in the step's context
+// (`defer_write`: the layer's last write is left to the next layer of this kind).  A layer may have no feed-forward (then no
+// norm2 and norm2b either).
+const char* const SANDWICH_PENDING = "sandwich.pending";
+class SandwichBlock final : public BlockPart {
+ public:
+  SandwichBlock(const std::string& prefix, const Json& p, const PartChildren& c) : BlockPart(prefix) {
+    auto norm = [](const std::shared_ptr<Part>& part) { return std::dynamic_pointer_cast<NormPart>(part); };
+    for (const auto& kv : c) {
+      if (kv.first == "norm1") norm1 = norm(kv.second);
+      if (kv.first == "norm1b") norm1b = norm(kv.second);
+      if (kv.first == "norm2") norm2 = norm(kv.second);
+      if (kv.first == "norm2b") norm2b = norm(kv.second);
+      if (kv.first == "mixer") mixer = std::dynamic_pointer_cast<MixerPart>(kv.second);
+      if (kv.first == "ffn") ffn = std::dynamic_pointer_cast<FeedForwardPart>(kv.second);
+    }
+    if (!norm1 || !norm1b || !mixer) throw ConfigError("block 'sandwich' needs norm1, mixer and norm1b parts (norm2, ffn and norm2b are optional)");
+    if ((ffn != nullptr) != (norm2 != nullptr) || (ffn != nullptr) != (norm2b != nullptr))
+      throw ConfigError("block 'sandwich': norm2, ffn and norm2b come together or not at all");
+    if (!norm1b->can_add() || (norm2b && !norm2b->can_add())) throw ConfigError("block 'sandwich': the norms behind its sublayers must be able to write into the residual");
+    if (!mixer->can_store() || (ffn && !ffn->can_store()))
+      throw ConfigError("block 'sandwich': its mixer and feed-forward must be able to write their output apart from the residual");
+    defer_write = p.has("defer_write") && p.at("defer_write").as_bool();
+    if (p.has("spare"))
+      for (const Json& t : p.at("spare").items()) spare.push_back(t.as_string());
+    if (!spare.empty()) dim = param_int(p, "dim");
+  }
+  const char* kind_name() const override { return "sandwich"; }
+  // `spare` (with `dim`): vectors that a checkpoint may carry for a layer that does not use them
+  std::vector<std::pair<std::string, TensorNeed>> tensors() const override {
+    std::vector<std::pair<std::string, TensorNeed>> t;
+    for (const std::string& n : spare) {
+      TensorNeed v;
+      v.shape = {dim};
+      v.role = TensorNeed::Vector;
+      v.optional = true;
+      t.emplace_back(n, v);
+    }
+    return t;
+  }
+  bool reads_through_ops() const override { return true; }
+  std::vector<std::shared_ptr<Part>> children() const override {
+    std::vector<std::shared_ptr<Part>> v = {norm1, mixer, norm1b};
+    if (ffn) v.insert(v.end(), {norm2, ffn, norm2b});
+    return v;
+  }
+  std::vector<std::string> child_slots() const override {
+    std::vector<std::string> v = {"norm1", "mixer", "norm1b"};
+    if (ffn) v.insert(v.end(), {"norm2", "ffn", "norm2b"});
+    return v;
+  }
+  // what a sublayer left for the residual: rows (their sum, a further branch) behind a norm of the given gain
+  struct Write {
+    Ops::GatheredRows rows;
+    Tensor gain;
+    float eps = 0.f;
+  };
+  // x += the write, then what `front` makes of x
+  static Rows write_read(StepContext& ctx, const Tensor& x, const Write& w, NormPart& front) {
+    Tensor gain;
+    float eps = 0.f;
+    if (front.rms_form(gain, eps)) {
+      Rows h;
+      h.t = ctx.buf("norm.out", ctx.act_dtype, {x.shape[0], x.shape[1]});
+      ctx.ops.norm_residual_next(x, w.rows.t, w.rows.gather, w.rows.n_gather, w.rows.plus, w.rows.plus_gate, w.gain, w.eps, gain, eps, h.t);
+      return h;
+    }
+    write(ctx, x, w);
+    return front.forward(ctx, x);
+  }
+  static void write(StepContext& ctx, const Tensor& x, const Write& w) {
+    ctx.ops.norm_residual_next(x, w.rows.t, w.rows.gather, w.rows.n_gather, w.rows.plus, w.rows.plus_gate, w.gain, w.eps);
+  }
+  void forward(StepContext& ctx, const Tensor& x) override {
+    ctx.ops.flush();
+    const int64_t M = x.shape[0];
+    Tensor y = ctx.buf("sandwich.y", DType::F32, {M, x.shape[1]});
+    Rows h;
+    const auto left = ctx.notes.find(SANDWICH_PENDING);
+    if (left != ctx.notes.end()) {      // the last write of the layer before
+      const StepContext::Note note = left->second;
+      ctx.notes.erase(left);
+      Write w;
+      w.rows.t = note.tensors[0];
+      w.rows.gather = note.tensors[1].ptr<int>();
+      w.rows.n_gather = (int)note.numbers[0];
+      w.rows.plus = note.tensors[2];
+      w.rows.plus_gate = note.tensors[3];
+      w.gain = note.tensors[4];
+      w.eps = (float)note.numbers[1];
+      h = write_read(ctx, x, w, *norm1);
+    } else {
+      h = norm1->forward(ctx, x, nullptr, 0, mixer->takes_lazy_norm() && norm1->can_be_lazy());
+    }
+    if (!mixer->reads_through_ops()) ctx.ops.flush();
+    mixer->forward_store(ctx, h, y);
+    Write w;
+    w.rows.t = y;
+    bool fusable = norm1b->rms_form(w.gain, w.eps);
+    if (ffn) {
+      if (fusable) {
+        h = write_read(ctx, x, w, *norm2);
+      } else {
+        norm1b->forward_add(ctx, y, x, true);
+        h = norm2->forward(ctx, x);
+      }
+      if (!ffn->reads_through_ops()) ctx.ops.flush();
+      fusable = norm2b->rms_form(w.gain, w.eps);
+      ffn->forward_rows(ctx, h, y, w.rows, fusable);
+    }
+    if (!fusable) {
+      (ffn ? norm2b : norm1b)->forward_add(ctx, w.rows.t, x, true, w.rows.gather, w.rows.n_gather);
+    } else if (defer_write) {
+      Tensor list;
+      if (w.rows.gather) list = Tensor((void*)w.rows.gather, DType::I32, {M, (int64_t)w.rows.n_gather});
+      ctx.notes[SANDWICH_PENDING] = StepContext::Note{{w.rows.t, list, w.rows.plus, w.rows.plus_gate, w.gain}, {(double)w.rows.n_gather, (double)w.eps}};
+    } else {
+      write(ctx, x, w);
+    }
+  }
+  std::shared_ptr<NormPart> norm1, norm1b, norm2, norm2b;
+  std::shared_ptr<MixerPart> mixer;
+  std::shared_ptr<FeedForwardPart> ffn;
+  bool defer_write = false;
+  std::vector<std::string> spare;
+  int64_t dim = 0;
 };
 
 // Two mixers side by side on the same input: y = left_scale * left(h) + right_scale * right(h), added in 32-bit.  `left`,
@@ -2649,8 +2964,8 @@ class SumMixer final : public MixerPart {
   void load(WeightSource& src) override {
     s_left = src.alloc(DType::F32, {dim});
     s_right = src.alloc(DType::F32, {dim});
-    DecayAttention::put_floats(s_left, std::vector<float>((size_t)dim, left_scale), src.to_host);
-    DecayAttention::put_floats(s_right, std::vector<float>((size_t)dim, right_scale), src.to_host);
+    put_floats(s_left, std::vector<float>((size_t)dim, left_scale), src.to_host);
+    put_floats(s_right, std::vector<float>((size_t)dim, right_scale), src.to_host);
   }
   void run(StepContext& ctx, const Rows& h, const Tensor& x) {
     const int64_t M = h.t.shape[0];
@@ -2691,6 +3006,12 @@ void register_builtin_parts() {
   register_part("mixer", "decay_attention", [](const std::string& prefix, const Json& p, const PartChildren&) {
     return std::make_shared<DecayAttention>(prefix, p);
   });
+  register_part("mixer", "mingru", [](const std::string& prefix, const Json& p, const PartChildren&) {
+    return std::make_shared<MinGRU>(prefix, p);
+  });
+  register_part("block", "sandwich",
+                [](const std::string& prefix, const Json& p, const PartChildren& c) { return std::make_shared<SandwichBlock>(prefix, p, c); },
+                {{"norm1", "norm"}, {"mixer", "mixer"}, {"norm1b", "norm"}, {"norm2", "norm?"}, {"ffn", "ffn?"}, {"norm2b", "norm?"}});
   register_part("mixer", "sum", [](const std::string& prefix, const Json& p, const PartChildren& c) {
     return std::make_shared<SumMixer>(prefix, p, c);
   });
@@ -2962,7 +3283,7 @@ float DiffAttention::lambda_of(const Tensor l[4], int dk, double diff, bool on_h
   }
   return std::exp(s1) - std::exp(s2) + (float)diff;
 }
-void DecayAttention::put_floats(const Tensor& dst, const std::vector<float>& values, bool on_host) {
+void put_floats(const Tensor& dst, const std::vector<float>& values, bool on_host) {
   if (on_host) {
     memcpy(dst.data, values.data(), values.size() * 4);
     return;
