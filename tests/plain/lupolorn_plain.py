@@ -133,7 +133,7 @@ def attention(h: np.ndarray, positions, m: dict, w: Dict[str, np.ndarray], name:
     q = unit_rms(rotate_pairs(q, positions, m.get("rot")), eps)
     k = unit_rms(rotate_pairs(k, positions, m.get("rot")), eps)
     gate = sigmoid(h @ w[name + ".g"].T)
-    vis = visible(T, (m.get("mask") or {}).get("size"))
+    vis = visible(T, None)
     o = np.zeros((T, H, dv))
     for j in range(H):
         g = j // (H // G)
