@@ -39,6 +39,13 @@ sized so that a token's experts do the arithmetic of the model's dense feed-forw
 with a sink, mixed values and gates, softmax attention beside linear attention with a fixed
 decay, a grouped router): `--mixers attention|parallel|alternate --ffn dense|moe --streams 2`.
 
+`--design lupolorn` does the same for a Lupolorn decoder (a norm on either side of every sublayer): as mixers `--mixers
+attention` (the model's heads rotated in pairs, unit norms, one more in the denominator, a gate a head), `latent` (latent
+attention with the model's heads of 128, latents of 512 for queries and for keys and values, a window of `--window`
+positions), `mingru` (an element-wise recurrence as wide as the model's heads together) or `alternate` (latent, attention,
+recurrence, ...); `--ffn dense` (squared relu, sized to do the arithmetic of the model's gated feed-forward) or `moe`
+(`--experts` of which a token takes `--top`, and a shared one behind a gate, together of the same arithmetic).
+
 `--design nazorax` does the same for a Nazorax decoder: parallel layers behind a Dynamic
 Tanh, as mixers `--mixers attention` (biased, rotated attention with the model's heads
 under a window of `--window` positions), `latent` (latent attention with the model's
@@ -142,6 +149,24 @@ def dubozen_config(base, mixers, ffn, experts, top, streams, value_size=0):
     return cfg
 
 
+def lupolorn_config(base, mixers, ffn, experts, top, window):
+    """A Lupolorn config.json with the layer widths of the Qwen3 configuration `base`."""
+    H, F, hd, heads = base["hidden_size"], base["intermediate_size"], base["head_dim"], base["num_attention_heads"]
+    ff = 3 * F // 2                                       # two matrices of 3F/2 do what three of F do
+    part = max(64, ff // (top + 1) // 64 * 64)            # ... and so do top experts and the shared one
+    mlp = dict(kind="dense", ff=ff) if ffn == "dense" else dict(kind="moe", expert=dict(ff=part), router=dict(experts=experts, top=top),
+                                                                shared=dict(ff=part))
+    attention = dict(type="attention", mlp=mlp, mixer=dict(
+        heads=heads, kv_heads=base["num_key_value_heads"], dim=hd, vdim=hd, scale=hd ** -0.5,
+        rot=dict(base=500000.0, dims=hd, scaling=dict(factor=8.0, low=1.0, high=4.0, original=8192))))
+    latent = dict(type="latent_attention", mlp=mlp, mixer=dict(heads=heads, dim=hd, vdim=hd, q_rank=4 * hd, kv_rank=4 * hd, scale=hd ** -0.5,
+                                                              mask=dict(size=window)))
+    mingru = dict(type="mingru", mlp=mlp, mixer=dict(width=heads * hd))
+    kinds = {"attention": [attention], "latent": [latent], "mingru": [mingru], "alternate": [latent, attention, mingru]}[mixers]
+    return dict(architecture="Lupolorn", width=H, vocab=base["vocab_size"], norm=dict(eps=1e-6), embedding=dict(scale=H ** 0.5),
+                layers=[kinds[i % len(kinds)] for i in range(base["num_hidden_layers"])])
+
+
 MAX_SEQ = 4096            # context length a request may reach (more if --context asks for it)
 PAGE = 16
 PEAK_HBM = 8.0e12         # bytes/s, MI355X
@@ -189,6 +214,9 @@ def model_numbers(model):
             v = getattr(need, "v_dim", None) or need.head_dim
             two_maps = getattr(part, "kind", "") == "diff_attention"     # its keys hold two maps; both read the values
             attn.append((part.params["heads"], need.head_dim, 2 * v if two_maps else v, need.window, getattr(need, "block", None)))
+        if getattr(part, "kind", "") == "latent_attention":      # every head against the cached rows, its values their latents
+            rank, rot = part.params["kv_rank"], part.params["rot_dim"]
+            attn.append((part.params["heads"], rank + rot, rank, need.window, None))
         if need is not None and hasattr(need, "shape") and not hasattr(need, "kv_heads"):
             cells.append(tuple(need.shape))
     # what a token's experts hold, and what a step of `batch` tokens reads of the experts if every token chooses alike at random
@@ -199,7 +227,9 @@ def model_numbers(model):
     # per cached token the keys and values of every cache layer (values of their own size where they have one); per
     # request the 32-bit state of every recurrent layer, read and written once a step
     state_bytes = sum(2 * 4 * int(np_prod(need.shape)) * n for need, n in model.cache_groups if not hasattr(need, "kv_heads") and hasattr(need, "shape"))
-    kv_bytes = lambda context: state_bytes + sum(need.kv_heads * (need.head_dim + (getattr(need, "v_dim", None) or need.head_dim)) * 2 * n *      # noqa: E731
+    row_bytes = lambda context: sum(2 * np_prod(need.row_shape) * n * min(context, need.window or context)      # noqa: E731
+                                    for need, n in model.cache_groups if hasattr(need, "row_shape"))      # latents, as rows and transposed
+    kv_bytes = lambda context: state_bytes + row_bytes(context) + sum(need.kv_heads * (need.head_dim + (getattr(need, "v_dim", None) or need.head_dim)) * 2 * n *      # noqa: E731
                                                  min(context, need.window or context, getattr(need, "block", None) or context)
                                                  for need, n in model.cache_groups if hasattr(need, "kv_heads"))
     return dict(layer_params=layer_params + active, head_params=head_params, weight_bytes=weight_bytes, weight_bytes_at=weight_bytes_at,
@@ -457,18 +487,18 @@ def main() -> int:
     ap.add_argument("--warmup", type=int, default=16)
     ap.add_argument("--model", choices=sorted(MODELS), default="0.6b", help="whose layer sizes the model has")
     ap.add_argument("--layers", type=int, default=None, help="run fewer layers than the configuration has")
-    ap.add_argument("--design", choices=["qwen3", "miterax", "mumasun", "nazorax", "dubozen"], default="qwen3",
-                    help="miterax / mumasun / nazorax / dubozen: a decoder of that design with the layer widths of --model instead (see --mixers; --experts, --top, --mask-size; --ffn, --window, --streams)")
-    ap.add_argument("--experts", type=int, default=8, help="--design mumasun / nazorax / dubozen: experts per layer")
-    ap.add_argument("--top", type=int, default=2, help="--design mumasun / nazorax / dubozen: experts a token takes")
-    ap.add_argument("--ffn", choices=["dense", "moe"], default="moe", help="--design nazorax / dubozen: the feed-forward of its layers")
+    ap.add_argument("--design", choices=["qwen3", "miterax", "mumasun", "nazorax", "dubozen", "lupolorn"], default="qwen3",
+                    help="miterax / mumasun / nazorax / dubozen / lupolorn: a decoder of that design with the layer widths of --model instead (see --mixers; --experts, --top, --mask-size; --ffn, --window, --streams)")
+    ap.add_argument("--experts", type=int, default=8, help="--design mumasun / nazorax / dubozen / lupolorn: experts per layer")
+    ap.add_argument("--top", type=int, default=2, help="--design mumasun / nazorax / dubozen / lupolorn: experts a token takes")
+    ap.add_argument("--ffn", choices=["dense", "moe"], default="moe", help="--design nazorax / dubozen / lupolorn: the feed-forward of its layers")
     ap.add_argument("--value-size", type=int, default=0, help="--design dubozen: the value size of its attention layers (0: the head size)")
     ap.add_argument("--streams", type=int, default=2, help="--design dubozen: copies of the residual (0: one plain residual)")
-    ap.add_argument("--window", type=int, default=1024, help="--design nazorax: positions an attention layer's window keeps")
+    ap.add_argument("--window", type=int, default=1024, help="--design nazorax / lupolorn: positions an attention (a latent attention) layer's window keeps")
     ap.add_argument("--mask-size", type=int, default=4096, help="--design mumasun: positions of a block of visible keys")
-    ap.add_argument("--mixers", choices=["attention", "mlstm", "latent", "parallel", "alternate"], default="alternate",
+    ap.add_argument("--mixers", choices=["attention", "mlstm", "latent", "parallel", "mingru", "alternate"], default="alternate",
                     help="--design miterax (attention, mlstm, alternate) / nazorax (attention, latent, alternate) / dubozen (attention, parallel, "
-                         "alternate): the mixer of its layers")
+                         "alternate) / lupolorn (attention, latent, mingru, alternate): the mixer of its layers")
     ap.add_argument("--batch", type=int, default=8)
     ap.add_argument("--context", type=int, default=2048, help="cached tokens each decoding request holds")
     ap.add_argument("--prefill-tokens", type=int, default=2048)
@@ -506,15 +536,23 @@ def main() -> int:
         cfg = mumasun_config(cfg, args.experts, args.top, args.mask_size)
         model_name = f"Mumasun ({args.top} of {args.experts} experts, blocks of {args.mask_size}) at {NAMES[args.model]} sizes"
     if args.design == "nazorax":
-        if args.mixers == "mlstm":
+        if args.mixers in ("mlstm", "mingru"):
             ap.error("--design nazorax has the mixers attention, latent and alternate")
         cfg = nazorax_config(cfg, args.mixers, args.ffn, args.experts, args.top, args.window)
         what = "dense feed-forward" if args.ffn == "dense" else f"{args.top} of {args.experts} experts and a shared one"
         model_name = f"Nazorax ({args.mixers} mixers, {what}) at {NAMES[args.model]} sizes"
-    elif args.mixers == "latent":
-        ap.error("--mixers latent goes with --design nazorax")
+    elif args.mixers == "latent" and args.design != "lupolorn":
+        ap.error("--mixers latent goes with --design nazorax and lupolorn")
+    if args.design == "lupolorn":
+        if args.mixers in ("mlstm", "parallel"):
+            ap.error("--design lupolorn has the mixers attention, latent, mingru and alternate")
+        cfg = lupolorn_config(cfg, args.mixers, args.ffn, args.experts, args.top, args.window)
+        what = "dense feed-forward" if args.ffn == "dense" else f"{args.top} of {args.experts} experts and a shared one"
+        model_name = f"Lupolorn ({args.mixers} mixers, {what}) at {NAMES[args.model]} sizes"
+    elif args.mixers == "mingru":
+        ap.error("--mixers mingru goes with --design lupolorn")
     if args.design == "dubozen":
-        if args.mixers in ("mlstm", "latent"):
+        if args.mixers in ("mlstm", "latent", "mingru"):
             ap.error("--design dubozen has the mixers attention, parallel and alternate")
         cfg = dubozen_config(cfg, args.mixers, args.ffn, args.experts, args.top, args.streams, args.value_size)
         what = "dense feed-forward" if args.ffn == "dense" else f"{args.top} of {args.experts} experts"
@@ -599,7 +637,7 @@ def main() -> int:
                    "hidden": sizes["hidden_size"], "heads": sizes["num_attention_heads"],
                    "kv_heads": sizes["num_key_value_heads"], "head_dim": sizes["head_dim"],
                    "intermediate": sizes["intermediate_size"], "vocab": sizes["vocab_size"],
-                   "tied_head": bool(sizes["tie_word_embeddings"]) and args.design == "qwen3",
+                   "tied_head": bool(sizes["tie_word_embeddings"]) and args.design in ("qwen3", "lupolorn"),
                    "global_batch": args.batch, "cached_tokens": context, "seq_len": max_seq, "page_size": PAGE,
                    "prefill_tokens": prefill_tokens, "parallelism": "single GPU", "decode_graph": True,
                    "sampling": f"temperature {args.temperature} top-k {args.top_k or 512} top-p {args.top_p}" if draw else "greedy"},
