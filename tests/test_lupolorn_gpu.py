@@ -397,6 +397,13 @@ def test_equal_scores_go_to_the_lower_index(ops):
     assert ids.cpu().tolist() == [[0, 1, 2]] * 3 and np.abs(f64(wts) - 0.125).max() < 1e-6
 
 
+def test_a_row_that_is_not_a_number_still_names_experts_that_exist(ops):
+    h = torch.full((2, 16), float("nan"), device="cuda")
+    ids, wts = torch.empty(2, 3, device="cuda", dtype=torch.int32), torch.empty(2, 3, device="cuda")
+    ops.moe_route_grouped(h, torch.ones(8, 16, device="cuda"), ids, wts, None, 3, renormalize=False, score="softmax")
+    assert all(0 <= i < 8 for row in ids.cpu().tolist() for i in row)
+
+
 # ---------------------------------------------------------------------------------- the engine
 REQUEST_LENGTHS = {"a": 97, "b": 45, "c": 130, "d": 33, "e": 71, "f": 58}
 PROMPT_LENGTHS = {"a": 60, "b": 12, "c": 101, "d": 30, "e": 2, "f": 41}

@@ -60,11 +60,11 @@ __device__ __forceinline__ void load_pair(const DiffPages& kv, int keyA, int las
   int rowA = keyA % kv.P, rowB = keyB % kv.P;
   if (pageA < 0) {
     pageA = kv.table[safe_key / kv.P];
-    rowA = safe_key % kv.P;
+    rowA = (safe_key % kv.P) & ~15;      // (a whole block of the page: from a row inside it the values' reads would leave the page)
   }
   if (pageB < 0) {
     pageB = kv.table[safe_key / kv.P];
-    rowB = safe_key % kv.P;
+    rowB = (safe_key % kv.P) & ~15;
   }
   const size_t page_elems = (size_t)kv.n_kv * kv.P * (2 * DK + DV);
   const bf16_t* ka = kv.pool + (size_t)pageA * page_elems + ((size_t)kv.kvh * kv.P + rowA) * (2 * DK);

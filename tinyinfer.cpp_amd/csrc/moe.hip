@@ -150,6 +150,7 @@ moe_route_kernel(const T* __restrict__ h, const float* __restrict__ router, int*
         at = oa;
       }
     }
+    if (at >= E) at = k;      // no score compares as larger (not a number): an expert that exists all the same
     if (corrected) best = s_plain[at];
     if (lane == 0) {
       ids[(size_t)m * top + k] = at;
