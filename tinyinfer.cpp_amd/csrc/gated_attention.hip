@@ -31,10 +31,73 @@ __device__ __forceinline__ void ga_rotation(const float* __restrict__ inv_freq, 
   }
 }
 
-// A wavefront per token and head: a query head, or a key head with its value head.  Grid (token, heads + kv heads in fours).
+// A wavefront per token and query or key head, four to a workgroup; behind them (blockIdx.y = the number of such workgroups a
+// token) workgroups of sixteen tokens and one value head each: the values pass through LDS, so that sixteen tokens that lie in a
+// page one after the other are written sixteen to a piece.  Values that are the keys as projected are written by the key heads.
 // pairs: entries 2i and 2i + 1 turn together (else i and i + rot_dims / 2); unit_norm: the head divided by its root mean square
 // behind the rotation
 #define GA_PREP_WAVES 4
+#define GA_V_TOKENS 16
+template <typename T>
+__device__ __forceinline__ void prep_values(const float* __restrict__ proj, int ld, int off_v, int mix_mode, const float* __restrict__ mix_lambda,
+                                            float* __restrict__ v_kept, const int* __restrict__ pos, const int* __restrict__ slot,
+                                            const int* __restrict__ table, int table_stride, T* __restrict__ pool, int M, int n_kv, int dk,
+                                            int dv, int dvr, int P) {
+  __shared__ T s_v[256][GA_V_TOKENS + 2];
+  __shared__ int s_page[GA_V_TOKENS], s_row[GA_V_TOKENS];
+  const int item = blockIdx.x;
+  const int n_groups = (M + GA_V_TOKENS - 1) / GA_V_TOKENS;
+  if (item >= n_groups * n_kv) return;
+  const int m0 = item / n_kv * GA_V_TOKENS, h = item % n_kv, n = min(GA_V_TOKENS, M - m0);
+  if (threadIdx.x < GA_V_TOKENS) {
+    const int i = threadIdx.x;
+    int page = -1, r = 0;
+    if (i < n) {
+      const int p = pos[m0 + i];
+      page = table[(size_t)slot[m0 + i] * table_stride + p / P];
+      r = p % P;
+    }
+    s_page[i] = page;
+    s_row[i] = r;
+  }
+  const float lam = mix_mode == 2 ? mix_lambda[0] : 0.f;
+  for (int e = threadIdx.x; e < n * dvr; e += TI_WAVE * GA_PREP_WAVES) {
+    const int i = e / dvr, d = e % dvr, m = m0 + i;
+    float x = 0.f;                                                    // rows beyond the value's size: zeros
+    if (d < dv) {
+      x = proj[(size_t)m * ld + off_v + (size_t)h * dv + d];
+      float* kept = v_kept ? v_kept + ((size_t)m * n_kv + h) * dv + d : nullptr;
+      if (mix_mode == 1) *kept = x;                                   // the layer whose values the later ones mix in
+      else if (mix_mode == 2) x = fmaf(lam, *kept, (1.0f - lam) * x);
+    }
+    st<T>(&s_v[d][i], x);
+  }
+  __syncthreads();
+  const size_t page_elems = (size_t)n_kv * P * (dk + dvr), v_off = (size_t)n_kv * P * dk + (size_t)h * dvr * P;
+  // one run of sixteen rows of one page, on a boundary of sixteen
+  bool run = n == GA_V_TOKENS && P % GA_V_TOKENS == 0 && s_page[0] >= 0 && s_row[0] % GA_V_TOKENS == 0 && (((uintptr_t)pool | (page_elems * sizeof(T)) | (v_off * sizeof(T))) & 15) == 0;
+#pragma unroll
+  for (int i = 1; i < GA_V_TOKENS; ++i) run = run && s_page[i] == s_page[0] && s_row[i] == s_row[0] + i;
+  if (run) {
+    constexpr int N = 16 / sizeof(T), PIECES = GA_V_TOKENS / N;       // elements of a piece of 16 bytes, pieces of a value's entry
+    T* base = pool + (size_t)s_page[0] * page_elems + v_off + s_row[0];
+    for (int e = threadIdx.x; e < dvr * PIECES; e += TI_WAVE * GA_PREP_WAVES) {
+      const int d = e / PIECES, k = e % PIECES;
+      T v[N];
+#pragma unroll
+      for (int j = 0; j < N; ++j) v[j] = s_v[d][k * N + j];
+      uint4 out;
+      __builtin_memcpy(&out, v, 16);
+      *reinterpret_cast<uint4*>(base + (size_t)d * P + k * N) = out;
+    }
+    return;
+  }
+  for (int e = threadIdx.x; e < n * dvr; e += TI_WAVE * GA_PREP_WAVES) {
+    const int i = e % n, d = e / n;
+    if (s_page[i] >= 0) pool[(size_t)s_page[i] * page_elems + v_off + (size_t)d * P + s_row[i]] = s_v[d][i];
+  }
+}
+
 template <typename T>
 __global__ void __launch_bounds__(TI_WAVE * GA_PREP_WAVES)
 gated_qkv_prep_kernel(const float* __restrict__ proj, int ld, int off_q, int off_k, int off_v, const float* __restrict__ q_w,
@@ -42,8 +105,14 @@ gated_qkv_prep_kernel(const float* __restrict__ proj, int ld, int off_q, int off
                       const float* __restrict__ rope_table, int table_len, float mag, int rot_dims, int mix_mode,
                       const float* __restrict__ mix_lambda, float* __restrict__ v_kept, const int* __restrict__ pos,
                       const int* __restrict__ slot, const int* __restrict__ table, int table_stride, T* __restrict__ pool,
-                      T* __restrict__ q_out, int n_head, int n_kv, int dk, int dv, int dvr, int P, int pairs, int unit_norm) {
+                      T* __restrict__ q_out, int M, int n_head, int n_kv, int dk, int dv, int dvr, int P, int pairs, int unit_norm) {
   __shared__ float s_all[GA_PREP_WAVES][256];
+  const int n_units = (n_head + n_kv + GA_PREP_WAVES - 1) / GA_PREP_WAVES;
+  if ((int)blockIdx.y >= n_units) {
+    prep_values<T>(proj, ld, off_v, mix_mode, mix_lambda, v_kept, pos, slot, table, table_stride, pool, M, n_kv, dk, dv, dvr, P);
+    return;
+  }
+  if ((int)blockIdx.x >= M) return;
   const int m = blockIdx.x, unit = blockIdx.y * GA_PREP_WAVES + threadIdx.x / TI_WAVE, lane = threadIdx.x % TI_WAVE;
   if (unit >= n_head + n_kv) return;      // (no barrier below: a wavefront keeps to itself)
   float* const s_h = s_all[threadIdx.x / TI_WAVE];
@@ -138,20 +207,6 @@ gated_qkv_prep_kernel(const float* __restrict__ proj, int ld, int off_q, int off
       if (d < dk) st<T>(dst + d, v[i]);
     }
   }
-  if (off_v < 0) return;
-  const float* vs = row + off_v + (size_t)h * dv;
-  float* kept = v_kept ? v_kept + ((size_t)m * n_kv + h) * dv : nullptr;
-  const float lam = mix_mode == 2 ? mix_lambda[0] : 0.f;
-  T* vbase = base + (size_t)n_kv * P * dk + (size_t)h * dvr * P + r;
-  for (int d = lane; d < dvr; d += TI_WAVE) {
-    float x = 0.f;                                                    // rows beyond the value's size: zeros
-    if (d < dv) {
-      x = vs[d];
-      if (mix_mode == 1) kept[d] = x;                                 // the layer whose values the later ones mix in
-      else if (mix_mode == 2) x = fmaf(lam, kept[d], (1.0f - lam) * x);
-    }
-    if (page >= 0) st<T>(vbase + (size_t)d * P, x);
-  }
 }
 
 extern "C" int ti_gated_qkv_prep(int dtype, const float* proj, int ld, int off_q, int off_k, int off_v, const float* q_w,
@@ -181,16 +236,17 @@ extern "C" int ti_gated_qkv_prep_form(int dtype, const float* proj, int ld, int 
   TI_REQUIRE(off_q >= 0 && off_k >= 0 && off_q + n_head * dk <= ld && off_k + n_kv * dk <= ld && (off_v < 0 || off_v + n_kv * dv <= ld),
              "gated_qkv_prep: the columns do not lie inside rows of %d", ld);
   if (M == 0) return 0;
-  const dim3 grid(M, (n_head + n_kv + GA_PREP_WAVES - 1) / GA_PREP_WAVES);
+  const int n_groups = off_v < 0 ? 0 : (M + GA_V_TOKENS - 1) / GA_V_TOKENS * n_kv;       // workgroups of the values
+  const dim3 grid(M > n_groups ? M : n_groups, (n_head + n_kv + GA_PREP_WAVES - 1) / GA_PREP_WAVES + (n_groups ? 1 : 0));
   if (dtype == TI_F32)
     gated_qkv_prep_kernel<float><<<grid, TI_WAVE * GA_PREP_WAVES, 0, stream>>>(proj, ld, off_q, off_k, off_v, q_w, k_w, eps, inv_freq, rope_table,
                                                                table_len, mag, rot_dims, mix_mode, mix_lambda, v_kept, pos, slot,
-                                                               table, table_stride, (float*)pool, (float*)q_out, n_head, n_kv, dk,
+                                                               table, table_stride, (float*)pool, (float*)q_out, M, n_head, n_kv, dk,
                                                                dv, dvr, page_size, pairs, unit_norm);
   else if (dtype == TI_BF16)
     gated_qkv_prep_kernel<bf16_t><<<grid, TI_WAVE * GA_PREP_WAVES, 0, stream>>>(proj, ld, off_q, off_k, off_v, q_w, k_w, eps, inv_freq, rope_table,
                                                                 table_len, mag, rot_dims, mix_mode, mix_lambda, v_kept, pos, slot,
-                                                                table, table_stride, (bf16_t*)pool, (bf16_t*)q_out, n_head, n_kv,
+                                                                table, table_stride, (bf16_t*)pool, (bf16_t*)q_out, M, n_head, n_kv,
                                                                 dk, dv, dvr, page_size, pairs, unit_norm);
   else
     TI_REQUIRE(false, "gated_qkv_prep: unknown dtype %d", dtype);

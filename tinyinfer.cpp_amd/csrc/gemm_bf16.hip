@@ -1983,9 +1983,9 @@ static bool pieces_serves(int M, int N, int K, int epi) {
   if ((epi < TI_EPI_STORE_F32 || epi > TI_EPI_SWIGLU) && epi != TI_EPI_RELU2) return false;
   // few tokens times a weight of few rows: a row per wavefront wins (and fills the compute units)
   if (row_per_wave_serves(M, N, K, epi)) return false;
-  // where the kernels with the norm in front take eight wavefronts, this one would give other bits
+  // where the kernels with the norm in front (K up to 4,096) take eight wavefronts, this one would give other bits
   const int grid = (epi == TI_EPI_SWIGLU) ? (N + 7) / 8 : (N + 15) / 16;
-  return skinny_waves_for(grid, K) == 4;
+  return K > 4096 || skinny_waves_for(grid, K) == 4;
 }
 // Into how many workgroups the pieces of K go when the product adds into the residual: a long K under
 // few rows of weight leaves a launch of few workgroups that each walk a long way (Qwen3-32B's down

@@ -3,7 +3,8 @@
 //   1. moe_group: counts the (token, expert) pairs of every expert, lays the experts' runs of rows one after
 //      the other and cuts them into tiles of 128 rows: offsets, the list of tiles, cursors at zero.
 //   2. moe_place: every pair takes a free row of its expert's run (which row does not matter: a row of a
-//      product depends on no other row) and writes its scaled input there, rounded to bfloat16.
+//      product depends on no other row) and writes its scaled input there, rounded to bfloat16; where the weights are
+//      on the outputs it leaves its token's number, and the first product gathers its rows from the step's own.
 //   3. two grouped products over the tiles: act = relu(A up_e^T)^2 (bfloat16), out = act down_e^T (32-bit).
 //      Weights are the A operand of v_mfma_f32_16x16x32_bf16 and tokens the 16 columns, both in their own
 //      layouts through LDS; a lane ends with four consecutive outputs of one token.
@@ -61,13 +62,14 @@ moe_group_kernel(const int* __restrict__ ids, int n_pairs, int E, int* __restric
   }
 }
 
-// A workgroup per 64 pairs: where[pair] = its row; rows[row] = bf16(s h[token]).  The workgroup counts its pairs per expert in
+// A workgroup per 64 pairs: where[pair] = its row; rows[row] = bf16(s h[token]), or, with `tokens` in the place of `rows` (inputs
+// without a factor), tokens[row] = its token, for a product that gathers its rows from h.  The workgroup counts its pairs per expert in
 // LDS and takes a run of rows from every expert's cursor at once (one atomic per expert it met, not one per pair); inside the
 // run a pair's place is its count in LDS.
 __global__ void __launch_bounds__(256)
 moe_place_kernel(const bf16_t* __restrict__ h, const int* __restrict__ ids, const float* __restrict__ wts, int* __restrict__ meta,
                  int E, int top, int W, int n_pairs, int* __restrict__ where, bf16_t* __restrict__ rows,
-                 const float* __restrict__ out_w = nullptr, float* __restrict__ row_w = nullptr) {
+                 const float* __restrict__ out_w = nullptr, float* __restrict__ row_w = nullptr, int* __restrict__ tokens = nullptr) {
   __shared__ int count[MOE_MAX_E];      // pairs of this workgroup per expert, then the first row of their run
   __shared__ int s_row[64];
   const int pair0 = blockIdx.x * 64;
@@ -87,7 +89,9 @@ moe_place_kernel(const bf16_t* __restrict__ h, const int* __restrict__ ids, cons
     where[pair0 + threadIdx.x] = r;
     if (row_w) row_w[r] = out_w[pair0 + threadIdx.x];      // weights on the experts' outputs: with the row
     s_row[threadIdx.x] = r;
+    if (tokens) tokens[r] = (pair0 + threadIdx.x) / top;
   }
+  if (tokens) return;
   __syncthreads();
   // a wavefront copies 16 of the rows, a lane 16 bytes at a time (W is a multiple of 32)
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -112,12 +116,12 @@ moe_place_kernel(const bf16_t* __restrict__ h, const int* __restrict__ ids, cons
 // wavefronts two by two, each 64 outputs (four blocks of 16) against 64 rows (four blocks of 16).  A step of 32 along k of both
 // operands is fetched once by the workgroup (thread t the 16-byte pieces t, t + 256) into one of two LDS stages while the step
 // before it is multiplied from the other; one barrier a step.  Rows of a stage are 80 bytes apart, so that the fragments'
-// reads spread over the banks.  EPI 0: relu^2, bfloat16; 1: 32-bit; 2: 32-bit, times the row's weight row_w[row].
+// reads spread over the banks.  tokens (null: none): row r of the operand is row tokens[r] of `rows`.  EPI 0: relu^2, bfloat16; 1: 32-bit; 2: 32-bit, times the row's weight row_w[row].
 #define MOE_LDS_ROW 40       // bfloat16 elements between rows of a stage (32 + 8)
 template <int EPI>
 __global__ void __launch_bounds__(256)
 moe_grouped_kernel(const bf16_t* __restrict__ rows, const bf16_t* __restrict__ w, const int* __restrict__ meta, int E, void* __restrict__ out,
-                   int N, int K, const float* __restrict__ row_w = nullptr) {
+                   int N, int K, const float* __restrict__ row_w = nullptr, const int* __restrict__ tokens = nullptr) {
   __shared__ __attribute__((aligned(16))) bf16_t lds[2][2][128 * MOE_LDS_ROW];      // [stage][weights | rows]
   const int n_tiles = meta[0];
   if ((int)blockIdx.x >= n_tiles) return;
@@ -131,8 +135,9 @@ moe_grouped_kernel(const bf16_t* __restrict__ rows, const bf16_t* __restrict__ w
   const int u0 = threadIdx.x, u1 = threadIdx.x + 256;
   const bf16_t* const src_w0 = w + ((size_t)e * N + min(n_blk + (u0 >> 2), N - 1)) * K + (u0 & 3) * 8;
   const bf16_t* const src_w1 = w + ((size_t)e * N + min(n_blk + (u1 >> 2), N - 1)) * K + (u1 & 3) * 8;
-  const bf16_t* const src_r0 = rows + (size_t)(row0 + min(u0 >> 2, n_rows - 1)) * K + (u0 & 3) * 8;
-  const bf16_t* const src_r1 = rows + (size_t)(row0 + min(u1 >> 2, n_rows - 1)) * K + (u1 & 3) * 8;
+  const int at0 = row0 + min(u0 >> 2, n_rows - 1), at1 = row0 + min(u1 >> 2, n_rows - 1);
+  const bf16_t* const src_r0 = rows + (size_t)(tokens ? tokens[at0] : at0) * K + (u0 & 3) * 8;
+  const bf16_t* const src_r1 = rows + (size_t)(tokens ? tokens[at1] : at1) * K + (u1 & 3) * 8;
   const int park0 = (u0 >> 2) * MOE_LDS_ROW + (u0 & 3) * 8, park1 = (u1 >> 2) * MOE_LDS_ROW + (u1 & 3) * 8;
   floatx4 acc[4][4];
 #pragma unroll
@@ -214,7 +219,7 @@ __global__ void moe_combine_kernel(const float* __restrict__ out, const int* __r
 extern "C" long ti_moe_grouped_meta_ints(int n_pairs, int E) { return 1 + (E + 1) + E + 3L * ((n_pairs + MOE_TILE - 1) / MOE_TILE + E); }
 
 // h bf16 [M, W]; ids, wts [M top]; up [E][F][W], down [E][W][F] bf16.  Scratch: meta int32 [ti_moe_grouped_meta_ints],
-// where int32 [M top], rows bf16 [M top][W], act bf16 [M top][F], out f32 [M top][W].  y (may be null): the tokens' sums;
+// where int32 [M top], rows bf16 [M top][W] (weights on the outputs: int32 [M top], the rows' tokens), act bf16 [M top][F], out f32 [M top][W].  y (may be null): the tokens' sums;
 // without it the caller adds the rows out[where[m top + k]] itself.  The weights multiply the experts' inputs (scale_input) or
 // their outputs (row_w: f32 scratch [M top]).  3: sizes not served (W, F multiples of 32, E <= 1024).
 extern "C" int ti_moe_experts_grouped_bf16(const void* h, const int* ids, const float* wts, const void* up, const void* down,
@@ -229,9 +234,11 @@ extern "C" int ti_moe_experts_grouped_bf16(const void* h, const int* ids, const 
   const int n_pairs = M * top;
   const int max_tiles = (n_pairs + MOE_TILE - 1) / MOE_TILE + E;
   moe_group_kernel<<<1, 1024, 0, stream>>>(ids, n_pairs, E, meta);
+  int* tokens = scale_input ? nullptr : (int*)rows;
   moe_place_kernel<<<(n_pairs + 63) / 64, 256, 0, stream>>>((const bf16_t*)h, ids, scale_input ? wts : nullptr, meta, E, top, W, n_pairs, where,
-                                                            (bf16_t*)rows, wts, scale_input ? nullptr : row_w);
-  moe_grouped_kernel<0><<<dim3(max_tiles, (F + 127) / 128), 256, 0, stream>>>((const bf16_t*)rows, (const bf16_t*)up, meta, E, act, F, W);
+                                                            (bf16_t*)rows, wts, scale_input ? nullptr : row_w, tokens);
+  moe_grouped_kernel<0><<<dim3(max_tiles, (F + 127) / 128), 256, 0, stream>>>((const bf16_t*)(tokens ? h : rows), (const bf16_t*)up, meta, E, act,
+                                                                              F, W, nullptr, tokens);
   const dim3 grid_down(max_tiles, (W + 127) / 128);
   if (scale_input) moe_grouped_kernel<1><<<grid_down, 256, 0, stream>>>((const bf16_t*)act, (const bf16_t*)down, meta, E, out, W, F);
   else moe_grouped_kernel<2><<<grid_down, 256, 0, stream>>>((const bf16_t*)act, (const bf16_t*)down, meta, E, out, W, F, row_w);
@@ -288,8 +295,11 @@ extern "C" int ti_moe_experts_grouped_gated_bf16(const void* h, const int* ids, 
   const int n_pairs = M * top;
   const int max_tiles = (n_pairs + MOE_TILE - 1) / MOE_TILE + E;
   moe_group_kernel<<<1, 1024, 0, stream>>>(ids, n_pairs, E, meta);
-  moe_place_kernel<<<(n_pairs + 63) / 64, 256, 0, stream>>>((const bf16_t*)h, ids, nullptr, meta, E, top, W, n_pairs, where, (bf16_t*)rows);
-  moe_grouped_kernel<1><<<dim3(max_tiles, (2 * F + 127) / 128), 256, 0, stream>>>((const bf16_t*)rows, (const bf16_t*)gate_up, meta, E, z, 2 * F, W);
+  int* tokens = (int*)rows;
+  moe_place_kernel<<<(n_pairs + 63) / 64, 256, 0, stream>>>((const bf16_t*)h, ids, nullptr, meta, E, top, W, n_pairs, where, nullptr, nullptr, nullptr,
+                                                            tokens);
+  moe_grouped_kernel<1><<<dim3(max_tiles, (2 * F + 127) / 128), 256, 0, stream>>>((const bf16_t*)h, (const bf16_t*)gate_up, meta, E, z, 2 * F, W,
+                                                                                  nullptr, tokens);
   const long n_act = (long)n_pairs * F;
   const unsigned blocks = (unsigned)((n_act + 255) / 256 < 16384 ? (n_act + 255) / 256 : 16384);
   moe_gate_rows_kernel<<<blocks, 256, 0, stream>>>(z, (bf16_t*)act, n_pairs, F, act_kind, limit, alpha);

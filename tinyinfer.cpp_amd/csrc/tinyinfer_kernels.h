@@ -368,13 +368,14 @@ int ti_moe_experts_rows_gated(int dtype, const void* h, const int* ids, const fl
 // by expert in tiles of 128 rows and both products run over the tiles.  Scratch: meta int32 [ti_moe_grouped_meta_ints(M top, E)],
 // where int32 [M top] (the row of every pair), rows bf16 [M top][W], act bf16 [M top][F], out f32 [M top][W].  y (may be
 // null): the tokens' sums; without it the caller adds the rows out[where[m top + k]] in ascending k.  The weights multiply the
-// experts' inputs (scale_input) or their outputs (row_w: f32 scratch [M top]).  3: sizes not served
+// experts' inputs (scale_input) or their outputs (row_w: f32 scratch [M top]; rows is int32 [M top] then, the rows' tokens).
+// 3: sizes not served
 long ti_moe_grouped_meta_ints(int n_pairs, int E);
 int ti_moe_experts_grouped_bf16(const void* h, const int* ids, const float* wts, const void* up, const void* down, int* meta,
                                 int* where, void* rows, void* act, float* out, float* y, int M, int W, int F, int E, int top,
                                 int scale_input, float* row_w, hipStream_t stream);
 
-// the gated experts of ti_moe_experts_rows_gated over such tiles; z: f32 scratch [M top][2F]; y is written (the tokens' weighted sums)
+// the gated experts of ti_moe_experts_rows_gated over such tiles; rows: int32 scratch [M top]; z: f32 scratch [M top][2F]; y is written (the tokens' weighted sums)
 int ti_moe_experts_grouped_gated_bf16(const void* h, const int* ids, const float* wts, const void* gate_up, const void* down,
                                       int* meta, int* where, void* rows, float* z, void* act, float* out, float* y, int M, int W,
                                       int F, int E, int top, int act_kind, float limit, float alpha, hipStream_t stream);

@@ -1115,7 +1115,7 @@ void Ops::latent_attention(const Tensor& proj, const Tensor& w_uk, const Tensor&
       int reach = lists->context;
       if (window > 0) reach = std::min(reach, window);
       int splits = 1;
-      if (reach > 0) splits = std::max(1, std::min({16, compute_units() / std::max(1, lists->n_rows * groups), reach / 128}));
+      if (reach > 0) splits = std::max(1, std::min({16, compute_units() / std::max(1, lists->n_rows * groups), reach / 64}));
       if (use.force_decode_splits > 0) splits = std::min(64, use.force_decode_splits);
       float* part = nullptr;
       if (splits > 1) {
@@ -1666,11 +1666,12 @@ void Ops::moe_experts(const Tensor& h, const Tensor& ids, const Tensor& wts, con
     const long meta_ints = KERNEL("moe_bf16", ti_moe_grouped_meta_ints)((int)pairs, experts);
     int* meta = (int*)ws.get("moe.meta", (size_t)meta_ints * 4);
     Tensor where = ws.tensor("moe.where", DType::I32, {pairs});
-    Tensor sorted = ws.tensor("moe.rows", DType::BF16, {pairs, W});
+    // scaled inputs are laid out expert by expert; unscaled ones stay where they are, a list names every row's token
+    void* sorted = ws.get("moe.rows", scale_input ? (size_t)(pairs * W) * 2 : (size_t)pairs * 4);
     Tensor act = ws.tensor("moe.act", DType::BF16, {pairs, F});
     Tensor out = ws.tensor("moe.out", DType::F32, {pairs, W});
     int rc = KERNEL("moe_bf16", ti_moe_experts_grouped_bf16)(h.data, (const int*)ids.data, (const float*)wts.data, up.data, down.data, meta,
-                                                             (int*)where.data, sorted.data, act.data, (float*)out.data,
+                                                             (int*)where.data, sorted, act.data, (float*)out.data,
                                                              rows ? nullptr : (float*)y.data, (int)M, (int)W, (int)F, experts, top,
                                                              scale_input ? 1 : 0,
                                                              scale_input ? nullptr : (float*)ws.get("moe.row_w", (size_t)pairs * 4),
@@ -1726,11 +1727,11 @@ void Ops::moe_experts_gated(const Tensor& h, const Tensor& ids, const Tensor& wt
     const long meta_ints = KERNEL("moe_bf16", ti_moe_grouped_meta_ints)((int)pairs, experts);
     int* meta = (int*)ws.get("moe.meta", (size_t)meta_ints * 4);
     Tensor where = ws.tensor("moe.where", DType::I32, {pairs});
-    Tensor sorted = ws.tensor("moe.rows", DType::BF16, {pairs, W});
+    void* sorted = ws.get("moe.rows", (size_t)pairs * 4);
     Tensor act = ws.tensor("moe.act", DType::BF16, {pairs, F});
     Tensor out = ws.tensor("moe.out", DType::F32, {pairs, W});
     int rc = KERNEL("moe_bf16", ti_moe_experts_grouped_gated_bf16)(h.data, (const int*)ids.data, (const float*)wts.data, gate_up.data,
-                                                                   down.data, meta, (int*)where.data, sorted.data, (float*)z.data, act.data,
+                                                                   down.data, meta, (int*)where.data, sorted, (float*)z.data, act.data,
                                                                    (float*)out.data, (float*)y.data, (int)M, (int)W, (int)F, experts, top,
                                                                    (int)kind, limit, alpha, (hipStream_t)launch_stream());
     if (rc == 0) {
