@@ -136,7 +136,8 @@ def rotation_inputs(rot, n_table):
 @pytest.mark.parametrize("heads,kv,dk,dv,P,rot_dims,normed,from_keys,gate,sink", [
     (4, 2, 16, 24, 16, 8, False, False, 1, True), (3, 3, 7, 7, 4, 6, True, True, 2, False), (6, 1, 40, 33, 64, 40, True, False, 1, True),
     (2, 2, 64, 64, 16, 32, True, True, 2, True), (2, 1, 64, 32, 16, 0, False, False, 0, True), (3, 1, 24, 16, 8, 12, False, False, 2, False),
-    (8, 2, 128, 128, 32, 64, True, True, 0, False), (1, 1, 256, 256, 16, 2, False, False, 1, True)])
+    (8, 2, 128, 128, 32, 64, True, True, 0, False), (1, 1, 256, 256, 16, 2, False, False, 1, True),
+    (20, 10, 24, 16, 16, 8, True, False, 2, True), (18, 9, 72, 72, 32, 66, True, True, 0, True)])
 def test_gated_attention(ops, dtype, heads, kv, dk, dv, P, rot_dims, normed, from_keys, gate, sink):
     """The projections of a whole request get their per-head norms and the rotation of their first entries and go into the
     pages in three portions (the last a single token); then the attention of every row with its sink and its gate.  The last

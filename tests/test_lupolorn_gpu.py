@@ -215,7 +215,8 @@ def test_the_parts_table_holds_the_stretched_frequencies(dims, base, scaling):
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("heads,kv,dk,dv,P,rot_dims,scaled", [
     (4, 2, 16, 24, 16, 8, True), (3, 3, 7, 5, 4, 6, True), (5, 1, 40, 33, 64, 40, False), (2, 2, 64, 64, 16, 64, True), (2, 1, 64, 32, 16, 0, False),
-    (8, 2, 128, 128, 32, 64, True), (1, 1, 256, 256, 16, 2, False), (7, 7, 32, 32, 8, 32, True), (3, 1, 130, 100, 16, 130, False)])
+    (8, 2, 128, 128, 32, 64, True), (1, 1, 256, 256, 16, 2, False), (7, 7, 32, 32, 8, 32, True), (3, 1, 130, 100, 16, 130, False),
+    (20, 10, 24, 16, 16, 16, True), (18, 9, 72, 40, 32, 70, False)])
 def test_attention_with_paired_rotation_unit_norms_and_one_more_in_the_denominator(ops, dtype, heads, kv, dk, dv, P, rot_dims, scaled):
     """The projections of a whole request are rotated, divided by their root mean square and written into the pages in three
     portions (the last a single token); then the attention of every row with a gate a head.  The last row's query points at

@@ -17,8 +17,6 @@
 
 TI_ERROR_API
 
-#define GA_MAX_DPL 4      // entries of a head a lane holds: heads up to 256
-
 __device__ __forceinline__ void ga_rotation(const float* __restrict__ inv_freq, const float* __restrict__ rope_table, int table_len,
                                             float mag, int half, int p, int i, float* c, float* s) {
   if (rope_table && p < table_len) {
@@ -31,11 +29,13 @@ __device__ __forceinline__ void ga_rotation(const float* __restrict__ inv_freq, 
   }
 }
 
-// A wavefront per token and query or key head, four to a workgroup; behind them (blockIdx.y = the number of such workgroups a
-// token) workgroups of sixteen tokens and one value head each: the values pass through LDS, so that sixteen tokens that lie in a
-// page one after the other are written sixteen to a piece.  Values that are the keys as projected are written by the key heads.
+// A wavefront per token and HPW query or key heads (one after the other in the order q, k), four wavefronts to a workgroup: the
+// position, its page and its angles are fetched once for the heads of a wavefront, whose loads are in flight together.  Behind
+// them (blockIdx.y = the number of such workgroups a token) workgroups of sixteen tokens and one value head each: the values pass
+// through LDS, so that sixteen tokens that lie in a page one after the other are written sixteen to a piece.  Values that are the
+// keys as projected are written by the key heads.
 // pairs: entries 2i and 2i + 1 turn together (else i and i + rot_dims / 2); unit_norm: the head divided by its root mean square
-// behind the rotation
+// behind the rotation.  DPL: entries of a head a lane holds.
 #define GA_PREP_WAVES 4
 #define GA_V_TOKENS 16
 template <typename T>
@@ -98,7 +98,7 @@ __device__ __forceinline__ void prep_values(const float* __restrict__ proj, int 
   }
 }
 
-template <typename T>
+template <typename T, int DPL, int HPW>
 __global__ void __launch_bounds__(TI_WAVE * GA_PREP_WAVES)
 gated_qkv_prep_kernel(const float* __restrict__ proj, int ld, int off_q, int off_k, int off_v, const float* __restrict__ q_w,
                       const float* __restrict__ k_w, float eps, const float* __restrict__ inv_freq,
@@ -106,105 +106,102 @@ gated_qkv_prep_kernel(const float* __restrict__ proj, int ld, int off_q, int off
                       const float* __restrict__ mix_lambda, float* __restrict__ v_kept, const int* __restrict__ pos,
                       const int* __restrict__ slot, const int* __restrict__ table, int table_stride, T* __restrict__ pool,
                       T* __restrict__ q_out, int M, int n_head, int n_kv, int dk, int dv, int dvr, int P, int pairs, int unit_norm) {
-  __shared__ float s_all[GA_PREP_WAVES][256];
-  const int n_units = (n_head + n_kv + GA_PREP_WAVES - 1) / GA_PREP_WAVES;
+  __shared__ float s_all[GA_PREP_WAVES][DPL * TI_WAVE];
+  const int per_group = GA_PREP_WAVES * HPW;
+  const int n_units = (n_head + n_kv + per_group - 1) / per_group;
   if ((int)blockIdx.y >= n_units) {
     prep_values<T>(proj, ld, off_v, mix_mode, mix_lambda, v_kept, pos, slot, table, table_stride, pool, M, n_kv, dk, dv, dvr, P);
     return;
   }
   if ((int)blockIdx.x >= M) return;
-  const int m = blockIdx.x, unit = blockIdx.y * GA_PREP_WAVES + threadIdx.x / TI_WAVE, lane = threadIdx.x % TI_WAVE;
-  if (unit >= n_head + n_kv) return;      // (no barrier below: a wavefront keeps to itself)
-  float* const s_h = s_all[threadIdx.x / TI_WAVE];
+  const int m = blockIdx.x, wave = threadIdx.x / TI_WAVE, lane = threadIdx.x % TI_WAVE;
+  const int first = blockIdx.y * per_group + wave * HPW, n = min(HPW, n_head + n_kv - first);
+  if (n <= 0) return;      // (no barrier below: a wavefront keeps to itself)
+  float* const s_h = s_all[wave];
   const int p = pos[m];
-  const bool is_q = unit < n_head;
-  const int h = is_q ? unit : unit - n_head;
   const float* row = proj + (size_t)m * ld;
-  const float* src = row + (is_q ? off_q : off_k) + (size_t)h * dk;
-  const float* nw = is_q ? q_w : k_w;
+  float v[HPW][DPL];
+#pragma unroll
+  for (int k = 0; k < HPW; ++k) {
+    const int unit = first + min(k, n - 1);      // (heads beyond the last: the last one again, not written)
+    const float* src = unit < n_head ? row + off_q + (size_t)unit * dk : row + off_k + (size_t)(unit - n_head) * dk;
+#pragma unroll
+    for (int i = 0; i < DPL; ++i) {
+      const int d = lane + i * TI_WAVE;
+      v[k][i] = d < dk ? src[d] : 0.f;
+    }
+  }
   const int page = table[(size_t)slot[m] * table_stride + p / P];
   const int r = p % P;
-  T* base = pool + (size_t)max(page, 0) * ((size_t)n_kv * P * (dk + dvr));
-  float v[GA_MAX_DPL];
-  float ss = 0.f;
-#pragma unroll
-  for (int i = 0; i < GA_MAX_DPL; ++i) {
-    const int d = lane + i * TI_WAVE;
-    v[i] = d < dk ? src[d] : 0.f;
-    ss = fmaf(v[i], v[i], ss);
-  }
-  if (!is_q && off_v < 0 && page >= 0) {
-    // the values are the keys as projected: before norm and rotation
-    T* vbase = base + (size_t)n_kv * P * dk + (size_t)h * dvr * P + r;
-#pragma unroll
-    for (int i = 0; i < GA_MAX_DPL; ++i) {
-      const int d = lane + i * TI_WAVE;
-      if (d < dv) st<T>(vbase + (size_t)d * P, v[i]);
-    }
-  }
-  if (nw) {
-    const float inv = 1.0f / sqrtf(group_sum<TI_WAVE>(ss) / (float)dk + eps);
-#pragma unroll
-    for (int i = 0; i < GA_MAX_DPL; ++i) {
-      const int d = lane + i * TI_WAVE;
-      if (d < dk) v[i] = v[i] * inv * nw[d];
-    }
-  }
   const int half = inv_freq ? rot_dims / 2 : 0;
-  if (half > 0 && pairs) {
-    // neighbours lie in neighbouring lanes
+  float c[DPL], s[DPL];
 #pragma unroll
-    for (int i = 0; i < GA_MAX_DPL; ++i) {
-      const int d = lane + i * TI_WAVE;
-      if (i * TI_WAVE < 2 * half) {      // (the same in every lane)
-        const float other = __shfl_xor(v[i], 1, TI_WAVE);
-        if (d < 2 * half) {
-          float c, s;
-          ga_rotation(inv_freq, rope_table, table_len, mag, half, p, d >> 1, &c, &s);
-          v[i] = (d & 1) ? v[i] * c + other * s : v[i] * c - other * s;
+  for (int i = 0; i < DPL; ++i) {
+    const int d = lane + i * TI_WAVE;
+    c[i] = 1.f;
+    s[i] = 0.f;
+    if (d < 2 * half) ga_rotation(inv_freq, rope_table, table_len, mag, half, p, pairs ? d >> 1 : d < half ? d : d - half, &c[i], &s[i]);
+  }
+  T* base = pool + (size_t)max(page, 0) * ((size_t)n_kv * P * (dk + dvr));
+#pragma unroll
+  for (int k = 0; k < HPW; ++k) {
+    const int unit = first + k;
+    const bool is_q = unit < n_head;
+    const int h = is_q ? unit : unit - n_head;
+    if (k < n && !is_q && off_v < 0 && page >= 0) {
+      // the values are the keys as projected: before norm and rotation
+      T* vbase = base + (size_t)n_kv * P * dk + (size_t)h * dvr * P + r;
+#pragma unroll
+      for (int i = 0; i < DPL; ++i) {
+        const int d = lane + i * TI_WAVE;
+        if (d < dv) st<T>(vbase + (size_t)d * P, v[k][i]);
+      }
+    }
+    const float* nw = is_q ? q_w : k_w;
+    if (nw) {
+      float ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < DPL; ++i) ss = fmaf(v[k][i], v[k][i], ss);      // (entries beyond the head are zero)
+      const float inv = 1.0f / sqrtf(group_sum<TI_WAVE>(ss) / (float)dk + eps);
+#pragma unroll
+      for (int i = 0; i < DPL; ++i) {
+        const int d = lane + i * TI_WAVE;
+        if (d < dk) v[k][i] = v[k][i] * inv * nw[d];
+      }
+    }
+    if (half > 0 && pairs) {
+      // neighbours lie in neighbouring lanes
+#pragma unroll
+      for (int i = 0; i < DPL; ++i)
+        if (i * TI_WAVE < 2 * half) {      // (the same in every lane)
+          const float other = __shfl_xor(v[k][i], 1, TI_WAVE);
+          if (lane + i * TI_WAVE < 2 * half) v[k][i] = (lane & 1) ? v[k][i] * c[i] + other * s[i] : v[k][i] * c[i] - other * s[i];
         }
+    } else if (half > 0) {
+#pragma unroll
+      for (int i = 0; i < DPL; ++i) s_h[lane + i * TI_WAVE] = v[k][i];
+      __threadfence_block();      // (a wavefront's LDS accesses are served in order)
+#pragma unroll
+      for (int i = 0; i < DPL; ++i) {
+        const int d = lane + i * TI_WAVE;
+        if (d < 2 * half) v[k][i] = d < half ? s_h[d] * c[i] - s_h[d + half] * s[i] : s_h[d] * c[i] + s_h[d - half] * s[i];
       }
+      __threadfence_block();
     }
-  } else if (half > 0) {
+    if (unit_norm) {
+      float sr = 0.f;
 #pragma unroll
-    for (int i = 0; i < GA_MAX_DPL; ++i) {
-      const int d = lane + i * TI_WAVE;
-      if (d < dk) s_h[d] = v[i];
+      for (int i = 0; i < DPL; ++i) sr = fmaf(v[k][i], v[k][i], sr);
+      const float inv = 1.0f / sqrtf(group_sum<TI_WAVE>(sr) / (float)dk + eps);
+#pragma unroll
+      for (int i = 0; i < DPL; ++i) v[k][i] *= inv;
     }
-    __threadfence_block();      // (a wavefront's LDS accesses are served in order)
+    if (k >= n || (!is_q && page < 0)) continue;      // the host reserves pages first; never write astray
+    T* dst = is_q ? q_out + ((size_t)m * n_head + h) * dk : base + ((size_t)h * P + r) * dk;
 #pragma unroll
-    for (int i = 0; i < GA_MAX_DPL; ++i) {
+    for (int i = 0; i < DPL; ++i) {
       const int d = lane + i * TI_WAVE;
-      if (d < 2 * half) {
-        float c, s;
-        ga_rotation(inv_freq, rope_table, table_len, mag, half, p, d < half ? d : d - half, &c, &s);
-        v[i] = d < half ? s_h[d] * c - s_h[d + half] * s : s_h[d] * c + s_h[d - half] * s;
-      }
-    }
-  }
-  if (unit_norm) {
-    float sr = 0.f;
-#pragma unroll
-    for (int i = 0; i < GA_MAX_DPL; ++i) sr = fmaf(v[i], v[i], sr);      // (entries beyond the head are zero)
-    const float inv = 1.0f / sqrtf(group_sum<TI_WAVE>(sr) / (float)dk + eps);
-#pragma unroll
-    for (int i = 0; i < GA_MAX_DPL; ++i) v[i] *= inv;
-  }
-  if (is_q) {
-    T* dst = q_out + ((size_t)m * n_head + h) * dk;
-#pragma unroll
-    for (int i = 0; i < GA_MAX_DPL; ++i) {
-      const int d = lane + i * TI_WAVE;
-      if (d < dk) st<T>(dst + d, v[i]);
-    }
-    return;
-  }
-  if (page >= 0) {      // the host reserves pages first; never write astray
-    T* dst = base + ((size_t)h * P + r) * dk;
-#pragma unroll
-    for (int i = 0; i < GA_MAX_DPL; ++i) {
-      const int d = lane + i * TI_WAVE;
-      if (d < dk) st<T>(dst + d, v[i]);
+      if (d < dk) st<T>(dst + d, v[k][i]);
     }
   }
 }
@@ -237,19 +234,35 @@ extern "C" int ti_gated_qkv_prep_form(int dtype, const float* proj, int ld, int 
              "gated_qkv_prep: the columns do not lie inside rows of %d", ld);
   if (M == 0) return 0;
   const int n_groups = off_v < 0 ? 0 : (M + GA_V_TOKENS - 1) / GA_V_TOKENS * n_kv;       // workgroups of the values
-  const dim3 grid(M > n_groups ? M : n_groups, (n_head + n_kv + GA_PREP_WAVES - 1) / GA_PREP_WAVES + (n_groups ? 1 : 0));
-  if (dtype == TI_F32)
-    gated_qkv_prep_kernel<float><<<grid, TI_WAVE * GA_PREP_WAVES, 0, stream>>>(proj, ld, off_q, off_k, off_v, q_w, k_w, eps, inv_freq, rope_table,
-                                                               table_len, mag, rot_dims, mix_mode, mix_lambda, v_kept, pos, slot,
-                                                               table, table_stride, (float*)pool, (float*)q_out, M, n_head, n_kv, dk,
-                                                               dv, dvr, page_size, pairs, unit_norm);
-  else if (dtype == TI_BF16)
-    gated_qkv_prep_kernel<bf16_t><<<grid, TI_WAVE * GA_PREP_WAVES, 0, stream>>>(proj, ld, off_q, off_k, off_v, q_w, k_w, eps, inv_freq, rope_table,
-                                                                table_len, mag, rot_dims, mix_mode, mix_lambda, v_kept, pos, slot,
-                                                                table, table_stride, (bf16_t*)pool, (bf16_t*)q_out, M, n_head, n_kv,
-                                                                dk, dv, dvr, page_size, pairs, unit_norm);
+  // few tokens: a wavefront a head; many: four heads a wavefront (the same arithmetic)
+  const int hpw = (long)M * (n_head + n_kv) > 8192 ? 4 : 1;
+  const int per_group = GA_PREP_WAVES * hpw;
+  const dim3 grid(M > n_groups ? M : n_groups, (n_head + n_kv + per_group - 1) / per_group + (n_groups ? 1 : 0));
+#define GA_PREP(T, D, N)                                                                                                               \
+  gated_qkv_prep_kernel<T, D, N><<<grid, TI_WAVE * GA_PREP_WAVES, 0, stream>>>(proj, ld, off_q, off_k, off_v, q_w, k_w, eps, inv_freq, \
+                                                                               rope_table, table_len, mag, rot_dims, mix_mode,         \
+                                                                               mix_lambda, v_kept, pos, slot, table, table_stride,     \
+                                                                               (T*)pool, (T*)q_out, M, n_head, n_kv, dk, dv, dvr,      \
+                                                                               page_size, pairs, unit_norm)
+#define GA_PREP_SIZE(T)                   \
+  do {                                    \
+    if (dk <= 64) {                       \
+      if (hpw == 4) GA_PREP(T, 1, 4);     \
+      else GA_PREP(T, 1, 1);              \
+    } else if (dk <= 128) {               \
+      if (hpw == 4) GA_PREP(T, 2, 4);     \
+      else GA_PREP(T, 2, 1);              \
+    } else {                              \
+      if (hpw == 4) GA_PREP(T, 4, 4);     \
+      else GA_PREP(T, 4, 1);              \
+    }                                     \
+  } while (0)
+  if (dtype == TI_F32) GA_PREP_SIZE(float);
+  else if (dtype == TI_BF16) GA_PREP_SIZE(bf16_t);
   else
     TI_REQUIRE(false, "gated_qkv_prep: unknown dtype %d", dtype);
+#undef GA_PREP_SIZE
+#undef GA_PREP
   TI_LAUNCH_CHECK();
   return 0;
 }
