@@ -63,9 +63,9 @@ moe_group_kernel(const int* __restrict__ ids, int n_pairs, int E, int* __restric
 }
 
 // A workgroup per 64 pairs: where[pair] = its row; rows[row] = bf16(s h[token]), or, with `tokens` in the place of `rows` (inputs
-// without a factor), tokens[row] = its token, for a product that gathers its rows from h.  The workgroup counts its pairs per expert in
-// LDS and takes a run of rows from every expert's cursor at once (one atomic per expert it met, not one per pair); inside the
-// run a pair's place is its count in LDS.
+// without a factor), tokens[row] = its token, for a product that gathers its rows from h.  The workgroup counts its pairs per
+// expert in LDS and takes a run of rows from every expert's cursor at once (one atomic per expert it met, not one per pair);
+// inside the run a pair's place is its count in LDS.
 __global__ void __launch_bounds__(256)
 moe_place_kernel(const bf16_t* __restrict__ h, const int* __restrict__ ids, const float* __restrict__ wts, int* __restrict__ meta,
                  int E, int top, int W, int n_pairs, int* __restrict__ where, bf16_t* __restrict__ rows,
@@ -116,7 +116,8 @@ moe_place_kernel(const bf16_t* __restrict__ h, const int* __restrict__ ids, cons
 // wavefronts two by two, each 64 outputs (four blocks of 16) against 64 rows (four blocks of 16).  A step of 32 along k of both
 // operands is fetched once by the workgroup (thread t the 16-byte pieces t, t + 256) into one of two LDS stages while the step
 // before it is multiplied from the other; one barrier a step.  Rows of a stage are 80 bytes apart, so that the fragments'
-// reads spread over the banks.  tokens (null: none): row r of the operand is row tokens[r] of `rows`.  EPI 0: relu^2, bfloat16; 1: 32-bit; 2: 32-bit, times the row's weight row_w[row].
+// reads spread over the banks.  tokens (null: none): row r of the operand is row tokens[r] of `rows`.  EPI 0: relu^2, bfloat16;
+// 1: 32-bit; 2: 32-bit, times the row's weight row_w[row].
 #define MOE_LDS_ROW 40       // bfloat16 elements between rows of a stage (32 + 8)
 template <int EPI>
 __global__ void __launch_bounds__(256)
@@ -219,8 +220,8 @@ __global__ void moe_combine_kernel(const float* __restrict__ out, const int* __r
 extern "C" long ti_moe_grouped_meta_ints(int n_pairs, int E) { return 1 + (E + 1) + E + 3L * ((n_pairs + MOE_TILE - 1) / MOE_TILE + E); }
 
 // h bf16 [M, W]; ids, wts [M top]; up [E][F][W], down [E][W][F] bf16.  Scratch: meta int32 [ti_moe_grouped_meta_ints],
-// where int32 [M top], rows bf16 [M top][W] (weights on the outputs: int32 [M top], the rows' tokens), act bf16 [M top][F], out f32 [M top][W].  y (may be null): the tokens' sums;
-// without it the caller adds the rows out[where[m top + k]] itself.  The weights multiply the experts' inputs (scale_input) or
+// where int32 [M top], rows bf16 [M top][W] (weights on the outputs: int32 [M top], the rows' tokens), act bf16 [M top][F],
+// out f32 [M top][W].  y (may be null): the tokens' sums; without it the caller adds the rows out[where[m top + k]] itself.  The weights multiply the experts' inputs (scale_input) or
 // their outputs (row_w: f32 scratch [M top]).  3: sizes not served (W, F multiples of 32, E <= 1024).
 extern "C" int ti_moe_experts_grouped_bf16(const void* h, const int* ids, const float* wts, const void* up, const void* down,
                                            int* meta, int* where, void* rows, void* act, float* out, float* y, int M, int W, int F,

@@ -537,6 +537,81 @@ def case_streams_gates_and_decay(ops, rng) -> int:
     return fails
 
 
+def case_sandwich_norms_gru_and_paired_rotation(ops, rng) -> int:
+    """A norm on either side of a sublayer, the minimal GRU, latents of queries and keys, rotation in pairs with unit norms,
+    experts weighted on their outputs with a gate beside the router."""
+    fails = 0
+    D = lambda a, dt=None: _dev(np.asarray(a), dt or (torch.int32 if np.asarray(a).dtype == np.int32 else torch.float32))      # noqa: E731
+    f32 = lambda a: np.asarray(a, dtype=np.float32).astype(np.float64)      # noqa: E731
+    sig = lambda z: 1.0 / (1.0 + np.exp(-z))      # noqa: E731
+    rms = lambda z, eps: z / np.sqrt((z * z).mean(-1, keepdims=True) + eps)      # noqa: E731
+    M, W = 7, 1028
+    x, y, plus = rng.normal(size=(M, W)), rng.normal(size=(2 * M, W)), rng.normal(size=(M, W))
+    gate, g, ng = rng.uniform(size=M), rng.normal(1, 0.2, size=W), rng.normal(1, 0.2, size=W)
+    want = f32(x) + rms(f32(y).reshape(M, 2, W).sum(1) + f32(gate)[:, None] * f32(plus), 1e-5) * f32(g)
+    xd, out = D(x), torch.empty(M, W, device="cuda")
+    ops.norm_residual_next(xd, D(y), D(g), 1e-5, None, 2, D(plus), D(gate), D(ng), 1e-6, out)
+    fails += _say("norm behind a sublayer, onto the residual", float(np.abs(_f64(xd) - want).max()), 5e-5)
+    fails += _say("  the norm in front of the next", float(np.abs(_f64(out) - rms(want, 1e-6) * f32(ng)).max()), 5e-5)
+    # minimal GRU: 150 tokens whole and in chunks of 64
+    T, N = 150, 70
+    proj, bz, bx = rng.normal(size=(T, 3 * N)) * 2, rng.normal(-2, 1, size=N), rng.normal(size=N)
+    p32 = f32(proj)
+    z, u = sig(p32[:, :N] + f32(bz)), p32[:, N:2 * N] + f32(bx)
+    c = np.where(u >= 0, u + 0.5, sig(u))
+    S, want = np.zeros(N), np.zeros((T, N))
+    for t in range(T):
+        S = (1 - z[t]) * S + z[t] * c[t]
+        want[t] = S * p32[t, 2 * N:] * sig(p32[t, 2 * N:])
+    entries = D(np.array([[0, T, 0, 0]], dtype=np.int32))
+    for name, extra in (("whole", ()), ("in chunks", (D(np.array([[0, 0, 64, 1], [0, 64, 64, 0], [0, 128, 22, 2]], dtype=np.int32)),
+                                                     D(np.array([[0, 3]], dtype=np.int32))))):
+        state, o = torch.zeros(1, N, device="cuda"), torch.empty(T, N, device="cuda")
+        ops.mingru_scan(D(proj), D(bz), D(bx), state, entries, o, N, (0, N, 2 * N), *extra)
+        fails += _say(f"minimal GRU, {name}", float(np.abs(_f64(o) - want).max()), 5e-5 * float(np.abs(want).max()))
+    # q and k heads of 24: neighbours of the first 16 entries turned, then divided by their root mean square
+    T, nh, nkv, d, P = 40, 3, 1, 24, 8
+    proj = rng.normal(size=(T, (nh + 2 * nkv) * d))
+    f = np.array([50.0 ** (-2.0 * i / 16) for i in range(8)])
+    ang = np.arange(T)[:, None] * f
+    q = f32(proj)[:, :nh * d].reshape(T, nh, d).copy()
+    a, b = q[:, :, 0:16:2].copy(), q[:, :, 1:16:2].copy()
+    q[:, :, 0:16:2], q[:, :, 1:16:2] = a * np.cos(ang)[:, None] - b * np.sin(ang)[:, None], b * np.cos(ang)[:, None] + a * np.sin(ang)[:, None]
+    table = np.arange(5, dtype=np.int32)[None, :]
+    pool, q_out = torch.zeros(5, nkv, P, 2 * d, device="cuda"), torch.empty(T, nh * d, device="cuda")
+    ops.gated_qkv_prep(D(proj), None, None, D(f), D(np.stack([np.cos(ang), np.sin(ang)], -1)), D(np.arange(T, dtype=np.int32)),
+                       D(np.zeros(T, dtype=np.int32)), D(table), pool, q_out, nh, nkv, d, d, (0, nh * d, (nh + nkv) * d), eps=1e-6, rot_dims=16,
+                       pairs=True, unit_norm=True)
+    fails += _say("rotation in pairs, then unit norms", float(np.abs(_f64(q_out).reshape(T, nh, d) - rms(q, 1e-6)).max()), 5e-5)
+    # both latents of a token normed
+    qr, R = 20, 32
+    proj, kn, qn = rng.normal(size=(T, qr + R)), rng.normal(1, 0.2, size=R), rng.normal(1, 0.2, size=qr)
+    pool, cq = torch.zeros(5, P, R, device="cuda"), torch.empty(T, qr, device="cuda")
+    ops.latent_prep_queries(D(proj), D(kn), D(qn), D(np.arange(T, dtype=np.int32)), D(np.zeros(T, dtype=np.int32)), D(table), pool, cq, qr, 1e-5, 0, qr, R)
+    err = max(np.abs(_f64(cq) - rms(f32(proj)[:, :qr], 1e-5) * f32(qn)).max(), np.abs(_f64(pool).reshape(T, R) - rms(f32(proj)[:, qr:], 1e-5) * f32(kn)).max())
+    fails += _say("latents of queries and of keys and values", float(err), 5e-5)
+    # squared-relu experts times their softmax scores, few tokens and many
+    E, top, W, F = 6, 2, 64, 32
+    router, sg = rng.normal(size=(E, W)) / 4, rng.normal(size=W) / 8
+    up, down = _bf16(rng.normal(size=(E * F, W)) / 6), _bf16(rng.normal(size=(E * W, F)) / 5)
+    for M in (5, 200):
+        h = _bf16(rng.normal(size=(M, W)))
+        ids, wts, gate = torch.empty(M, top, device="cuda", dtype=torch.int32), torch.empty(M, top, device="cuda"), torch.empty(M, device="cuda")
+        hd = D(h, torch.bfloat16)
+        ops.moe_route_grouped(hd, D(router), ids, wts, None, top, renormalize=False, score="softmax", gate_row=D(sg), gate_out=gate)
+        y = torch.empty(M, W, device="cuda")
+        ops.moe_experts(hd, ids, wts, D(up, torch.bfloat16), D(down, torch.bfloat16), y, E, scale_input=False)
+        sc = np.exp(h @ f32(router).T)
+        sc /= sc.sum(1, keepdims=True)
+        want = np.zeros((M, W))
+        for t in range(M):
+            for e in ids.cpu().numpy()[t]:
+                want[t] += sc[t, e] * (down.reshape(E, W, F)[e] @ np.maximum(up.reshape(E, F, W)[e] @ h[t], 0) ** 2)
+        fails += _say(f"experts weighted on their outputs, {M} tokens", float(np.abs(_f64(y) - want).max()), 1e-2 * float(np.abs(want).max()))
+        fails += _say("  the gate beside the router", float(np.abs(_f64(gate) - sig(h @ f32(sg))).max()), 1e-5)
+    return fails
+
+
 def run_selftest() -> int:
     if not torch.cuda.is_available():
         print("[selftest] no GPU: the kernels of this framework run on an AMD GPU (gfx950) only", flush=True)
@@ -565,6 +640,7 @@ def run_selftest() -> int:
     fails += case_diff_attention(ops, rng, nh=4, nkv=2, dk=32, dv=64, T=200, block=150, taps=4, rot=32, dtype=torch.bfloat16)
     fails += case_diff_attention(ops, rng, nh=8, nkv=1, dk=64, dv=128, T=130, block=64, taps=2, rot=16, dtype=torch.bfloat16)
     fails += case_streams_gates_and_decay(ops, rng)
+    fails += case_sandwich_norms_gru_and_paired_rotation(ops, rng)
     fails += case_embed_argmax_sample(ops, rng)
     fails += case_model_shapes(ops, rng)
     fails += case_head_bandwidth(ops, rng)
