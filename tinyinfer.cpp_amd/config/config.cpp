@@ -397,6 +397,7 @@ void ensure_builtin_architectures() {
     architectures().push_back({"Nazorax", nazorax_spec, nazorax_typed_config});
     architectures().push_back({"Dubozen", dubozen_spec, dubozen_typed_config});
     architectures().push_back({"Lupolorn", lupolorn_spec, lupolorn_typed_config});
+    architectures().push_back({"Ruzolorn", ruzolorn_spec, ruzolorn_typed_config});
   });
 }
 

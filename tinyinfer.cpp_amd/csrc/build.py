@@ -30,7 +30,7 @@ FLAGS = ["-O3", "-std=c++17", f"--offload-arch={ARCH}", "-fPIC", "-shared",
          "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
          "-mllvm", "-amdgpu-kernarg-preload-count=16",
          "-Wno-unused-command-line-argument"]
-HEADERS = ["common.h", "qk_prep.h", "tinyinfer_kernels.h", "tinyinfer_kernels_tuning.h"]
+HEADERS = ["common.h", "qk_prep.h", "short_conv.h", "tinyinfer_kernels.h", "tinyinfer_kernels_tuning.h"]
 # flags of single libraries.  The attention kernels rescale their MFMA accumulators with
 # vector instructions; kept in the accumulation registers they would be copied out and back
 # on every turn of the loop, so their MFMAs are told to work on ordinary vector registers.
@@ -53,13 +53,15 @@ ON_DEMAND = ("measure",)
 
 # libraries that only some architectures call into (by the name config.json gives the architecture); every other
 # library serves them all
-ONLY_FOR = {"pointwise": ("Miterax", "Nazorax", "Dubozen"), "recurrent": ("Miterax",), "residual": ("Mumasun", "Lupolorn"), "diff_attention": ("Mumasun",),
-            "diff_attention_bf16": ("Mumasun",), "moe": ("Mumasun", "Nazorax", "Dubozen", "Lupolorn"),
-            "moe_bf16": ("Mumasun", "Nazorax", "Dubozen", "Lupolorn"), "latent_attention": ("Nazorax", "Lupolorn"),
-            "latent_attention_bf16": ("Nazorax", "Lupolorn"), "hyper": ("Dubozen",), "gated_attention": ("Dubozen", "Lupolorn"),
-            "linear_attention": ("Dubozen",), "mingru": ("Lupolorn",)}
+ONLY_FOR = {"pointwise": ("Miterax", "Nazorax", "Dubozen"), "recurrent": ("Miterax",),
+            "residual": ("Mumasun", "Lupolorn", "Ruzolorn"), "diff_attention": ("Mumasun",),
+            "diff_attention_bf16": ("Mumasun",), "moe": ("Mumasun", "Nazorax", "Dubozen", "Lupolorn", "Ruzolorn"),
+            "moe_bf16": ("Mumasun", "Nazorax", "Dubozen", "Lupolorn", "Ruzolorn"), "latent_attention": ("Nazorax", "Lupolorn"),
+            "latent_attention_bf16": ("Nazorax", "Lupolorn"), "hyper": ("Dubozen", "Ruzolorn"),
+            "gated_attention": ("Dubozen", "Lupolorn", "Ruzolorn"), "linear_attention": ("Dubozen", "Ruzolorn"), "mingru": ("Lupolorn",),
+            "short_conv": ("Mumasun", "Ruzolorn")}
 # ... and libraries that a named architecture never calls into
-NOT_FOR = {"attention_generic": ("Mumasun", "Dubozen", "Lupolorn"), "attention_bf16": ("Mumasun",)}
+NOT_FOR = {"attention_generic": ("Mumasun", "Dubozen", "Lupolorn", "Ruzolorn"), "attention_bf16": ("Mumasun",)}
 
 
 def libraries_for(dtype: str, architecture: str = None) -> List[str]:
@@ -94,7 +96,7 @@ def architecture_of(model_dir: str):
 # and the C interface the Python package binds): C++17, no device code
 PKG = os.path.dirname(HERE)
 HOST_SOURCES = ["config/json.cpp", "config/config.cpp", "config/miterax.cpp", "config/mumasun.cpp", "config/nazorax.cpp", "config/dubozen.cpp",
-                "config/lupolorn.cpp", "ops/ops.cpp", "parts/parts.cpp", "weights/weights.cpp",
+                "config/lupolorn.cpp", "config/ruzolorn.cpp", "ops/ops.cpp", "parts/parts.cpp", "weights/weights.cpp",
                 "models/model.cpp", "cache/cache_manager.cpp", "engine/engine.cpp", "engine/scheduler.cpp",
                 "sampling/sampler.cpp", "engine/c_api.cpp"]
 HOST_HEADERS = ["include/inference.h", "config/read.h", "weights/weights.h", "csrc/tinyinfer_kernels.h"]

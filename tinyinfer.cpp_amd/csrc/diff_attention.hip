@@ -1,7 +1,6 @@
 // Differential attention for any sizes, float32 or bfloat16 storage, 32-bit arithmetic:
-//   a short causal convolution over time on the channels of a fused q/k/v projection, with the last
-//   taps - 1 projected rows of every request kept as its state;
-//   the preparation of queries and keys (RMS norm per head and map, rotation of the first `rot_dims`
+//   the preparation of queries and keys (a short causal convolution over time on the channels of the fused projection
+//   where a layer has one, RMS norm per head and map, rotation of the first `rot_dims`
 //   entries in the half-split layout) and the cache write;
 //   the attention itself: every query head holds two maps (two queries against two keys, one value),
 //   each an ordinary softmax over the visible keys; o = a1 - lambda a2, divided by its root mean
@@ -10,63 +9,10 @@
 // counted from position 0 (block 0: no blocks) and, with a window, at most window - 1 behind.
 // A page is K [n_kv][P][2 dk] (a row's two maps side by side) | V [n_kv][dv][P].
 #include "common.h"
+#include "short_conv.h"
 #include "tinyinfer_kernels.h"
 
 TI_ERROR_API
-
-// ------------------------------------------------------------ short convolution over time
-// out[m, c] = sum_j taps[c][j] * u(p - (K - 1) + j)[c], p the position of row m.  Rows of positions from the
-// entry's start on are rows of this step; earlier ones are the request's state [K - 1][C] (row i is position
-// start - (K - 1) + i; zeros at admission stand for what lies before the sequence).  Ascending j, fused
-// multiply-adds: the same bits however the tokens were cut into steps.
-__global__ void __launch_bounds__(256)
-short_conv_kernel(const float* __restrict__ u, const float* __restrict__ taps, const float* __restrict__ state,
-                  const int* __restrict__ entries, const int* __restrict__ entry_of, const int* __restrict__ pos,
-                  float* __restrict__ out, int C, int K) {
-  const int m = blockIdx.x;
-  const int e = entry_of[m];
-  const int row0 = entries[4 * e], start = entries[4 * e + 2], slot = entries[4 * e + 3];
-  const int p = pos[m];
-  const float* st_rows = state + (size_t)slot * (K - 1) * C;
-  for (int c = threadIdx.x; c < C; c += 256) {
-    float acc = 0.f;
-    for (int j = 0; j < K; ++j) {
-      const int s = p - (K - 1) + j;
-      const float v = s >= start ? u[(size_t)(row0 + s - start) * C + c] : st_rows[(size_t)(s - start + K - 1) * C + c];
-      acc = fmaf(taps[(size_t)c * K + j], v, acc);
-    }
-    out[(size_t)m * C + c] = acc;
-  }
-}
-
-// the state after the step: the last K - 1 rows of the sequence so far.  A thread owns a channel and walks the
-// state's rows upwards: what it still reads of the old state lies above what it has written.
-__global__ void __launch_bounds__(256)
-short_conv_state_kernel(const float* __restrict__ u, float* __restrict__ state, const int* __restrict__ entries, int C, int K) {
-  const int e = blockIdx.x;
-  const int row0 = entries[4 * e], n = entries[4 * e + 1], slot = entries[4 * e + 3];
-  float* st_rows = state + (size_t)slot * (K - 1) * C;
-  for (int c = blockIdx.y * 256 + threadIdx.x; c < C; c += gridDim.y * 256)
-    for (int i = 0; i < K - 1; ++i) {
-      const int r = n - (K - 1) + i;      // the step's row that lands here; below zero: a row the state already holds
-      st_rows[(size_t)i * C + c] = r >= 0 ? u[(size_t)(row0 + r) * C + c] : st_rows[(size_t)(i + n) * C + c];
-    }
-}
-
-extern "C" int ti_short_conv(const float* u, const float* taps, float* state, const int* entries, int n_entries,
-                             const int* entry_of, const int* pos, float* out, int M, int C, int K, hipStream_t stream) {
-  TI_REQUIRE(M >= 0 && C > 0 && K >= 1 && n_entries >= 0, "short_conv: bad sizes M=%d C=%d taps=%d", M, C, K);
-  TI_REQUIRE(K == 1 || state, "short_conv: %d taps need a state", K);
-  if (M == 0) return 0;
-  short_conv_kernel<<<M, 256, 0, stream>>>(u, taps, state, entries, entry_of, pos, out, C, K);
-  TI_LAUNCH_CHECK();
-  if (K > 1 && n_entries > 0) {
-    dim3 grid(n_entries, (C + 255) / 256 < 64 ? (C + 255) / 256 : 64);
-    short_conv_state_kernel<<<grid, 256, 0, stream>>>(u, state, entries, C, K);
-    TI_LAUNCH_CHECK();
-  }
-  return 0;
-}
 
 // ------------------------------------------------------------ queries and keys prepared, cache written
 // qkv f32 [M, n_head 2 dk + n_kv 2 dk + n_kv dv].  Every run of dk entries of q and k (a head's map) is divided
@@ -74,8 +20,8 @@ extern "C" int ti_short_conv(const float* u, const float* taps, float* state, co
 // first rot_dims entries are turned: entry i with entry i + rot_dims / 2 by the angle pos * inv_freq[i], cosine and
 // sine times `mag` (the table [table_len][rot_dims / 2][2] holds them ready for positions below table_len).
 // q goes to q_out (T) [M, n_head 2 dk], k and v into the page of the token's position.
-// CONV: the rows of qkv are what the projection left, and every channel first passes the short convolution above (taps,
-// state, entries, entry_of as in short_conv_kernel; the state itself is moved on by short_conv_state_kernel afterwards):
+// CONV: the rows of qkv are what the projection left, and every channel first passes the short convolution of ti_short_conv
+// (taps, state, entries, entry_of as there; the state itself is moved on by short_conv_state_kernel afterwards):
 // the same sums in the same order as the convolution on its own, so the same bits.
 template <typename T, bool CONV>
 __global__ void __launch_bounds__(256)
@@ -197,7 +143,7 @@ extern "C" int ti_diff_qk_prep(int dtype, const float* qkv, const float* taps, f
   if (taps && K > 1 && n_entries > 0) {
     const int C = n_head * 2 * dk + n_kv * (2 * dk + dv);
     dim3 grid(n_entries, (C + 255) / 256 < 64 ? (C + 255) / 256 : 64);
-    short_conv_state_kernel<<<grid, 256, 0, stream>>>(qkv, state, entries, C, K);
+    short_conv_state_kernel<<<grid, 256, 0, stream>>>(qkv, C, state, entries, C, K);
     TI_LAUNCH_CHECK();
   }
   return 0;

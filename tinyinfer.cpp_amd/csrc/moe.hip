@@ -256,19 +256,14 @@ __device__ __forceinline__ void next_pairs(const int* __restrict__ ids, int n_pa
   }
 }
 
-// z[r][p] = rows[p] . b[r] for the NP rows in LDS (T) and MOE_ROWS rows of the weight in memory, K apart (rows of the weight
-// beyond the last one are read as the last one): the loads of all the weight's rows are in flight together.  Every sum runs
-// over a lane's pieces in ascending order, then a butterfly.
+// z[r][p] = rows[p] . br[r] for the NP rows in LDS (T) and MOE_ROWS rows of the weight in memory: the loads of all the weight's
+// rows are in flight together.  Every sum runs over a lane's pieces in ascending order, then a butterfly.
 template <typename T, bool VEC, int NP>
-__device__ __forceinline__ void wave_dots(const T* rows, int n_live, const T* __restrict__ b, int n_rows_w, int K, int lane,
-                                          float (*z)[NP]) {
+__device__ __forceinline__ void wave_dots(const T* rows, int n_live, const T* const* br, int K, int lane, float (*z)[NP]) {
 #pragma unroll
   for (int r = 0; r < MOE_ROWS; ++r)
 #pragma unroll
     for (int p = 0; p < NP; ++p) z[r][p] = 0.f;
-  const T* br[MOE_ROWS];
-#pragma unroll
-  for (int r = 0; r < MOE_ROWS; ++r) br[r] = b + (size_t)(r < n_rows_w ? r : n_rows_w - 1) * K;
   if (VEC) {
     constexpr int N = Piece<T>::N;
     for (int c = lane * N; c < K; c += 64 * N) {
@@ -306,52 +301,80 @@ __device__ __forceinline__ void wave_dots(const T* rows, int n_live, const T* __
     for (int p = 0; p < NP; ++p) z[r][p] = group_sum<64>(z[r][p]);
 }
 
-// DOWN false: rows are the tokens' inputs h (scaled by the score where it scales the input), K = W, outputs F, relu^2 to act.
-// DOWN true: rows are act, K = F, outputs W, 32-bit to part (times the score where it scales the output).
-// plain (DOWN false): the sums are stored as they are, in 32-bit (a gated activation over [gate | up] follows in a kernel of its own).
-template <typename T, bool VEC, int NP, bool DOWN>
+// a gated expert's activation of the two sums.  kind 0: silu(g) u; 1: g = min(g, limit), u = clamp(u, -limit, limit),
+// g sigmoid(alpha g) (u + 1)
+__device__ __forceinline__ float moe_gate(float g, float u, int kind, float limit, float alpha) {
+  if (kind == 0) return g / (1.0f + expf(-g)) * u;
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+}
+
+// what a workgroup per (expert, outputs) does
+#define MOE_UP 0       // in: the tokens' inputs h (scaled by the score where it scales the input), K = W, N = F outputs: relu^2 to act (T)
+#define MOE_GATED 1    // in: h, K = W, N = F: an expert's weight is [2 F][W], gate rows above up rows; the gated activation to act (T)
+#define MOE_DOWN 2     // in: act, K = F, N = W: 32-bit to part (times the score where it scales the output)
+// ids from E on are identity experts: MOE_DOWN's workgroups of blockIdx.x = E (launched where there are any) write their
+// pairs' rows of part, the score times the token's row of `self`.
+struct MoeRows { int n_pairs, K, N, top, scale_input, E, kind; float limit, alpha; };
+template <typename T, bool VEC, int NP, int FORM>
 __global__ void __launch_bounds__(256)
 moe_expert_rows_kernel(const T* __restrict__ in, const int* __restrict__ ids, const float* __restrict__ wts, const T* __restrict__ w,
-                       void* __restrict__ out, int n_pairs, int K, int N, int top, int scale_input, int plain) {
+                       void* __restrict__ out, const T* __restrict__ self, const MoeRows a) {
   extern __shared__ __attribute__((aligned(16))) unsigned char raw[];
   T* rows = reinterpret_cast<T*>(raw);      // [NP][K]
   __shared__ int s_pairs[NP], s_found[2];
-  const int e = blockIdx.x;
+  const int e = blockIdx.x, K = a.K, N = a.N;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int n0 = (blockIdx.y * 4 + wave) * MOE_ROWS;
-  const T* we = w + (size_t)e * N * K;
+  if (FORM == MOE_DOWN && e == a.E) {
+    for (int pair = blockIdx.y; pair < a.n_pairs; pair += gridDim.y) {
+      if (ids[pair] < a.E) continue;
+      const float s = wts[pair];
+      for (int c = threadIdx.x; c < N; c += 256) ((float*)out)[(size_t)pair * N + c] = ld<T>(self + (size_t)(pair / a.top) * N + c) * s;
+    }
+    return;
+  }
+  constexpr int OUT = FORM == MOE_GATED ? MOE_ROWS / 2 : MOE_ROWS;      // outputs a wavefront
+  const int n0 = (blockIdx.y * 4 + wave) * OUT;
+  const T* we = w + (size_t)e * (FORM == MOE_GATED ? 2 * N : N) * K;
+  const T* br[MOE_ROWS];      // (outputs beyond the last one: the last one's rows)
+#pragma unroll
+  for (int r = 0; r < MOE_ROWS; ++r) {
+    const int n = min(n0 + r % OUT, N - 1);
+    br[r] = we + (size_t)(r < OUT ? n : N + n) * K;
+  }
   int next = 0;
-  while (next < n_pairs) {
-    if (wave == 0) next_pairs<NP>(ids, n_pairs, e, next, s_pairs, s_found);
+  while (next < a.n_pairs) {
+    if (wave == 0) next_pairs<NP>(ids, a.n_pairs, e, next, s_pairs, s_found);
     __syncthreads();
     const int n_live = s_found[0];
     next = s_found[1];
     if (n_live == 0) break;
     for (int p = 0; p < n_live; ++p) {
       const int pair = s_pairs[p];
-      const T* src = DOWN ? in + (size_t)pair * K : in + (size_t)(pair / top) * K;
-      const float s = (!DOWN && scale_input) ? wts[pair] : 1.f;
-      for (int c = threadIdx.x; c < K; c += 256) st<T>(rows + (size_t)p * K + c, DOWN ? ld<T>(src + c) : ld<T>(src + c) * s);
+      const T* src = FORM == MOE_DOWN ? in + (size_t)pair * K : in + (size_t)(pair / a.top) * K;
+      const float s = (FORM == MOE_UP && a.scale_input) ? wts[pair] : 1.f;
+      for (int c = threadIdx.x; c < K; c += 256) st<T>(rows + (size_t)p * K + c, FORM == MOE_UP ? ld<T>(src + c) * s : ld<T>(src + c));
     }
     __syncthreads();
     if (n0 < N) {
       float z[MOE_ROWS][NP];
-      const int n_rows_w = min(MOE_ROWS, N - n0);
-      wave_dots<T, VEC, NP>(rows, n_live, we + (size_t)n0 * K, n_rows_w, K, lane, z);
+      wave_dots<T, VEC, NP>(rows, n_live, br, K, lane, z);
       if (lane == 0) {
 #pragma unroll
-        for (int r = 0; r < MOE_ROWS; ++r)
+        for (int r = 0; r < OUT; ++r)
 #pragma unroll
           for (int p = 0; p < NP; ++p)
-            if (r < n_rows_w && p < n_live) {
-              const int pair = s_pairs[p], n = n0 + r;
-              if (DOWN) {
-                ((float*)out)[(size_t)pair * N + n] = scale_input ? z[r][p] : z[r][p] * wts[pair];
-              } else if (plain) {      // the sums themselves, 32-bit: an activation over several of them follows
-                ((float*)out)[(size_t)pair * N + n] = z[r][p];
+            if (n0 + r < N && p < n_live) {
+              const int pair = s_pairs[p];
+              const size_t at = (size_t)pair * N + n0 + r;
+              if (FORM == MOE_DOWN) {
+                ((float*)out)[at] = a.scale_input ? z[r][p] : z[r][p] * wts[pair];
+              } else if (FORM == MOE_GATED) {
+                st<T>((T*)out + at, moe_gate(z[r][p], z[(r + OUT) % MOE_ROWS][p], a.kind, a.limit, a.alpha));
               } else {
-                const float a = fmaxf(z[r][p], 0.f);
-                st<T>((T*)out + (size_t)pair * N + n, a * a);
+                const float v = fmaxf(z[r][p], 0.f);
+                st<T>((T*)out + at, v * v);
               }
             }
       }
@@ -370,51 +393,55 @@ __global__ void moe_sum_pairs_kernel(const float* __restrict__ part, float* __re
   }
 }
 
-template <typename T, bool VEC, int NP, bool DOWN>
-static void launch_expert_rows(const void* in, const int* ids, const float* wts, const void* w, void* out, int n_pairs, int K, int N,
-                               int top, int scale_input, int E, hipStream_t stream, int plain) {
-  const dim3 grid(E, (N + 4 * MOE_ROWS - 1) / (4 * MOE_ROWS));
-  moe_expert_rows_kernel<T, VEC, NP, DOWN><<<grid, 256, (size_t)NP * K * sizeof(T), stream>>>((const T*)in, ids, wts, (const T*)w, out,
-                                                                                               n_pairs, K, N, top, scale_input, plain);
+template <typename T, bool VEC, int NP, int FORM>
+static void launch_expert_rows(const void* in, const int* ids, const float* wts, const void* w, void* out, const void* self, const MoeRows& a,
+                               hipStream_t stream) {
+  const int each = 4 * (FORM == MOE_GATED ? MOE_ROWS / 2 : MOE_ROWS);
+  const dim3 grid(a.E + (FORM == MOE_DOWN && self ? 1 : 0), (a.N + each - 1) / each);
+  moe_expert_rows_kernel<T, VEC, NP, FORM><<<grid, 256, (size_t)NP * a.K * sizeof(T), stream>>>((const T*)in, ids, wts, (const T*)w, out,
+                                                                                                 (const T*)self, a);
 }
-template <typename T, bool VEC, bool DOWN>
-static int expert_rows(const void* in, const int* ids, const float* wts, const void* w, void* out, int n_pairs, int K, int N, int top,
-                       int scale_input, int E, hipStream_t stream, int plain = 0) {
-  const size_t row = (size_t)K * sizeof(T), room = 48 * 1024;      // rows of the pairs a round holds in LDS
-  if (4 * row <= room) launch_expert_rows<T, VEC, 4, DOWN>(in, ids, wts, w, out, n_pairs, K, N, top, scale_input, E, stream, plain);
-  else if (2 * row <= room) launch_expert_rows<T, VEC, 2, DOWN>(in, ids, wts, w, out, n_pairs, K, N, top, scale_input, E, stream, plain);
-  else if (row <= 64 * 1024) launch_expert_rows<T, VEC, 1, DOWN>(in, ids, wts, w, out, n_pairs, K, N, top, scale_input, E, stream, plain);
+template <typename T, bool VEC, int FORM>
+static int expert_rows(const void* in, const int* ids, const float* wts, const void* w, void* out, const void* self, const MoeRows& a,
+                       hipStream_t stream) {
+  const size_t row = (size_t)a.K * sizeof(T), room = 48 * 1024;      // rows of the pairs a round holds in LDS
+  if (4 * row <= room) launch_expert_rows<T, VEC, 4, FORM>(in, ids, wts, w, out, self, a, stream);
+  else if (2 * row <= room) launch_expert_rows<T, VEC, 2, FORM>(in, ids, wts, w, out, self, a, stream);
+  else if (row <= 64 * 1024) launch_expert_rows<T, VEC, 1, FORM>(in, ids, wts, w, out, self, a, stream);
   else return 1;
   return 0;
 }
 
-// act: scratch in the dtype of h, [M top][F]; part: f32 [M top][W], a token's rows to be added in ascending order: into y where
-// y is given, else by the caller
-extern "C" int ti_moe_experts_rows(int dtype, const void* h, const int* ids, const float* wts, const void* up, const void* down,
-                                   void* act, float* part, float* y, int M, int W, int F, int E, int top, int scale_input,
-                                   hipStream_t stream) {
+// both products of all pairs: act (T) [n_pairs][F], part f32 [n_pairs][W]
+template <typename T, bool VEC, int UP>
+static int experts_rows(const void* h, const int* ids, const float* wts, const void* up, const void* down, void* act, float* part, int M, int W,
+                        int F, int E, int top, int scale_input, int identity, int kind, float limit, float alpha, hipStream_t stream) {
+  MoeRows a = {M * top, W, F, top, scale_input, E, kind, limit, alpha};
+  int rc = expert_rows<T, VEC, UP>(h, ids, wts, up, act, nullptr, a, stream);
+  a.K = F;
+  a.N = W;
+  if (rc == 0) rc = expert_rows<T, VEC, MOE_DOWN>(act, ids, wts, down, part, identity ? h : nullptr, a, stream);
+  return rc;
+}
+
+template <int UP>
+static int experts_rows_any(int dtype, const void* h, const int* ids, const float* wts, const void* up, const void* down, void* act, float* part,
+                            float* y, int M, int W, int F, int E, int top, int scale_input, int identity, int kind, float limit, float alpha,
+                            hipStream_t stream) {
   TI_REQUIRE(M >= 0 && W > 0 && F > 0 && top > 0 && E > 0, "moe_experts: bad sizes M=%d W=%d F=%d top=%d", M, W, F, top);
+  TI_REQUIRE(dtype == TI_F32 || dtype == TI_BF16, "moe_experts: unknown dtype %d", dtype);
   if (M == 0) return 0;
-  TI_REQUIRE((F + 4 * MOE_ROWS - 1) / (4 * MOE_ROWS) <= 65535 && (W + 4 * MOE_ROWS - 1) / (4 * MOE_ROWS) <= 65535,
-             "moe_experts: sizes W=%d F=%d are too large", W, F);
-  const int es = dtype == TI_F32 ? 4 : 2;
-  const int piece = 16 / es;
+  TI_REQUIRE((F + 7) / 8 <= 65535 && (W + 15) / 16 <= 65535, "moe_experts: sizes W=%d F=%d are too large", W, F);
+  const int piece = 16 / (dtype == TI_F32 ? 4 : 2);
   const bool vec = W % piece == 0 && F % piece == 0 && (((uintptr_t)up | (uintptr_t)down | (uintptr_t)act | (uintptr_t)h) & 15) == 0;
-  const int n_pairs = M * top;
   int rc;
-#define MOE_BOTH(T, V)                                                                                              \
-  do {                                                                                                              \
-    rc = expert_rows<T, V, false>(h, ids, wts, up, act, n_pairs, W, F, top, scale_input, E, stream);                \
-    if (rc == 0) rc = expert_rows<T, V, true>(act, ids, wts, down, part, n_pairs, F, W, top, scale_input, E, stream); \
-  } while (0)
+#define MOE_BOTH(T, V) rc = experts_rows<T, V, UP>(h, ids, wts, up, down, act, part, M, W, F, E, top, scale_input, identity, kind, limit, alpha, stream)
   if (dtype == TI_F32) {
     if (vec) MOE_BOTH(float, true);
     else MOE_BOTH(float, false);
-  } else if (dtype == TI_BF16) {
+  } else {
     if (vec) MOE_BOTH(bf16_t, true);
     else MOE_BOTH(bf16_t, false);
-  } else {
-    TI_REQUIRE(false, "moe_experts: unknown dtype %d", dtype);
   }
 #undef MOE_BOTH
   TI_REQUIRE(rc == 0, "moe_experts: a row of %d or %d entries does not fit the workgroup's 64 KB", W, F);
@@ -423,64 +450,20 @@ extern "C" int ti_moe_experts_rows(int dtype, const void* h, const int* ids, con
   return 0;
 }
 
-// ------------------------------------------------------------ gated experts
-// y[m] = sum_k s_k W_down[e_k] act(W_gate[e_k] h, W_up[e_k] h): gate_up [E][2F][W] holds an expert's gate rows above its up rows.
-//   act_kind 1: g = min(g, limit), u = clamp(u, -limit, limit); g * sigmoid(alpha g) * (u + 1)        0: silu(g) * u
-// z: f32 scratch [M top][2F] (the two products' sums), act: scratch of the dtype of h [M top][F], part: f32 [M top][W].
-template <typename T>
-__global__ void moe_gate_kernel(const float* __restrict__ z, T* __restrict__ act, long n_pairs, int F, int kind, float limit, float alpha) {
-  const long n = n_pairs * F;
-  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long)gridDim.x * blockDim.x) {
-    const long pair = i / F;
-    const int f = (int)(i % F);
-    float g = z[pair * 2 * F + f], u = z[pair * 2 * F + F + f];
-    float y;
-    if (kind == 0) {
-      y = g / (1.0f + expf(-g)) * u;
-    } else {
-      g = fminf(g, limit);
-      u = fminf(fmaxf(u, -limit), limit);
-      y = g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
-    }
-    st<T>(act + i, y);
-  }
+// act: scratch in the dtype of h, [M top][F]; part: f32 [M top][W], a token's rows to be added in ascending order: into y where
+// y is given, else by the caller.  identity: ids from E on are identity experts
+extern "C" int ti_moe_experts_rows(int dtype, const void* h, const int* ids, const float* wts, const void* up, const void* down,
+                                   void* act, float* part, float* y, int M, int W, int F, int E, int top, int scale_input, int identity,
+                                   hipStream_t stream) {
+  return experts_rows_any<MOE_UP>(dtype, h, ids, wts, up, down, act, part, y, M, W, F, E, top, scale_input, identity, 0, 0.f, 0.f, stream);
 }
 
+// gated experts: y[m] = sum_k s_k W_down[e_k] act(W_gate[e_k] h, W_up[e_k] h): gate_up [E][2F][W] holds an expert's gate rows above
+// its up rows; act_kind as moe_gate's
 extern "C" int ti_moe_experts_rows_gated(int dtype, const void* h, const int* ids, const float* wts, const void* gate_up, const void* down,
-                                         float* z, void* act, float* part, float* y, int M, int W, int F, int E, int top, int act_kind,
-                                         float limit, float alpha, hipStream_t stream) {
-  TI_REQUIRE(M >= 0 && W > 0 && F > 0 && top > 0 && E > 0, "moe_experts: bad sizes M=%d W=%d F=%d top=%d", M, W, F, top);
+                                         void* act, float* part, float* y, int M, int W, int F, int E, int top, int act_kind, float limit,
+                                         float alpha, int identity, hipStream_t stream) {
   TI_REQUIRE(act_kind == 0 || act_kind == 1, "moe_experts: unknown gated activation %d", act_kind);
-  if (M == 0) return 0;
-  TI_REQUIRE((2 * F + 4 * MOE_ROWS - 1) / (4 * MOE_ROWS) <= 65535 && (W + 4 * MOE_ROWS - 1) / (4 * MOE_ROWS) <= 65535,
-             "moe_experts: sizes W=%d F=%d are too large", W, F);
-  const int es = dtype == TI_F32 ? 4 : 2;
-  const int piece = 16 / es;
-  const bool vec = W % piece == 0 && F % piece == 0 && (((uintptr_t)gate_up | (uintptr_t)down | (uintptr_t)act | (uintptr_t)h) & 15) == 0;
-  const int n_pairs = M * top;
-  const long n_act = (long)n_pairs * F;
-  const unsigned blocks = (unsigned)((n_act + 255) / 256 < 16384 ? (n_act + 255) / 256 : 16384);
-  int rc;
-#define MOE_GATED(T, V)                                                                                                 \
-  do {                                                                                                                  \
-    rc = expert_rows<T, V, false>(h, ids, wts, gate_up, z, n_pairs, W, 2 * F, top, 0, E, stream, 1);                    \
-    if (rc == 0) {                                                                                                      \
-      moe_gate_kernel<T><<<blocks, 256, 0, stream>>>(z, (T*)act, n_pairs, F, act_kind, limit, alpha);                   \
-      rc = expert_rows<T, V, true>(act, ids, wts, down, part, n_pairs, F, W, top, 0, E, stream);                        \
-    }                                                                                                                   \
-  } while (0)
-  if (dtype == TI_F32) {
-    if (vec) MOE_GATED(float, true);
-    else MOE_GATED(float, false);
-  } else if (dtype == TI_BF16) {
-    if (vec) MOE_GATED(bf16_t, true);
-    else MOE_GATED(bf16_t, false);
-  } else {
-    TI_REQUIRE(false, "moe_experts: unknown dtype %d", dtype);
-  }
-#undef MOE_GATED
-  TI_REQUIRE(rc == 0, "moe_experts: a row of %d or %d entries does not fit the workgroup's 64 KB", W, F);
-  if (y) moe_sum_pairs_kernel<<<M, 256, 0, stream>>>(part, y, W, top);
-  TI_LAUNCH_CHECK();
-  return 0;
+  return experts_rows_any<MOE_GATED>(dtype, h, ids, wts, gate_up, down, act, part, y, M, W, F, E, top, 0, identity, act_kind, limit, alpha,
+                                     stream);
 }

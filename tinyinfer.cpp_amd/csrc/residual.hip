@@ -78,19 +78,21 @@ extern "C" int ti_norm_residual(float* x, const float* y, const float* g, const 
 }
 
 // Layers with a norm on either side of a sublayer, both in one pass over the row:
-//   x[m] += y'[m] / sqrt(mean(y'[m]^2) + eps) * g,   then   out[m] = x[m] / sqrt(mean(x[m]^2) + next_eps) * next_g  (RT)
-// y'[m]: the rows of y as above, in ascending order, and behind them plus_gate[m] plus[m] (plus null: none; plus_gate null:
-// times one).  out null: the first line alone.  A workgroup per row; x, y' and both gains are asked for before the first
-// sum is known and stay in registers: NV pieces of four elements a thread (NV 0: any width, element by element from memory).
+//   x[m] += factor N(y'[m]) g,   then   out[m] = N(x[m]) next_g  (RT)
+// with N(z) = z / sqrt(mean(z^2) + eps), or, centered, (z - mean z) / sqrt(mean((z - mean z)^2) + eps).
+// y'[m]: y_scale times the rows of y as above, in ascending order, and behind them plus_scale plus_gate[m] plus[m] (plus null:
+// none; plus_gate null: one).  out null: the first line alone.  A workgroup per row; x, y' and both gains are asked for before
+// the first sum is known and stay in registers: NV pieces of four elements a thread (NV 0: any width, element by element from
+// memory).
 template <typename RT, int NV>
 __global__ void __launch_bounds__(256)
 norm_residual_next_kernel(float* __restrict__ x, const float* __restrict__ y, const int* __restrict__ gather, int n_gather,
-                          const float* __restrict__ plus, const float* __restrict__ plus_gate, const float* __restrict__ g, float eps,
-                          const float* __restrict__ next_g, float next_eps, RT* __restrict__ out, int H) {
+                          const float* __restrict__ plus, const float* __restrict__ plus_gate, const ti_norm_pair p, RT* __restrict__ out,
+                          int H) {
   __shared__ float red[4];
   const int m = blockIdx.x;
   const int terms = (gather || n_gather > 1) ? n_gather : 1;
-  const float pg = plus_gate ? plus_gate[m] : 1.f;
+  const float pg = p.plus_scale * (plus_gate ? plus_gate[m] : 1.f);
   float* const row = x + (size_t)m * H;
   auto source = [&](int k) { return y + (gather ? (size_t)gather[(size_t)m * n_gather + k] : (size_t)m * terms + k) * H; };
   if constexpr (NV > 0) {
@@ -102,8 +104,8 @@ norm_residual_next_kernel(float* __restrict__ x, const float* __restrict__ y, co
       v[j] = xv[j] = gv[j] = nv[j] = zero;
       if (i < H) {
         xv[j] = *reinterpret_cast<const float4*>(row + i);
-        gv[j] = *reinterpret_cast<const float4*>(g + i);
-        if (out) nv[j] = *reinterpret_cast<const float4*>(next_g + i);
+        gv[j] = *reinterpret_cast<const float4*>(p.g + i);
+        if (out) nv[j] = *reinterpret_cast<const float4*>(p.next_g + i);
       }
     }
     for (int k = 0; k < terms; ++k) {
@@ -117,28 +119,46 @@ norm_residual_next_kernel(float* __restrict__ x, const float* __restrict__ y, co
         }
       }
     }
-    float ss = 0.f;
+    if (p.y_scale != 1.f) {
 #pragma unroll
-    for (int j = 0; j < NV; ++j) {
-      const int i = (j * 256 + threadIdx.x) * 4;
-      if (plus && i < H) {
-        const float4 a = *reinterpret_cast<const float4*>(plus + (size_t)m * H + i);
-        v[j] = make_float4(fmaf(pg, a.x, v[j].x), fmaf(pg, a.y, v[j].y), fmaf(pg, a.z, v[j].z), fmaf(pg, a.w, v[j].w));
-      }
-      ss = rms_accumulate(ss, v[j]);
+      for (int j = 0; j < NV; ++j) v[j] = make_float4(v[j].x * p.y_scale, v[j].y * p.y_scale, v[j].z * p.y_scale, v[j].w * p.y_scale);
     }
-    const float scale = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)H + eps);
-    float s2 = 0.f;
+    if (plus) {
+#pragma unroll
+      for (int j = 0; j < NV; ++j) {
+        const int i = (j * 256 + threadIdx.x) * 4;
+        if (i < H) {
+          const float4 a = *reinterpret_cast<const float4*>(plus + (size_t)m * H + i);
+          v[j] = make_float4(fmaf(pg, a.x, v[j].x), fmaf(pg, a.y, v[j].y), fmaf(pg, a.z, v[j].z), fmaf(pg, a.w, v[j].w));
+        }
+      }
+    }
+    // the row in the threads' registers becomes what N divides (its mean off where centered), the result is the divisor's inverse
+    auto inverse = [&](float4* z, int centered, float eps) {
+      if (centered) {
+        float sum = 0.f;
+#pragma unroll
+        for (int j = 0; j < NV; ++j) sum += (z[j].x + z[j].y) + (z[j].z + z[j].w);      // (zeros beyond the row)
+        const float mean = block_sum<256>(sum, red) / (float)H;
+#pragma unroll
+        for (int j = 0; j < NV; ++j)
+          if ((j * 256 + (int)threadIdx.x) * 4 < H) z[j] = make_float4(z[j].x - mean, z[j].y - mean, z[j].z - mean, z[j].w - mean);
+      }
+      float ss = 0.f;
+#pragma unroll
+      for (int j = 0; j < NV; ++j) ss = rms_accumulate(ss, z[j]);
+      return 1.0f / sqrtf(block_sum<256>(ss, red) / (float)H + eps);
+    };
+    const float scale = p.factor * inverse(v, p.centered, p.eps);
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int i = (j * 256 + threadIdx.x) * 4;
       xv[j] = make_float4(xv[j].x + v[j].x * scale * gv[j].x, xv[j].y + v[j].y * scale * gv[j].y, xv[j].z + v[j].z * scale * gv[j].z,
                           xv[j].w + v[j].w * scale * gv[j].w);
       if (i < H) *reinterpret_cast<float4*>(row + i) = xv[j];
-      s2 = rms_accumulate(s2, xv[j]);
     }
     if (!out) return;
-    const float next = 1.0f / sqrtf(block_sum<256>(s2, red) / (float)H + next_eps);
+    const float next = inverse(xv, p.next_centered, p.next_eps);
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int i = (j * 256 + threadIdx.x) * 4;
@@ -158,34 +178,41 @@ norm_residual_next_kernel(float* __restrict__ x, const float* __restrict__ y, co
         const float a = source(k)[i];
         v = k == 0 ? a : v + a;
       }
+      v *= p.y_scale;
       return plus ? fmaf(pg, plus[(size_t)m * H + i], v) : v;
     };
-    float ss = 0.f, s2 = 0.f;
-    for (int i = threadIdx.x; i < H; i += 256) {
-      const float v = value(i);
-      ss = fmaf(v, v, ss);
-    }
-    const float scale = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)H + eps);
-    for (int i = threadIdx.x; i < H; i += 256) {
-      const float now = row[i] + value(i) * scale * g[i];
-      row[i] = now;
-      s2 = fmaf(now, now, s2);
-    }
+    auto inverse = [&](auto z, int centered, float eps, float* mean) {
+      *mean = 0.f;
+      if (centered) {
+        float sum = 0.f;
+        for (int i = threadIdx.x; i < H; i += 256) sum += z(i);
+        *mean = block_sum<256>(sum, red) / (float)H;
+      }
+      float ss = 0.f;
+      for (int i = threadIdx.x; i < H; i += 256) {
+        const float v = z(i) - *mean;
+        ss = fmaf(v, v, ss);
+      }
+      return 1.0f / sqrtf(block_sum<256>(ss, red) / (float)H + eps);
+    };
+    float mean;
+    const float scale = p.factor * inverse(value, p.centered, p.eps, &mean);
+    for (int i = threadIdx.x; i < H; i += 256) row[i] = row[i] + (value(i) - mean) * scale * p.g[i];
     if (!out) return;
-    const float next = 1.0f / sqrtf(block_sum<256>(s2, red) / (float)H + next_eps);
-    for (int i = threadIdx.x; i < H; i += 256) st<RT>(out + (size_t)m * H + i, row[i] * next * next_g[i]);      // (its own elements)
+    const float next = inverse([&](int i) { return row[i]; }, p.next_centered, p.next_eps, &mean);      // (its own elements)
+    for (int i = threadIdx.x; i < H; i += 256) st<RT>(out + (size_t)m * H + i, (row[i] - mean) * next * p.next_g[i]);
   }
 }
 
 extern "C" int ti_norm_residual_next(float* x, const float* y, const int* gather, int n_gather, const float* plus, const float* plus_gate,
-                                     const float* g, float eps, const float* next_g, float next_eps, void* out, int out_dtype, int M,
-                                     int H, hipStream_t stream) {
-  TI_REQUIRE(M >= 0 && H > 0 && (!gather || n_gather > 0) && (!out || next_g), "norm_residual_next: bad sizes M=%d H=%d gather=%d", M, H, n_gather);
+                                     const ti_norm_pair* norms, void* out, int out_dtype, int M, int H, hipStream_t stream) {
+  TI_REQUIRE(M >= 0 && H > 0 && (!gather || n_gather > 0) && norms && norms->g && (!out || norms->next_g),
+             "norm_residual_next: bad sizes M=%d H=%d gather=%d", M, H, n_gather);
   TI_REQUIRE(!out || out_dtype == TI_F32 || out_dtype == TI_BF16, "norm_residual_next: unknown dtype %d", out_dtype);
   if (M == 0) return 0;
-  const bool v4 = H % 4 == 0 && H <= 8192 && (((uintptr_t)x | (uintptr_t)y | (uintptr_t)g | (uintptr_t)plus | (uintptr_t)next_g | (uintptr_t)out) & 15) == 0;
-#define TI_NRN(RT, NV)                                                                                                             \
-  norm_residual_next_kernel<RT, NV><<<M, 256, 0, stream>>>(x, y, gather, n_gather, plus, plus_gate, g, eps, next_g, next_eps, (RT*)out, H)
+  const bool v4 = H % 4 == 0 && H <= 8192 &&
+                  (((uintptr_t)x | (uintptr_t)y | (uintptr_t)norms->g | (uintptr_t)plus | (uintptr_t)(out ? norms->next_g : nullptr) | (uintptr_t)out) & 15) == 0;
+#define TI_NRN(RT, NV) norm_residual_next_kernel<RT, NV><<<M, 256, 0, stream>>>(x, y, gather, n_gather, plus, plus_gate, *norms, (RT*)out, H)
 #define TI_NRN_WIDTH(RT)               \
   do {                                 \
     if (!v4) TI_NRN(RT, 0);            \

@@ -250,19 +250,37 @@ int ti_gated_attention_rows(int dtype, const void* q, const void* pool, const in
                             int n_head, int n_kv, int dk, int dv, int dv_rows, int page_size, float scale, int window,
                             hipStream_t stream);
 
-// ---- libti_linear_attention: linear attention with a fixed decay per head, and the gated norm behind it
-// S_t = decay_h S_(t-1) + k_t v_t^T, o_t = S_t^T q_t with q, k, v = silu of the given columns of proj f32 [M, ld]; state f32
-// [slots][heads][dk][dv]; entry_meta [n_entries][4] = (row0, tokens, start, slot); o f32 [M, heads dv]
-int ti_decay_scan(const float* proj, int ld, int off_q, int off_k, int off_v, const float* decay, float* state, long slot_stride,
-                  const int* entry_meta, int n_entries, float* o, int heads, int dk, int dv, hipStream_t stream);
-// the same with the entries' tokens in chunks that run side by side (chunks [n_chunks][4] = (entry, first row, tokens, 1: the
-// entry's first chunk + 2: its last), spans [n_entries][2] = (first chunk, chunks); scratch float [n_chunks][heads][dk dv])
-int ti_decay_scan_chunked(const float* proj, int ld, int off_q, int off_k, int off_v, const float* decay, float* state,
-                          long slot_stride, const int* entry_meta, int n_entries, const int* chunks, int n_chunks, const int* spans,
-                          float* scratch, float* o, int heads, int dk, int dv, hipStream_t stream);
-// out = o / rms(o over the whole row) * w * sigmoid(gate), gate in rows of ld floats from column off_g on
-int ti_gated_row_norm(int out_dtype, const float* o, const float* gate, int ld, int off_g, const float* w, void* out, int M, int W,
-                      float eps, hipStream_t stream);
+// ---- libti_linear_attention: linear attention as a scan, and the gated norms behind it
+// What enters the recurrence S_t = a_t S_(t-1) + d_t k_t v_t^T, o_t = S_t^T q_t (+ skip_h v_t): q, k (qk_heads x dk, head h of
+// `heads` reads head h / (heads / qk_heads)) and v (heads x dv) from the given columns of proj f32 [M, ld]
+typedef struct ti_scan_inputs {
+  const float* proj;
+  int ld, off_q, off_k, off_v, qk_heads;
+  int act;                      // 1: silu on q, k and v
+  float k_scale;                // k times this (behind activation or rotation)
+  // rotation of the first rot_dims entries of q and k (entry i with i + rot_dims / 2; 0: none), positions int32 [M];
+  // rope_table [table_len][rot_dims / 2][2] may be null
+  const float *inv_freq, *rope_table;
+  int table_len, rot_dims;
+  const int* pos;
+  const float* decay;           // [heads]: a_t = decay_h, d_t = 1; or null and, with dt in rows of dt_ld floats (already at its
+  const float *dt, *dt_bias, *a_log;     // first column): d_t = softplus(dt_h + dt_bias_h), a_t = exp(-exp(a_log_h) d_t)
+  int dt_ld;
+  const float* skip;            // [heads] or null
+} ti_scan_inputs;
+// state f32 [slots][heads][dk][dv]; entry_meta [n_entries][4] = (row0, tokens, start, slot); o f32 [M, heads dv]
+int ti_linear_scan(const ti_scan_inputs* in, float* state, long slot_stride, const int* entry_meta, int n_entries, float* o, int heads,
+                   int dk, int dv, hipStream_t stream);
+// the same with the entries' tokens in chunks of up to 64 that run side by side (chunks [n_chunks][4] = (entry, first row, tokens,
+// 1: the entry's first chunk + 2: its last), spans [n_entries][2] = (first chunk, chunks); scratch float
+// [n_chunks][heads][dk dv + 1])
+int ti_linear_scan_chunked(const ti_scan_inputs* in, float* state, long slot_stride, const int* entry_meta, int n_entries,
+                           const int* chunks, int n_chunks, const int* spans, float* scratch, float* o, int heads, int dk, int dv,
+                           hipStream_t stream);
+// out = o / rms(o) * w * act(gate) with the rms over each of `groups` equal runs of a row (w null: none; act 0 sigmoid, 1 silu;
+// gate_first: o times act(gate) is what is normed), gate in rows of ld floats from column off_g on
+int ti_gated_group_norm(int out_dtype, const float* o, const float* gate, int ld, int off_g, const float* w, void* out, int M, int W,
+                        int groups, float eps, int silu, int gate_first, hipStream_t stream);
 
 // ---- libti_mingru: S <- (1 - s) S + s c element by element, s = sigmoid(z + bias_z), c = u + 1/2 (u >= 0) or sigmoid(u) with
 // u = x + bias_x; out = S g sigmoid(g).  proj f32 [M, ld] with W columns of z, x and g from off_z, off_x, off_g on; state f32
@@ -281,11 +299,21 @@ int ti_mingru_scan_chunked(int out_dtype, const float* proj, int ld, int off_z, 
 // [M][H] of rounded_dtype, the new x rounded for the product that reads it next
 int ti_norm_residual(float* x, const float* y, const float* g, const int* gather, int n_gather, int M, int H, float eps,
                      int accumulate, void* rounded, int rounded_dtype, hipStream_t stream);
-// x[m] += y'[m] / sqrt(mean(y'[m]^2) + eps) * g, y' as above plus plus_gate[m] plus[m] (plus f32 [M][H], null: none; plus_gate
-// f32 [M], null: times one); then out[m] = x[m] / sqrt(mean(x[m]^2) + next_eps) * next_g in out_dtype (out null: not written)
+// A norm behind a sublayer and the one in front of the next: x[m] += factor N(y'[m]) g, then out[m] = N(x[m]) next_g in out_dtype
+// (out null: not written).  N divides by the root mean square (plus eps) or, centered, takes the mean off first and divides by the
+// standard deviation.  y': y_scale times the rows of y as above, plus plus_scale plus_gate[m] plus[m] (plus f32 [M][H], null: none;
+// plus_gate f32 [M], null: one)
+typedef struct ti_norm_pair {
+  const float* g;
+  float eps;
+  int centered;
+  const float* next_g;
+  float next_eps;
+  int next_centered;
+  float y_scale, plus_scale, factor;
+} ti_norm_pair;
 int ti_norm_residual_next(float* x, const float* y, const int* gather, int n_gather, const float* plus, const float* plus_gate,
-                          const float* g, float eps, const float* next_g, float next_eps, void* out, int out_dtype, int M, int H,
-                          hipStream_t stream);
+                          const ti_norm_pair* norms, void* out, int out_dtype, int M, int H, hipStream_t stream);
 // y[m] += gate[m] plus[m] (gate null: times one)
 int ti_add_gated_rows(float* y, const float* plus, const float* gate, int M, int H, hipStream_t stream);
 // out = x rounded to out_dtype
@@ -293,12 +321,15 @@ int ti_round_rows(int out_dtype, const float* x, void* out, long n, hipStream_t 
 // x *= s
 int ti_scale(float* x, float s, long n, hipStream_t stream);
 
-// ---- libti_diff_attention: a short convolution over time with carried state, and differential attention
-// out[m, c] = sum_j taps[c][j] u(pos[m] - (K - 1) + j)[c]; u f32 [M, C] holds the step's rows, state f32
-// [slots][K - 1][C] the K - 1 rows before each entry's start (entries int32 [n][4] = (row0, tokens, start, slot);
-// entry_of[m]: the entry of row m), which the call then replaces by the last K - 1 rows up to the step's end
-int ti_short_conv(const float* u, const float* taps, float* state, const int* entries, int n_entries, const int* entry_of,
-                  const int* pos, float* out, int M, int C, int K, hipStream_t stream);
+// ---- libti_short_conv: a short causal convolution over time with carried state
+// out[m, c] = act(bias[c] + sum_j taps[c][j] u(pos[m] - (K - 1) + j)[c]) (bias null: none; silu 0: no activation); u f32, M rows
+// of ld floats, holds the step's rows, state f32 [slots][K - 1][C] the K - 1 rows before each entry's start (entries int32 [n][4]
+// = (row0, tokens, start, slot); entry_of[m]: the entry of row m), which the call then replaces by the last K - 1 rows up to
+// the step's end; out f32 [M, C]
+int ti_short_conv(const float* u, long ld, const float* taps, const float* bias, int silu, float* state, const int* entries,
+                  int n_entries, const int* entry_of, const int* pos, float* out, int M, int C, int K, hipStream_t stream);
+
+// ---- libti_diff_attention: differential attention
 // qkv f32 [M, n_head 2 dk + n_kv 2 dk + n_kv dv] (each query head and kv head holds two maps of dk): per map RMS
 // norm with the weights q_w / k_w [dk] (may be null), rotation of the first rot_dims entries (entry i with entry
 // i + rot_dims / 2; cos and sin times mag; rope_table [table_len][rot_dims / 2][2] may be null), q to q_out, k and v
@@ -353,32 +384,30 @@ int ti_moe_route_gate(int dtype, const void* h, const float* router, const float
 // y f32 [M, W] = sum_k down[e_k] relu(up[e_k] (s_k h))^2 (scale_input) or sum_k s_k down[e_k] relu(up[e_k] h)^2;
 // up [E][F][W], down [E][W][F] in the dtype of h; act: scratch of that dtype, [M top][F]; part: f32 [M top][W].  A workgroup
 // per expert and 16 outputs walks its weights once for all the pairs that chose the expert: steps of few tokens, and float32.
-// A token's rows of part are added in ascending order into y where y is given, else left to the caller
+// A token's rows of part are added in ascending order into y where y is given, else left to the caller.  identity: ids from E on
+// are identity experts, their row of part is s_k h
 int ti_moe_experts_rows(int dtype, const void* h, const int* ids, const float* wts, const void* up, const void* down, void* act,
-                        float* part, float* y, int M, int W, int F, int E, int top, int scale_input, hipStream_t stream);
+                        float* part, float* y, int M, int W, int F, int E, int top, int scale_input, int identity, hipStream_t stream);
 
 // experts with a gate: y[m] = sum_k s_k down[e_k] act(gate[e_k] h, up[e_k] h); gate_up [E][2F][W] holds an expert's gate rows
 // above its up rows.  act_kind 0: silu(g) u; 1: g = min(g, limit), u = clamp(u, -limit, limit), g sigmoid(alpha g) (u + 1).
-// z: f32 scratch [M top][2F]; act, part, y as above
+// act, part, y, identity as above
 int ti_moe_experts_rows_gated(int dtype, const void* h, const int* ids, const float* wts, const void* gate_up, const void* down,
-                              float* z, void* act, float* part, float* y, int M, int W, int F, int E, int top, int act_kind,
-                              float limit, float alpha, hipStream_t stream);
+                              void* act, float* part, float* y, int M, int W, int F, int E, int top, int act_kind, float limit,
+                              float alpha, int identity, hipStream_t stream);
 
 // ---- libti_moe_bf16: the experts for steps of many tokens, on the matrix cores: the (token, expert) pairs are laid out expert
 // by expert in tiles of 128 rows and both products run over the tiles.  Scratch: meta int32 [ti_moe_grouped_meta_ints(M top, E)],
 // where int32 [M top] (the row of every pair), rows bf16 [M top][W], act bf16 [M top][F], out f32 [M top][W].  y (may be
 // null): the tokens' sums; without it the caller adds the rows out[where[m top + k]] in ascending k.  The weights multiply the
 // experts' inputs (scale_input) or their outputs (row_w: f32 scratch [M top]; rows is int32 [M top] then, the rows' tokens).
-// 3: sizes not served
+// act_kind < 0: relu^2; 0, 1: the gated experts of ti_moe_experts_rows_gated (up is their gate_up), weights on the outputs.
+// identity: ids from E on are identity experts.  3: sizes not served
 long ti_moe_grouped_meta_ints(int n_pairs, int E);
 int ti_moe_experts_grouped_bf16(const void* h, const int* ids, const float* wts, const void* up, const void* down, int* meta,
                                 int* where, void* rows, void* act, float* out, float* y, int M, int W, int F, int E, int top,
-                                int scale_input, float* row_w, hipStream_t stream);
-
-// the gated experts of ti_moe_experts_rows_gated over such tiles; rows: int32 scratch [M top]; z: f32 scratch [M top][2F]; y is written (the tokens' weighted sums)
-int ti_moe_experts_grouped_gated_bf16(const void* h, const int* ids, const float* wts, const void* gate_up, const void* down,
-                                      int* meta, int* where, void* rows, float* z, void* act, float* out, float* y, int M, int W,
-                                      int F, int E, int top, int act_kind, float limit, float alpha, hipStream_t stream);
+                                int scale_input, float* row_w, int act_kind, float limit, float alpha, int identity,
+                                hipStream_t stream);
 
 // ---- libti_attention_bf16: the same on the matrix cores (head sizes 32, 64, 128; pages of 16 n rows)
 // rows of single tokens; n_splits > 1 needs part_o f32 [n_rows, n_head, n_splits, hd] and part_ml f32

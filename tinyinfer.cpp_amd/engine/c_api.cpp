@@ -1296,20 +1296,38 @@ int ti_ops_call(void* ops_, const char* op_, const ti_tensor* t, int n_t, const 
     if (g.mode) g.proj = arg(6);
     ops.gated_attention(arg(0), arg(1), view_of(2, arg(1)), iptr(3), iptr(4), arg(5), g, arg(7), (int)num(0), (int)num(1), (int)num(2),
                         (int)num(3), (float)num(4), (int)num(5));
-  } else if (op == "decay_scan") {
-    // proj, decay, state, entries [R, 4], o; heads, dk, dv, columns of q, k, v
-    Ops::QkvColumns c;
-    c.q = (int)num(3);
-    c.k = (int)num(4);
-    c.v = (int)num(5);
-    // optional: chunks [n][4] and spans [R][2] (tensors 5 and 6): the chunked form
-    const bool chunked = n_t > 6 && arg(5).defined();
-    ops.decay_scan(arg(0), c, arg(1), arg(2), iptr(3), (int)arg(3).shape[0], arg(4), (int)num(0), (int)num(1), (int)num(2),
-                   chunked ? iptr(5) : nullptr, chunked ? (int)arg(5).shape[0] : 0, chunked ? iptr(6) : nullptr,
-                   chunked ? &workspace_of(&ops) : nullptr);
-  } else if (op == "gated_row_norm") {
-    // o, proj, w, out; gate column, eps
-    ops.gated_row_norm(arg(0), arg(1), (int)num(0), arg(2), (float)num(1), arg(3));
+  } else if (op == "linear_scan") {
+    // rows, state, entries [R, 4], o, chunks [n][4], spans [R][2] (the last two may be absent), decay, inv_freq, rope_table, positions,
+    // dt, dt_bias, a_log, skip (each may be absent); heads, dk, dv, columns of q, k, v, q/k heads, silu, k_scale, rotated entries, dt column
+    Ops::LinearScan in;
+    in.rows = arg(0);
+    in.cols.q = (int)num(3);
+    in.cols.k = (int)num(4);
+    in.cols.v = (int)num(5);
+    in.qk_heads = (int)num(6);
+    in.silu = num(7) != 0;
+    in.k_scale = (float)num(8);
+    in.decay = arg(6);
+    if (arg(7).defined()) {
+      in.rot = rotation(7, 8);
+      in.rot.dims = (int)num(9);
+      in.positions = iptr(9);
+    }
+    in.dt = arg(10);
+    in.dt_bias = arg(11);
+    in.a_log = arg(12);
+    in.skip = arg(13);
+    in.dt_col = (int)num(10);
+    const bool chunked = arg(4).defined();
+    ops.linear_scan(in, arg(1), iptr(2), (int)arg(2).shape[0], arg(3), (int)num(0), (int)num(1), (int)num(2), chunked ? iptr(4) : nullptr,
+                    chunked ? (int)arg(4).shape[0] : 0, chunked ? iptr(5) : nullptr, chunked ? &workspace_of(&ops) : nullptr);
+  } else if (op == "gated_group_norm") {
+    // o, proj, w (may be absent), out; gate column, eps, runs of a row, silu, gate in front of the norm
+    Ops::GroupNorm form;
+    form.groups = (int)num(2);
+    form.silu = num(3) != 0;
+    form.gate_first = num(4) != 0;
+    ops.gated_group_norm(arg(0), arg(1), (int)num(0), arg(2), (float)num(1), arg(3), form);
   } else if (op == "moe_route_grouped") {
     // h, router, ids, wts, correction (may be absent), [gate row, gate out]; top, score, renormalize, groups, keep, weight scale, sum floor
     Ops::RouterGroups g;
@@ -1349,10 +1367,18 @@ int ti_ops_call(void* ops_, const char* op_, const ti_tensor* t, int n_t, const 
                     chunked ? (int)arg(6).shape[0] : 0, chunked ? iptr(7) : nullptr, chunked ? &workspace_of(&ops) : nullptr);
   } else if (op == "norm_residual_next") {
     // x, y, gain, gather [M, n] (may be absent), plus, plus_gate, next_gain, next_out (each may be absent); eps, next_eps,
-    // rows of y a row of x sums where no list names them
+    // rows of y a row of x sums where no list names them, centered, next centered, factor, y_scale, plus_scale
     const bool g = arg(3).defined();
-    ops.norm_residual_next(arg(0), arg(1), g ? iptr(3) : nullptr, g ? (int)arg(3).shape[1] : (int)num(2), arg(4), arg(5), arg(2), (float)num(0),
-                           arg(6), (float)num(1), arg(7));
+    Ops::GatheredRows y;
+    y.t = arg(1);
+    y.gather = g ? iptr(3) : nullptr;
+    y.n_gather = g ? (int)arg(3).shape[1] : (int)num(2);
+    y.plus = arg(4);
+    y.plus_gate = arg(5);
+    y.y_scale = (float)num(6);
+    y.plus_scale = (float)num(7);
+    Ops::RowNorm norm{arg(2), (float)num(0), num(3) != 0}, next{arg(6), (float)num(1), num(4) != 0};
+    ops.norm_residual_next(arg(0), y, norm, (float)num(5), next, arg(7));
   } else if (op == "add_gated_rows") {
     ops.add_gated_rows(arg(0), arg(1), n_t > 2 ? arg(2) : Tensor());
   } else if (op == "latent_attention") {
@@ -1378,9 +1404,9 @@ int ti_ops_call(void* ops_, const char* op_, const ti_tensor* t, int n_t, const 
   } else if (op == "latent_transpose") {
     ops.latent_transpose(arg(0), arg(1), (int)num(0));
   } else if (op == "moe_experts_gated") {
-    // h, ids, wts, gate_up, down, y; experts, kind, limit, alpha
+    // h, ids, wts, gate_up, down, y; experts, kind, limit, alpha, [identity experts]
     ops.moe_experts_gated(arg(0), arg(1), arg(2), arg(3), arg(4), arg(5), (int)num(0), (Ops::GatedAct)(int)num(1), (float)num(2),
-                          (float)num(3), workspace_of(&ops));
+                          (float)num(3), workspace_of(&ops), nullptr, n_s > 4 ? (int)num(4) : 0);
   } else if (op == "attention_capped") {
     // q, pool, table, positions, slots, out; heads, kv_heads, dk, dv, scale, softcap, window
     ops.attention_capped(arg(0), arg(1), view_of(2, arg(1)), iptr(3), iptr(4), arg(5), (int)num(0), (int)num(1), (int)num(2),
@@ -1412,8 +1438,9 @@ int ti_ops_call(void* ops_, const char* op_, const ti_tensor* t, int n_t, const 
   } else if (op == "scale") {
     ops.scale(arg(0), (float)num(0));
   } else if (op == "short_conv") {
-    // u, taps, state, entries [R, 4], entry of every row, positions, out
-    ops.short_conv(arg(0), arg(1), arg(2), iptr(3), (int)arg(3).shape[0], iptr(4), iptr(5), arg(6));
+    // u, taps, state, entries [R, 4], entry of every row, positions, out, [bias]; [silu]
+    ops.short_conv(arg(0), arg(1), arg(2), iptr(3), (int)arg(3).shape[0], iptr(4), iptr(5), arg(6), n_t > 7 ? arg(7) : Tensor(),
+                   n_s > 0 && num(0) != 0);
   } else if (op == "diff_qk_prep") {
     // qkv, q_w, k_w, inv_freq, rope_table, positions, slots, table, pool, q_out, [taps, state, entries [R, 4]: the short
     // convolution inside]; eps, heads, kv_heads, dk, dv, rotated entries, mag
@@ -1457,8 +1484,9 @@ int ti_ops_call(void* ops_, const char* op_, const ti_tensor* t, int n_t, const 
     // h, router, ids, wts; top, score kind, renormalize
     ops.moe_route(arg(0), arg(1), arg(2), arg(3), (int)num(0), (Ops::RouterScore)(int)num(1), num(2) != 0);
   } else if (op == "moe_experts") {
-    // h, ids, wts, up, down, y; experts, scale_input
-    ops.moe_experts(arg(0), arg(1), arg(2), arg(3), arg(4), arg(5), (int)num(0), num(1) != 0, workspace_of(&ops));
+    // h, ids, wts, up, down, y; experts, scale_input, [identity experts]
+    ops.moe_experts(arg(0), arg(1), arg(2), arg(3), arg(4), arg(5), (int)num(0), num(1) != 0, workspace_of(&ops), nullptr,
+                    n_s > 2 ? (int)num(2) : 0);
   } else if (op == "argmax") {
     ops.argmax(arg(0), arg(1).ptr<int>());
   } else if (op == "sample") {

@@ -173,8 +173,11 @@ ModelSpec nazorax_spec(const Json& config);
 Json dubozen_typed_config(const Json& config);
 ModelSpec dubozen_spec(const Json& config);
 // the Lupolorn decoder (config/lupolorn.cpp)
+// the Ruzolorn decoder (config/ruzolorn.cpp)
 Json lupolorn_typed_config(const Json& config);
+Json ruzolorn_typed_config(const Json& config);
 ModelSpec lupolorn_spec(const Json& config);
+ModelSpec ruzolorn_spec(const Json& config);
 // {"architecture": the registered name that matched, "config": the typed configuration (the input itself if
 // the architecture registered no reader)}; ConfigError as spec_from_config
 Json typed_config(const Json& config);
@@ -439,15 +442,31 @@ class Ops {
   void gated_attention(const Tensor& q, const Tensor& pool, const CacheView& view, const int* positions, const int* slots,
                        const Tensor& sink, const AttentionGate& gate, const Tensor& out, int heads, int kv_heads, int dk, int dv,
                        float scale, int window, const AttentionWork* work = nullptr, Workspace* ws = nullptr);
-  // Linear attention with a fixed decay per head over each entry's tokens, from and into its state slot: S <- decay_h S + k v^T,
-  // o = S^T q with q, k, v = silu of proj's columns; decay f32 [heads]; state f32 [slots][heads][dk dv]; o f32 [M, heads dv]
-  // chunks (device int32 [n_chunks][4] = (entry, first row, tokens, 1: the entry's first chunk + 2: its last)) and spans
+  // Linear attention over each entry's tokens, from and into its state slot: S <- a S + d k v^T, o = S^T q + skip_h v.  q, k
+  // (qk_heads x dk; 0: as many as heads; head h reads head h / (heads / qk_heads)) and v (heads x dv) are columns of rows f32
+  // [M, N]: with silu, or q and k rotated (rot, positions), or as they are; k times k_scale behind that.  Fixed decay: a =
+  // decay_h (f32 [heads]), d = 1; else d = softplus(dt + dt_bias_h) with dt f32 [M, N'] from column dt_col on, a = exp(-exp(a_log_h) d)
+  struct LinearScan {
+    Tensor rows;
+    QkvColumns cols;
+    int qk_heads = 0;
+    bool silu = false;
+    float k_scale = 1.f;
+    Rotation rot;
+    const int* positions = nullptr;
+    Tensor decay;
+    Tensor dt, dt_bias, a_log, skip;
+    int dt_col = 0;
+  };
+  // state f32 [slots][heads][dk dv]; o f32 [M, heads dv]
+  // chunks (device int32 [n_chunks][4] = (entry, first row, tokens up to 64, 1: the entry's first chunk + 2: its last)) and spans
   // ([n_entries][2] = (first chunk, chunks)): long portions run as chunks side by side, through scratch of `ws`
-  void decay_scan(const Tensor& proj, const QkvColumns& cols, const Tensor& decay, const Tensor& state, const int* entry_meta,
-                  int n_entries, const Tensor& o, int heads, int dk, int dv, const int* chunks = nullptr, int n_chunks = 0,
-                  const int* spans = nullptr, Workspace* ws = nullptr);
-  // out = o / rms(o over the whole row) * w * sigmoid(gate columns of proj), in the compute dtype
-  void gated_row_norm(const Tensor& o, const Tensor& proj, int gate_col, const Tensor& w, float eps, const Tensor& out);
+  void linear_scan(const LinearScan& in, const Tensor& state, const int* entry_meta, int n_entries, const Tensor& o, int heads, int dk,
+                   int dv, const int* chunks = nullptr, int n_chunks = 0, const int* spans = nullptr, Workspace* ws = nullptr);
+  // out = o / rms(o) * w * act(gate columns of proj), in the compute dtype: the rms over each of `groups` equal runs of a row, w
+  // undefined: none; silu: act is silu, else sigmoid; gate_first: the norm is of o times act(gate)
+  struct GroupNorm { int groups = 1; bool silu = false, gate_first = false; };
+  void gated_group_norm(const Tensor& o, const Tensor& proj, int gate_col, const Tensor& w, float eps, const Tensor& out, const GroupNorm& form);
   // ---- layers that norm what a sublayer returns; short convolutions; differential attention; mixtures of experts
   // x (+)= y / rms(y) * gain (32-bit; gain is the factor itself).  accumulate false: x is overwritten (y may be x).
   // gather (device int32 [M][n_gather]): row m of y is the sum of the rows y[gather[m][k]], k ascending; no list and
@@ -455,11 +474,24 @@ class Ops {
   // rounded (may be null): also receives the new x in its own dtype, for the product that reads the residual next
   void norm_residual(const Tensor& x, const Tensor& y, const Tensor& gain, float eps, bool accumulate, const int* gather = nullptr,
                      int n_gather = 0, const Tensor* rounded = nullptr);
-  // a norm on either side of a sublayer, both in one pass over the row: x += y' / rms(y') * gain, then next_out = x / rms(x) *
-  // next_gain in its own dtype (next_out undefined: the sum alone).  y': the rows of y as above, and behind them the row of
-  // `plus` (f32 [M, H], undefined: none) times plus_gate (f32 [M], undefined: one)
-  void norm_residual_next(const Tensor& x, const Tensor& y, const int* gather, int n_gather, const Tensor& plus, const Tensor& plus_gate,
-                          const Tensor& gain, float eps, const Tensor& next_gain = Tensor(), float next_eps = 0.f, const Tensor& next_out = Tensor());
+  // rows whose sums are a sublayer's output, left to whoever reads it: row m is y_scale times the sum of the rows t[gather[m][k]], k
+  // ascending (gather: device int32 [M][n_gather]; no list: of the rows t[m n_gather + k]), and a further branch of it, for readers
+  // that say so: plus f32 [M, W] (undefined: none) times plus_gate f32 [M] (undefined: one) times plus_scale
+  struct GatheredRows {
+    Tensor t;
+    const int* gather = nullptr;
+    int n_gather = 0;
+    Tensor plus, plus_gate;
+    float y_scale = 1.f, plus_scale = 1.f;
+  };
+  // what a norm of a row divides by: the root mean square (plus eps), or, centered, the standard deviation of the row without its mean
+  struct RowNorm { Tensor gain; float eps = 0.f; bool centered = false; };
+  // a norm on either side of a sublayer, both in one pass over the row: x += factor N(y') gain, then next_out = N'(x) next gain in
+  // its own dtype (next_out undefined: the sum alone); y': the rows' sums as above
+  void norm_residual_next(const Tensor& x, const GatheredRows& y, const RowNorm& norm, float factor, const RowNorm& next, const Tensor& next_out);
+  void norm_residual_next(const Tensor& x, const GatheredRows& y, const RowNorm& norm, float factor) {
+    norm_residual_next(x, y, norm, factor, norm, Tensor());
+  }
   void add_gated_rows(const Tensor& y, const Tensor& plus, const Tensor& gate);      // y[m] += gate[m] plus[m] (gate undefined: one)
   // The minimal GRU over each entry's tokens, from and into its state slot: S <- (1 - s) S + s c with s = sigmoid(z + bias_z),
   // c = u + 1/2 (u >= 0) or sigmoid(u), u = x + bias_x; out = S silu(g).  proj f32 [M, N]: `width` columns each of z, x and g;
@@ -470,10 +502,11 @@ class Ops {
                    const int* spans = nullptr, Workspace* ws = nullptr);
   void round_rows(const Tensor& x, const Tensor& out);                               // out = x in out's dtype
   void scale(const Tensor& x, float s);                                              // x *= s (float32)
-  // out[m, c] = sum_j taps[c, j] u(position of m - (K - 1) + j)[c] over each entry's rows, the K - 1 rows before an
-  // entry's start taken from its state slot f32 [slots][K - 1][C]; the slot then gets the entry's last K - 1 rows
+  // out[m, c] = act(bias[c] + sum_j taps[c, j] u(position of m - (K - 1) + j)[c]) over each entry's rows, the K - 1 rows before an
+  // entry's start taken from its state slot f32 [slots][K - 1][C]; the slot then gets the entry's last K - 1 rows.  u: f32 [M, C],
+  // or C columns of wider rows; bias undefined: none; silu: the activation
   void short_conv(const Tensor& u, const Tensor& taps, const Tensor& state, const int* entry_meta, int n_entries,
-                  const int* entry_of, const int* positions, const Tensor& out);
+                  const int* entry_of, const int* positions, const Tensor& out, const Tensor& bias = Tensor(), bool silu = false);
   // qkv f32 [M, heads 2 dk + kv_heads 2 dk + kv_heads dv] (two maps a head): per-map norm, rotation of the first
   // rot.dims entries, q to q_out, k and v into pages K [kv][P][2 dk] | V [kv][dv][P]
   // conv (may be null): the short convolution of `short_conv` on every channel first, inside the same kernel
@@ -507,17 +540,14 @@ class Ops {
                  bool renormalize, const RouterGroups& grouped);
   // y f32 [M, W] = sum over a token's experts of down_e relu(up_e h)^2, the weight on the expert's input or output;
   // up [E F, W], down [E W, F]; scratch comes from `ws`.  With `rows` (and bfloat16, many tokens, sizes the matrix-core kernels
-  // take) y may stay unwritten: then rows->t is f32 [M top, W] and rows->gather device int32 [M][top]: row m of the result is
-  // the sum of the rows rows->t[gather[m][k]], k ascending (no list: of the rows m n_gather + k), left to the norm that
-  // reads it (Ops::norm_residual)
-  // plus, plus_gate: a further branch of the result, f32 [M, W] times f32 [M] (undefined: none / one), for readers that say so
-  struct GatheredRows { Tensor t; const int* gather = nullptr; int n_gather = 0; Tensor plus, plus_gate; };
+  // take) y may stay unwritten: then the result is what `rows` says, left to the norm that reads it.
+  // identity > 0: so many ids from `experts` on are identity experts, whose output is h itself
   void moe_experts(const Tensor& h, const Tensor& ids, const Tensor& wts, const Tensor& up, const Tensor& down, const Tensor& y,
-                   int experts, bool scale_input, Workspace& ws, GatheredRows* rows = nullptr);
+                   int experts, bool scale_input, Workspace& ws, GatheredRows* rows = nullptr, int identity = 0);
   // experts with a gate: y = sum_k s_k down_e act(gate_e h, up_e h); gate_up [E 2F, W] holds an expert's gate rows above its up rows
   void moe_experts_gated(const Tensor& h, const Tensor& ids, const Tensor& wts, const Tensor& gate_up, const Tensor& down,
                          const Tensor& y, int experts, GatedAct kind, float limit, float alpha, Workspace& ws,
-                         GatheredRows* rows = nullptr);
+                         GatheredRows* rows = nullptr, int identity = 0);
   void argmax(const Tensor& logits, int* out);
   void sample(const Tensor& logits, const float* temperature, const int* top_k, const float* top_p, const float* uniform,
               int* out);
@@ -559,6 +589,9 @@ class Ops {
 
  private:
   void* launch_stream();
+  void experts_of(const char* what, const Tensor& h, const Tensor& ids, const Tensor& wts, const Tensor& up, const Tensor& down, const Tensor& y,
+                  int experts, bool scale_input, bool gated, GatedAct kind, float limit, float alpha, Workspace& ws, GatheredRows* rows,
+                  int identity);
   void took(const char* what);       // the call under way names the kernel it took (seen in the list of calls)
   void* stream_ = nullptr;
   int units_ = 0;
@@ -753,8 +786,8 @@ class NormPart : public Part { public: using Part::Part; const char* family() co
   // that keep the residual in several streams
   virtual bool can_mix() const { return false; }
   virtual Rows forward_mixed(StepContext& ctx, const Tensor& streams, const Tensor& coef);
-  // a plain RMS norm with a gain per channel says what it is, for kernels that take it in (false: it is something else)
-  virtual bool rms_form(Tensor& weight, float& eps) const { return false; }
+  // a plain RMS or layer norm with a gain per channel says what it is, for kernels that take it in (false: it is something else)
+  virtual bool row_form(Ops::RowNorm& norm) const { return false; }
   // for a writer of the streams that takes the next read in: the norm's weight, eps and the rows it would write (null: no such form)
   virtual bool mixed_form(StepContext& ctx, int64_t M, Tensor& weight, float& eps, Rows& rows) { return false; } };
 class PositionPart : public Part { public: using Part::Part; const char* family() const override { return "pos"; }

@@ -97,13 +97,13 @@ _LIB_OF = {"embed": "core", "rmsnorm": "core", "rope_neox": "core", "rope_table"
            "fill_random": "core", "fill_zero": "core", "add_sinusoid": "pointwise", "add_row": "pointwise", "xielu": "pointwise",
            "scaled_add": "pointwise", "qkv_split_write": "pointwise", "attention_capped": "attention_generic",
            "mlstm_scan": "recurrent", "gated_head_norm": "recurrent", "norm_residual": "residual", "round_rows": "residual",
-           "scale": "residual", "short_conv": "diff_attention", "diff_qk_prep": "diff_attention", "diff_attention": "diff_attention",
+           "scale": "residual", "short_conv": "short_conv", "diff_qk_prep": "diff_attention", "diff_attention": "diff_attention",
            "moe_route": "moe", "moe_experts": "moe", "moe_experts_gated": "moe", "qkv_prep_write": "pointwise", "dyt": "pointwise",
            "gated_act": "pointwise", "concat_round": "pointwise", "latent_prep": "latent_attention",
            "latent_attention": "latent_attention", "latent_transpose": "latent_attention", "layernorm": "hyper",
            "layernorm_mixed": "hyper", "hyper_combine": "hyper", "hyper_spread": "hyper", "hyper_write": "hyper",
-           "gated_qkv_prep": "gated_attention", "gated_attention": "gated_attention", "decay_scan": "linear_attention",
-           "gated_row_norm": "linear_attention", "moe_route_grouped": "moe",
+           "gated_qkv_prep": "gated_attention", "gated_attention": "gated_attention", "linear_scan": "linear_attention",
+           "gated_group_norm": "linear_attention", "moe_route_grouped": "moe",
            "latent_prep_queries": "latent_attention", "mingru_scan": "mingru", "norm_residual_next": "residual", "add_gated_rows": "residual"}
 
 
@@ -372,10 +372,11 @@ class Ops:
     def scale(self, x, s):
         self._call("scale", [x], [s])
 
-    def short_conv(self, u, taps, state, entries, entry_of, positions, out):
-        """out[m, c] = sum_j taps[c, j] u(pos[m] - (K - 1) + j)[c]; state f32 [slots, K - 1, C] holds the rows before each
-        entry's start and is left with the last K - 1 rows; entries int32 [R, 4] = (first row, tokens, start, slot)."""
-        self._call("short_conv", [u, taps, state, entries, entry_of, positions, out])
+    def short_conv(self, u, taps, state, entries, entry_of, positions, out, bias=None, silu=False):
+        """out[m, c] = act(bias[c] + sum_j taps[c, j] u(pos[m] - (K - 1) + j)[c]); u may be columns of wider rows; state f32
+        [slots, K - 1, C] holds the rows before each entry's start and is left with the last K - 1 rows; entries int32 [R, 4] =
+        (first row, tokens, start, slot)."""
+        self._call("short_conv", [u, taps, state, entries, entry_of, positions, out, bias], [int(bool(silu))])
 
     def diff_qk_prep(self, qkv, q_w, k_w, inv_freq, rope_table, positions, slots, table, pool, q_out, eps, heads, kv_heads, dk, dv,
                      rot_dims=0, mag=1.0, taps=None, state=None, entries=None):
@@ -407,10 +408,12 @@ class Ops:
         """score "softmax_chosen": the largest logits are chosen and the weights are the softmax over the chosen logits alone."""
         self._call("moe_route", [h, router, ids, wts], [top, {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2}[score], int(bool(renormalize))])
 
-    def moe_experts_gated(self, h, ids, wts, gate_up, down, y, experts, activation="clamped", limit=0.0, alpha=1.702):
-        """y f32 [M, W] = sum_k s_k down_e act(gate_e h, up_e h); gate_up [experts 2F, W] holds an expert's gate rows above its up rows."""
+    def moe_experts_gated(self, h, ids, wts, gate_up, down, y, experts, activation="clamped", limit=0.0, alpha=1.702, identity=0):
+        """y f32 [M, W] = sum_k s_k down_e act(gate_e h, up_e h); gate_up [experts 2F, W] holds an expert's gate rows above its up
+        rows; identity: so many ids from `experts` on stand for h itself."""
         libs = ["moe"] + (["moe_bf16"] if h.dtype == native.torch().bfloat16 else [])
-        self._call("moe_experts_gated", [h, ids, wts, gate_up, down, y], [experts, {"silu": 0, "clamped": 1}[activation], limit, alpha], libs=libs)
+        self._call("moe_experts_gated", [h, ids, wts, gate_up, down, y], [experts, {"silu": 0, "clamped": 1}[activation], limit, alpha, identity],
+                   libs=libs)
 
     # ---- Dynamic Tanh, gated activations, biased and partly rotated q/k/v, latent attention
     def dyt(self, x, alpha, w, b, out, rows=None):
@@ -457,14 +460,27 @@ class Ops:
         self._call("gated_attention", [q, pool, table, positions, slots, sink, gate_proj, out],
                    [heads, kv_heads, dk, dv, scale, int(window or 0), gate_col, gate_mode])
 
+    def linear_scan(self, rows, state, entries, o, heads, dk, dv, columns, decay=None, chunks=None, spans=None, qk_heads=0, silu=False,
+                    k_scale=1.0, inv_freq=None, rope_table=None, positions=None, rot_dims=0, dt=None, dt_col=0, dt_bias=None, a_log=None,
+                    skip=None):
+        """entries int32 [R, 4] = (first row, tokens, -, state slot); S <- a S + d k v^T, o = S^T q + skip v with q, k, v the columns
+        of `rows` (with silu, or q and k rotated), k times k_scale; decay f32 [heads]: a = decay, d = 1; else d = softplus(dt + dt_bias),
+        a = exp(-exp(a_log) d).  chunks int32 [n, 4] = (entry, first row, tokens up to 64, 1: the entry's first chunk + 2: its last)
+        and spans int32 [R, 2] = (first chunk, chunks): the entries' tokens run as chunks side by side."""
+        self._call("linear_scan", [rows, state, entries, o, chunks, spans, decay, inv_freq, rope_table, positions, dt, dt_bias, a_log, skip],
+                   [heads, dk, dv] + list(columns) + [qk_heads or heads, int(bool(silu)), k_scale, rot_dims, dt_col])
+
     def decay_scan(self, proj, decay, state, entries, o, heads, dk, dv, columns, chunks=None, spans=None):
-        """entries int32 [R, 4] = (first row, tokens, -, state slot); S <- decay S + k v^T, o = S^T q on silu'd columns of proj.
-        chunks int32 [n, 4] = (entry, first row, tokens, 1: the entry's first chunk + 2: its last) and spans int32 [R, 2] = (first
-        chunk, chunks): the entries' tokens run as chunks side by side."""
-        self._call("decay_scan", [proj, decay, state, entries, o, chunks, spans], [heads, dk, dv] + list(columns))
+        """`linear_scan` with a fixed decay per head on silu'd columns."""
+        self.linear_scan(proj, state, entries, o, heads, dk, dv, columns, decay=decay, chunks=chunks, spans=spans, silu=True)
+
+    def gated_group_norm(self, o, proj, gate_col, w, eps, out, groups=1, silu=False, gate_first=False):
+        """out = o / rms(o) * w * act(gate): the rms over each of `groups` equal runs of a row; w None: none; gate_first: the norm is
+        of o times act(gate)."""
+        self._call("gated_group_norm", [o, proj, w, out], [gate_col, eps, groups, int(bool(silu)), int(bool(gate_first))])
 
     def gated_row_norm(self, o, proj, gate_col, w, eps, out):
-        self._call("gated_row_norm", [o, proj, w, out], [gate_col, eps])
+        self.gated_group_norm(o, proj, gate_col, w, eps, out)
 
     def moe_route_grouped(self, h, router, ids, wts, correction, top, groups=0, keep=0, weight_scale=1.0, sum_floor=0.0, renormalize=True,
                           score="sigmoid", gate_row=None, gate_out=None):
@@ -474,10 +490,13 @@ class Ops:
                    [top, {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2}[score], int(bool(renormalize)), groups, keep, weight_scale, sum_floor])
 
     # ---- norms on either side of a sublayer, the minimal GRU, queries from a latent
-    def norm_residual_next(self, x, y, gain, eps, gather=None, n_sum=0, plus=None, plus_gate=None, next_gain=None, next_eps=0.0, next_out=None):
-        """x += y' / rms(y') * gain, then next_out = x / rms(x) * next_gain (where given); y' = y, or the sum of the rows y[gather[m, k]]
-        (no list and n_sum > 1: y[m n_sum + k]), plus plus_gate[m] plus[m]."""
-        self._call("norm_residual_next", [x, y, gain, gather, plus, plus_gate, next_gain, next_out], [eps, next_eps, n_sum])
+    def norm_residual_next(self, x, y, gain, eps, gather=None, n_sum=0, plus=None, plus_gate=None, next_gain=None, next_eps=0.0, next_out=None,
+                           centered=False, next_centered=False, factor=1.0, y_scale=1.0, plus_scale=1.0):
+        """x += factor N(y') gain, then next_out = N'(x) next_gain (where given); N divides by the root mean square or, centered, is a
+        layer norm; y' = y_scale times y, or the sum of the rows y[gather[m, k]] (no list and n_sum > 1: y[m n_sum + k]), plus
+        plus_scale plus_gate[m] plus[m]."""
+        self._call("norm_residual_next", [x, y, gain, gather, plus, plus_gate, next_gain, next_out],
+                   [eps, next_eps, n_sum, int(bool(centered)), int(bool(next_centered)), factor, y_scale, plus_scale])
 
     def add_gated_rows(self, y, plus, gate=None):
         """y[m] += gate[m] plus[m]."""
@@ -527,10 +546,10 @@ class Ops:
         """dst [heads cols, rows] = src [heads rows, cols], every head's matrix transposed."""
         self._call("latent_transpose", [src, dst], [heads])
 
-    def moe_experts(self, h, ids, wts, up, down, y, experts, scale_input=True):
+    def moe_experts(self, h, ids, wts, up, down, y, experts, scale_input=True, identity=0):
         """y f32 [M, W] = sum over a token's experts; up [experts F, W], down [experts W, F]."""
         libs = ["moe"] + (["moe_bf16"] if h.dtype == native.torch().bfloat16 else [])
-        self._call("moe_experts", [h, ids, wts, up, down, y], [experts, int(bool(scale_input))], libs=libs)
+        self._call("moe_experts", [h, ids, wts, up, down, y], [experts, int(bool(scale_input)), identity], libs=libs)
 
     def argmax(self, logits, out):
         if out.dtype != native.torch().int32 or out.shape[0] < logits.shape[0]:

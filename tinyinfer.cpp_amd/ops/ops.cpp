@@ -1369,47 +1369,80 @@ void Ops::gated_attention(const Tensor& q, const Tensor& pool, const CacheView& 
   check("gated_attention", rc, "gated_attention");
 }
 
-void Ops::decay_scan(const Tensor& proj, const QkvColumns& cols, const Tensor& decay, const Tensor& state, const int* entry_meta,
-                     int n_entries, const Tensor& o, int heads, int dk, int dv, const int* chunks, int n_chunks, const int* spans,
-                     Workspace* ws) {
-  TIMED("decay_scan " + dims(proj) + " entries=" + std::to_string(n_entries) + (chunks ? " chunks=" + std::to_string(n_chunks) : ""));
-  require(proj.ndim == 2 && proj.dtype == DType::F32 && proj.contiguous(), "decay_scan: proj must be contiguous float32 [M, N]");
-  const int64_t per_slot = (int64_t)heads * dk * dv;
+void Ops::linear_scan(const LinearScan& in, const Tensor& state, const int* entry_meta, int n_entries, const Tensor& o, int heads, int dk,
+                      int dv, const int* chunks, int n_chunks, const int* spans, Workspace* ws) {
+  TIMED("linear_scan " + dims(in.rows) + (in.decay.defined() ? "" : " selective") + " entries=" + std::to_string(n_entries) +
+        (chunks ? " chunks=" + std::to_string(n_chunks) : ""));
+  const Tensor& rows = in.rows;
+  require(rows.ndim == 2 && rows.dtype == DType::F32 && rows.contiguous(), "linear_scan: the rows must be contiguous float32 [M, N]");
+  const int64_t per_slot = (int64_t)heads * dk * dv, M = rows.shape[0];
   require(state.dtype == DType::F32 && state.contiguous() && state.ndim >= 2 && state.numel() == state.shape[0] * per_slot,
-          "decay_scan: state " + state.describe() + " does not fit [slots, " + std::to_string(heads) + ", " + std::to_string(dk * dv) + "]");
-  require(decay.dtype == DType::F32 && decay.numel() == heads, "decay_scan: decay " + decay.describe() + " must be float32 [heads]");
-  require(o.dtype == DType::F32 && o.contiguous() && o.ndim == 2 && o.shape[0] == proj.shape[0] && o.shape[1] == (int64_t)heads * dv,
-          "decay_scan: o " + o.describe() + " does not fit");
-  require(entry_meta != nullptr || n_entries == 0, "decay_scan: no entry records");
+          "linear_scan: state " + state.describe() + " does not fit [slots, " + std::to_string(heads) + ", " + std::to_string(dk * dv) + "]");
+  require(o.dtype == DType::F32 && o.contiguous() && o.ndim == 2 && o.shape[0] == M && o.shape[1] == (int64_t)heads * dv,
+          "linear_scan: o " + o.describe() + " does not fit");
+  require(entry_meta != nullptr || n_entries == 0, "linear_scan: no entry records");
+  auto per_head = [&](const Tensor& t) { return t.dtype == DType::F32 && t.contiguous() && t.numel() == heads; };
+  ti_scan_inputs si = {};
+  si.proj = (const float*)rows.data;
+  si.ld = (int)rows.shape[1];
+  si.off_q = in.cols.q;
+  si.off_k = in.cols.k;
+  si.off_v = in.cols.v;
+  si.qk_heads = in.qk_heads > 0 ? in.qk_heads : heads;
+  si.act = in.silu ? 1 : 0;
+  si.k_scale = in.k_scale;
+  if (in.rot.inv_freq) {
+    require(in.positions != nullptr && !in.silu && !in.rot.pairs && in.rot.mag == 1.f, "linear_scan: a rotation in pairs, with another magnitude or behind an activation is not served");
+    si.inv_freq = in.rot.inv_freq;
+    si.rope_table = in.rot.table;
+    si.table_len = in.rot.table_len;
+    si.rot_dims = in.rot.dims > 0 ? in.rot.dims : dk;
+    si.pos = in.positions;
+  }
+  if (in.decay.defined()) {
+    require(per_head(in.decay), "linear_scan: decay " + in.decay.describe() + " must be float32 [heads]");
+    si.decay = (const float*)in.decay.data;
+  } else {
+    require(in.dt.ndim == 2 && in.dt.dtype == DType::F32 && in.dt.contiguous() && in.dt.shape[0] == M && in.dt_col >= 0 &&
+                in.dt_col + heads <= in.dt.shape[1] && per_head(in.dt_bias) && per_head(in.a_log),
+            "linear_scan: the step sizes' columns, biases or rates do not fit");
+    si.dt = (const float*)in.dt.data + in.dt_col;
+    si.dt_ld = (int)in.dt.shape[1];
+    si.dt_bias = (const float*)in.dt_bias.data;
+    si.a_log = (const float*)in.a_log.data;
+  }
+  if (in.skip.defined()) {
+    require(per_head(in.skip), "linear_scan: skip " + in.skip.describe() + " must be float32 [heads]");
+    si.skip = (const float*)in.skip.data;
+  }
   if (chunks) {
-    require(spans && ws && n_chunks >= n_entries, "decay_scan: chunks need spans and a workspace");
-    float* scratch = (float*)ws->get("decay.chunk_states", (size_t)n_chunks * per_slot * 4);
-    int rc = KERNEL("linear_attention", ti_decay_scan_chunked)((const float*)proj.data, (int)proj.shape[1], cols.q, cols.k, cols.v,
-                                                               (const float*)decay.data, (float*)state.data, (long)per_slot, entry_meta,
-                                                               n_entries, chunks, n_chunks, spans, scratch, (float*)o.data, heads, dk, dv,
-                                                               (hipStream_t)launch_stream());
-    check("linear_attention", rc, "decay_scan(chunked)");
+    require(spans && ws && n_chunks >= n_entries, "linear_scan: chunks need spans and a workspace");
+    float* scratch = (float*)ws->get("scan.chunk_states", (size_t)n_chunks * (per_slot + heads) * 4);
+    int rc = KERNEL("linear_attention", ti_linear_scan_chunked)(&si, (float*)state.data, (long)per_slot, entry_meta, n_entries, chunks, n_chunks,
+                                                                spans, scratch, (float*)o.data, heads, dk, dv, (hipStream_t)launch_stream());
+    check("linear_attention", rc, "linear_scan(chunked)");
     took("[chunked]");
     return;
   }
-  int rc = KERNEL("linear_attention", ti_decay_scan)((const float*)proj.data, (int)proj.shape[1], cols.q, cols.k, cols.v,
-                                                     (const float*)decay.data, (float*)state.data, (long)per_slot, entry_meta, n_entries,
-                                                     (float*)o.data, heads, dk, dv, (hipStream_t)launch_stream());
-  check("linear_attention", rc, "decay_scan");
+  int rc = KERNEL("linear_attention", ti_linear_scan)(&si, (float*)state.data, (long)per_slot, entry_meta, n_entries, (float*)o.data, heads, dk,
+                                                      dv, (hipStream_t)launch_stream());
+  check("linear_attention", rc, "linear_scan");
 }
 
-void Ops::gated_row_norm(const Tensor& o, const Tensor& proj, int gate_col, const Tensor& w, float eps, const Tensor& out) {
-  TIMED("gated_row_norm " + dims(o));
-  require(o.ndim == 2 && o.dtype == DType::F32 && o.contiguous(), "gated_row_norm: o must be contiguous float32 [M, W]");
+void Ops::gated_group_norm(const Tensor& o, const Tensor& proj, int gate_col, const Tensor& w, float eps, const Tensor& out, const GroupNorm& form) {
+  TIMED("gated_group_norm " + dims(o) + (form.groups > 1 ? " groups=" + std::to_string(form.groups) : ""));
+  require(o.ndim == 2 && o.dtype == DType::F32 && o.contiguous(), "gated_group_norm: o must be contiguous float32 [M, W]");
   const int64_t M = o.shape[0], W = o.shape[1];
-  require(out.ndim == 2 && out.shape[0] == M && out.shape[1] == W && out.contiguous() && w.dtype == DType::F32 && w.numel() == W,
-          "gated_row_norm: out " + out.describe() + " or w " + w.describe() + " do not fit");
+  require(form.groups > 0 && W % form.groups == 0, "gated_group_norm: rows of " + std::to_string(W) + " in " + std::to_string(form.groups) + " runs");
+  require(out.ndim == 2 && out.shape[0] == M && out.shape[1] == W && out.contiguous() && (!w.defined() || (w.dtype == DType::F32 && w.numel() == W)),
+          "gated_group_norm: out " + out.describe() + " or w " + w.describe() + " do not fit");
   require(proj.ndim == 2 && proj.dtype == DType::F32 && proj.contiguous() && proj.shape[0] == M && gate_col >= 0 && gate_col + W <= proj.shape[1],
-          "gated_row_norm: the gate's columns do not lie inside proj " + proj.describe());
-  int rc = KERNEL("linear_attention", ti_gated_row_norm)(code(out.dtype, "gated_row_norm"), (const float*)o.data, (const float*)proj.data,
-                                                         (int)proj.shape[1], gate_col, (const float*)w.data, out.data, (int)M, (int)W, eps,
-                                                         (hipStream_t)launch_stream());
-  check("linear_attention", rc, "gated_row_norm");
+          "gated_group_norm: the gate's columns do not lie inside proj " + proj.describe());
+  int rc = KERNEL("linear_attention", ti_gated_group_norm)(code(out.dtype, "gated_group_norm"), (const float*)o.data, (const float*)proj.data,
+                                                           (int)proj.shape[1], gate_col, w.defined() ? (const float*)w.data : nullptr, out.data,
+                                                           (int)M, (int)W, form.groups, eps, form.silu ? 1 : 0, form.gate_first ? 1 : 0,
+                                                           (hipStream_t)launch_stream());
+  check("linear_attention", rc, "gated_group_norm");
 }
 
 // ------------------------------------------------- post-norm layers, short convolutions, differential attention, experts
@@ -1428,24 +1461,34 @@ void Ops::norm_residual(const Tensor& x, const Tensor& y, const Tensor& gain, fl
   check("residual", rc, "norm_residual");
 }
 
-void Ops::norm_residual_next(const Tensor& x, const Tensor& y, const int* gather, int n_gather, const Tensor& plus, const Tensor& plus_gate,
-                             const Tensor& gain, float eps, const Tensor& next_gain, float next_eps, const Tensor& next_out) {
-  TIMED("norm_residual_next " + dims(x) + (plus.defined() ? " plus" : "") + (next_out.defined() ? " +norm" : ""));
+void Ops::norm_residual_next(const Tensor& x, const GatheredRows& y, const RowNorm& norm, float factor, const RowNorm& next, const Tensor& next_out) {
+  TIMED("norm_residual_next " + dims(x) + (norm.centered ? " centered" : "") + (y.plus.defined() ? " plus" : "") + (next_out.defined() ? " +norm" : ""));
   const int64_t H = x.ndim == 2 ? x.shape[1] : 0;
-  require(x.ndim == 2 && x.dtype == DType::F32 && x.contiguous() && y.ndim == 2 && y.dtype == DType::F32 && y.contiguous() &&
-              y.shape[1] == H && (gather ? n_gather > 0 : y.shape[0] == x.shape[0] * std::max(1, n_gather)) &&
-              gain.dtype == DType::F32 && gain.numel() == H,
-          "norm_residual_next: x " + x.describe() + ", y " + y.describe() + " or gain " + gain.describe() + " do not fit");
-  require((!plus.defined() || (plus.dtype == DType::F32 && plus.contiguous() && plus.numel() == x.numel())) &&
-              (!plus_gate.defined() || (plus_gate.dtype == DType::F32 && plus_gate.contiguous() && plus_gate.numel() == x.shape[0])),
-          "norm_residual_next: the further branch " + plus.describe() + " or its gate do not fit");
-  require(!next_out.defined() || (next_out.contiguous() && next_out.numel() == x.numel() && next_gain.dtype == DType::F32 && next_gain.numel() == H),
+  require(x.ndim == 2 && x.dtype == DType::F32 && x.contiguous() && y.t.ndim == 2 && y.t.dtype == DType::F32 && y.t.contiguous() &&
+              y.t.shape[1] == H && (y.gather ? y.n_gather > 0 : y.t.shape[0] == x.shape[0] * std::max(1, y.n_gather)) &&
+              norm.gain.dtype == DType::F32 && norm.gain.numel() == H,
+          "norm_residual_next: x " + x.describe() + ", y " + y.t.describe() + " or gain " + norm.gain.describe() + " do not fit");
+  require((!y.plus.defined() || (y.plus.dtype == DType::F32 && y.plus.contiguous() && y.plus.numel() == x.numel())) &&
+              (!y.plus_gate.defined() || (y.plus_gate.dtype == DType::F32 && y.plus_gate.contiguous() && y.plus_gate.numel() == x.shape[0])),
+          "norm_residual_next: the further branch " + y.plus.describe() + " or its gate do not fit");
+  require(!next_out.defined() || (next_out.contiguous() && next_out.numel() == x.numel() && next.gain.dtype == DType::F32 && next.gain.numel() == H),
           "norm_residual_next: the next norm's rows or gain do not fit x");
-  int rc = KERNEL("residual", ti_norm_residual_next)(
-      (float*)x.data, (const float*)y.data, gather, n_gather, plus.defined() ? (const float*)plus.data : nullptr,
-      plus_gate.defined() ? (const float*)plus_gate.data : nullptr, (const float*)gain.data, eps,
-      next_out.defined() ? (const float*)next_gain.data : nullptr, next_eps, next_out.defined() ? next_out.data : nullptr,
-      next_out.defined() ? code(next_out.dtype, "norm_residual_next") : 0, (int)x.shape[0], (int)H, (hipStream_t)launch_stream());
+  ti_norm_pair p = {};
+  p.g = (const float*)norm.gain.data;
+  p.eps = norm.eps;
+  p.centered = norm.centered ? 1 : 0;
+  p.next_g = next_out.defined() ? (const float*)next.gain.data : nullptr;
+  p.next_eps = next.eps;
+  p.next_centered = next.centered ? 1 : 0;
+  p.y_scale = y.y_scale;
+  p.plus_scale = y.plus_scale;
+  p.factor = factor;
+  int rc = KERNEL("residual", ti_norm_residual_next)((float*)x.data, (const float*)y.t.data, y.gather, y.n_gather,
+                                                     y.plus.defined() ? (const float*)y.plus.data : nullptr,
+                                                     y.plus_gate.defined() ? (const float*)y.plus_gate.data : nullptr, &p,
+                                                     next_out.defined() ? next_out.data : nullptr,
+                                                     next_out.defined() ? code(next_out.dtype, "norm_residual_next") : 0, (int)x.shape[0],
+                                                     (int)H, (hipStream_t)launch_stream());
   check("residual", rc, "norm_residual_next");
 }
 
@@ -1507,23 +1550,25 @@ void Ops::scale(const Tensor& x, float s) {
 }
 
 void Ops::short_conv(const Tensor& u, const Tensor& taps, const Tensor& state, const int* entry_meta, int n_entries,
-                     const int* entry_of, const int* positions, const Tensor& out) {
-  TIMED("short_conv " + dims(u));
-  require(u.ndim == 2 && u.dtype == DType::F32 && u.contiguous() && out.ndim == 2 && out.dtype == DType::F32 && out.contiguous() &&
-              out.shape[0] == u.shape[0] && out.shape[1] == u.shape[1] && out.data != u.data,
-          "short_conv: u " + u.describe() + " and out " + out.describe() + " must be distinct contiguous float32 [M, C]");
+                     const int* entry_of, const int* positions, const Tensor& out, const Tensor& bias, bool silu) {
+  TIMED("short_conv " + dims(u) + (bias.defined() ? " bias" : "") + (silu ? " silu" : ""));
+  require(u.ndim == 2 && u.dtype == DType::F32 && u.stride[1] == 1 && u.stride[0] >= u.shape[1] && out.ndim == 2 && out.dtype == DType::F32 &&
+              out.contiguous() && out.shape[0] == u.shape[0] && out.shape[1] == u.shape[1] && out.data != u.data,
+          "short_conv: u " + u.describe() + " and out " + out.describe() + " must be distinct float32 [M, C]");
   const int64_t C = u.shape[1];
-  require(taps.ndim == 2 && taps.dtype == DType::F32 && taps.contiguous() && taps.shape[0] == C && taps.shape[1] >= 1,
-          "short_conv: taps " + taps.describe() + " must be float32 [C, taps]");
+  require(taps.ndim == 2 && taps.dtype == DType::F32 && taps.contiguous() && taps.shape[0] == C && taps.shape[1] >= 1 &&
+              (!bias.defined() || (bias.dtype == DType::F32 && bias.numel() == C)),
+          "short_conv: taps " + taps.describe() + " must be float32 [C, taps], a bias float32 [C]");
   const int64_t K = taps.shape[1];
   require(K == 1 || (state.defined() && state.dtype == DType::F32 && state.contiguous() && state.ndim == 3 &&
                      state.shape[1] == K - 1 && state.shape[2] == C),
           "short_conv: state " + state.describe() + " does not fit [slots, " + std::to_string(K - 1) + ", " + std::to_string(C) + "]");
   require(entry_meta != nullptr && entry_of != nullptr && positions != nullptr, "short_conv: no entry records");
-  int rc = KERNEL("diff_attention", ti_short_conv)((const float*)u.data, (const float*)taps.data, (float*)state.data, entry_meta,
-                                                   n_entries, entry_of, positions, (float*)out.data, (int)u.shape[0], (int)C, (int)K,
-                                                   (hipStream_t)launch_stream());
-  check("diff_attention", rc, "short_conv");
+  int rc = KERNEL("short_conv", ti_short_conv)((const float*)u.data, (long)u.stride[0], (const float*)taps.data,
+                                               bias.defined() ? (const float*)bias.data : nullptr, silu ? 1 : 0, (float*)state.data, entry_meta,
+                                               n_entries, entry_of, positions, (float*)out.data, (int)u.shape[0], (int)C, (int)K,
+                                               (hipStream_t)launch_stream());
+  check("short_conv", rc, "short_conv");
 }
 
 void Ops::diff_qk_prep(const Tensor& qkv, const float* q_w, const float* k_w, float eps, const Rotation& rot, const int* positions,
@@ -1644,19 +1689,32 @@ void Ops::moe_route(const Tensor& h, const Tensor& router, const Tensor& ids, co
 }
 
 void Ops::moe_experts(const Tensor& h, const Tensor& ids, const Tensor& wts, const Tensor& up, const Tensor& down, const Tensor& y,
-                      int experts, bool scale_input, Workspace& ws, GatheredRows* rows) {
-  TIMED("moe_experts " + dims(h) + " * " + dims(up));
+                      int experts, bool scale_input, Workspace& ws, GatheredRows* rows, int identity) {
+  experts_of("moe_experts", h, ids, wts, up, down, y, experts, scale_input, false, Silu, 0.f, 0.f, ws, rows, identity);
+}
+
+void Ops::moe_experts_gated(const Tensor& h, const Tensor& ids, const Tensor& wts, const Tensor& gate_up, const Tensor& down,
+                            const Tensor& y, int experts, GatedAct kind, float limit, float alpha, Workspace& ws, GatheredRows* rows, int identity) {
+  experts_of("moe_experts_gated", h, ids, wts, gate_up, down, y, experts, false, true, kind, limit, alpha, ws, rows, identity);
+}
+
+void Ops::experts_of(const char* name, const Tensor& h, const Tensor& ids, const Tensor& wts, const Tensor& up, const Tensor& down,
+                     const Tensor& y, int experts, bool scale_input, bool gated, GatedAct kind, float limit, float alpha, Workspace& ws,
+                     GatheredRows* rows, int identity) {
+  const std::string what = name;
+  TIMED(what + " " + dims(h) + " * " + dims(up) + (identity ? " +identity" : ""));
   require(h.ndim == 2 && h.contiguous() && up.ndim == 2 && down.ndim == 2 && up.contiguous() && down.contiguous() &&
-              up.dtype == h.dtype && down.dtype == h.dtype && experts > 0,
-          "moe_experts: h, up and down must be matrices of one dtype");
+              up.dtype == h.dtype && down.dtype == h.dtype && experts > 0 && identity >= 0,
+          what + ": h, up and down must be matrices of one dtype");
   const int64_t M = h.shape[0], W = h.shape[1];
-  require(up.shape[1] == W && up.shape[0] % experts == 0, "moe_experts: up " + up.describe() + " does not fit");
-  const int64_t F = up.shape[0] / experts;
-  require(down.shape[0] == (int64_t)experts * W && down.shape[1] == F, "moe_experts: down " + down.describe() + " does not fit");
+  const int64_t per = (gated ? 2 : 1) * (int64_t)experts;
+  require(up.shape[1] == W && up.shape[0] % per == 0, what + ": up " + up.describe() + " does not fit");
+  const int64_t F = up.shape[0] / per;
+  require(down.shape[0] == (int64_t)experts * W && down.shape[1] == F, what + ": down " + down.describe() + " does not fit");
   require(y.ndim == 2 && y.dtype == DType::F32 && y.contiguous() && y.shape[0] == M && y.shape[1] == W,
-          "moe_experts: y " + y.describe() + " does not fit");
+          what + ": y " + y.describe() + " does not fit");
   require(ids.dtype == DType::I32 && wts.dtype == DType::F32 && ids.numel() == wts.numel() && (M == 0 || ids.numel() % M == 0),
-          "moe_experts: ids and wts must be int32 / float32 [M, top]");
+          what + ": ids and wts must be int32 / float32 [M, top]");
   if (rows) *rows = GatheredRows();
   if (M == 0) return;
   const int top = (int)(ids.numel() / M);
@@ -1675,6 +1733,7 @@ void Ops::moe_experts(const Tensor& h, const Tensor& ids, const Tensor& wts, con
                                                              rows ? nullptr : (float*)y.data, (int)M, (int)W, (int)F, experts, top,
                                                              scale_input ? 1 : 0,
                                                              scale_input ? nullptr : (float*)ws.get("moe.row_w", (size_t)pairs * 4),
+                                                             gated ? (int)kind : -1, limit, alpha, identity > 0 ? 1 : 0,
                                                              (hipStream_t)launch_stream());
     if (rc == 0) {
       took(rows ? "[mfma, grouped, sums left]" : "[mfma, grouped]");
@@ -1685,70 +1744,24 @@ void Ops::moe_experts(const Tensor& h, const Tensor& ids, const Tensor& wts, con
       }
       return;
     }
-    if (rc != 3) check("moe_bf16", rc, "moe_experts(grouped)");
+    if (rc != 3) check("moe_bf16", rc, (what + "(grouped)").c_str());
   }
   took(rows && top > 1 ? "[rows, sums left]" : "[rows]");
   Tensor act = ws.tensor("moe.act", h.dtype, {pairs, F});
   // one expert a token: its row is the result; else the pairs' rows, added by this call or left to the norm that reads them
   Tensor part = top == 1 ? y : ws.tensor("moe.out", DType::F32, {pairs, W});
   const bool left = rows && top > 1;
-  int rc = KERNEL("moe", ti_moe_experts_rows)(code(h.dtype, "moe_experts"), h.data, (const int*)ids.data, (const float*)wts.data,
-                                              up.data, down.data, act.data, (float*)part.data, (top == 1 || left) ? nullptr : (float*)y.data,
-                                              (int)M, (int)W, (int)F, experts, top, scale_input ? 1 : 0, (hipStream_t)launch_stream());
-  check("moe", rc, "moe_experts");
-  if (left) {
-    rows->t = part;
-    rows->gather = nullptr;
-    rows->n_gather = top;
-  }
-}
-
-void Ops::moe_experts_gated(const Tensor& h, const Tensor& ids, const Tensor& wts, const Tensor& gate_up, const Tensor& down,
-                            const Tensor& y, int experts, GatedAct kind, float limit, float alpha, Workspace& ws, GatheredRows* rows) {
-  TIMED("moe_experts_gated " + dims(h) + " * " + dims(gate_up));
-  require(h.ndim == 2 && h.contiguous() && gate_up.ndim == 2 && down.ndim == 2 && gate_up.contiguous() && down.contiguous() &&
-              gate_up.dtype == h.dtype && down.dtype == h.dtype && experts > 0,
-          "moe_experts_gated: h, gate_up and down must be matrices of one dtype");
-  const int64_t M = h.shape[0], W = h.shape[1];
-  require(gate_up.shape[1] == W && gate_up.shape[0] % (2 * experts) == 0, "moe_experts_gated: gate_up " + gate_up.describe() + " does not fit");
-  const int64_t F = gate_up.shape[0] / (2 * experts);
-  require(down.shape[0] == (int64_t)experts * W && down.shape[1] == F, "moe_experts_gated: down " + down.describe() + " does not fit");
-  require(y.ndim == 2 && y.dtype == DType::F32 && y.contiguous() && y.shape[0] == M && y.shape[1] == W,
-          "moe_experts_gated: y " + y.describe() + " does not fit");
-  require(ids.dtype == DType::I32 && wts.dtype == DType::F32 && ids.numel() == wts.numel() && (M == 0 || ids.numel() % M == 0),
-          "moe_experts_gated: ids and wts must be int32 / float32 [M, top]");
-  if (rows) *rows = GatheredRows();
-  if (M == 0) return;
-  const int top = (int)(ids.numel() / M);
-  const int64_t pairs = M * top;
-  Tensor z = ws.tensor("moe.z", DType::F32, {pairs, 2 * F});
-  // many tokens: the pairs grouped by expert, both products on the matrix cores
-  if (h.dtype == DType::BF16 && use.fast_gemm && pairs >= 128 && kernel_library_available("moe_bf16")) {
-    const long meta_ints = KERNEL("moe_bf16", ti_moe_grouped_meta_ints)((int)pairs, experts);
-    int* meta = (int*)ws.get("moe.meta", (size_t)meta_ints * 4);
-    Tensor where = ws.tensor("moe.where", DType::I32, {pairs});
-    void* sorted = ws.get("moe.rows", (size_t)pairs * 4);
-    Tensor act = ws.tensor("moe.act", DType::BF16, {pairs, F});
-    Tensor out = ws.tensor("moe.out", DType::F32, {pairs, W});
-    int rc = KERNEL("moe_bf16", ti_moe_experts_grouped_gated_bf16)(h.data, (const int*)ids.data, (const float*)wts.data, gate_up.data,
-                                                                   down.data, meta, (int*)where.data, sorted, (float*)z.data, act.data,
-                                                                   (float*)out.data, (float*)y.data, (int)M, (int)W, (int)F, experts, top,
-                                                                   (int)kind, limit, alpha, (hipStream_t)launch_stream());
-    if (rc == 0) {
-      took("[mfma, grouped]");
-      return;
-    }
-    if (rc != 3) check("moe_bf16", rc, "moe_experts_gated(grouped)");
-  }
-  took(rows && top > 1 ? "[rows, sums left]" : "[rows]");
-  Tensor act = ws.tensor("moe.act", h.dtype, {pairs, F});
-  Tensor part = top == 1 ? y : ws.tensor("moe.out", DType::F32, {pairs, W});
-  const bool left = rows && top > 1;
-  int rc = KERNEL("moe", ti_moe_experts_rows_gated)(code(h.dtype, "moe_experts_gated"), h.data, (const int*)ids.data, (const float*)wts.data,
-                                                    gate_up.data, down.data, (float*)z.data, act.data, (float*)part.data,
-                                                    (top == 1 || left) ? nullptr : (float*)y.data, (int)M, (int)W, (int)F, experts, top,
-                                                    (int)kind, limit, alpha, (hipStream_t)launch_stream());
-  check("moe", rc, "moe_experts_gated");
+  float* sums = (top == 1 || left) ? nullptr : (float*)y.data;
+  int rc;
+  if (gated)
+    rc = KERNEL("moe", ti_moe_experts_rows_gated)(code(h.dtype, name), h.data, (const int*)ids.data, (const float*)wts.data, up.data,
+                                                  down.data, act.data, (float*)part.data, sums, (int)M, (int)W, (int)F, experts, top,
+                                                  (int)kind, limit, alpha, identity > 0 ? 1 : 0, (hipStream_t)launch_stream());
+  else
+    rc = KERNEL("moe", ti_moe_experts_rows)(code(h.dtype, name), h.data, (const int*)ids.data, (const float*)wts.data, up.data, down.data,
+                                            act.data, (float*)part.data, sums, (int)M, (int)W, (int)F, experts, top, scale_input ? 1 : 0,
+                                            identity > 0 ? 1 : 0, (hipStream_t)launch_stream());
+  check("moe", rc, name);
   if (left) {
     rows->t = part;
     rows->gather = nullptr;

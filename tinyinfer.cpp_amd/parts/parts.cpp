@@ -58,6 +58,13 @@
 //   mixer     "sum"         two mixers side by side on the same input, added with fixed factors
 //   ffn       "glu" with `activation` "gelu_tanh"; "moe" with `correction`, `groups`, `weight_scale`, `sum_floor`
 //
+//   mixer     "decay_attention" with `activation` "none", `pos`, `k_scale`, `norm` "head", `gate` "silu" (retention)
+//   mixer     "mamba2"      a short convolution, then a matrix state per head under a decay the token sets, a gate in front of a
+//                           norm in parts; state and convolution rows per request
+//   filter    "short_conv" with `bias`, `activation` "silu"
+//   block     "sandwich" with `factor`, layer norms and mixers of two branches
+//   ffn       "moe" with `identity`: experts that return their input
+//
 // A part gets every size and constant as a parameter and never looks at the model it sits in.
 #include <algorithm>
 #include <cmath>
@@ -332,9 +339,10 @@ class RMSNorm final : public NormPart {
     weight = src.alloc(DType::F32, {dim});
     spread(one, weight, src.to_host);
   }
-  bool rms_form(Tensor& w, float& e) const override {
-    w = weight;
-    e = eps;
+  bool row_form(Ops::RowNorm& norm) const override {
+    norm.gain = weight;
+    norm.eps = eps;
+    norm.centered = false;
     return true;
   }
   static void spread(const Tensor& one, const Tensor& all, bool on_host);     // all[:] = one[0]
@@ -586,10 +594,11 @@ class Attention final : public MixerPart {
       if (vm != "first" && vm != "mix") throw ConfigError("attention: v_mix '" + vm + "' is not served (first, mix)");
       mix_mode = vm == "first" ? 1 : 2;
     }
-    gated = has_sink || fixed_sink || gate_mode != 0 || values_from_keys || mix_mode != 0 || unit_norm;
+    const bool own_values = v_dim != head_dim || (p.has("general") && p.at("general").as_bool());
+    gated = has_sink || fixed_sink || gate_mode != 0 || values_from_keys || mix_mode != 0 || unit_norm || (qk_norm && own_values);
     if (gated) {
       if (softcap > 0.f || temp_coef != 0.f || bias || (p.has("shares_kv") && p.at("shares_kv").as_bool()))
-        throw ConfigError("attention: a sink, a gate, values from the keys or mixed values go with neither capped scores, a query "
+        throw ConfigError("attention: a sink, a gate, values from the keys, mixed values or a norm beside a value size go with neither capped scores, a query "
                           "temperature, biases nor a shared cache");
       if (values_from_keys && v_dim != head_dim) throw ConfigError("attention: values that are the keys have the keys' size");
       if (values_from_keys && mix_mode) throw ConfigError("attention: values that are the keys are not mixed");
@@ -950,7 +959,7 @@ class Attention final : public MixerPart {
   int64_t hidden = 0, nq = 0, nk = 0, nv = 0, no = 0, ng = 0;
   int heads = 0, kv_heads = 0, head_dim = 0, v_dim = 0, window = 0, temp_every = 0;
   bool qk_norm = true, shares_kv = false, general = false, bias = false;
-  bool gated = false;             // any of the four below: the gated kernels run
+  bool gated = false;             // any of the below, or a per-head norm beside values of their own size: the gated kernels run
   bool unit_norm = false;         // `qk_norm` "unit_after": q and k heads divided by their root mean square behind the rotation
   bool fixed_sink = false;        // `sink_value`: the same number for every head, in the place of a learned sink
   float sink_value = 0.f;
@@ -1444,9 +1453,10 @@ class RotaryPartial final : public PositionPart {
 };
 
 // A causal convolution over time on every channel of the rows it is given: y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros
-// before a sequence's start, no bias.  `segments`: [[tensor name, channels], ...], the taps [channels, taps] of runs of
-// channels side by side (the parts of a fused projection each bring their own tensor).  The last taps - 1 rows of every
-// request are its state (32-bit, zeroed at admission: the zeros before the start).
+// before a sequence's start.  `segments`: [[tensor name, channels], ...], the taps [channels, taps] of runs of
+// channels side by side (the parts of a fused projection each bring their own tensor).  `bias`: plus a number a channel (the
+// segments' names with ".b").  `activation` "silu": of the result.  The last taps - 1 rows of every request are its state (32-bit,
+// zeroed at admission: the zeros before the start).
 class ShortConv final : public FilterPart {
  public:
   ShortConv(const std::string& prefix, const Json& p) : FilterPart(prefix) {
@@ -1460,6 +1470,11 @@ class ShortConv final : public FilterPart {
       segments.emplace_back(s[0].as_string(), s[1].as_int());
       channels += s[1].as_int();
     }
+    bias = p.has("bias") && p.at("bias").as_bool();
+    if (p.has("activation")) {
+      if (p.at("activation").as_string() != "silu") throw ConfigError("short_conv: activation '" + p.at("activation").as_string() + "' is not served (silu)");
+      silu = true;
+    }
   }
   const char* kind_name() const override { return "short_conv"; }
   bool reads_through_ops() const override { return true; }
@@ -1472,14 +1487,23 @@ class ShortConv final : public FilterPart {
       n.a = 1.0 / taps;
       n.b = 0.3;
       t.emplace_back(s.first, n);
+      if (bias) {
+        TensorNeed b;
+        b.shape = {s.second};
+        b.role = TensorNeed::Vector;
+        b.b = 0.2;
+        t.emplace_back(s.first + ".b", b);
+      }
     }
     return t;
   }
   void load(WeightSource& src) override {
     w = src.alloc(DType::F32, {channels, (int64_t)taps});
+    if (bias) b = src.alloc(DType::F32, {channels});
     int64_t at = 0;
     for (const auto& s : segments) {
       src.fill(s.first, w.rows(at, s.second));
+      if (bias) src.fill(s.first + ".b", b.rows(at, s.second));
       at += s.second;
     }
   }
@@ -1496,9 +1520,10 @@ class ShortConv final : public FilterPart {
     return ctx.state(bound.first, bound.second);
   }
   void forward(StepContext& ctx, const Tensor& u, const Tensor& out) override {
-    ctx.ops.short_conv(u, w, state_of(ctx), ctx.entry_meta, (int)ctx.entries.size(), ctx.slots, ctx.positions, out);
+    ctx.ops.short_conv(u, w, state_of(ctx), ctx.entry_meta, (int)ctx.entries.size(), ctx.slots, ctx.positions, out, b, silu);
   }
   bool fused(StepContext& ctx, Ops::ShortConv& conv) override {
+    if (bias || silu) return false;
     conv.taps = w;
     conv.state = state_of(ctx);
     conv.entry_meta = ctx.entry_meta;
@@ -1506,11 +1531,12 @@ class ShortConv final : public FilterPart {
     conv.entry_of = ctx.slots;
     return true;
   }
-  std::vector<std::pair<std::string, Tensor>> held() const override { return {{"w", w}}; }
+  std::vector<std::pair<std::string, Tensor>> held() const override { return {{"w", w}, {"b", b}}; }
   int taps = 1;
   int64_t channels = 0;
+  bool bias = false, silu = false;
   std::vector<std::pair<std::string, int64_t>> segments;
-  Tensor w;
+  Tensor w, b;
 };
 
 // Differential attention.  Every one of the `heads` query heads holds two maps: q has heads x 2 x head_dim rows, k has
@@ -1736,7 +1762,8 @@ class DiffAttention final : public MixerPart {
 // scores are divided by their sum.  `scale_input` true: the score multiplies the expert's input, the output is
 // sum_e expert_e(s_e h); false: its output.  `activation`: "relu2", the square of relu.  `shared_gate`: the output of the
 // `shared` feed-forward is multiplied by sigmoid(w . h), one number a token (tensor `shared_gate_tensor` [1, hidden], default
-// prefix.shared.gate); the router's kernel takes that row along.
+// prefix.shared.gate); the router's kernel takes that row along.  `identity`: so many rows more in the router (and the correction),
+// behind the experts': identity experts, whose output is h itself; they hold no weights.
 class MoE final : public FeedForwardPart {
  public:
   MoE(const std::string& prefix, const Json& p, const PartChildren& children = {}) : FeedForwardPart(prefix) {
@@ -1746,7 +1773,9 @@ class MoE final : public FeedForwardPart {
     top = (int)param_int(p, "top");
     if (hidden <= 0 || intermediate <= 0) throw ConfigError("moe: sizes must be positive");
     if (experts < 1 || experts > 1024) throw ConfigError("moe: " + std::to_string(experts) + " experts are not served (1 to 1024)");
-    if (top < 1 || top > experts || top > 64)
+    identity = p.has("identity") ? (int)param_int(p, "identity") : 0;
+    if (identity < 0 || experts + identity > 1024) throw ConfigError("moe: " + std::to_string(identity) + " identity experts are not served");
+    if (top < 1 || top > experts + identity || top > 64)
       throw ConfigError("moe: top " + std::to_string(top) + " must lie between 1 and the number of experts (and at most 64)");
     if (hidden * 4 > 64 * 1024 || intermediate * 4 > 64 * 1024)
       throw ConfigError("moe: a width of " + std::to_string(hidden) + " / an expert size of " + std::to_string(intermediate) +
@@ -1776,6 +1805,7 @@ class MoE final : public FeedForwardPart {
     if (p.has("groups")) {
       groups = (int)param_int(p.at("groups"), "count");
       keep = (int)param_int(p.at("groups"), "keep");
+      if (identity) throw ConfigError("moe: identity experts do not go with groups");
       if (groups < 1 || experts % groups || keep < 1 || keep > groups || (int64_t)keep * (experts / groups) < top)
         throw ConfigError("moe: " + std::to_string(groups) + " groups of which " + std::to_string(keep) + " are kept do not fit " +
                           std::to_string(experts) + " experts and top " + std::to_string(top));
@@ -1811,7 +1841,7 @@ class MoE final : public FeedForwardPart {
     TensorNeed up, down, router;
     up.shape = {intermediate, hidden};
     down.shape = {hidden, intermediate};
-    router.shape = {(int64_t)experts, hidden};
+    router.shape = {(int64_t)experts + identity, hidden};
     router.role = TensorNeed::Vector;      // held in 32-bit whatever the engine's dtype
     router.b = 0.1;
     for (int e = 0; e < experts; ++e) {
@@ -1829,7 +1859,7 @@ class MoE final : public FeedForwardPart {
     }
     if (corrected) {
       TensorNeed c;
-      c.shape = {(int64_t)experts};
+      c.shape = {(int64_t)experts + identity};
       c.role = TensorNeed::Vector;
       c.b = 0.3;
       t.emplace_back(n_correction, c);
@@ -1848,7 +1878,7 @@ class MoE final : public FeedForwardPart {
       src.fill(expert_name(e, "down"), w_down.rows((int64_t)e * hidden, hidden));
     }
     TensorNeed router;
-    router.shape = {(int64_t)experts, hidden};
+    router.shape = {(int64_t)experts + identity, hidden};
     router.role = TensorNeed::Vector;
     w_router = src.fetch(n_router, router);
     if (shared_gate) {
@@ -1859,7 +1889,7 @@ class MoE final : public FeedForwardPart {
     }
     if (corrected) {
       TensorNeed c;
-      c.shape = {(int64_t)experts};
+      c.shape = {(int64_t)experts + identity};
       c.role = TensorNeed::Vector;
       correction = src.fetch(n_correction, c);
     }
@@ -1884,8 +1914,8 @@ class MoE final : public FeedForwardPart {
     } else {
       ctx.ops.moe_route(rows, w_router, ids, wts, top, score, renormalize);
     }
-    if (gated) ctx.ops.moe_experts_gated(rows, ids, wts, w_up, w_down, y, experts, act_kind, limit, alpha, ctx.ws, left);
-    else ctx.ops.moe_experts(rows, ids, wts, w_up, w_down, y, experts, scale_input, ctx.ws, left);
+    if (gated) ctx.ops.moe_experts_gated(rows, ids, wts, w_up, w_down, y, experts, act_kind, limit, alpha, ctx.ws, left, identity);
+    else ctx.ops.moe_experts(rows, ids, wts, w_up, w_down, y, experts, scale_input, ctx.ws, left, identity);
   }
   void forward_store(StepContext& ctx, const Rows& h, const Tensor& y) override {
     run(ctx, h, y, nullptr);
@@ -1925,7 +1955,7 @@ class MoE final : public FeedForwardPart {
     return {{"w_up", w_up}, {"w_down", w_down}, {"w_router", w_router}, {"w_shared_gate", w_shared_gate}};
   }
   int64_t hidden = 0, intermediate = 0;
-  int experts = 0, top = 0;
+  int experts = 0, top = 0, identity = 0;
   Ops::RouterScore score = Ops::Sigmoid;
   bool renormalize = false, scale_input = true;
   bool gated = false;                      // `activation` glu_*: experts hold gate, up and down; the weight is on the output
@@ -1985,7 +2015,7 @@ class DynamicTanh final : public NormPart {
 // gelu(g) = g / 2 (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))); "clamped" (`limit`, `alpha` default 1.702):
 // g = min(g, limit), u = clamp(u, -limit, limit), g sigmoid(alpha g) (u + 1).  `bias`: every projection has a bias (the
 // tensor's name with ".b").  The first product leaves 32-bit sums of [gate | up] (one stacked weight), the activation is
-// taken in 32-bit and rounded once.  Tensor names: prefix + ".gate", ".up", ".down" unless the parameters give them.
+// taken in 32-bit and rounded once (silu without biases: inside the product).  Tensor names: prefix + ".gate", ".up", ".down" unless the parameters give them.
 class GatedFFN final : public FeedForwardPart {
  public:
   GatedFFN(const std::string& prefix, const Json& p) : FeedForwardPart(prefix) {
@@ -2044,10 +2074,14 @@ class GatedFFN final : public FeedForwardPart {
   }
   void run(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
     const int64_t M = h.t.shape[0];
-    Tensor z = ctx.buf("glu.z", DType::F32, {M, 2 * intermediate});
-    ctx.ops.linear(h, w_gate_up, z, Ops::Store);
     Tensor y = ctx.buf("glu.y", ctx.act_dtype, {M, intermediate});
-    ctx.ops.gated_act(z, b_gate_up, y, kind, limit, alpha);
+    if (kind == Ops::Silu && !bias) {      // the activation in the product's epilogue
+      ctx.ops.linear(h, w_gate_up, y, Ops::SwiGLU);
+    } else {
+      Tensor z = ctx.buf("glu.z", DType::F32, {M, 2 * intermediate});
+      ctx.ops.linear(h, w_gate_up, z, Ops::Store);
+      ctx.ops.gated_act(z, b_gate_up, y, kind, limit, alpha);
+    }
     ctx.ops.linear(y, w_down, out, epi, false);
     if (bias) ctx.ops.add_row(out, b_down);
   }
@@ -2436,6 +2470,12 @@ class LayerNorm final : public NormPart {
     if (accumulate || gather || n_gather > 1 || rounded) throw EngineError("layernorm: it norms 32-bit rows in place, nothing else");
     ctx.ops.layernorm(y, weight, eps, x);
   }
+  bool row_form(Ops::RowNorm& norm) const override {
+    norm.gain = weight;
+    norm.eps = eps;
+    norm.centered = true;
+    return true;
+  }
   bool can_mix() const override { return true; }
   Rows forward_mixed(StepContext& ctx, const Tensor& streams, const Tensor& coef) override {
     Rows r;
@@ -2637,15 +2677,18 @@ class HyperBlock final : public BlockPart {
   Tensor w_in[2], w_out[2], w_mix[2];
 };
 
-// Linear attention with a fixed decay per head.  q = silu(W_q h), k = silu(W_k h) (heads x head_dim), v = silu(W_v h)
-// (heads x v_head_dim); per head S_t = decay_h S_(t-1) + k_t v_t^T and o_t = S_t^T q_t, no other scale; the heads side by side
-// are divided by their root mean square over the whole row (eps), multiplied by the vector `norm` and by sigmoid(W_g h), and W_o
-// maps them back.  q, k, v and the gate come from one product with the stacked weight [q; k; v; g].  S (heads x head_dim x
-// v_head_dim) is per-request state in 32-bit, zero at admission; activations, state, outputs and the norm are 32-bit.
+// Linear attention with a fixed decay per head.  q = act(W_q h), k = act(W_k h) (heads x head_dim), v = act(W_v h)
+// (heads x v_head_dim), act silu (`activation` "silu", the default) or nothing ("none"); without an activation q and k may be
+// rotated (the child `pos`); k times `k_scale` (default 1) behind that.  Per head S_t = decay_h S_(t-1) + k_t v_t^T and
+// o_t = S_t^T q_t, no other scale.  `norm` "row" (the default): the heads side by side are divided by their root mean square over
+// the whole row (eps) and multiplied by the vector `norm`; "head": each head by its own, no vector.  Then times sigmoid(W_g h) or
+// silu(W_g h) (`gate` "sigmoid", the default, or "silu"), and W_o maps them back.  q, k, v and the gate come from one product with
+// the stacked weight [q; k; v; g].  S (heads x head_dim x v_head_dim) is per-request state in 32-bit, zero at admission; what
+// enters the recurrence, the state, outputs and the norm are 32-bit.
 // `decay`: the heads' factors.  Tensor names: prefix + ".q", ".k", ".v", ".g", ".o", ".norm".
 class DecayAttention final : public MixerPart {
  public:
-  DecayAttention(const std::string& prefix, const Json& p) : MixerPart(prefix) {
+  DecayAttention(const std::string& prefix, const Json& p, const PartChildren& children = {}) : MixerPart(prefix) {
     hidden = param_int(p, "hidden");
     heads = (int)param_int(p, "heads");
     dk = (int)param_int(p, "head_dim");
@@ -2659,6 +2702,21 @@ class DecayAttention final : public MixerPart {
       if (!v.is_number()) throw ConfigError("decay_attention: 'decay' must hold numbers");
       decay.push_back((float)v.as_double());
     }
+    auto choice = [&](const char* key, const char* first, const char* second) {      // true: the second
+      if (!p.has(key)) return false;
+      const std::string v = p.at(key).as_string();
+      if (v != first && v != second) throw ConfigError(std::string("decay_attention: ") + key + " '" + v + "' is not served (" + first + ", " + second + ")");
+      return v == second;
+    };
+    silu = !choice("activation", "silu", "none");
+    head_norm = choice("norm", "row", "head");
+    form.groups = head_norm ? heads : 1;
+    form.silu = choice("gate", "sigmoid", "silu");
+    k_scale = p.has("k_scale") ? (float)param_float(p, "k_scale") : 1.f;
+    for (const auto& c : children)
+      if (c.first == "pos") pos = std::dynamic_pointer_cast<PositionPart>(c.second);
+    if (!pos && p.has("pos")) pos = std::dynamic_pointer_cast<PositionPart>(build_part("pos", PartSpec::from_json(p.at("pos")), prefix));
+    if (pos && silu) throw ConfigError("decay_attention: a rotation does not go with an activation on q and k");
     nq = (int64_t)heads * dk;
     nv = (int64_t)heads * dv;
     width = 2 * nq + 2 * nv;
@@ -2667,6 +2725,14 @@ class DecayAttention final : public MixerPart {
   bool takes_lazy_norm() const override { return true; }
   bool reads_through_ops() const override { return true; }
   bool can_store() const override { return true; }
+  std::vector<std::shared_ptr<Part>> children() const override {
+    if (pos) return {pos};
+    return {};
+  }
+  std::vector<std::string> child_slots() const override {
+    if (pos) return {"pos"};
+    return {};
+  }
   std::string name(const char* t) const { return join(prefix, t); }
   std::vector<std::pair<std::string, TensorNeed>> tensors() const override {
     TensorNeed qk, v, o, nw;
@@ -2677,7 +2743,9 @@ class DecayAttention final : public MixerPart {
     nw.role = TensorNeed::Vector;
     nw.a = 1.0;
     nw.b = 0.1;
-    return {{name("q"), qk}, {name("k"), qk}, {name("v"), v}, {name("g"), v}, {name("o"), o}, {name("norm"), nw}};
+    std::vector<std::pair<std::string, TensorNeed>> t = {{name("q"), qk}, {name("k"), qk}, {name("v"), v}, {name("g"), v}, {name("o"), o}};
+    if (!head_norm) t.emplace_back(name("norm"), nw);
+    return t;
   }
   void load(WeightSource& src) override {
     w_in = src.alloc(src.matrix_dtype, {width, hidden});
@@ -2687,7 +2755,7 @@ class DecayAttention final : public MixerPart {
     src.fill(name("g"), w_in.rows(2 * nq + nv, nv));
     const auto t = tensors();
     w_o = src.fetch(t[4].first, t[4].second);
-    norm_w = src.fetch(t[5].first, t[5].second);
+    if (!head_norm) norm_w = src.fetch(t[5].first, t[5].second);
     w_decay = src.alloc(DType::F32, {(int64_t)heads});
     put_floats(w_decay, decay, src.to_host);
   }
@@ -2699,25 +2767,33 @@ class DecayAttention final : public MixerPart {
     return n;
   }
   // A step with a long portion: every entry's tokens in chunks of CHUNK that run side by side (the state is carried from chunk
-  // to chunk element by element), from CHUNK_FROM tokens on.  The lists are the same for every such mixer of the model; the
-  // first one builds them.
-  static constexpr int CHUNK = 64, CHUNK_FROM = 128;
-  void plan(StepPlan& plan) const override { plan_chunks(plan, "decay", CHUNK, CHUNK_FROM); }
+  // to chunk element by element), from CHUNK_FROM tokens on.  The lists are the same for every mixer of the model that scans so;
+  // the first one builds them.
+  static constexpr int CHUNK = 64, CHUNK_FROM = 64;
+  void plan(StepPlan& plan) const override { plan_chunks(plan, "scan", CHUNK, CHUNK_FROM); }
+  // the scan of a step over the part's state slots, in chunks where the step has them
+  static void scan(StepContext& ctx, const MixerPart* part, const Ops::LinearScan& in, const Tensor& o, int heads, int dk, int dv) {
+    const auto bound = ctx.binding(part);
+    ctx.ops.linear_scan(in, ctx.state(bound.first, bound.second), ctx.entry_meta, (int)ctx.entries.size(), o, heads, dk, dv,
+                        ctx.planned("scan.chunks"), (int)(ctx.planned_size("scan.chunks") / 4), ctx.planned("scan.spans"), &ctx.ws);
+  }
   void run(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
     const int64_t M = h.t.shape[0];
     Tensor proj = ctx.buf("decay.proj", DType::F32, {M, width});
     ctx.ops.linear(h, w_in, proj, Ops::Store);
-    const auto bound = ctx.binding(this);
-    const Tensor state = ctx.state(bound.first, bound.second);
     Tensor o = ctx.buf("decay.o", DType::F32, {M, nv});
-    Ops::QkvColumns cols;
-    cols.q = 0;
-    cols.k = (int)nq;
-    cols.v = (int)(2 * nq);
-    ctx.ops.decay_scan(proj, cols, w_decay, state, ctx.entry_meta, (int)ctx.entries.size(), o, heads, dk, dv, ctx.planned("decay.chunks"),
-                       (int)(ctx.planned_size("decay.chunks") / 4), ctx.planned("decay.spans"), &ctx.ws);
+    Ops::LinearScan in;
+    in.rows = proj;
+    in.cols.k = (int)nq;
+    in.cols.v = (int)(2 * nq);
+    in.silu = silu;
+    in.k_scale = k_scale;
+    in.decay = w_decay;
+    if (pos && !pos->fused(in.rot)) throw EngineError("decay_attention: the position encoding '" + std::string(pos->kind_name()) + "' has no fused form");
+    in.positions = ctx.positions;
+    scan(ctx, this, in, o, heads, dk, dv);
     Tensor a = ctx.buf("decay.gated", ctx.act_dtype, {M, nv});
-    ctx.ops.gated_row_norm(o, proj, (int)(2 * nq + nv), norm_w, eps, a);
+    ctx.ops.gated_group_norm(o, proj, (int)(2 * nq + nv), norm_w, eps, a, form);
     ctx.ops.linear(a, w_o, out, epi, epi == Ops::Add);
   }
   void forward(StepContext& ctx, const Rows& h, const Tensor& x) override { run(ctx, h, x, Ops::Add); }
@@ -2727,9 +2803,126 @@ class DecayAttention final : public MixerPart {
   }
   int64_t hidden = 0, nq = 0, nv = 0, width = 0;
   int heads = 0, dk = 0, dv = 0;
-  float eps = 1e-6f;
+  float eps = 1e-6f, k_scale = 1.f;
+  bool silu = true, head_norm = false;
+  Ops::GroupNorm form;
+  std::shared_ptr<PositionPart> pos;
   std::vector<float> decay;
   Tensor w_in, w_o, norm_w, w_decay;
+};
+
+// A Mamba-2 layer (state-space duality).  W_in h = [z: inner | x: inner | B: groups state | C: groups state | dt: heads], inner =
+// heads x v_head_dim.  x, B and C together pass a short causal convolution over time (`conv` taps, a bias) and silu.  Per head,
+// with d = softplus(dt + dt_bias) and head j reading group floor(j / (heads / groups)) of B and C:
+//   S_t = exp(-exp(A_log) d) S_(t-1) + d B_t x_t^T  (state x v_head_dim),   y_t = S_t^T C_t + D x_t.
+// y times silu(z) is divided by its root mean square (eps) in `norm_groups` equal parts, multiplied by the vector `norm`, and W_o
+// maps it back.  S and the convolution's last inputs are per-request state in 32-bit, zero at admission; everything between the two
+// products is 32-bit.  Tensor names: prefix + ".in", ".conv", ".conv.b", ".dt_bias", ".A_log", ".D", ".norm", ".o".
+class Mamba2 final : public MixerPart {
+ public:
+  Mamba2(const std::string& prefix, const Json& p, const PartChildren& children) : MixerPart(prefix) {
+    hidden = param_int(p, "hidden");
+    heads = (int)param_int(p, "heads");
+    dv = (int)param_int(p, "v_head_dim");
+    state = (int)param_int(p, "state");
+    groups = p.has("groups") ? (int)param_int(p, "groups") : 1;
+    eps = (float)param_float(p, "eps");
+    form.groups = p.has("norm_groups") ? (int)param_int(p, "norm_groups") : 1;
+    form.silu = form.gate_first = true;
+    if (hidden <= 0 || heads <= 0 || dv <= 0 || state <= 0) throw ConfigError("mamba2: sizes must be positive");
+    if (groups < 1 || heads % groups) throw ConfigError("mamba2: " + std::to_string(heads) + " heads do not fit " + std::to_string(groups) + " groups");
+    if (dv > 256 || state > 256) throw ConfigError("mamba2: a state of " + std::to_string(state) + " x " + std::to_string(dv) + " a head is not served (up to 256 x 256)");
+    inner = (int64_t)heads * dv;
+    channels = inner + 2 * (int64_t)groups * state;
+    width = inner + channels + heads;
+    if (form.groups < 1 || inner % form.groups) throw ConfigError("mamba2: " + std::to_string(inner) + " channels do not fit " + std::to_string(form.groups) + " parts of a norm");
+    for (const auto& c : children)
+      if (c.first == "conv") conv = std::dynamic_pointer_cast<FilterPart>(c.second);
+    if (!conv) {
+      Json cp = Json::object(), segment = Json::array(), segments = Json::array();
+      segment.push(Json(join(prefix, "conv")));
+      segment.push(Json(channels));
+      segments.push(segment);
+      cp.set("taps", param_int(p, "conv"));
+      cp.set("segments", segments);
+      cp.set("bias", true);
+      cp.set("activation", "silu");
+      PartSpec spec;
+      spec.kind = "short_conv";
+      spec.params = cp;
+      conv = std::dynamic_pointer_cast<FilterPart>(build_part("filter", spec, join(prefix, "conv")));
+    }
+  }
+  const char* kind_name() const override { return "mamba2"; }
+  bool takes_lazy_norm() const override { return true; }
+  bool reads_through_ops() const override { return true; }
+  bool can_store() const override { return true; }
+  std::vector<std::shared_ptr<Part>> children() const override { return {conv}; }
+  std::vector<std::string> child_slots() const override { return {"conv"}; }
+  std::string name(const char* t) const { return join(prefix, t); }
+  std::vector<std::pair<std::string, TensorNeed>> tensors() const override {
+    TensorNeed in, o, bias, rate, skip, nw;
+    in.shape = {width, hidden};
+    o.shape = {hidden, inner};
+    bias.shape = rate.shape = skip.shape = {(int64_t)heads};
+    nw.shape = {inner};
+    bias.role = rate.role = skip.role = nw.role = TensorNeed::Vector;
+    bias.init = rate.init = "uniform";
+    bias.a = -4.0;      // step sizes of a few hundredths
+    bias.b = -1.0;
+    rate.a = 0.0;
+    rate.b = 2.5;
+    skip.a = nw.a = 1.0;
+    skip.b = nw.b = 0.1;
+    return {{name("in"), in}, {name("o"), o}, {name("dt_bias"), bias}, {name("A_log"), rate}, {name("D"), skip}, {name("norm"), nw}};
+  }
+  void load(WeightSource& src) override {
+    const auto t = tensors();
+    Tensor* const to[] = {&w_in, &w_o, &dt_bias, &a_log, &skip, &norm_w};
+    for (size_t i = 0; i < t.size(); ++i) *to[i] = src.fetch(t[i].first, t[i].second);
+  }
+  bool has_cache() const override { return true; }
+  CacheNeed cache_need() const override {
+    CacheNeed n;
+    n.kind = CacheNeed::State;
+    n.state_shape = {heads, (int64_t)state * dv};
+    return n;
+  }
+  void plan(StepPlan& plan) const override { plan_chunks(plan, "scan", DecayAttention::CHUNK, DecayAttention::CHUNK_FROM); }
+  void run(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
+    const int64_t M = h.t.shape[0], GN = (int64_t)groups * state;
+    Tensor proj = ctx.buf("mamba2.proj", DType::F32, {M, width});
+    ctx.ops.linear(h, w_in, proj, Ops::Store);
+    Tensor xbc = ctx.buf("mamba2.xbc", DType::F32, {M, channels});
+    conv->forward(ctx, proj.cols(inner, channels), xbc);
+    Tensor y = ctx.buf("mamba2.y", DType::F32, {M, inner});
+    Ops::LinearScan in;
+    in.rows = xbc;
+    in.cols.q = (int)(inner + GN);
+    in.cols.k = (int)inner;
+    in.cols.v = 0;
+    in.qk_heads = groups;
+    in.dt = proj;
+    in.dt_col = (int)(inner + channels);
+    in.dt_bias = dt_bias;
+    in.a_log = a_log;
+    in.skip = skip;
+    DecayAttention::scan(ctx, this, in, y, heads, state, dv);
+    Tensor a = ctx.buf("mamba2.gated", ctx.act_dtype, {M, inner});
+    ctx.ops.gated_group_norm(y, proj, 0, norm_w, eps, a, form);
+    ctx.ops.linear(a, w_o, out, epi, epi == Ops::Add);
+  }
+  void forward(StepContext& ctx, const Rows& h, const Tensor& x) override { run(ctx, h, x, Ops::Add); }
+  void forward_store(StepContext& ctx, const Rows& h, const Tensor& y) override { run(ctx, h, y, Ops::Store); }
+  std::vector<std::pair<std::string, Tensor>> held() const override {
+    return {{"w_in", w_in}, {"w_o", w_o}, {"dt_bias", dt_bias}, {"a_log", a_log}, {"skip", skip}, {"norm_w", norm_w}};
+  }
+  int64_t hidden = 0, inner = 0, channels = 0, width = 0;
+  int heads = 0, dv = 0, state = 0, groups = 1;
+  float eps = 1e-6f;
+  Ops::GroupNorm form;
+  std::shared_ptr<FilterPart> conv;
+  Tensor w_in, w_o, dt_bias, a_log, skip, norm_w;
 };
 
 // A minimal GRU: an element-wise recurrence over `width` channels whose gate and candidate read the current token only.
@@ -2803,10 +2996,10 @@ class MinGRU final : public MixerPart {
   Tensor w_in, b_z, b_x, w_o;
 };
 
-// A norm in front of every sublayer and another behind it: x += norm1b(mixer(norm1(x))); x += norm2b(ffn(norm2(x))).  The
-// sublayers write apart from the residual.  Where both norms at hand are plain RMS norms, the norm behind a sublayer, the
-// residual sum and the norm in front of the next sublayer are one kernel (Ops::norm_residual_next), which also adds what the
-// feed-forward left unsummed: within a layer directly, from layer to layer through a note in the step's context
+// A norm in front of every sublayer and another behind it: x += m norm1b(mixer(norm1(x))); x += m norm2b(ffn(norm2(x))), m a
+// number (`factor`, default 1).  The sublayers write apart from the residual.  Where both norms at hand are plain RMS or layer
+// norms, the norm behind a sublayer, the residual sum and the norm in front of the next sublayer are one kernel
+// (Ops::norm_residual_next), which also adds what a mixer of two branches or the feed-forward left unsummed: within a layer directly, from layer to layer through a note in the step's context
 // (`defer_write`: the layer's last write is left to the next layer of this kind).  A layer may have no feed-forward (then no
 // norm2 and norm2b either).
 const char* const SANDWICH_PENDING = "sandwich.pending";
@@ -2825,7 +3018,11 @@ class SandwichBlock final : public BlockPart {
     if (!norm1 || !norm1b || !mixer) throw ConfigError("block 'sandwich' needs norm1, mixer and norm1b parts (norm2, ffn and norm2b are optional)");
     if ((ffn != nullptr) != (norm2 != nullptr) || (ffn != nullptr) != (norm2b != nullptr))
       throw ConfigError("block 'sandwich': norm2, ffn and norm2b come together or not at all");
-    if (!norm1b->can_add() || (norm2b && !norm2b->can_add())) throw ConfigError("block 'sandwich': the norms behind its sublayers must be able to write into the residual");
+    Ops::RowNorm form;
+    if (p.has("factor")) factor = (float)param_float(p, "factor");
+    for (const auto& n : {norm1b, norm2b})
+      if (n && !n->row_form(form) && (!n->can_add() || factor != 1.f))
+        throw ConfigError("block 'sandwich': the norms behind its sublayers must be able to write into the residual");
     if (!mixer->can_store() || (ffn && !ffn->can_store()))
       throw ConfigError("block 'sandwich': its mixer and feed-forward must be able to write their output apart from the residual");
     defer_write = p.has("defer_write") && p.at("defer_write").as_bool();
@@ -2857,27 +3054,22 @@ class SandwichBlock final : public BlockPart {
     if (ffn) v.insert(v.end(), {"norm2", "ffn", "norm2b"});
     return v;
   }
-  // what a sublayer left for the residual: rows (their sum, a further branch) behind a norm of the given gain
+  // what a sublayer left for the residual: rows (their sum, a further branch) behind a norm
   struct Write {
     Ops::GatheredRows rows;
-    Tensor gain;
-    float eps = 0.f;
+    Ops::RowNorm norm;
   };
   // x += the write, then what `front` makes of x
-  static Rows write_read(StepContext& ctx, const Tensor& x, const Write& w, NormPart& front) {
-    Tensor gain;
-    float eps = 0.f;
-    if (front.rms_form(gain, eps)) {
+  Rows write_read(StepContext& ctx, const Tensor& x, const Write& w, NormPart& front) const {
+    Ops::RowNorm next;
+    if (front.row_form(next)) {
       Rows h;
       h.t = ctx.buf("norm.out", ctx.act_dtype, {x.shape[0], x.shape[1]});
-      ctx.ops.norm_residual_next(x, w.rows.t, w.rows.gather, w.rows.n_gather, w.rows.plus, w.rows.plus_gate, w.gain, w.eps, gain, eps, h.t);
+      ctx.ops.norm_residual_next(x, w.rows, w.norm, factor, next, h.t);
       return h;
     }
-    write(ctx, x, w);
+    ctx.ops.norm_residual_next(x, w.rows, w.norm, factor);
     return front.forward(ctx, x);
-  }
-  static void write(StepContext& ctx, const Tensor& x, const Write& w) {
-    ctx.ops.norm_residual_next(x, w.rows.t, w.rows.gather, w.rows.n_gather, w.rows.plus, w.rows.plus_gate, w.gain, w.eps);
   }
   void forward(StepContext& ctx, const Tensor& x) override {
     ctx.ops.flush();
@@ -2894,17 +3086,25 @@ class SandwichBlock final : public BlockPart {
       w.rows.n_gather = (int)note.numbers[0];
       w.rows.plus = note.tensors[2];
       w.rows.plus_gate = note.tensors[3];
-      w.gain = note.tensors[4];
-      w.eps = (float)note.numbers[1];
+      w.norm.gain = note.tensors[4];
+      w.norm.eps = (float)note.numbers[1];
+      w.norm.centered = note.numbers[2] != 0;
+      w.rows.y_scale = (float)note.numbers[3];
+      w.rows.plus_scale = (float)note.numbers[4];
       h = write_read(ctx, x, w, *norm1);
     } else {
       h = norm1->forward(ctx, x, nullptr, 0, mixer->takes_lazy_norm() && norm1->can_be_lazy());
     }
     if (!mixer->reads_through_ops()) ctx.ops.flush();
-    mixer->forward_store(ctx, h, y);
     Write w;
+    bool fusable = norm1b->row_form(w.norm);
     w.rows.t = y;
-    bool fusable = norm1b->rms_form(w.gain, w.eps);
+    if (fusable && mixer->leaves_pair()) {      // two branches: added by the kernel that norms their sum
+      w.rows.plus = ctx.buf("sandwich.y2", DType::F32, {M, x.shape[1]});
+      mixer->forward_pair(ctx, h, y, w.rows.plus, w.rows.y_scale, w.rows.plus_scale);
+    } else {
+      mixer->forward_store(ctx, h, y);
+    }
     if (ffn) {
       if (fusable) {
         h = write_read(ctx, x, w, *norm2);
@@ -2913,7 +3113,8 @@ class SandwichBlock final : public BlockPart {
         h = norm2->forward(ctx, x);
       }
       if (!ffn->reads_through_ops()) ctx.ops.flush();
-      fusable = norm2b->rms_form(w.gain, w.eps);
+      w = Write();
+      fusable = norm2b->row_form(w.norm);
       ffn->forward_rows(ctx, h, y, w.rows, fusable);
     }
     if (!fusable) {
@@ -2921,15 +3122,18 @@ class SandwichBlock final : public BlockPart {
     } else if (defer_write) {
       Tensor list;
       if (w.rows.gather) list = Tensor((void*)w.rows.gather, DType::I32, {M, (int64_t)w.rows.n_gather});
-      ctx.notes[SANDWICH_PENDING] = StepContext::Note{{w.rows.t, list, w.rows.plus, w.rows.plus_gate, w.gain}, {(double)w.rows.n_gather, (double)w.eps}};
+      ctx.notes[SANDWICH_PENDING] = StepContext::Note{{w.rows.t, list, w.rows.plus, w.rows.plus_gate, w.norm.gain},
+                                                      {(double)w.rows.n_gather, (double)w.norm.eps, w.norm.centered ? 1.0 : 0.0,
+                                                       (double)w.rows.y_scale, (double)w.rows.plus_scale}};
     } else {
-      write(ctx, x, w);
+      ctx.ops.norm_residual_next(x, w.rows, w.norm, factor);
     }
   }
   std::shared_ptr<NormPart> norm1, norm1b, norm2, norm2b;
   std::shared_ptr<MixerPart> mixer;
   std::shared_ptr<FeedForwardPart> ffn;
   bool defer_write = false;
+  float factor = 1.f;
   std::vector<std::string> spare;
   int64_t dim = 0;
 };
@@ -3003,8 +3207,11 @@ void register_builtin_parts() {
   register_part("block", "hyper",
                 [](const std::string& prefix, const Json& p, const PartChildren& c) { return std::make_shared<HyperBlock>(prefix, p, c); },
                 {{"norm1", "norm"}, {"mixer", "mixer"}, {"norm2", "norm?"}, {"ffn", "ffn?"}});
-  register_part("mixer", "decay_attention", [](const std::string& prefix, const Json& p, const PartChildren&) {
-    return std::make_shared<DecayAttention>(prefix, p);
+  register_part("mixer", "decay_attention", [](const std::string& prefix, const Json& p, const PartChildren& c) {
+    return std::make_shared<DecayAttention>(prefix, p, c);
+  });
+  register_part("mixer", "mamba2", [](const std::string& prefix, const Json& p, const PartChildren& c) {
+    return std::make_shared<Mamba2>(prefix, p, c);
   });
   register_part("mixer", "mingru", [](const std::string& prefix, const Json& p, const PartChildren&) {
     return std::make_shared<MinGRU>(prefix, p);
