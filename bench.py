@@ -46,6 +46,11 @@ positions), `mingru` (an element-wise recurrence as wide as the model's heads to
 recurrence, ...); `--ffn dense` (squared relu, sized to do the arithmetic of the model's gated feed-forward) or `moe`
 (`--experts` of which a token takes `--top`, and a shared one behind a gate, together of the same arithmetic).
 
+`--design ruzolorn` does the same for a Ruzolorn decoder (layer norms on either side of every sublayer): as mixers `--mixers parallel`
+(window attention with the model's heads, values of `--value-size`, beside a Mamba-2 layer of twice the model's width in heads of 64
+with a state of 128), `retention` (as many heads as the model has kv heads, 128 x 128 each) or `alternate` (retention, parallel,
+...); experts as for Lupolorn, gated, `--identity` of the router's rows standing for the input itself.
+
 `--design nazorax` does the same for a Nazorax decoder: parallel layers behind a Dynamic
 Tanh, as mixers `--mixers attention` (biased, rotated attention with the model's heads
 under a window of `--window` positions), `latent` (latent attention with the model's
@@ -167,6 +172,21 @@ def lupolorn_config(base, mixers, ffn, experts, top, window):
                 layers=[kinds[i % len(kinds)] for i in range(base["num_hidden_layers"])])
 
 
+def ruzolorn_config(base, mixers, experts, top, identity, window, value_size=0):
+    """A Ruzolorn config.json with the layer widths of the Qwen3 configuration `base`."""
+    H, F, hd, kv = base["hidden_size"], base["intermediate_size"], base["head_dim"], base["num_key_value_heads"]
+    part = max(64, F // (top + 1) // 64 * 64)            # top experts and the shared one do what the gated dense one of F does
+    mlp = dict(kind="moe", expert=dict(ff=part), router=dict(experts=experts, top=top, identity=identity), shared=dict(ff=part))
+    left = dict(heads=base["num_attention_heads"], kv_heads=kv, dim=hd, vdim=value_size or hd, scale=hd ** -0.5, mask=dict(size=window))
+    right = dict(heads=2 * H // 64, vdim=64, state=128, groups=1, conv=4, norm_groups=1)
+    parallel = dict(type="parallel", mlp=mlp, mixer=dict(left=left, right=right, left_scale=0.7, right_scale=0.7))
+    decay = [1.0 - 2.0 ** (-5.0 - 3.0 * j / max(1, kv - 1)) for j in range(kv)]
+    retention = dict(type="retention", mlp=mlp, mixer=dict(heads=kv, dim=hd, vdim=hd, decay=decay, rot=dict(base=1000000.0, dims=hd)))
+    kinds = {"parallel": [parallel], "retention": [retention], "alternate": [retention, parallel]}[mixers]
+    return dict(architecture="Ruzolorn", width=H, vocab=base["vocab_size"], norm=dict(eps=1e-6), embedding=dict(scale=4.0), residual_mult=0.5,
+                layers=[kinds[i % len(kinds)] for i in range(base["num_hidden_layers"])])
+
+
 MAX_SEQ = 4096            # context length a request may reach (more if --context asks for it)
 PAGE = 16
 PEAK_HBM = 8.0e12         # bytes/s, MI355X
@@ -208,7 +228,7 @@ def model_numbers(model):
             else:
                 layer_params += n
         if experts:
-            routed.append((experts, part.params["experts"], part.params["top"]))
+            routed.append((experts, part.params["experts"] + part.params.get("identity", 0), part.params["top"]))      # (rows of the router)
         need = part.cache_need()
         if need is not None and hasattr(need, "kv_heads") and "heads" in getattr(part, "params", {}):
             v = getattr(need, "v_dim", None) or need.head_dim
@@ -312,8 +332,8 @@ def decode_floor(engine, rids, last, nums, context, batch):
         if c["name"].startswith("moe_experts") and nums["routed"]:
             n_all, e, top = nums["routed"][0]
             per_call = int(n_all * (1.0 - (1.0 - top / e) ** batch) * 2)      # the experts the step's tokens chose
-        if c["name"].startswith("mlstm_scan") and nums["cells"]:
-            per_call = 2 * 4 * np_prod(nums["cells"][0]) * batch      # the requests' state, read and written
+        if c["name"].startswith(("mlstm_scan", "linear_scan")) and nums["cells"]:
+            per_call = 2 * 4 * max(np_prod(s) for s in nums["cells"]) * batch      # the requests' state, read and written
         sizes += [per_call] * c["calls"]
         if c["name"].startswith("attention") and "runs" in c["name"]:
             sizes += [4096] * c["calls"]              # the kernel that merges the runs of a context
@@ -487,18 +507,19 @@ def main() -> int:
     ap.add_argument("--warmup", type=int, default=16)
     ap.add_argument("--model", choices=sorted(MODELS), default="0.6b", help="whose layer sizes the model has")
     ap.add_argument("--layers", type=int, default=None, help="run fewer layers than the configuration has")
-    ap.add_argument("--design", choices=["qwen3", "miterax", "mumasun", "nazorax", "dubozen", "lupolorn"], default="qwen3",
-                    help="miterax / mumasun / nazorax / dubozen / lupolorn: a decoder of that design with the layer widths of --model instead (see --mixers; --experts, --top, --mask-size; --ffn, --window, --streams)")
-    ap.add_argument("--experts", type=int, default=8, help="--design mumasun / nazorax / dubozen / lupolorn: experts per layer")
-    ap.add_argument("--top", type=int, default=2, help="--design mumasun / nazorax / dubozen / lupolorn: experts a token takes")
+    ap.add_argument("--design", choices=["qwen3", "miterax", "mumasun", "nazorax", "dubozen", "lupolorn", "ruzolorn"], default="qwen3",
+                    help="miterax / mumasun / nazorax / dubozen / lupolorn / ruzolorn: a decoder of that design with the layer widths of --model instead (see --mixers; --experts, --top, --mask-size; --ffn, --window, --streams)")
+    ap.add_argument("--experts", type=int, default=8, help="--design mumasun / nazorax / dubozen / lupolorn / ruzolorn: experts per layer")
+    ap.add_argument("--top", type=int, default=2, help="--design mumasun / nazorax / dubozen / lupolorn / ruzolorn: experts a token takes")
     ap.add_argument("--ffn", choices=["dense", "moe"], default="moe", help="--design nazorax / dubozen / lupolorn: the feed-forward of its layers")
-    ap.add_argument("--value-size", type=int, default=0, help="--design dubozen: the value size of its attention layers (0: the head size)")
+    ap.add_argument("--value-size", type=int, default=0, help="--design dubozen / ruzolorn: the value size of its attention layers (0: the head size)")
+    ap.add_argument("--identity", type=int, default=2, help="--design ruzolorn: rows of the router that stand for the input itself")
     ap.add_argument("--streams", type=int, default=2, help="--design dubozen: copies of the residual (0: one plain residual)")
-    ap.add_argument("--window", type=int, default=1024, help="--design nazorax / lupolorn: positions an attention (a latent attention) layer's window keeps")
+    ap.add_argument("--window", type=int, default=1024, help="--design nazorax / lupolorn / ruzolorn: positions an attention (a latent attention) layer's window keeps")
     ap.add_argument("--mask-size", type=int, default=4096, help="--design mumasun: positions of a block of visible keys")
-    ap.add_argument("--mixers", choices=["attention", "mlstm", "latent", "parallel", "mingru", "alternate"], default="alternate",
+    ap.add_argument("--mixers", choices=["attention", "mlstm", "latent", "parallel", "mingru", "retention", "alternate"], default="alternate",
                     help="--design miterax (attention, mlstm, alternate) / nazorax (attention, latent, alternate) / dubozen (attention, parallel, "
-                         "alternate) / lupolorn (attention, latent, mingru, alternate): the mixer of its layers")
+                         "alternate) / lupolorn (attention, latent, mingru, alternate) / ruzolorn (parallel, retention, alternate): the mixer of its layers")
     ap.add_argument("--batch", type=int, default=8)
     ap.add_argument("--context", type=int, default=2048, help="cached tokens each decoding request holds")
     ap.add_argument("--prefill-tokens", type=int, default=2048)
@@ -536,7 +557,7 @@ def main() -> int:
         cfg = mumasun_config(cfg, args.experts, args.top, args.mask_size)
         model_name = f"Mumasun ({args.top} of {args.experts} experts, blocks of {args.mask_size}) at {NAMES[args.model]} sizes"
     if args.design == "nazorax":
-        if args.mixers in ("mlstm", "mingru"):
+        if args.mixers in ("mlstm", "mingru", "parallel", "retention"):
             ap.error("--design nazorax has the mixers attention, latent and alternate")
         cfg = nazorax_config(cfg, args.mixers, args.ffn, args.experts, args.top, args.window)
         what = "dense feed-forward" if args.ffn == "dense" else f"{args.top} of {args.experts} experts and a shared one"
@@ -544,7 +565,7 @@ def main() -> int:
     elif args.mixers == "latent" and args.design != "lupolorn":
         ap.error("--mixers latent goes with --design nazorax and lupolorn")
     if args.design == "lupolorn":
-        if args.mixers in ("mlstm", "parallel"):
+        if args.mixers in ("mlstm", "parallel", "retention"):
             ap.error("--design lupolorn has the mixers attention, latent, mingru and alternate")
         cfg = lupolorn_config(cfg, args.mixers, args.ffn, args.experts, args.top, args.window)
         what = "dense feed-forward" if args.ffn == "dense" else f"{args.top} of {args.experts} experts and a shared one"
@@ -552,13 +573,21 @@ def main() -> int:
     elif args.mixers == "mingru":
         ap.error("--mixers mingru goes with --design lupolorn")
     if args.design == "dubozen":
-        if args.mixers in ("mlstm", "latent", "mingru"):
+        if args.mixers in ("mlstm", "latent", "mingru", "retention"):
             ap.error("--design dubozen has the mixers attention, parallel and alternate")
         cfg = dubozen_config(cfg, args.mixers, args.ffn, args.experts, args.top, args.streams, args.value_size)
         what = "dense feed-forward" if args.ffn == "dense" else f"{args.top} of {args.experts} experts"
         model_name = f"Dubozen ({args.mixers} mixers, {what}, {args.streams or 'no'} streams) at {NAMES[args.model]} sizes"
-    elif args.mixers == "parallel":
-        ap.error("--mixers parallel goes with --design dubozen")
+    elif args.mixers == "parallel" and args.design != "ruzolorn":
+        ap.error("--mixers parallel goes with --design dubozen and ruzolorn")
+    if args.design == "ruzolorn":
+        if args.mixers not in ("parallel", "retention", "alternate"):
+            ap.error("--design ruzolorn has the mixers parallel, retention and alternate")
+        cfg = ruzolorn_config(cfg, args.mixers, args.experts, args.top, args.identity, args.window, args.value_size)
+        model_name = (f"Ruzolorn ({args.mixers} mixers, {args.top} of {args.experts} experts and {args.identity} identities and a shared one) at "
+                      f"{NAMES[args.model]} sizes")
+    elif args.mixers == "retention":
+        ap.error("--mixers retention goes with --design ruzolorn")
     rng = np.random.default_rng(0)
     context, prefill_tokens = args.context, args.prefill_tokens
     max_seq = max(MAX_SEQ, context + args.warmup + args.steps + 64, prefill_tokens, args.cached + args.portion)
