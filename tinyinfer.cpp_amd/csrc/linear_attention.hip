@@ -26,31 +26,38 @@ TI_ERROR_API
 __device__ __forceinline__ float la_silu(float z) { return z * __frcp_rn(1.0f + __expf(-z)); }
 __device__ __forceinline__ float la_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 
-// entry i of a query or key head of row m at position p, as it enters the recurrence (`head`: the head's columns of the row)
-__device__ __forceinline__ float scan_entry(const ti_scan_inputs& in, const float* __restrict__ head, int i, int p) {
-  const float x = head[i];
-  if (in.act) return la_silu(x);
-  if (i >= in.rot_dims) return x;
-  const int half = in.rot_dims / 2, f = i < half ? i : i - half;
-  const float other = head[i < half ? i + half : i - half];
-  float c, s;
+#define SCAN_NT 256         // threads of a workgroup
+#define SCAN_TB 16          // tokens staged together
+// how q, k, v and the decays come about
+#define SCAN_SILU 0         // silu on all three, fixed decays
+#define SCAN_ROTATED 1      // q and k rotated, or as they are; fixed decays
+#define SCAN_SELECTIVE 2    // as they are; step sizes
+__device__ __forceinline__ void scan_angle(const ti_scan_inputs& in, int p, int half, int f, float* c, float* s) {
   if (in.rope_table && p < in.table_len) {
-    c = in.rope_table[((size_t)p * half + f) * 2];
-    s = in.rope_table[((size_t)p * half + f) * 2 + 1];
+    *c = in.rope_table[((size_t)p * half + f) * 2];
+    *s = in.rope_table[((size_t)p * half + f) * 2 + 1];
   } else {
     const float a = (float)p * in.inv_freq[f];
-    c = cosf(a);
-    s = sinf(a);
+    *c = cosf(a);
+    *s = sinf(a);
   }
-  return i < half ? x * c - other * s : x * c + other * s;
 }
-__device__ __forceinline__ float scan_value(const ti_scan_inputs& in, float x) { return in.act ? la_silu(x) : x; }
+// entry i of a query or key head of row m at position p, as it enters the recurrence (`head`: the head's columns of the row)
+template <int FORM> __device__ __forceinline__ float scan_entry(const ti_scan_inputs& in, const float* __restrict__ head, int i, int p) {
+  const float x = head[i];
+  if (FORM == SCAN_SILU) return la_silu(x);
+  if (FORM == SCAN_SELECTIVE || i >= in.rot_dims) return x;
+  const int half = in.rot_dims / 2;
+  float c, s;
+  scan_angle(in, p, half, i < half ? i : i - half, &c, &s);
+  return i < half ? x * c - head[i + half] * s : x * c + head[i - half] * s;
+}
 // the step size of row m, head h
 __device__ __forceinline__ float scan_dt(const ti_scan_inputs& in, int m, int h) {
   return la_softplus(in.dt[(size_t)m * in.dt_ld + h] + in.dt_bias[h]);
 }
 
-template <int NT, int RPT, int TB>
+template <int FORM, int NT, int RPT, int TB>
 __global__ void __launch_bounds__(NT)
 scan_tokens_kernel(const ti_scan_inputs in, float* __restrict__ state, long slot_stride, const int* __restrict__ entry_meta,
                    float* __restrict__ o, int heads, int dk, int dv, int dvs, int dvp) {
@@ -70,7 +77,7 @@ scan_tokens_kernel(const ti_scan_inputs in, float* __restrict__ state, long slot
   float* s_a = s_part + TB * NT;                  // [TB] the tokens' decays
   float* s_d = s_a + TB;                          // [TB] ... and step sizes
   float* S = state + (size_t)slot * slot_stride + (size_t)h * dk * dv;
-  const float fixed = in.decay ? in.decay[h] : 0.f, rate = in.decay ? 0.f : expf(in.a_log[h]);
+  const float fixed = FORM == SCAN_SELECTIVE ? 0.f : in.decay[h], rate = FORM == SCAN_SELECTIVE ? expf(in.a_log[h]) : 0.f;
   const float skip = in.skip ? in.skip[h] : 0.f;
   float reg[RPT];
 #pragma unroll
@@ -82,15 +89,22 @@ scan_tokens_kernel(const ti_scan_inputs in, float* __restrict__ state, long slot
     for (int x = threadIdx.x; x < nt * width; x += NT) {
       const int tt = x / width, c = x % width, m = row0 + t0 + tt;
       const float* row = in.proj + (size_t)m * in.ld;
-      const int p = in.rot_dims ? in.pos[m] : 0;
-      if (c < dkp) s_q[tt * dkp + c] = c < dk ? scan_entry(in, row + in.off_q + hq * dk, c, p) : 0.f;
-      else if (c < 2 * dkp) s_k[tt * dkp + c - dkp] = c - dkp < dk ? scan_entry(in, row + in.off_k + hq * dk, c - dkp, p) * in.k_scale : 0.f;
-      else s_v[tt * dvs + c - 2 * dkp] = col0 + c - 2 * dkp < dv ? scan_value(in, row[in.off_v + h * dv + col0 + c - 2 * dkp]) : 0.f;
+      const int p = FORM == SCAN_ROTATED && in.rot_dims ? in.pos[m] : 0;
+      if (c < 2 * dkp) {
+        const bool is_q = c < dkp;
+        const int i = is_q ? c : c - dkp;
+        const float e = i < dk ? scan_entry<FORM>(in, row + (is_q ? in.off_q : in.off_k) + hq * dk, i, p) : 0.f;
+        (is_q ? s_q : s_k)[tt * dkp + i] = is_q ? e : e * in.k_scale;
+      } else {
+        const int i = c - 2 * dkp;
+        const float e = col0 + i < dv ? row[in.off_v + h * dv + col0 + i] : 0.f;
+        s_v[tt * dvs + i] = FORM == SCAN_SILU ? la_silu(e) : e;
+      }
     }
     if (threadIdx.x < nt) {
-      const float d = in.decay ? 1.f : scan_dt(in, row0 + t0 + threadIdx.x, h);
+      const float d = FORM == SCAN_SELECTIVE ? scan_dt(in, row0 + t0 + threadIdx.x, h) : 1.f;
       s_d[threadIdx.x] = d;
-      s_a[threadIdx.x] = in.decay ? fixed : expf(-rate * d);
+      s_a[threadIdx.x] = FORM == SCAN_SELECTIVE ? expf(-rate * d) : fixed;
     }
     __syncthreads();
     for (int tt = 0; tt < nt; ++tt) {
@@ -148,8 +162,8 @@ struct ChunkWeights {
   float pw[SC_N + 1], d[SC_N];
   double L[SC_N];
 };
-__device__ __forceinline__ void chunk_weights(const ti_scan_inputs& in, ChunkWeights& w, int row0, int n, int h) {
-  if (in.decay) {
+template <bool SELECTIVE> __device__ __forceinline__ void chunk_weights(const ti_scan_inputs& in, ChunkWeights& w, int row0, int n, int h) {
+  if (!SELECTIVE) {
     if (threadIdx.x <= SC_N) {
       double p = 1.0;
       const double a = (double)in.decay[h];
@@ -172,40 +186,91 @@ __device__ __forceinline__ void chunk_weights(const ti_scan_inputs& in, ChunkWei
   }
 }
 // e^(L_t - L_s) for s <= t; e^(L_t) with s = -1
-__device__ __forceinline__ float chunk_factor(const ti_scan_inputs& in, const ChunkWeights& w, int t, int s) {
-  if (in.decay) return w.pw[t - s];
+template <bool SELECTIVE> __device__ __forceinline__ float chunk_factor(const ChunkWeights& w, int t, int s) {
+  if (!SELECTIVE) return w.pw[t - s];
   return expf((float)(s < 0 ? w.L[t] : w.L[t] - w.L[s]));
 }
+
+// A block of 64 rows x 64 columns of 32-bit numbers on its way into LDS: a thread asks for four pieces of four neighbouring columns
+// (rows threadIdx.x / 16 + 16 k), all in flight together, and puts them down later.  Rows from n_rows and columns from n_cols on
+// are zeros.  VEC: the pieces are aligned to 16 bytes and n_cols is a multiple of four.
+template <bool VEC> struct Block64 {
+  float4 v[4];
+  __device__ __forceinline__ void load(const float* __restrict__ src, size_t ld, int n_rows, int n_cols) {
+    const int c = (threadIdx.x & 15) * 4;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const int r = (threadIdx.x >> 4) + 16 * k;
+      const float* p = src + (size_t)min(r, n_rows - 1) * ld;      // (a row that is not there: the last one's numbers, dropped below)
+      float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (VEC) {
+        x = *reinterpret_cast<const float4*>(p + min(c, n_cols - 4));
+      } else {
+        x.x = p[min(c, n_cols - 1)];
+        x.y = p[min(c + 1, n_cols - 1)];
+        x.z = p[min(c + 2, n_cols - 1)];
+        x.w = p[min(c + 3, n_cols - 1)];
+      }
+      v[k] = x;
+    }
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const bool row = (int)(threadIdx.x >> 4) + 16 * k < n_rows;
+      v[k].x = row && c < n_cols ? v[k].x : 0.f;
+      v[k].y = row && c + 1 < n_cols ? v[k].y : 0.f;
+      v[k].z = row && c + 2 < n_cols ? v[k].z : 0.f;
+      v[k].w = row && c + 3 < n_cols ? v[k].w : 0.f;
+    }
+  }
+  __device__ __forceinline__ void silu() {      // (of zero: zero)
+#pragma unroll
+    for (int k = 0; k < 4; ++k) v[k] = make_float4(la_silu(v[k].x), la_silu(v[k].y), la_silu(v[k].z), la_silu(v[k].w));
+  }
+  template <class F> __device__ __forceinline__ void scale_rows(F f) {
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const float s = f((int)(threadIdx.x >> 4) + 16 * k);
+      v[k] = make_float4(v[k].x * s, v[k].y * s, v[k].z * s, v[k].w * s);
+    }
+  }
+  template <int ROW> __device__ __forceinline__ void put(float (*dst)[ROW]) const {
+#pragma unroll
+    for (int k = 0; k < 4; ++k) *reinterpret_cast<float4*>(&dst[(threadIdx.x >> 4) + 16 * k][(threadIdx.x & 15) * 4]) = v[k];
+  }
+};
 
 // scratch [chunk][head][dk][dv] = what the chunk adds to an empty state, chunk_decay [chunk][head] = e^(L_n).  A workgroup per
 // (chunk, head, block of 64 x 64 of the state); its four wavefronts two by two, each 32 x 32: the sum over the chunk's tokens as
 // matrix products k^T v.
+template <int FORM, bool VEC>
 __global__ void __launch_bounds__(256)
 scan_chunk_states_kernel(const ti_scan_inputs in, const int* __restrict__ chunks, float* __restrict__ scratch, float* __restrict__ chunk_decay,
                          int heads, int dk, int dv, int col_blocks) {
-  __shared__ float s_k[SC_N][SC_COL], s_v[SC_N][SC_COL];
+  __shared__ __attribute__((aligned(16))) float s_k[SC_N][SC_COL], s_v[SC_N][SC_COL];
   __shared__ ChunkWeights w;
+  constexpr bool SEL = FORM == SCAN_SELECTIVE;
   const int h = blockIdx.y, hq = h / (heads / in.qk_heads);
   const int row0 = chunks[4 * blockIdx.x + 1], n = chunks[4 * blockIdx.x + 2];
   const int i0 = blockIdx.z / col_blocks * SC_N, j0 = blockIdx.z % col_blocks * SC_N;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, quad = lane >> 4;
-  const int c = threadIdx.x & 63;
-  chunk_weights(in, w, row0, n, h);
+  const float* rows = in.proj + (size_t)row0 * in.ld;
+  Block64<VEC> k, v;
+  k.load(rows + in.off_k + hq * dk + i0, in.ld, n, dk - i0);
+  v.load(rows + in.off_v + h * dv + j0, in.ld, n, dv - j0);
+  chunk_weights<SEL>(in, w, row0, n, h);
   __syncthreads();
-#pragma unroll
-  for (int k = 0; k < SC_N / 4; ++k) {
-    const int t = wave + 4 * k, m = row0 + t;
-    float kv = 0.f, vv = 0.f;
-    if (t < n) {
-      const float* row = in.proj + (size_t)m * in.ld;
-      const float f = in.decay ? chunk_factor(in, w, n - 1, t) : chunk_factor(in, w, n - 1, t) * w.d[t];
-      if (i0 + c < dk) kv = scan_entry(in, row + in.off_k + hq * dk, i0 + c, in.rot_dims ? in.pos[m] : 0) * in.k_scale * f;
-      if (j0 + c < dv) vv = scan_value(in, row[in.off_v + h * dv + j0 + c]);
-    }
-    s_k[t][c] = kv;
-    s_v[t][c] = vv;
+  if (FORM == SCAN_SILU) {
+    k.silu();
+    v.silu();
   }
-  if (blockIdx.z == 0 && threadIdx.x == 0) chunk_decay[(size_t)blockIdx.x * heads + h] = chunk_factor(in, w, n - 1, -1);
+  k.scale_rows([&](int t) {
+    if (t >= n) return 0.f;
+    const float f = chunk_factor<SEL>(w, n - 1, t) * in.k_scale;
+    return SEL ? f * w.d[t] : f;
+  });
+  k.put(s_k);
+  v.put(s_v);
+  if (blockIdx.z == 0 && threadIdx.x == 0) chunk_decay[(size_t)blockIdx.x * heads + h] = chunk_factor<SEL>(w, n - 1, -1);
   __syncthreads();
   const int wy = (wave >> 1) * 32, wx = (wave & 1) * 32;
   sc_float4 acc[2][2] = {};
@@ -265,41 +330,49 @@ __global__ void scan_carry_kernel(float* __restrict__ scratch, const float* __re
 }
 
 // The outputs of a chunk from the state it starts from: a workgroup per (chunk, head, 64 columns of the state), its four
-// wavefronts two by two over 64 tokens x 64 columns.  q . k and q . S over blocks of 64 of the state's rows, then the weighted
-// and masked q . k against the values.
+// wavefronts two by two over 64 tokens x 64 columns.  q . k and q . S over blocks of 64 of the state's rows (the next block is on
+// its way from memory meanwhile), then the weighted and masked q . k against the values.
+template <int FORM, bool VEC>
 __global__ void __launch_bounds__(256)
 scan_chunk_outputs_kernel(const ti_scan_inputs in, const int* __restrict__ chunks, const float* __restrict__ scratch, float* __restrict__ o,
                           int heads, int dk, int dv) {
-  __shared__ __attribute__((aligned(16))) float s_q[SC_N][SC_ROW], s_k[SC_N][SC_ROW];
-  __shared__ float s_s[SC_N][SC_COL];
+  __shared__ __attribute__((aligned(16))) float s_q[SC_N][SC_ROW], s_k[SC_N][SC_ROW], s_s[SC_N][SC_COL];
   __shared__ ChunkWeights w;
+  constexpr bool SEL = FORM == SCAN_SELECTIVE;
   const int h = blockIdx.y, hq = h / (heads / in.qk_heads);
   const int row0 = chunks[4 * blockIdx.x + 1], n = chunks[4 * blockIdx.x + 2];
   const int j0 = blockIdx.z * SC_N;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, quad = lane >> 4;
-  const int c = threadIdx.x & 63;
   const int wy = (wave >> 1) * 32, wx = (wave & 1) * 32;
-  const float* S = scratch + ((size_t)blockIdx.x * heads + h) * dk * dv;
   const bool masked = wy + 31 < wx;      // none of this wavefront's (token, earlier token) pairs is in order
-  chunk_weights(in, w, row0, n, h);
+  const float* S = scratch + ((size_t)blockIdx.x * heads + h) * dk * dv + j0;
+  const float* rows = in.proj + (size_t)row0 * in.ld;
+  const float* row_q = rows + in.off_q + hq * dk;
+  const float* row_k = rows + in.off_k + hq * dk;
+  Block64<VEC> q, k, v;      // v: the state's rows, behind the last block the values
+  q.load(row_q, in.ld, n, dk);
+  k.load(row_k, in.ld, n, dk);
+  v.load(S, dv, dk, dv - j0);
+  chunk_weights<SEL>(in, w, row0, n, h);
   sc_float4 P[2][2] = {}, O[2][2] = {};
   for (int i0 = 0; i0 < dk; i0 += SC_N) {
     __syncthreads();
-#pragma unroll
-    for (int k = 0; k < SC_N / 4; ++k) {
-      const int t = wave + 4 * k, m = row0 + t;
-      float qv = 0.f, kv = 0.f;
-      if (t < n && i0 + c < dk) {
-        const float* row = in.proj + (size_t)m * in.ld;
-        const int p = in.rot_dims ? in.pos[m] : 0;
-        qv = scan_entry(in, row + in.off_q + hq * dk, i0 + c, p);
-        kv = scan_entry(in, row + in.off_k + hq * dk, i0 + c, p) * in.k_scale;
-      }
-      s_q[t][c] = qv;
-      s_k[t][c] = kv;
-      s_s[t][c] = (i0 + t < dk && j0 + c < dv) ? S[(size_t)(i0 + t) * dv + j0 + c] : 0.f;
+    if (FORM == SCAN_SILU) {
+      q.silu();
+      k.silu();
     }
+    q.put(s_q);
+    k.put(s_k);
+    v.put(s_s);
     __syncthreads();
+    const int next = i0 + SC_N;
+    if (next < dk) {
+      q.load(row_q + next, in.ld, n, dk - next);
+      k.load(row_k + next, in.ld, n, dk - next);
+      v.load(S + (size_t)next * dv, dv, dk - next, dv - j0);
+    } else {
+      v.load(rows + in.off_v + h * dv + j0, in.ld, n, dv - j0);
+    }
 #pragma unroll
     for (int i = 0; i < SC_N; i += 16) {
       // lane group g holds the rows i + 4 g .. i + 4 g + 3 of the sum: product e takes entry e of every group
@@ -307,19 +380,19 @@ scan_chunk_outputs_kernel(const ti_scan_inputs in, const int* __restrict__ chunk
 #pragma unroll
       for (int x = 0; x < 2; ++x) {
         a[x] = *reinterpret_cast<const float4*>(&s_q[wy + 16 * x + r16][i + 4 * quad]);
-        if (!masked) b[x] = *reinterpret_cast<const float4*>(&s_k[wx + 16 * x + r16][i + 4 * quad]);
+        b[x] = *reinterpret_cast<const float4*>(&s_k[wx + 16 * x + r16][i + 4 * quad]);
       }
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        float v[2];
+        float sv[2];
 #pragma unroll
-        for (int y = 0; y < 2; ++y) v[y] = s_s[i + 4 * quad + e][wx + 16 * y + r16];
+        for (int y = 0; y < 2; ++y) sv[y] = s_s[i + 4 * quad + e][wx + 16 * y + r16];
 #pragma unroll
         for (int x = 0; x < 2; ++x) {
           const float ax = e == 0 ? a[x].x : e == 1 ? a[x].y : e == 2 ? a[x].z : a[x].w;
 #pragma unroll
           for (int y = 0; y < 2; ++y) {
-            O[x][y] = __builtin_amdgcn_mfma_f32_16x16x4f32(ax, v[y], O[x][y], 0, 0, 0);
+            O[x][y] = __builtin_amdgcn_mfma_f32_16x16x4f32(ax, sv[y], O[x][y], 0, 0, 0);
             if (!masked) {
               const float by = e == 0 ? b[y].x : e == 1 ? b[y].y : e == 2 ? b[y].z : b[y].w;
               P[x][y] = __builtin_amdgcn_mfma_f32_16x16x4f32(ax, by, P[x][y], 0, 0, 0);
@@ -336,21 +409,18 @@ scan_chunk_outputs_kernel(const ti_scan_inputs in, const int* __restrict__ chunk
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int t = wy + 16 * x + 4 * quad + r;
-      const float f = t < n ? chunk_factor(in, w, t, -1) : 0.f;
+      const float f = t < n ? chunk_factor<SEL>(w, t, -1) : 0.f;
 #pragma unroll
       for (int y = 0; y < 2; ++y) {
         O[x][y][r] *= f;
         const int s = wx + 16 * y + r16;
         float p = 0.f;
-        if (s <= t && t < n) p = P[x][y][r] * chunk_factor(in, w, t, s) * (in.decay ? 1.f : w.d[s]);
+        if (s <= t && t < n) p = P[x][y][r] * chunk_factor<SEL>(w, t, s) * in.k_scale * (SEL ? w.d[s] : 1.f);
         s_q[t][s] = p;
       }
     }
-#pragma unroll
-  for (int k = 0; k < SC_N / 4; ++k) {
-    const int t = wave + 4 * k;
-    s_s[t][c] = (t < n && j0 + c < dv) ? scan_value(in, in.proj[(size_t)(row0 + t) * in.ld + in.off_v + h * dv + j0 + c]) : 0.f;
-  }
+  if (FORM == SCAN_SILU) v.silu();
+  v.put(s_s);
   __syncthreads();
 #pragma unroll
   for (int i = 0; i < SC_N; i += 16) {
@@ -360,14 +430,14 @@ scan_chunk_outputs_kernel(const ti_scan_inputs in, const int* __restrict__ chunk
     for (int x = 0; x < 2; ++x) a[x] = *reinterpret_cast<const float4*>(&s_q[wy + 16 * x + r16][i + 4 * quad]);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      float v[2];
+      float sv[2];
 #pragma unroll
-      for (int y = 0; y < 2; ++y) v[y] = s_s[i + 4 * quad + e][wx + 16 * y + r16];
+      for (int y = 0; y < 2; ++y) sv[y] = s_s[i + 4 * quad + e][wx + 16 * y + r16];
 #pragma unroll
       for (int x = 0; x < 2; ++x) {
         const float ax = e == 0 ? a[x].x : e == 1 ? a[x].y : e == 2 ? a[x].z : a[x].w;
 #pragma unroll
-        for (int y = 0; y < 2; ++y) O[x][y] = __builtin_amdgcn_mfma_f32_16x16x4f32(ax, v[y], O[x][y], 0, 0, 0);
+        for (int y = 0; y < 2; ++y) O[x][y] = __builtin_amdgcn_mfma_f32_16x16x4f32(ax, sv[y], O[x][y], 0, 0, 0);
       }
     }
   }
@@ -380,18 +450,37 @@ scan_chunk_outputs_kernel(const ti_scan_inputs in, const int* __restrict__ chunk
       for (int r = 0; r < 4; ++r) {
         const int t = wy + 16 * x + 4 * quad + r, j = wx + 16 * y + r16;
         if (t >= n || j0 + j >= dv) continue;
-        float v = O[x][y][r];
-        if (in.skip) v = fmaf(skip, s_s[t][j], v);
-        o[(size_t)(row0 + t) * heads * dv + (size_t)h * dv + j0 + j] = v;
+        float y_t = O[x][y][r];
+        if (in.skip) y_t = fmaf(skip, s_s[t][j], y_t);
+        o[(size_t)(row0 + t) * heads * dv + (size_t)h * dv + j0 + j] = y_t;
       }
 }
 
-template <int NT, int TB>
+// The rotation of the step's queries and keys in place, in front of the chunks (which then take them as they are): a thread per
+// pair of entries.
+__global__ void __launch_bounds__(256) scan_rotate_kernel(float* __restrict__ proj, const ti_scan_inputs in, int dk, long n_pairs) {
+  const int half = in.rot_dims / 2;
+  for (long x = (long)blockIdx.x * 256 + threadIdx.x; x < n_pairs; x += (long)gridDim.x * 256) {
+    const int f = (int)(x % half);
+    const long unit = x / half;
+    const int u = (int)(unit % (2 * in.qk_heads));
+    const long m = unit / (2 * in.qk_heads);
+    float* head = proj + m * in.ld + (u < in.qk_heads ? in.off_q + u * dk : in.off_k + (u - in.qk_heads) * dk);
+    float c, s;
+    scan_angle(in, in.pos[m], half, f, &c, &s);
+    const float a = head[f], b = head[f + half];
+    head[f] = a * c - b * s;
+    head[f + half] = b * c + a * s;
+  }
+}
+
+template <int FORM>
 static int launch_scan(int rpt, dim3 grid, size_t lds, hipStream_t stream, const ti_scan_inputs& in, float* state, long slot_stride,
                        const int* entry_meta, float* o, int heads, int dk, int dv, int dvs, int dvp) {
-#define LA_CASE(R)                                                                                                                  \
-  case R:                                                                                                                           \
-    scan_tokens_kernel<NT, R, TB><<<grid, NT, lds, stream>>>(in, state, slot_stride, entry_meta, o, heads, dk, dv, dvs, dvp);       \
+#define LA_CASE(R)                                                                                                                        \
+  case R:                                                                                                                                 \
+    scan_tokens_kernel<FORM, SCAN_NT, R, SCAN_TB><<<grid, SCAN_NT, lds, stream>>>(in, state, slot_stride, entry_meta, o, heads, dk, dv,   \
+                                                                                  dvs, dvp);                                              \
     return 0;
   switch (rpt) {
     LA_CASE(1) LA_CASE(2) LA_CASE(4) LA_CASE(8) LA_CASE(16) LA_CASE(32) LA_CASE(64)
@@ -401,22 +490,20 @@ static int launch_scan(int rpt, dim3 grid, size_t lds, hipStream_t stream, const
 }
 
 // wide states are cut into slices of 64 columns, a workgroup each: more workgroups, and fewer rows a thread
-struct ScanShape { int dvs, slices, dvp, nt, tb, rpt; size_t lds; bool big; };
+struct ScanShape { int dvs, slices, dvp, rpt; size_t lds; };
 static ScanShape scan_shape(int dk, int dv) {
   ScanShape s;
   s.dvs = dv > 64 ? 64 : dv;
   s.slices = (dv + s.dvs - 1) / s.dvs;
   s.dvp = 1;
   while (s.dvp < s.dvs) s.dvp *= 2;
-  s.big = (long)dk * s.dvp > 64L * 256;
-  s.nt = s.big ? 1024 : 256;
-  s.tb = s.big ? 4 : 16;
-  const int rgs = s.nt / s.dvp;
+  const int rgs = SCAN_NT / s.dvp;
   s.rpt = 1;
   while (s.rpt * rgs < dk) s.rpt *= 2;
-  s.lds = ((size_t)s.tb * (2 * s.rpt * rgs + s.dvs) + (size_t)s.tb * s.nt + 2 * s.tb) * 4;
+  s.lds = ((size_t)SCAN_TB * (2 * s.rpt * rgs + s.dvs) + (size_t)SCAN_TB * SCAN_NT + 2 * SCAN_TB) * 4;
   return s;
 }
+static int scan_form(const ti_scan_inputs* in) { return in->act ? SCAN_SILU : in->decay ? SCAN_ROTATED : SCAN_SELECTIVE; }
 
 static int check_scan(const char* what, const ti_scan_inputs* in, long slot_stride, int heads, int dk, int dv) {
   TI_REQUIRE(heads > 0 && heads <= 65535 && dk > 0 && dk <= 256 && dv > 0 && dv <= 256, "%s: bad sizes heads=%d dk=%d dv=%d (up to 256)",
@@ -427,7 +514,8 @@ static int check_scan(const char* what, const ti_scan_inputs* in, long slot_stri
              "%s: the columns do not lie inside rows of %d", what, in->ld);
   TI_REQUIRE(in->rot_dims >= 0 && in->rot_dims % 2 == 0 && in->rot_dims <= dk && (!in->rot_dims || (in->inv_freq && in->pos && !in->act)),
              "%s: a rotation of %d of %d entries is not served", what, in->rot_dims, dk);
-  TI_REQUIRE(in->decay || (in->dt && in->dt_bias && in->a_log && in->dt_ld >= heads), "%s: neither fixed decays nor step sizes", what);
+  TI_REQUIRE(in->decay || (in->dt && in->dt_bias && in->a_log && in->dt_ld >= heads && !in->act && !in->rot_dims),
+             "%s: neither fixed decays nor step sizes, or step sizes beside an activation or a rotation", what);
   TI_REQUIRE(slot_stride >= (long)heads * dk * dv, "%s: a slot of %ld floats does not hold the state", what, slot_stride);
   return 0;
 }
@@ -441,8 +529,14 @@ extern "C" int ti_linear_scan(const ti_scan_inputs* in, float* state, long slot_
   const ScanShape s = scan_shape(dk, dv);
   TI_REQUIRE(s.rpt <= 64, "linear_scan: a state of %d x %d is not served", dk, dv);
   const dim3 grid(n_entries, heads, s.slices);
-  const int rc = s.big ? launch_scan<1024, 4>(s.rpt, grid, s.lds, stream, *in, state, slot_stride, entry_meta, o, heads, dk, dv, s.dvs, s.dvp)
-                       : launch_scan<256, 16>(s.rpt, grid, s.lds, stream, *in, state, slot_stride, entry_meta, o, heads, dk, dv, s.dvs, s.dvp);
+  int rc;
+#define SCAN_CALL(F) rc = launch_scan<F>(s.rpt, grid, s.lds, stream, *in, state, slot_stride, entry_meta, o, heads, dk, dv, s.dvs, s.dvp)
+  switch (scan_form(in)) {
+    case SCAN_SILU: SCAN_CALL(SCAN_SILU); break;
+    case SCAN_ROTATED: SCAN_CALL(SCAN_ROTATED); break;
+    default: SCAN_CALL(SCAN_SELECTIVE);
+  }
+#undef SCAN_CALL
   TI_REQUIRE(rc == 0, "linear_scan: no kernel for %d rows a thread", s.rpt);
   TI_LAUNCH_CHECK();
   return 0;
@@ -451,75 +545,142 @@ extern "C" int ti_linear_scan(const ti_scan_inputs* in, float* state, long slot_
 // The same with every entry's tokens cut into chunks of up to 64 that run side by side.  chunks int [n_chunks][4] = (entry, first
 // row, tokens, flags), spans int [n_entries][2] = (first chunk, chunks), both in device memory; scratch float
 // [n_chunks][heads][dk dv + 1]
-extern "C" int ti_linear_scan_chunked(const ti_scan_inputs* in, float* state, long slot_stride, const int* entry_meta, int n_entries,
-                                      const int* chunks, int n_chunks, const int* spans, float* scratch, float* o, int heads, int dk,
-                                      int dv, hipStream_t stream) {
-  if (check_scan("linear_scan", in, slot_stride, heads, dk, dv)) return 1;
-  TI_REQUIRE(chunks && spans && scratch && n_chunks >= n_entries, "linear_scan: chunks need their lists and scratch");
-  if (n_entries == 0) return 0;
+template <int FORM, bool VEC>
+static void launch_chunks(const ti_scan_inputs& in, float* state, long slot_stride, const int* entry_meta, int n_entries, const int* chunks,
+                          int n_chunks, const int* spans, float* scratch, float* o, int heads, int dk, int dv, hipStream_t stream) {
   const int rb = (dk + SC_N - 1) / SC_N, cb = (dv + SC_N - 1) / SC_N, per_head = dk * dv;
   float* chunk_decay = scratch + (size_t)n_chunks * heads * per_head;
-  scan_chunk_states_kernel<<<dim3(n_chunks, heads, rb * cb), 256, 0, stream>>>(*in, chunks, scratch, chunk_decay, heads, dk, dv, cb);
+  scan_chunk_states_kernel<FORM, VEC><<<dim3(n_chunks, heads, rb * cb), 256, 0, stream>>>(in, chunks, scratch, chunk_decay, heads, dk, dv, cb);
   scan_carry_kernel<<<dim3(n_entries, heads, (per_head + 255) / 256), 256, 0, stream>>>(scratch, chunk_decay, spans, entry_meta, state, slot_stride,
                                                                                       heads, per_head);
-  scan_chunk_outputs_kernel<<<dim3(n_chunks, heads, cb), 256, 0, stream>>>(*in, chunks, scratch, o, heads, dk, dv);
+  scan_chunk_outputs_kernel<FORM, VEC><<<dim3(n_chunks, heads, cb), 256, 0, stream>>>(in, chunks, scratch, o, heads, dk, dv);
+}
+
+// (rotated queries and keys are turned in place: the columns of proj are overwritten)
+extern "C" int ti_linear_scan_chunked(const ti_scan_inputs* inputs, int M, float* state, long slot_stride, const int* entry_meta, int n_entries,
+                                      const int* chunks, int n_chunks, const int* spans, float* scratch, float* o, int heads, int dk,
+                                      int dv, hipStream_t stream) {
+  ti_scan_inputs in = *inputs;
+  if (check_scan("linear_scan", &in, slot_stride, heads, dk, dv)) return 1;
+  TI_REQUIRE(chunks && spans && scratch && n_chunks >= n_entries, "linear_scan: chunks need their lists and scratch");
+  if (n_entries == 0 || M == 0) return 0;
+  if (in.rot_dims) {
+    const long pairs = (long)M * 2 * in.qk_heads * (in.rot_dims / 2);
+    const unsigned blocks = (unsigned)((pairs + 255) / 256 < 8192 ? (pairs + 255) / 256 : 8192);
+    scan_rotate_kernel<<<blocks, 256, 0, stream>>>((float*)in.proj, in, dk, pairs);
+    in.rot_dims = 0;
+  }
+  const bool vec = dk % 4 == 0 && dv % 4 == 0 && in.ld % 4 == 0 && in.off_q % 4 == 0 && in.off_k % 4 == 0 && in.off_v % 4 == 0 &&
+                   (((uintptr_t)in.proj | (uintptr_t)scratch) & 15) == 0;
+#define SCAN_CHUNKS(F)                                                                                                                    \
+  do {                                                                                                                                    \
+    if (vec) launch_chunks<F, true>(in, state, slot_stride, entry_meta, n_entries, chunks, n_chunks, spans, scratch, o, heads, dk, dv, stream); \
+    else launch_chunks<F, false>(in, state, slot_stride, entry_meta, n_entries, chunks, n_chunks, spans, scratch, o, heads, dk, dv, stream);    \
+  } while (0)
+  switch (scan_form(&in)) {
+    case SCAN_SILU: SCAN_CHUNKS(SCAN_SILU); break;
+    case SCAN_ROTATED: SCAN_CHUNKS(SCAN_ROTATED); break;
+    default: SCAN_CHUNKS(SCAN_SELECTIVE);
+  }
+#undef SCAN_CHUNKS
   TI_LAUNCH_CHECK();
   return 0;
 }
 
 // The norm behind such a mixer and its gate: a row of W entries in `groups` equal runs, each divided by its own root mean square,
 // times w (null: none), with the gate's activation of gate columns off_g .. (0: sigmoid, 1: silu) multiplied in behind the
-// norm, or in front of it (gate_first); rounded once to T.  WAVES: a wavefront per run (runs of up to 1024 entries, in
-// registers), else a workgroup.
-template <typename T, bool WAVES>
+// norm, or in front of it (gate_first); rounded once to T.  TPR threads a run (a wavefront or the whole workgroup), each N
+// neighbouring entries at a time (N 4: everything aligned to 16 bytes), PIECES of them in registers (0: any length, from memory).
+template <typename T, int TPR, int N, int PIECES>
 __global__ void __launch_bounds__(256)
 gated_group_norm_kernel(const float* __restrict__ o, const float* __restrict__ gate, int ld, int off_g, const float* __restrict__ w,
                         T* __restrict__ out, int M, int W, int groups, float eps, int silu, int gate_first) {
   __shared__ float red[4];
   const int size = W / groups;
-  auto gate_of = [&](float g) { return silu ? la_silu(g) : 1.0f / (1.0f + expf(-g)); };
-  if constexpr (WAVES) {
-    const long run = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (run >= (long)M * groups) return;
-    const int lane = threadIdx.x & 63;
-    const size_t m = run / groups;
-    const int c0 = (int)(run % groups) * size;
-    const float* src = o + m * W + c0;
-    const float* g = gate + m * ld + off_g + c0;
-    float v[16], f[16];
+  const long run = (long)blockIdx.x * (256 / TPR) + threadIdx.x / TPR;
+  if (run >= (long)M * groups) return;      // (whole wavefronts; with a workgroup a run there is none)
+  const int lane = threadIdx.x % TPR;
+  const size_t m = run / groups;
+  const int c0 = (int)(run % groups) * size;
+  const float* src = o + m * W + c0;
+  const float* g = gate + m * ld + off_g + c0;
+  const float* wr = w ? w + c0 : nullptr;
+  T* dst = out + m * W + c0;
+  auto gate_of = [&](float z) { return silu ? la_silu(z) : 1.0f / (1.0f + expf(-z)); };
+  auto total = [&](float ss) {
+    if (TPR == 256) return block_sum<256>(ss, red);
+    return group_sum<TI_WAVE>(ss);
+  };
+  if constexpr (PIECES > 0) {
+    float v[PIECES][N], f[PIECES][N];
+#pragma unroll
+    for (int i = 0; i < PIECES; ++i) {
+      const int c = (lane + TPR * i) * N;
+#pragma unroll
+      for (int j = 0; j < N; ++j) v[i][j] = f[i][j] = 0.f;
+      if (c < size) {
+        if constexpr (N == 4) {
+          const float4 a = *reinterpret_cast<const float4*>(src + c), b = *reinterpret_cast<const float4*>(g + c);
+          v[i][0] = a.x; v[i][1] = a.y; v[i][2] = a.z; v[i][3] = a.w;
+          f[i][0] = b.x; f[i][1] = b.y; f[i][2] = b.z; f[i][3] = b.w;
+        } else {
+          v[i][0] = src[c];
+          f[i][0] = g[c];
+        }
+      }
+    }
     float ss = 0.f;
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int c = lane + 64 * i;
-      if (64 * i >= size) break;
-      v[i] = f[i] = 0.f;
-      if (c < size) {
-        f[i] = gate_of(g[c]);
-        v[i] = src[c];
-        if (gate_first) v[i] *= f[i];
-      }
-      ss = fmaf(v[i], v[i], ss);
-    }
-    const float inv = 1.0f / sqrtf(group_sum<TI_WAVE>(ss) / (float)size + eps);
+    for (int i = 0; i < PIECES; ++i)
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int c = lane + 64 * i;
-      if (64 * i >= size) break;
-      if (c < size) st<T>(out + m * W + c0 + c, v[i] * inv * (w ? w[c0 + c] : 1.f) * (gate_first ? 1.f : f[i]));
+      for (int j = 0; j < N; ++j) {
+        f[i][j] = gate_of(f[i][j]);
+        if (gate_first) v[i][j] *= f[i][j];
+        ss = fmaf(v[i][j], v[i][j], ss);
+      }
+    const float inv = 1.0f / sqrtf(total(ss) / (float)size + eps);
+#pragma unroll
+    for (int i = 0; i < PIECES; ++i) {
+      const int c = (lane + TPR * i) * N;
+      if (c >= size) continue;
+      float y[N];
+#pragma unroll
+      for (int j = 0; j < N; ++j) y[j] = v[i][j] * inv * (wr ? wr[c + j] : 1.f) * (gate_first ? 1.f : f[i][j]);
+      if constexpr (N == 4) {
+        if constexpr (sizeof(T) == 2) *reinterpret_cast<uint2*>(dst + c) = make_uint2(pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3]));
+        else *reinterpret_cast<float4*>(dst + c) = make_float4(y[0], y[1], y[2], y[3]);
+      } else {
+        st<T>(dst + c, y[0]);
+      }
     }
   } else {
-    const size_t m = blockIdx.x / groups;
-    const int c0 = (int)(blockIdx.x % groups) * size;
-    const float* src = o + m * W + c0;
-    const float* g = gate + m * ld + off_g + c0;
     float ss = 0.f;
-    for (int c = threadIdx.x; c < size; c += 256) {
+    for (int c = lane; c < size; c += TPR) {
       const float v = gate_first ? src[c] * gate_of(g[c]) : src[c];
       ss = fmaf(v, v, ss);
     }
-    const float inv = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)size + eps);
-    for (int c = threadIdx.x; c < size; c += 256) st<T>(out + m * W + c0 + c, src[c] * inv * (w ? w[c0 + c] : 1.f) * gate_of(g[c]));
+    const float inv = 1.0f / sqrtf(total(ss) / (float)size + eps);
+    for (int c = lane; c < size; c += TPR) st<T>(dst + c, src[c] * inv * (wr ? wr[c] : 1.f) * gate_of(g[c]));
   }
+}
+
+template <typename T>
+static void launch_group_norm(bool vec, const float* o, const float* gate, int ld, int off_g, const float* w, void* out, int M, int W, int groups,
+                              float eps, int silu, int gate_first, hipStream_t stream) {
+  const int size = W / groups;
+  const long runs = (long)M * groups;
+#define GGN(TPR, N, P)                                                                                                              \
+  gated_group_norm_kernel<T, TPR, N, P><<<(unsigned)((runs + 256 / TPR - 1) / (256 / TPR)), 256, 0, stream>>>(o, gate, ld, off_g, w, (T*)out, M, W, \
+                                                                                                           groups, eps, silu, gate_first)
+  if (vec && size <= 256) GGN(64, 4, 1);
+  else if (!vec && size <= 64) GGN(64, 1, 1);
+  else if (!vec && size <= 256) GGN(64, 1, 4);
+  else if (vec && size <= 1024) GGN(256, 4, 1);
+  else if (vec && size <= 2048) GGN(256, 4, 2);
+  else if (vec && size <= 4096) GGN(256, 4, 4);
+  else if (vec && size <= 8192) GGN(256, 4, 8);
+  else GGN(256, 1, 0);
+#undef GGN
 }
 
 extern "C" int ti_gated_group_norm(int out_dtype, const float* o, const float* gate, int ld, int off_g, const float* w, void* out, int M,
@@ -528,18 +689,9 @@ extern "C" int ti_gated_group_norm(int out_dtype, const float* o, const float* g
              "gated_group_norm: bad sizes M=%d W=%d in %d runs, gate columns %d of %d", M, W, groups, off_g, ld);
   TI_REQUIRE(out_dtype == TI_F32 || out_dtype == TI_BF16, "gated_group_norm: unknown dtype %d", out_dtype);
   if (M == 0) return 0;
-  const bool waves = groups > 1 && W / groups <= 1024;
-  const long runs = (long)M * groups;
-  const unsigned blocks = (unsigned)(waves ? (runs + 3) / 4 : runs);
-#define GGN(T, V) gated_group_norm_kernel<T, V><<<blocks, 256, 0, stream>>>(o, gate, ld, off_g, w, (T*)out, M, W, groups, eps, silu, gate_first)
-  if (out_dtype == TI_F32) {
-    if (waves) GGN(float, true);
-    else GGN(float, false);
-  } else {
-    if (waves) GGN(bf16_t, true);
-    else GGN(bf16_t, false);
-  }
-#undef GGN
+  const bool vec = (W / groups) % 4 == 0 && ld % 4 == 0 && off_g % 4 == 0 && (((uintptr_t)o | (uintptr_t)gate | (uintptr_t)out) & 15) == 0;
+  if (out_dtype == TI_F32) launch_group_norm<float>(vec, o, gate, ld, off_g, w, out, M, W, groups, eps, silu, gate_first, stream);
+  else launch_group_norm<bf16_t>(vec, o, gate, ld, off_g, w, out, M, W, groups, eps, silu, gate_first, stream);
   TI_LAUNCH_CHECK();
   return 0;
 }

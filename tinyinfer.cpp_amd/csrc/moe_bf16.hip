@@ -74,9 +74,10 @@ moe_place_kernel(const bf16_t* __restrict__ h, const int* __restrict__ ids, cons
                  int E, int R, int top, int W, int n_pairs, int* __restrict__ where, bf16_t* __restrict__ rows,
                  float* __restrict__ row_w, int* __restrict__ tokens, float* __restrict__ out) {
   __shared__ int count[MOE_MAX_E + 1];      // pairs of this workgroup per expert, then the first row of their run
-  __shared__ int s_row[64], s_self[64];
+  __shared__ int s_row[64], s_self[64], s_n_self;
   const int pair0 = blockIdx.x * 64;
   for (int e = threadIdx.x; e < R; e += 256) count[e] = 0;
+  if (threadIdx.x == 0) s_n_self = 0;
   __syncthreads();
   int e_mine = -1, local = 0;
   if (threadIdx.x < 64 && pair0 + threadIdx.x < n_pairs) {
@@ -92,39 +93,43 @@ moe_place_kernel(const bf16_t* __restrict__ h, const int* __restrict__ ids, cons
     where[pair0 + threadIdx.x] = r;
     if (row_w) row_w[r] = wts[pair0 + threadIdx.x];      // weights on the experts' outputs: with the row
     s_row[threadIdx.x] = r;
-    s_self[threadIdx.x] = e_mine >= E ? 1 : 0;
+    if (e_mine >= E) s_self[atomicAdd(&s_n_self, 1)] = threadIdx.x;      // an identity expert's pair (in any order: a pair is a row of its own)
     if (tokens) tokens[r] = (pair0 + threadIdx.x) / top;
   }
   if (tokens && R == E) return;
   __syncthreads();
-  // a wavefront takes 16 of the pairs, a lane 16 bytes at a time (W is a multiple of 32)
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  for (int i = 0; i < 16; ++i) {
-    const int pair = pair0 + wave * 16 + i;
-    if (pair >= n_pairs) break;
-    const bool self = s_self[wave * 16 + i] != 0;
-    if (tokens && !self) continue;
-    const float s = wts[pair];
-    const bf16_t* src = h + (size_t)(pair / top) * W;
-    const size_t row = (size_t)s_row[wave * 16 + i];
-    for (int c = lane * 8; c < W; c += 64 * 8) {
-      const uint4 a = *reinterpret_cast<const uint4*>(src + c);
-      const unsigned w[4] = {a.x, a.y, a.z, a.w};
-      float f[8];
+  // 16 bytes of a row at a time (W is a multiple of 32)
+  auto piece = [&](int local_pair, int c, float* f) {
+    const float s = wts[pair0 + local_pair];
+    const uint4 a = *reinterpret_cast<const uint4*>(h + (size_t)((pair0 + local_pair) / top) * W + c);
+    const unsigned w[4] = {a.x, a.y, a.z, a.w};
 #pragma unroll
-      for (int k = 0; k < 4; ++k) {
-        f[2 * k] = __uint_as_float(w[k] << 16) * s;
-        f[2 * k + 1] = __uint_as_float(w[k] & 0xffff0000u) * s;
-      }
-      if (self) {
-        float4* dst = reinterpret_cast<float4*>(out + row * W + c);
-        dst[0] = make_float4(f[0], f[1], f[2], f[3]);
-        dst[1] = make_float4(f[4], f[5], f[6], f[7]);
-      } else {
-        *reinterpret_cast<uint4*>(rows + row * W + c) =
+    for (int k = 0; k < 4; ++k) {
+      f[2 * k] = __uint_as_float(w[k] << 16) * s;
+      f[2 * k + 1] = __uint_as_float(w[k] & 0xffff0000u) * s;
+    }
+  };
+  const int pieces = W / 8;
+  if (!tokens) {      // scaled inputs, laid out expert by expert: a wavefront copies 16 of the rows
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    for (int i = 0; i < 16; ++i) {
+      const int p = wave * 16 + i;
+      if (pair0 + p >= n_pairs) break;
+      for (int c = lane * 8; c < W; c += 64 * 8) {
+        float f[8];
+        piece(p, c, f);
+        *reinterpret_cast<uint4*>(rows + (size_t)s_row[p] * W + c) =
             make_uint4(pack_bf16x2(f[0], f[1]), pack_bf16x2(f[2], f[3]), pack_bf16x2(f[4], f[5]), pack_bf16x2(f[6], f[7]));
       }
     }
+  }
+  for (int x = threadIdx.x; x < s_n_self * pieces; x += 256) {
+    const int p = s_self[x / pieces], c = x % pieces * 8;
+    float f[8];
+    piece(p, c, f);
+    float4* dst = reinterpret_cast<float4*>(out + (size_t)s_row[p] * W + c);
+    dst[0] = make_float4(f[0], f[1], f[2], f[3]);
+    dst[1] = make_float4(f[4], f[5], f[6], f[7]);
   }
 }
 

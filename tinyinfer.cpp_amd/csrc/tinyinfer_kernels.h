@@ -273,8 +273,8 @@ int ti_linear_scan(const ti_scan_inputs* in, float* state, long slot_stride, con
                    int dk, int dv, hipStream_t stream);
 // the same with the entries' tokens in chunks of up to 64 that run side by side (chunks [n_chunks][4] = (entry, first row, tokens,
 // 1: the entry's first chunk + 2: its last), spans [n_entries][2] = (first chunk, chunks); scratch float
-// [n_chunks][heads][dk dv + 1])
-int ti_linear_scan_chunked(const ti_scan_inputs* in, float* state, long slot_stride, const int* entry_meta, int n_entries,
+// [n_chunks][heads][dk dv + 1]; M: the step's rows).  Rotated queries and keys are turned in place: proj is written
+int ti_linear_scan_chunked(const ti_scan_inputs* in, int M, float* state, long slot_stride, const int* entry_meta, int n_entries,
                            const int* chunks, int n_chunks, const int* spans, float* scratch, float* o, int heads, int dk, int dv,
                            hipStream_t stream);
 // out = o / rms(o) * w * act(gate) with the rms over each of `groups` equal runs of a row (w null: none; act 0 sigmoid, 1 silu;

@@ -460,7 +460,8 @@ class Ops {
   };
   // state f32 [slots][heads][dk dv]; o f32 [M, heads dv]
   // chunks (device int32 [n_chunks][4] = (entry, first row, tokens up to 64, 1: the entry's first chunk + 2: its last)) and spans
-  // ([n_entries][2] = (first chunk, chunks)): long portions run as chunks side by side, through scratch of `ws`
+  // ([n_entries][2] = (first chunk, chunks)): long portions run as chunks side by side, through scratch of `ws` (the
+  // columns of q and k that are to be rotated are then turned in place)
   void linear_scan(const LinearScan& in, const Tensor& state, const int* entry_meta, int n_entries, const Tensor& o, int heads, int dk,
                    int dv, const int* chunks = nullptr, int n_chunks = 0, const int* spans = nullptr, Workspace* ws = nullptr);
   // out = o / rms(o) * w * act(gate columns of proj), in the compute dtype: the rms over each of `groups` equal runs of a row, w

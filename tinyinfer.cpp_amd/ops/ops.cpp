@@ -1418,7 +1418,7 @@ void Ops::linear_scan(const LinearScan& in, const Tensor& state, const int* entr
   if (chunks) {
     require(spans && ws && n_chunks >= n_entries, "linear_scan: chunks need spans and a workspace");
     float* scratch = (float*)ws->get("scan.chunk_states", (size_t)n_chunks * (per_slot + heads) * 4);
-    int rc = KERNEL("linear_attention", ti_linear_scan_chunked)(&si, (float*)state.data, (long)per_slot, entry_meta, n_entries, chunks, n_chunks,
+    int rc = KERNEL("linear_attention", ti_linear_scan_chunked)(&si, (int)M, (float*)state.data, (long)per_slot, entry_meta, n_entries, chunks, n_chunks,
                                                                 spans, scratch, (float*)o.data, heads, dk, dv, (hipStream_t)launch_stream());
     check("linear_attention", rc, "linear_scan(chunked)");
     took("[chunked]");
