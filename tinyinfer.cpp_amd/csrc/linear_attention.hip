@@ -456,21 +456,29 @@ scan_chunk_outputs_kernel(const ti_scan_inputs in, const int* __restrict__ chunk
       }
 }
 
-// The rotation of the step's queries and keys in place, in front of the chunks (which then take them as they are): a thread per
-// pair of entries.
-__global__ void __launch_bounds__(256) scan_rotate_kernel(float* __restrict__ proj, const ti_scan_inputs in, int dk, long n_pairs) {
-  const int half = in.rot_dims / 2;
-  for (long x = (long)blockIdx.x * 256 + threadIdx.x; x < n_pairs; x += (long)gridDim.x * 256) {
-    const int f = (int)(x % half);
-    const long unit = x / half;
-    const int u = (int)(unit % (2 * in.qk_heads));
-    const long m = unit / (2 * in.qk_heads);
-    float* head = proj + m * in.ld + (u < in.qk_heads ? in.off_q + u * dk : in.off_k + (u - in.qk_heads) * dk);
-    float c, s;
-    scan_angle(in, in.pos[m], half, f, &c, &s);
-    const float a = head[f], b = head[f + half];
-    head[f] = a * c - b * s;
-    head[f + half] = b * c + a * s;
+// The rotation of the step's queries and keys in place, in front of the chunks (which then take them as they are): a workgroup per
+// (row, 1024 pairs of entries), four neighbouring pairs a thread (VEC: aligned to 16 bytes) or one.
+template <bool VEC> __global__ void __launch_bounds__(256) scan_rotate_kernel(float* __restrict__ proj, const ti_scan_inputs in, int dk) {
+  constexpr int N = VEC ? 4 : 1;
+  const int half = in.rot_dims / 2, n_pairs = 2 * in.qk_heads * half;
+  float* const row = proj + (size_t)blockIdx.x * in.ld;
+  const int p = in.pos[blockIdx.x];
+  for (int x = (blockIdx.y * 256 + threadIdx.x) * N; x < n_pairs; x += gridDim.y * 256 * N) {
+    const int f = x % half, u = x / half;      // (VEC: half is a multiple of four, the pairs lie in one head)
+    float* a = row + (u < in.qk_heads ? in.off_q + u * dk : in.off_k + (u - in.qk_heads) * dk) + f;
+    float* b = a + half;
+    float c[N], s[N];
+#pragma unroll
+    for (int i = 0; i < N; ++i) scan_angle(in, p, half, f + i, &c[i], &s[i]);
+    if constexpr (VEC) {
+      const float4 va = *reinterpret_cast<const float4*>(a), vb = *reinterpret_cast<const float4*>(b);
+      *reinterpret_cast<float4*>(a) = make_float4(va.x * c[0] - vb.x * s[0], va.y * c[1] - vb.y * s[1], va.z * c[2] - vb.z * s[2], va.w * c[3] - vb.w * s[3]);
+      *reinterpret_cast<float4*>(b) = make_float4(vb.x * c[0] + va.x * s[0], vb.y * c[1] + va.y * s[1], vb.z * c[2] + va.z * s[2], vb.w * c[3] + va.w * s[3]);
+    } else {
+      const float va = *a, vb = *b;
+      *a = va * c[0] - vb * s[0];
+      *b = vb * c[0] + va * s[0];
+    }
   }
 }
 
@@ -565,9 +573,12 @@ extern "C" int ti_linear_scan_chunked(const ti_scan_inputs* inputs, int M, float
   TI_REQUIRE(chunks && spans && scratch && n_chunks >= n_entries, "linear_scan: chunks need their lists and scratch");
   if (n_entries == 0 || M == 0) return 0;
   if (in.rot_dims) {
-    const long pairs = (long)M * 2 * in.qk_heads * (in.rot_dims / 2);
-    const unsigned blocks = (unsigned)((pairs + 255) / 256 < 8192 ? (pairs + 255) / 256 : 8192);
-    scan_rotate_kernel<<<blocks, 256, 0, stream>>>((float*)in.proj, in, dk, pairs);
+    const int half = in.rot_dims / 2;
+    const bool vec = half % 4 == 0 && dk % 4 == 0 && in.ld % 4 == 0 && in.off_q % 4 == 0 && in.off_k % 4 == 0 && ((uintptr_t)in.proj & 15) == 0;
+    const int each = vec ? 1024 : 256, pieces = (2 * in.qk_heads * half + each - 1) / each;
+    const dim3 grid(M, pieces < 64 ? pieces : 64);
+    if (vec) scan_rotate_kernel<true><<<grid, 256, 0, stream>>>((float*)in.proj, in, dk);
+    else scan_rotate_kernel<false><<<grid, 256, 0, stream>>>((float*)in.proj, in, dk);
     in.rot_dims = 0;
   }
   const bool vec = dk % 4 == 0 && dv % 4 == 0 && in.ld % 4 == 0 && in.off_q % 4 == 0 && in.off_k % 4 == 0 && in.off_v % 4 == 0 &&

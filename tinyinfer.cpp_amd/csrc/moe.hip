@@ -38,98 +38,127 @@ template <> struct Piece<bf16_t> {
   }
 };
 
-// the wavefront's share of a . b over n elements: a in LDS or memory as floats through `fa`, b a row of the weight
-template <typename T, bool VEC, class FA>
-__device__ __forceinline__ float wave_dot(FA fa, const T* __restrict__ b, int n, int lane) {
-  float z = 0.f;
-  if (VEC) {
-    constexpr int N = Piece<T>::N;
-    for (int c = lane * N; c < n; c += 64 * N) {
-      float v[N];
-      Piece<T>::load(b + c, v);
-#pragma unroll
-      for (int i = 0; i < N; ++i) z = fmaf(fa(c + i), v[i], z);
-    }
-  } else {
-    for (int c = lane; c < n; c += 64) z = fmaf(fa(c), ld<T>(b + c), z);
-  }
-  return group_sum<64>(z);
-}
-
 // ------------------------------------------------------------ router
-// A workgroup per token.  Logits: wavefront w takes experts w, w + 4, ...; lanes share the token's row in pieces of
-// 16 bytes (lane l the pieces l, l + 64, ... in ascending order, then a butterfly).  Choice: the first wavefront
-// holds the scores (lane l the experts l, l + 64, ...) and takes the largest `top` times.
-template <typename T, bool VEC>
+// A workgroup per TM tokens (1, or 4 in long steps: a row of the router is fetched once for four tokens).  Logits: wavefront w takes
+// experts w, w + 4, ...; lanes share the tokens' rows in pieces of 16 bytes (lane l the pieces l, l + 64, ... in ascending order,
+// then a butterfly).  Choice: wavefront t holds token t's scores (lane l the experts l, l + 64, ...) and takes the largest `top`
+// times.  The order of every sum is the same whatever TM.
+struct RouteForm {
+  int W, E, top, score_kind, renormalize, n_groups, keep;
+  float weight_scale, sum_floor;
+};
+// what lanes of the wavefront left in LDS is there for its other lanes
+__device__ __forceinline__ void wave_publish() {
+  __builtin_amdgcn_wave_barrier();
+  __threadfence_block();
+}
+template <typename T, bool VEC, int TM>
 __global__ void __launch_bounds__(256)
-moe_route_kernel(const T* __restrict__ h, const float* __restrict__ router, int* __restrict__ ids, float* __restrict__ wts,
-                 int W, int E, int top, int score_kind, int renormalize, const float* __restrict__ correction = nullptr,
-                 int n_groups = 0, int keep = 0, float weight_scale = 1.f, float sum_floor = 0.f,
-                 const float* __restrict__ gate_row = nullptr, float* __restrict__ gate_out = nullptr) {
-  __shared__ float s_score[MOE_MAX_EXPERTS];
-  __shared__ float s_plain[MOE_MAX_EXPERTS];      // the scores the weights are taken from, where the choice reads corrected ones
-  __shared__ float s_group[MOE_MAX_EXPERTS];
-  __shared__ float red[4];
-  const bool corrected = correction != nullptr || n_groups > 1;
-  const int m = blockIdx.x;
+moe_route_kernel(const T* __restrict__ h, const float* __restrict__ router, int* __restrict__ ids, float* __restrict__ wts, int M,
+                 const RouteForm a, const float* __restrict__ correction, const float* __restrict__ gate_row, float* __restrict__ gate_out) {
+  extern __shared__ float s_route[];      // [TM][E] scores, [TM][E] the scores the weights are taken from, [TM][groups]
+  const int E = a.E, W = a.W;
+  const bool corrected = correction != nullptr || a.n_groups > 1;
+  const int m0 = blockIdx.x * TM;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const T* row = h + (size_t)m * W;
+  const T* rows[TM];
+#pragma unroll
+  for (int t = 0; t < TM; ++t) rows[t] = h + (size_t)min(m0 + t, M - 1) * W;
+  auto dots = [&](const float* __restrict__ w, float* z) {      // w . every token's row
+#pragma unroll
+    for (int t = 0; t < TM; ++t) z[t] = 0.f;
+    if (VEC) {
+      constexpr int N = Piece<T>::N;
+      for (int c = lane * N; c < W; c += 64 * N) {
+        float f[N];
+#pragma unroll
+        for (int i = 0; i < N; ++i) f[i] = w[c + i];
+#pragma unroll
+        for (int t = 0; t < TM; ++t) {
+          float v[N];
+          Piece<T>::load(rows[t] + c, v);
+#pragma unroll
+          for (int i = 0; i < N; ++i) z[t] = fmaf(f[i], v[i], z[t]);
+        }
+      }
+    } else {
+      for (int c = lane; c < W; c += 64) {
+        const float f = w[c];
+#pragma unroll
+        for (int t = 0; t < TM; ++t) z[t] = fmaf(f, ld<T>(rows[t] + c), z[t]);
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < TM; ++t) z[t] = group_sum<64>(z[t]);
+  };
   for (int e = wave; e < E; e += 4) {
-    const float z = wave_dot<T, VEC>([&](int c) { return router[(size_t)e * W + c]; }, row, W, lane);
-    if (lane == 0) s_score[e] = z;
+    float z[TM];
+    dots(router + (size_t)e * W, z);
+    if (lane == 0) {
+#pragma unroll
+      for (int t = 0; t < TM; ++t) s_route[t * E + e] = z[t];
+    }
   }
   if (gate_row && wave == E % 4) {      // one more row beside the router's: sigmoid(gate_row . h), a factor for another branch
-    const float z = wave_dot<T, VEC>([&](int c) { return gate_row[c]; }, row, W, lane);
-    if (lane == 0) gate_out[m] = 1.0f / (1.0f + expf(-z));
+    float z[TM];
+    dots(gate_row, z);
+    if (lane == 0) {
+#pragma unroll
+      for (int t = 0; t < TM; ++t)
+        if (m0 + t < M) gate_out[m0 + t] = 1.0f / (1.0f + expf(-z[t]));
+    }
   }
   __syncthreads();
-  if (score_kind == MOE_SOFTMAX) {
-    float mx = -INFINITY;
-    for (int e = threadIdx.x; e < E; e += 256) mx = fmaxf(mx, s_score[e]);
-    mx = block_max<256>(mx, red);
-    float sum = 0.f;
-    for (int e = threadIdx.x; e < E; e += 256) sum += expf(s_score[e] - mx);
-    sum = block_sum<256>(sum, red);
-    for (int e = threadIdx.x; e < E; e += 256) s_score[e] = expf(s_score[e] - mx) / sum;
-  } else if (score_kind == MOE_SIGMOID) {
-    for (int e = threadIdx.x; e < E; e += 256) s_score[e] = 1.0f / (1.0f + expf(-s_score[e]));
+  if (wave >= TM || m0 + wave >= M) return;
+  const int m = m0 + wave;
+  float* const s_score = s_route + wave * E;
+  float* const s_plain = s_route + (TM + wave) * E;
+  if (a.score_kind == MOE_SOFTMAX) {
+    float mx = -INFINITY, sum = 0.f;
+    for (int e = lane; e < E; e += 64) mx = fmaxf(mx, s_score[e]);
+    mx = group_max<64>(mx);
+    for (int e = lane; e < E; e += 64) sum += expf(s_score[e] - mx);
+    sum = group_sum<64>(sum);
+    for (int e = lane; e < E; e += 64) s_score[e] = expf(s_score[e] - mx) / sum;
+  } else if (a.score_kind == MOE_SIGMOID) {
+    for (int e = lane; e < E; e += 64) s_score[e] = 1.0f / (1.0f + expf(-s_score[e]));
   }
-  __syncthreads();
   if (corrected) {
     // the choice reads score + correction; the weights keep the score itself
-    for (int e = threadIdx.x; e < E; e += 256) {
+    for (int e = lane; e < E; e += 64) {
       s_plain[e] = s_score[e];
       if (correction) s_score[e] += correction[e];
     }
-    __syncthreads();
-    if (n_groups > 1) {
+    wave_publish();
+    if (a.n_groups > 1) {
       // groups of E / n_groups neighbours: a group's score is the sum of its two largest choice scores; experts outside
       // the `keep` best groups (ties to the lower group) cannot be chosen
-      const int per = E / n_groups;
-      for (int g = threadIdx.x; g < n_groups; g += 256) {
-        float a = -INFINITY, b = -INFINITY;
+      float* const s_group = s_route + 2 * TM * E + wave * a.n_groups;
+      const int per = E / a.n_groups;
+      for (int g = lane; g < a.n_groups; g += 64) {
+        float x = -INFINITY, y = -INFINITY;
         for (int e = g * per; e < (g + 1) * per; ++e) {
           const float s = s_score[e];
-          if (s > a) {
-            b = a;
-            a = s;
-          } else if (s > b) {
-            b = s;
+          if (s > x) {
+            y = x;
+            x = s;
+          } else if (s > y) {
+            y = s;
           }
         }
-        s_group[g] = per > 1 ? a + b : a;
+        s_group[g] = per > 1 ? x + y : x;
       }
-      __syncthreads();
-      for (int g = threadIdx.x; g < n_groups; g += 256) {
+      wave_publish();
+      for (int g = lane; g < a.n_groups; g += 64) {
         int better = 0;
-        for (int o = 0; o < n_groups; ++o) better += (s_group[o] > s_group[g] || (s_group[o] == s_group[g] && o < g)) ? 1 : 0;
-        if (better >= keep)
+        for (int o = 0; o < a.n_groups; ++o) better += (s_group[o] > s_group[g] || (s_group[o] == s_group[g] && o < g)) ? 1 : 0;
+        if (better >= a.keep)
           for (int e = g * per; e < (g + 1) * per; ++e) s_score[e] = -INFINITY;
       }
-      __syncthreads();
     }
   }
-  if (wave != 0) return;
+  wave_publish();
+  const int top = a.top;
   float total = 0.f, first = 0.f;
   for (int k = 0; k < top; ++k) {
     float best = -INFINITY;
@@ -157,7 +186,7 @@ moe_route_kernel(const T* __restrict__ h, const float* __restrict__ router, int*
       wts[(size_t)m * top + k] = best;
       s_score[at] = -INFINITY;
     }
-    if (score_kind == MOE_SOFTMAX_CHOSEN) {
+    if (a.score_kind == MOE_SOFTMAX_CHOSEN) {
       // the first choice is the largest logit: every weight is exp(z - z_first) over the sum of those, in the order of choice
       if (k == 0) first = best;
       const float w = expf(best - first);
@@ -166,11 +195,10 @@ moe_route_kernel(const T* __restrict__ h, const float* __restrict__ router, int*
     } else {
       total += best;
     }
-    __builtin_amdgcn_wave_barrier();
-    __threadfence_block();
+    wave_publish();
   }
-  if ((renormalize || score_kind == MOE_SOFTMAX_CHOSEN) && lane < top) wts[(size_t)m * top + lane] /= total + sum_floor;
-  if (weight_scale != 1.f && lane < top) wts[(size_t)m * top + lane] *= weight_scale;
+  if ((a.renormalize || a.score_kind == MOE_SOFTMAX_CHOSEN) && lane < top) wts[(size_t)m * top + lane] /= total + a.sum_floor;
+  if (a.weight_scale != 1.f && lane < top) wts[(size_t)m * top + lane] *= a.weight_scale;
 }
 
 extern "C" int ti_moe_route(int dtype, const void* h, const float* router, int* ids, float* wts, int M, int W, int E, int top,
@@ -203,7 +231,14 @@ extern "C" int ti_moe_route_gate(int dtype, const void* h, const float* router, 
   if (M == 0) return 0;
   const int piece = dtype == TI_F32 ? 4 : 8;
   const bool vec = W % piece == 0 && ((uintptr_t)h & 15) == 0;
-#define MOE_ROUTE(T, V) moe_route_kernel<T, V><<<M, 256, 0, stream>>>((const T*)h, router, ids, wts, W, E, top, score_kind, renormalize, correction, n_groups, keep, weight_scale, sum_floor, gate_row, gate_out)
+  const RouteForm form = {W, E, top, score_kind, renormalize, n_groups, keep, weight_scale, sum_floor};
+  const size_t per_token = ((size_t)2 * E + (n_groups > 1 ? n_groups : 0)) * 4;
+  const bool four = M >= 512 && 4 * per_token <= 64 * 1024;
+#define MOE_ROUTE(T, V)                                                                                                                          \
+  do {                                                                                                                                           \
+    if (four) moe_route_kernel<T, V, 4><<<(M + 3) / 4, 256, 4 * per_token, stream>>>((const T*)h, router, ids, wts, M, form, correction, gate_row, gate_out); \
+    else moe_route_kernel<T, V, 1><<<M, 256, per_token, stream>>>((const T*)h, router, ids, wts, M, form, correction, gate_row, gate_out);        \
+  } while (0)
   if (dtype == TI_F32) {
     if (vec) MOE_ROUTE(float, true);
     else MOE_ROUTE(float, false);

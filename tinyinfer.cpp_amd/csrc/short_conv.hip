@@ -71,12 +71,20 @@ short_conv_rows_kernel(const float* __restrict__ u, long ld, const float* __rest
   for (int x = 0; x < N; ++x)
 #pragma unroll
     for (int j = 0; j < K; ++j) w[x][j] = taps[(size_t)(c + x) * K + j];
+  int first[ROWS], slots[ROWS];      // of the rows' entries: all asked for before the first is needed
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) first[i] = entry_of[min(m0 + i, M - 1)];
 #pragma unroll
   for (int i = 0; i < ROWS; ++i) {
-    const int m = m0 + i;
+    const int e = first[i];
+    first[i] = entries[4 * e];
+    slots[i] = entries[4 * e + 3];
+  }
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    const int m = m0 + i, row0 = first[i];
     if (m >= M) break;
-    const int e = entry_of[m], row0 = entries[4 * e], slot = entries[4 * e + 3];
-    float* st_rows = state + (size_t)slot * (K - 1) * C + c;
+    float* st_rows = state + (size_t)slots[i] * (K - 1) * C + c;
     ScPiece<N> back[K];
 #pragma unroll
     for (int j = 0; j < K; ++j) {
