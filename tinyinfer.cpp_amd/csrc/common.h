@@ -50,14 +50,65 @@ template <typename T> __device__ __forceinline__ void st(T* p, float v);
 template <> __device__ __forceinline__ void st<float>(float* p, float v) { *p = v; }
 template <> __device__ __forceinline__ void st<bf16_t>(bf16_t* p, float v) { *p = f2bf(v); }
 
+// The value of lane i xor O, where lanes that differ in the bits above O (inside their group) hold the same value, as in a
+// butterfly that starts at the widest distance: rotations inside rows of 16 lanes and swaps between rows, without a trip through
+// LDS.  For O = 8 and above no such condition is needed.
+template <int O> __device__ __forceinline__ float lane_xor(float v) {
+  const int x = __float_as_int(v);
+  if (O == 8) return __int_as_float(__builtin_amdgcn_update_dpp(x, x, 0x128, 0xf, 0xf, false));       // row_ror:8
+  if (O == 4) return __int_as_float(__builtin_amdgcn_update_dpp(x, x, 0x124, 0xf, 0xf, false));       // row_ror:4
+  if (O == 2) return __int_as_float(__builtin_amdgcn_update_dpp(x, x, 0x4e, 0xf, 0xf, false));        // quad_perm:[2,3,0,1]
+  return __int_as_float(__builtin_amdgcn_update_dpp(x, x, 0xb1, 0xf, 0xf, false));                    // quad_perm:[1,0,3,2]
+}
+struct LanePair { float a, b; };
+// the values of lanes i and i xor 32 (16), in the same order in both
+template <int O> __device__ __forceinline__ LanePair lane_pair(float v) {
+  const unsigned x = (unsigned)__float_as_int(v);
+  if (O == 32) {
+    const auto r = __builtin_amdgcn_permlane32_swap(x, x, false, false);
+    return {__int_as_float((int)r[0]), __int_as_float((int)r[1])};
+  }
+  const auto r = __builtin_amdgcn_permlane16_swap(x, x, false, false);
+  return {__int_as_float((int)r[0]), __int_as_float((int)r[1])};
+}
+
 // sum over the `width` consecutive lanes a lane belongs to (width: power of two <= 64);
 // every lane of the group ends with the total
 template <int WIDTH> __device__ __forceinline__ float group_sum(float v) {
+  if constexpr (WIDTH >= 16) {
+    if constexpr (WIDTH >= 64) {
+      const LanePair p = lane_pair<32>(v);
+      v = p.a + p.b;
+    }
+    if constexpr (WIDTH >= 32) {
+      const LanePair p = lane_pair<16>(v);
+      v = p.a + p.b;
+    }
+    v += lane_xor<8>(v);
+    v += lane_xor<4>(v);
+    v += lane_xor<2>(v);
+    v += lane_xor<1>(v);
+    return v;
+  }
 #pragma unroll
   for (int o = WIDTH / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, TI_WAVE);
   return v;
 }
 template <int WIDTH> __device__ __forceinline__ float group_max(float v) {
+  if constexpr (WIDTH >= 16) {
+    if constexpr (WIDTH >= 64) {
+      const LanePair p = lane_pair<32>(v);
+      v = fmaxf(p.a, p.b);
+    }
+    if constexpr (WIDTH >= 32) {
+      const LanePair p = lane_pair<16>(v);
+      v = fmaxf(p.a, p.b);
+    }
+    v = fmaxf(v, lane_xor<8>(v));
+    v = fmaxf(v, lane_xor<4>(v));
+    v = fmaxf(v, lane_xor<2>(v));
+    return fmaxf(v, lane_xor<1>(v));
+  }
 #pragma unroll
   for (int o = WIDTH / 2; o > 0; o >>= 1) v = fmaxf(v, __shfl_xor(v, o, TI_WAVE));
   return v;

@@ -254,81 +254,75 @@ extern "C" int ti_moe_route_gate(int dtype, const void* h, const float* router, 
 }
 
 // ------------------------------------------------------------ the experts, an output a wavefront
-// up [E][F][W], down [E][W][F] in T.  Two kernels, both with a workgroup per (expert, 16 outputs): the workgroup finds the
-// pairs (token, choice) of its expert, NP at a time, keeps their input rows in LDS and walks its rows of the weight once for
-// all of them: an expert's weights are read once a step however many tokens chose it.
+// up [E][F][W], down [E][W][F] in T.  Two kernels, a wavefront per (expert, a few outputs), on its own from beginning to end: it
+// finds the pairs (token, choice) of its expert, up to eight at a time, and walks its rows of the weight once for all of them: an
+// expert's weights are read once a step for every eight tokens that chose it.
 //   act[pair][f] = relu(up[e][f] . (s h[token]))^2 rounded to T;   part[pair][c] = down[e][c] . act[pair]
 // and a token's rows of `part` are added in the order its experts were chosen by whoever reads them (moe_sum_pairs, or the
-// norm that follows).  A wavefront owns four outputs; its lanes share a row of the weight in pieces of 16 bytes (lane l the
+// norm that follows).  A wavefront owns four rows of the weight; its lanes share a row in pieces of 16 bytes (lane l the
 // pieces l, l + 64, ... in ascending order, then a butterfly): the order of every sum is fixed, whatever else the step holds.
-#define MOE_ROWS 4      // outputs a wavefront
+#define MOE_ROWS 4      // rows of the weight a wavefront
+#define MOE_PAIRS 8     // pairs at a time
 
-// the next pairs of expert e from pair `next` on, at most NP: their indices to s_pairs, (count, where to go on) to s_found.
-// Called by the first wavefront.
-template <int NP>
-__device__ __forceinline__ void next_pairs(const int* __restrict__ ids, int n_pairs, int e, int next, int* s_pairs, int* s_found) {
-  const int lane = threadIdx.x & 63;
+// the next pairs of expert e from pair `next` on, at most MOE_PAIRS: lane p gets the p-th one's index; returns how many, `next` goes on
+__device__ __forceinline__ int next_pairs(const int* __restrict__ ids, int n_pairs, int e, int lane, int& next, int& mine) {
   int n = 0, i = next;
-  while (i < n_pairs && n < NP) {
+  while (i < n_pairs && n < MOE_PAIRS) {
     const bool hit = i + lane < n_pairs && ids[i + lane] == e;
     unsigned long long mask = __ballot(hit);
     int consumed = 64;
     while (mask) {
       const int b = __ffsll((long long)mask) - 1;
-      if (n == NP) {       // this one waits for the next round
+      if (n == MOE_PAIRS) {       // this one waits for the next round
         consumed = b;
         break;
       }
-      if (lane == 0) s_pairs[n] = i + b;
+      if (lane == n) mine = i + b;
       ++n;
       mask &= mask - 1;
     }
     i += consumed;
   }
-  if (lane == 0) {
-    s_found[0] = n;
-    s_found[1] = i;
-  }
+  next = i;
+  return n;
 }
 
-// z[r][p] = rows[p] . br[r] for the NP rows in LDS (T) and MOE_ROWS rows of the weight in memory: the loads of all the weight's
-// rows are in flight together.  Every sum runs over a lane's pieces in ascending order, then a butterfly.
-template <typename T, bool VEC, int NP>
-__device__ __forceinline__ void wave_dots(const T* rows, int n_live, const T* const* br, int K, int lane, float (*z)[NP]) {
+// one element of a pair's row as a product reads it: in T, times the score where that scales the input
+template <typename T> __device__ __forceinline__ float scaled_input(float v, float s);
+template <> __device__ __forceinline__ float scaled_input<float>(float v, float s) { return v * s; }
+template <> __device__ __forceinline__ float scaled_input<bf16_t>(float v, float s) { return bf2f(f2bf(v * s)); }
+
+// z[r][p] = row p of the pairs . br[r]: the loads of all the weight's rows and of all the pairs' rows are in flight together.  Every
+// sum runs over a lane's pieces in ascending order, then a butterfly.  SCALED: a pair's row is multiplied by s[p] first.
+template <typename T, bool VEC, int NP, bool SCALED>
+__device__ __forceinline__ void wave_dots(const T* const* rows, const float* s, const T* const* br, int K, int lane, float (*z)[MOE_PAIRS]) {
 #pragma unroll
   for (int r = 0; r < MOE_ROWS; ++r)
 #pragma unroll
     for (int p = 0; p < NP; ++p) z[r][p] = 0.f;
-  if (VEC) {
-    constexpr int N = Piece<T>::N;
-    for (int c = lane * N; c < K; c += 64 * N) {
-      float v[MOE_ROWS][N];
+  constexpr int N = VEC ? Piece<T>::N : 1;
+  constexpr int AHEAD = NP <= 4 ? 2 : 1;
+#pragma unroll AHEAD
+  for (int c = lane * N; c < K; c += 64 * N) {
+    float v[MOE_ROWS][N], a[NP][N];
 #pragma unroll
-      for (int r = 0; r < MOE_ROWS; ++r) Piece<T>::load(br[r] + c, v[r]);
-#pragma unroll
-      for (int p = 0; p < NP; ++p)
-        if (p < n_live) {
-          float a[N];
-          Piece<T>::load(rows + (size_t)p * K + c, a);
-#pragma unroll
-          for (int r = 0; r < MOE_ROWS; ++r)
-#pragma unroll
-            for (int i = 0; i < N; ++i) z[r][p] = fmaf(a[i], v[r][i], z[r][p]);
-        }
+    for (int r = 0; r < MOE_ROWS; ++r) {
+      if constexpr (VEC) Piece<T>::load(br[r] + c, v[r]);
+      else v[r][0] = ld<T>(br[r] + c);
     }
-  } else {
-    for (int c = lane; c < K; c += 64) {
-      float v[MOE_ROWS];
 #pragma unroll
-      for (int r = 0; r < MOE_ROWS; ++r) v[r] = ld<T>(br[r] + c);
-#pragma unroll
-      for (int p = 0; p < NP; ++p)
-        if (p < n_live) {
-          const float a = ld<T>(rows + (size_t)p * K + c);
-#pragma unroll
-          for (int r = 0; r < MOE_ROWS; ++r) z[r][p] = fmaf(a, v[r], z[r][p]);
-        }
+    for (int p = 0; p < NP; ++p) {
+      if constexpr (VEC) Piece<T>::load(rows[p] + c, a[p]);
+      else a[p][0] = ld<T>(rows[p] + c);
     }
+#pragma unroll
+    for (int p = 0; p < NP; ++p)
+#pragma unroll
+      for (int i = 0; i < N; ++i) {
+        const float x = SCALED ? scaled_input<T>(a[p][i], s[p]) : a[p][i];
+#pragma unroll
+        for (int r = 0; r < MOE_ROWS; ++r) z[r][p] = fmaf(x, v[r][i], z[r][p]);
+      }
   }
 #pragma unroll
   for (int r = 0; r < MOE_ROWS; ++r)
@@ -345,20 +339,17 @@ __device__ __forceinline__ float moe_gate(float g, float u, int kind, float limi
   return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
 }
 
-// what a workgroup per (expert, outputs) does
+// what a wavefront per (expert, outputs) does
 #define MOE_UP 0       // in: the tokens' inputs h (scaled by the score where it scales the input), K = W, N = F outputs: relu^2 to act (T)
 #define MOE_GATED 1    // in: h, K = W, N = F: an expert's weight is [2 F][W], gate rows above up rows; the gated activation to act (T)
 #define MOE_DOWN 2     // in: act, K = F, N = W: 32-bit to part (times the score where it scales the output)
 // ids from E on are identity experts: MOE_DOWN's workgroups of blockIdx.x = E (launched where there are any) write their
 // pairs' rows of part, the score times the token's row of `self`.
 struct MoeRows { int n_pairs, K, N, top, scale_input, E, kind; float limit, alpha; };
-template <typename T, bool VEC, int NP, int FORM>
-__global__ void __launch_bounds__(256)
+template <typename T, bool VEC, int FORM>
+__global__ void __launch_bounds__(256, 3)
 moe_expert_rows_kernel(const T* __restrict__ in, const int* __restrict__ ids, const float* __restrict__ wts, const T* __restrict__ w,
                        void* __restrict__ out, const T* __restrict__ self, const MoeRows a) {
-  extern __shared__ __attribute__((aligned(16))) unsigned char raw[];
-  T* rows = reinterpret_cast<T*>(raw);      // [NP][K]
-  __shared__ int s_pairs[NP], s_found[2];
   const int e = blockIdx.x, K = a.K, N = a.N;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   if (FORM == MOE_DOWN && e == a.E) {
@@ -371,6 +362,7 @@ moe_expert_rows_kernel(const T* __restrict__ in, const int* __restrict__ ids, co
   }
   constexpr int OUT = FORM == MOE_GATED ? MOE_ROWS / 2 : MOE_ROWS;      // outputs a wavefront
   const int n0 = (blockIdx.y * 4 + wave) * OUT;
+  if (n0 >= N) return;      // (no barrier below)
   const T* we = w + (size_t)e * (FORM == MOE_GATED ? 2 * N : N) * K;
   const T* br[MOE_ROWS];      // (outputs beyond the last one: the last one's rows)
 #pragma unroll
@@ -380,41 +372,45 @@ moe_expert_rows_kernel(const T* __restrict__ in, const int* __restrict__ ids, co
   }
   int next = 0;
   while (next < a.n_pairs) {
-    if (wave == 0) next_pairs<NP>(ids, a.n_pairs, e, next, s_pairs, s_found);
-    __syncthreads();
-    const int n_live = s_found[0];
-    next = s_found[1];
+    int mine = 0;
+    const int n_live = next_pairs(ids, a.n_pairs, e, lane, next, mine);
     if (n_live == 0) break;
-    for (int p = 0; p < n_live; ++p) {
-      const int pair = s_pairs[p];
-      const T* src = FORM == MOE_DOWN ? in + (size_t)pair * K : in + (size_t)(pair / a.top) * K;
-      const float s = (FORM == MOE_UP && a.scale_input) ? wts[pair] : 1.f;
-      for (int c = threadIdx.x; c < K; c += 256) st<T>(rows + (size_t)p * K + c, FORM == MOE_UP ? ld<T>(src + c) * s : ld<T>(src + c));
+    int pairs[MOE_PAIRS];
+    const T* rows[MOE_PAIRS];
+    float s[MOE_PAIRS];
+#pragma unroll
+    for (int p = 0; p < MOE_PAIRS; ++p) {      // (places beyond the last pair: the first one again, not written)
+      pairs[p] = __builtin_amdgcn_readlane(mine, p < n_live ? p : 0);
+      rows[p] = in + (size_t)(FORM == MOE_DOWN ? pairs[p] : pairs[p] / a.top) * K;
+      s[p] = FORM == MOE_GATED ? 1.f : wts[pairs[p]];
     }
-    __syncthreads();
-    if (n0 < N) {
-      float z[MOE_ROWS][NP];
-      wave_dots<T, VEC, NP>(rows, n_live, br, K, lane, z);
-      if (lane == 0) {
+    float z[MOE_ROWS][MOE_PAIRS];
+#define MOE_DOTS(NP)                                                                                         \
+  do {                                                                                                       \
+    if (FORM == MOE_UP && a.scale_input) wave_dots<T, VEC, NP, true>(rows, s, br, K, lane, z);               \
+    else wave_dots<T, VEC, NP, false>(rows, s, br, K, lane, z);                                              \
+  } while (0)
+    if (n_live <= 2) MOE_DOTS(2);
+    else if (n_live <= 4) MOE_DOTS(4);
+    else MOE_DOTS(8);
+#undef MOE_DOTS
+    if (lane == 0) {
 #pragma unroll
-        for (int r = 0; r < OUT; ++r)
+      for (int r = 0; r < OUT; ++r)
 #pragma unroll
-          for (int p = 0; p < NP; ++p)
-            if (n0 + r < N && p < n_live) {
-              const int pair = s_pairs[p];
-              const size_t at = (size_t)pair * N + n0 + r;
-              if (FORM == MOE_DOWN) {
-                ((float*)out)[at] = a.scale_input ? z[r][p] : z[r][p] * wts[pair];
-              } else if (FORM == MOE_GATED) {
-                st<T>((T*)out + at, moe_gate(z[r][p], z[(r + OUT) % MOE_ROWS][p], a.kind, a.limit, a.alpha));
-              } else {
-                const float v = fmaxf(z[r][p], 0.f);
-                st<T>((T*)out + at, v * v);
-              }
+        for (int p = 0; p < MOE_PAIRS; ++p)
+          if (n0 + r < N && p < n_live) {
+            const size_t at = (size_t)pairs[p] * N + n0 + r;
+            if (FORM == MOE_DOWN) {
+              ((float*)out)[at] = a.scale_input ? z[r][p] : z[r][p] * s[p];
+            } else if (FORM == MOE_GATED) {
+              st<T>((T*)out + at, moe_gate(z[r][p], z[(r + OUT) % MOE_ROWS][p], a.kind, a.limit, a.alpha));
+            } else {
+              const float v = fmaxf(z[r][p], 0.f);
+              st<T>((T*)out + at, v * v);
             }
-      }
+          }
     }
-    __syncthreads();      // the rows and the list are read to the end before the next round writes them
   }
 }
 
@@ -428,35 +424,23 @@ __global__ void moe_sum_pairs_kernel(const float* __restrict__ part, float* __re
   }
 }
 
-template <typename T, bool VEC, int NP, int FORM>
-static void launch_expert_rows(const void* in, const int* ids, const float* wts, const void* w, void* out, const void* self, const MoeRows& a,
-                               hipStream_t stream) {
+template <typename T, bool VEC, int FORM>
+static void expert_rows(const void* in, const int* ids, const float* wts, const void* w, void* out, const void* self, const MoeRows& a,
+                        hipStream_t stream) {
   const int each = 4 * (FORM == MOE_GATED ? MOE_ROWS / 2 : MOE_ROWS);
   const dim3 grid(a.E + (FORM == MOE_DOWN && self ? 1 : 0), (a.N + each - 1) / each);
-  moe_expert_rows_kernel<T, VEC, NP, FORM><<<grid, 256, (size_t)NP * a.K * sizeof(T), stream>>>((const T*)in, ids, wts, (const T*)w, out,
-                                                                                                 (const T*)self, a);
-}
-template <typename T, bool VEC, int FORM>
-static int expert_rows(const void* in, const int* ids, const float* wts, const void* w, void* out, const void* self, const MoeRows& a,
-                       hipStream_t stream) {
-  const size_t row = (size_t)a.K * sizeof(T), room = 48 * 1024;      // rows of the pairs a round holds in LDS
-  if (4 * row <= room) launch_expert_rows<T, VEC, 4, FORM>(in, ids, wts, w, out, self, a, stream);
-  else if (2 * row <= room) launch_expert_rows<T, VEC, 2, FORM>(in, ids, wts, w, out, self, a, stream);
-  else if (row <= 64 * 1024) launch_expert_rows<T, VEC, 1, FORM>(in, ids, wts, w, out, self, a, stream);
-  else return 1;
-  return 0;
+  moe_expert_rows_kernel<T, VEC, FORM><<<grid, 256, 0, stream>>>((const T*)in, ids, wts, (const T*)w, out, (const T*)self, a);
 }
 
 // both products of all pairs: act (T) [n_pairs][F], part f32 [n_pairs][W]
 template <typename T, bool VEC, int UP>
-static int experts_rows(const void* h, const int* ids, const float* wts, const void* up, const void* down, void* act, float* part, int M, int W,
+static void experts_rows(const void* h, const int* ids, const float* wts, const void* up, const void* down, void* act, float* part, int M, int W,
                         int F, int E, int top, int scale_input, int identity, int kind, float limit, float alpha, hipStream_t stream) {
   MoeRows a = {M * top, W, F, top, scale_input, E, kind, limit, alpha};
-  int rc = expert_rows<T, VEC, UP>(h, ids, wts, up, act, nullptr, a, stream);
+  expert_rows<T, VEC, UP>(h, ids, wts, up, act, nullptr, a, stream);
   a.K = F;
   a.N = W;
-  if (rc == 0) rc = expert_rows<T, VEC, MOE_DOWN>(act, ids, wts, down, part, identity ? h : nullptr, a, stream);
-  return rc;
+  expert_rows<T, VEC, MOE_DOWN>(act, ids, wts, down, part, identity ? h : nullptr, a, stream);
 }
 
 template <int UP>
@@ -469,8 +453,7 @@ static int experts_rows_any(int dtype, const void* h, const int* ids, const floa
   TI_REQUIRE((F + 7) / 8 <= 65535 && (W + 15) / 16 <= 65535, "moe_experts: sizes W=%d F=%d are too large", W, F);
   const int piece = 16 / (dtype == TI_F32 ? 4 : 2);
   const bool vec = W % piece == 0 && F % piece == 0 && (((uintptr_t)up | (uintptr_t)down | (uintptr_t)act | (uintptr_t)h) & 15) == 0;
-  int rc;
-#define MOE_BOTH(T, V) rc = experts_rows<T, V, UP>(h, ids, wts, up, down, act, part, M, W, F, E, top, scale_input, identity, kind, limit, alpha, stream)
+#define MOE_BOTH(T, V) experts_rows<T, V, UP>(h, ids, wts, up, down, act, part, M, W, F, E, top, scale_input, identity, kind, limit, alpha, stream)
   if (dtype == TI_F32) {
     if (vec) MOE_BOTH(float, true);
     else MOE_BOTH(float, false);
@@ -479,7 +462,6 @@ static int experts_rows_any(int dtype, const void* h, const int* ids, const floa
     else MOE_BOTH(bf16_t, false);
   }
 #undef MOE_BOTH
-  TI_REQUIRE(rc == 0, "moe_experts: a row of %d or %d entries does not fit the workgroup's 64 KB", W, F);
   if (y) moe_sum_pairs_kernel<<<M, 256, 0, stream>>>(part, y, W, top);
   TI_LAUNCH_CHECK();
   return 0;

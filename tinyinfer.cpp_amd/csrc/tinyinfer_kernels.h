@@ -382,8 +382,8 @@ int ti_moe_route_gate(int dtype, const void* h, const float* router, const float
                       int top, int score_kind, int renormalize, int n_groups, int keep, float weight_scale, float sum_floor,
                       const float* gate_row, float* gate_out, hipStream_t stream);
 // y f32 [M, W] = sum_k down[e_k] relu(up[e_k] (s_k h))^2 (scale_input) or sum_k s_k down[e_k] relu(up[e_k] h)^2;
-// up [E][F][W], down [E][W][F] in the dtype of h; act: scratch of that dtype, [M top][F]; part: f32 [M top][W].  A workgroup
-// per expert and 16 outputs walks its weights once for all the pairs that chose the expert: steps of few tokens, and float32.
+// up [E][F][W], down [E][W][F] in the dtype of h; act: scratch of that dtype, [M top][F]; part: f32 [M top][W].  A wavefront
+// per expert and a few outputs walks its weights once for every eight pairs that chose the expert: steps of few tokens, and float32.
 // A token's rows of part are added in ascending order into y where y is given, else left to the caller.  identity: ids from E on
 // are identity experts, their row of part is s_k h
 int ti_moe_experts_rows(int dtype, const void* h, const int* ids, const float* wts, const void* up, const void* down, void* act,

@@ -1861,7 +1861,7 @@ class MoE final : public FeedForwardPart {
       TensorNeed c;
       c.shape = {(int64_t)experts + identity};
       c.role = TensorNeed::Vector;
-      c.b = 0.3;
+      c.b = score == Ops::Softmax ? 0.3 / (experts + identity) : 0.3;      // of the size of the scores it joins, or smaller
       t.emplace_back(n_correction, c);
     }
     return t;
