@@ -255,14 +255,14 @@ extern "C" int ti_moe_route_gate(int dtype, const void* h, const float* router, 
 
 // ------------------------------------------------------------ the experts, an output a wavefront
 // up [E][F][W], down [E][W][F] in T.  Two kernels, a wavefront per (expert, a few outputs), on its own from beginning to end: it
-// finds the pairs (token, choice) of its expert, up to eight at a time, and walks its rows of the weight once for all of them: an
-// expert's weights are read once a step for every eight tokens that chose it.
+// finds the pairs (token, choice) of its expert, up to four at a time, and walks its rows of the weight once for all of them: an
+// expert's weights are read once a step for every four tokens that chose it.
 //   act[pair][f] = relu(up[e][f] . (s h[token]))^2 rounded to T;   part[pair][c] = down[e][c] . act[pair]
 // and a token's rows of `part` are added in the order its experts were chosen by whoever reads them (moe_sum_pairs, or the
 // norm that follows).  A wavefront owns four rows of the weight; its lanes share a row in pieces of 16 bytes (lane l the
 // pieces l, l + 64, ... in ascending order, then a butterfly): the order of every sum is fixed, whatever else the step holds.
 #define MOE_ROWS 4      // rows of the weight a wavefront
-#define MOE_PAIRS 8     // pairs at a time
+#define MOE_PAIRS 4     // pairs at a time
 
 // the next pairs of expert e from pair `next` on, at most MOE_PAIRS: lane p gets the p-th one's index; returns how many, `next` goes on
 __device__ __forceinline__ int next_pairs(const int* __restrict__ ids, int n_pairs, int e, int lane, int& next, int& mine) {
@@ -301,8 +301,7 @@ __device__ __forceinline__ void wave_dots(const T* const* rows, const float* s, 
 #pragma unroll
     for (int p = 0; p < NP; ++p) z[r][p] = 0.f;
   constexpr int N = VEC ? Piece<T>::N : 1;
-  constexpr int AHEAD = NP <= 4 ? 2 : 1;
-#pragma unroll AHEAD
+#pragma unroll 2
   for (int c = lane * N; c < K; c += 64 * N) {
     float v[MOE_ROWS][N], a[NP][N];
 #pragma unroll
@@ -347,7 +346,7 @@ __device__ __forceinline__ float moe_gate(float g, float u, int kind, float limi
 // pairs' rows of part, the score times the token's row of `self`.
 struct MoeRows { int n_pairs, K, N, top, scale_input, E, kind; float limit, alpha; };
 template <typename T, bool VEC, int FORM>
-__global__ void __launch_bounds__(256, 3)
+__global__ void __launch_bounds__(256)
 moe_expert_rows_kernel(const T* __restrict__ in, const int* __restrict__ ids, const float* __restrict__ wts, const T* __restrict__ w,
                        void* __restrict__ out, const T* __restrict__ self, const MoeRows a) {
   const int e = blockIdx.x, K = a.K, N = a.N;
@@ -390,9 +389,8 @@ moe_expert_rows_kernel(const T* __restrict__ in, const int* __restrict__ ids, co
     if (FORM == MOE_UP && a.scale_input) wave_dots<T, VEC, NP, true>(rows, s, br, K, lane, z);               \
     else wave_dots<T, VEC, NP, false>(rows, s, br, K, lane, z);                                              \
   } while (0)
-    if (n_live <= 2) MOE_DOTS(2);
-    else if (n_live <= 4) MOE_DOTS(4);
-    else MOE_DOTS(8);
+    if (n_live == 1) MOE_DOTS(1);
+    else MOE_DOTS(MOE_PAIRS);
 #undef MOE_DOTS
     if (lane == 0) {
 #pragma unroll
@@ -463,6 +461,15 @@ static int experts_rows_any(int dtype, const void* h, const int* ids, const floa
   }
 #undef MOE_BOTH
   if (y) moe_sum_pairs_kernel<<<M, 256, 0, stream>>>(part, y, W, top);
+  TI_LAUNCH_CHECK();
+  return 0;
+}
+
+// y[m] = the sum of a token's rows of part f32 [M top][W], in ascending order
+extern "C" int ti_moe_sum_pairs(const float* part, float* y, int M, int W, int top, hipStream_t stream) {
+  TI_REQUIRE(M >= 0 && W > 0 && top > 0, "moe_sum_pairs: bad sizes M=%d W=%d top=%d", M, W, top);
+  if (M == 0) return 0;
+  moe_sum_pairs_kernel<<<M, 256, 0, stream>>>(part, y, W, top);
   TI_LAUNCH_CHECK();
   return 0;
 }

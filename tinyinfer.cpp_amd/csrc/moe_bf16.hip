@@ -1,4 +1,5 @@
-// The experts of a mixture of experts for steps of many tokens, bfloat16 on the matrix cores of gfx950.
+// The experts of a mixture of experts, bfloat16 on the matrix cores of gfx950.  Steps of few tokens: moe_few (at the end of this
+// file).  Steps of many tokens:
 //
 //   1. moe_group: counts the (token, expert) pairs of every expert, lays the experts' runs of rows one after
 //      the other and cuts them into tiles of 128 rows: offsets, the list of tiles, cursors at zero.
@@ -302,6 +303,140 @@ extern "C" int ti_moe_experts_grouped_bf16(const void* h, const int* ids, const 
   if (scale_input) moe_grouped_kernel<1><<<grid_down, 256, 0, stream>>>((const bf16_t*)act, (const bf16_t*)down, meta, R, out, W, F);
   else moe_grouped_kernel<2><<<grid_down, 256, 0, stream>>>((const bf16_t*)act, (const bf16_t*)down, meta, R, out, W, F, row_w);
   if (y) moe_combine_kernel<<<M, 256, 0, stream>>>(out, where, y, W, top);
+  TI_LAUNCH_CHECK();
+  return 0;
+}
+
+// ------------------------------------------------------------ steps of few tokens
+// A workgroup per (expert, 16 outputs): the expert's rows of the weight are the A operand of v_mfma_f32_16x16x32_bf16, up to sixteen
+// of the pairs that chose it the columns; both come straight from memory in their own layouts.  The four wavefronts take the steps
+// of 32 along k in turn, eight of a wavefront's in flight together; their sums are added in LDS in a fixed order.  A workgroup
+// whose expert nobody chose ends at once; more than sixteen pairs take another round.
+//   FORM 0: act = relu(up (s h))^2 (s 1 unless the score scales the input), 1: act = the gated activation of (gate h, up h) (w
+// [E][2 N][K], gate rows above up rows), 2: part = s down act, or down act where the score was in the input.
+// ids from E on are identity experts: FORM 2's workgroups of blockIdx.x = E write their pairs' rows, s self[token].
+#define FEW_AHEAD 8
+struct MoeFew { int n_pairs, K, N, top, scale_input, E, kind; float limit, alpha; };
+template <int FORM, bool SCALED>
+__global__ void __launch_bounds__(256)
+moe_few_kernel(const bf16_t* __restrict__ in, const int* __restrict__ ids, const float* __restrict__ wts, const bf16_t* __restrict__ w,
+               void* __restrict__ out, const bf16_t* __restrict__ self, const MoeFew a) {
+  constexpr int SETS = FORM == 1 ? 2 : 1;      // runs of 16 rows of the weight
+  __shared__ int s_pairs[4][16];
+  __shared__ float s_sum[4][SETS][256];
+  const int e = blockIdx.x, K = a.K, N = a.N;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, quad = lane >> 4;
+  if (FORM == 2 && e == a.E) {
+    for (int pair = blockIdx.y; pair < a.n_pairs; pair += gridDim.y) {
+      if (ids[pair] < a.E) continue;
+      const float s = wts[pair];
+      for (int c = threadIdx.x; c < N; c += 256) ((float*)out)[(size_t)pair * N + c] = bf2f(self[(size_t)(pair / a.top) * N + c]) * s;
+    }
+    return;
+  }
+  const int n0 = blockIdx.y * 16, steps = K / 32;
+  const bf16_t* src_w[SETS];
+#pragma unroll
+  for (int x = 0; x < SETS; ++x) src_w[x] = w + ((size_t)e * SETS * N + (size_t)x * N + min(n0 + r16, N - 1)) * K + quad * 8;
+  for (int base = 0;; base += 16) {
+    // the expert's pairs base .. base + 15, every wavefront for itself
+    int n_live = 0;
+    for (int i = 0; i < a.n_pairs; i += 64) {
+      const bool hit = i + lane < a.n_pairs && ids[i + lane] == e;
+      const unsigned long long mask = __ballot(hit);
+      const int rank = n_live + __popcll(mask & ((1ull << lane) - 1ull)) - base;
+      if (hit && rank >= 0 && rank < 16) s_pairs[wave][rank] = i + lane;
+      n_live += __popcll(mask);
+    }
+    n_live = min(16, n_live - base);
+    if (n_live <= 0) return;      // (the same in all four)
+    __builtin_amdgcn_wave_barrier();
+    __threadfence_block();
+    const int mine = s_pairs[wave][r16 < n_live ? r16 : 0];      // (columns beyond the last pair: the first one again, not written)
+    const bf16_t* src_p = in + (size_t)(FORM == 2 ? mine : mine / a.top) * K + quad * 8;
+    const float s = SCALED ? wts[mine] : 1.f;
+    floatx4 acc[SETS];
+#pragma unroll
+    for (int x = 0; x < SETS; ++x) acc[x] = floatx4{0.f, 0.f, 0.f, 0.f};
+    for (int step = wave; step < steps; step += 4 * FEW_AHEAD) {
+      Frag8 fw[FEW_AHEAD][SETS], fp[FEW_AHEAD];
+#pragma unroll
+      for (int j = 0; j < FEW_AHEAD; ++j) {
+        const int k = min(step + 4 * j, steps - 1) * 32;      // (a step that is not there: the last one's operands, not multiplied)
+#pragma unroll
+        for (int x = 0; x < SETS; ++x) fw[j][x].u = *reinterpret_cast<const uint4*>(src_w[x] + k);
+        fp[j].u = *reinterpret_cast<const uint4*>(src_p + k);
+      }
+#pragma unroll
+      for (int j = 0; j < FEW_AHEAD; ++j) {
+        if (step + 4 * j >= steps) break;
+        if (SCALED) {
+          const unsigned v[4] = {fp[j].u.x, fp[j].u.y, fp[j].u.z, fp[j].u.w};
+          unsigned o[4];
+#pragma unroll
+          for (int i = 0; i < 4; ++i) o[i] = pack_bf16x2(__uint_as_float(v[i] << 16) * s, __uint_as_float(v[i] & 0xffff0000u) * s);
+          fp[j].u = make_uint4(o[0], o[1], o[2], o[3]);
+        }
+#pragma unroll
+        for (int x = 0; x < SETS; ++x) acc[x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fw[j][x].v, fp[j].v, acc[x], 0, 0, 0);
+      }
+    }
+    // lane: outputs 4 quad + i of column r16
+#pragma unroll
+    for (int x = 0; x < SETS; ++x) *reinterpret_cast<floatx4*>(&s_sum[wave][x][lane * 4]) = acc[x];
+    __syncthreads();
+    const int row = threadIdx.x & 15, col = threadIdx.x >> 4;
+    const int at = ((row >> 2) * 16 + col) * 4 + (row & 3);
+    float z[SETS];
+#pragma unroll
+    for (int x = 0; x < SETS; ++x) z[x] = ((s_sum[0][x][at] + s_sum[1][x][at]) + s_sum[2][x][at]) + s_sum[3][x][at];
+    if (col < n_live && n0 + row < N) {
+      const int pair = s_pairs[wave][col];
+      const size_t to = (size_t)pair * N + n0 + row;
+      if (FORM == 0) {
+        const float v = fmaxf(z[0], 0.f);
+        ((bf16_t*)out)[to] = f2bf(v * v);
+      } else if (FORM == 1) {
+        float g = z[0], u = z[SETS - 1];
+        if (a.kind == 0) {
+          g = g / (1.0f + expf(-g)) * u;
+        } else {
+          g = fminf(g, a.limit);
+          u = fminf(fmaxf(u, -a.limit), a.limit);
+          g = g / (1.0f + expf(-a.alpha * g)) * (u + 1.0f);
+        }
+        ((bf16_t*)out)[to] = f2bf(g);
+      } else {
+        ((float*)out)[to] = a.scale_input ? z[0] : z[0] * wts[pair];
+      }
+    }
+    __syncthreads();      // sums and pairs are read to the end before the next round writes them
+  }
+}
+
+// the same contract as ti_moe_experts_rows (act_kind < 0: relu^2) / ti_moe_experts_rows_gated for bfloat16 and W, F multiples of 32
+// (3: sizes not served); part f32 [M top][W], a token's rows to be added by the caller
+extern "C" int ti_moe_experts_few_bf16(const void* h, const int* ids, const float* wts, const void* up, const void* down, void* act, float* part,
+                                       int M, int W, int F, int E, int top, int scale_input, int act_kind, float limit, float alpha, int identity,
+                                       hipStream_t stream) {
+  if (W % 32 || F % 32 || (((uintptr_t)h | (uintptr_t)up | (uintptr_t)down | (uintptr_t)act) & 15) != 0 || (W + 15) / 16 > 65535 || (F + 15) / 16 > 65535) {
+    ti_set_error("moe_experts (few): W=%d, F=%d are not served", W, F);
+    return 3;
+  }
+  TI_REQUIRE(M >= 0 && top > 0 && E > 0 && act_kind <= 1 && !(act_kind >= 0 && scale_input), "moe_experts (few): bad arguments");
+  if (M == 0) return 0;
+  MoeFew a = {M * top, W, F, top, scale_input, E, act_kind, limit, alpha};
+  const dim3 grid_up(E, (F + 15) / 16);
+  if (act_kind >= 0)
+    moe_few_kernel<1, false><<<grid_up, 256, 0, stream>>>((const bf16_t*)h, ids, wts, (const bf16_t*)up, act, nullptr, a);
+  else if (scale_input)
+    moe_few_kernel<0, true><<<grid_up, 256, 0, stream>>>((const bf16_t*)h, ids, wts, (const bf16_t*)up, act, nullptr, a);
+  else
+    moe_few_kernel<0, false><<<grid_up, 256, 0, stream>>>((const bf16_t*)h, ids, wts, (const bf16_t*)up, act, nullptr, a);
+  a.K = F;
+  a.N = W;
+  moe_few_kernel<2, false><<<dim3(E + (identity ? 1 : 0), (W + 15) / 16), 256, 0, stream>>>((const bf16_t*)act, ids, wts, (const bf16_t*)down, part,
+                                                                                          (const bf16_t*)h, a);
   TI_LAUNCH_CHECK();
   return 0;
 }

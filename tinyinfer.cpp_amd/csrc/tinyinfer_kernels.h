@@ -383,7 +383,7 @@ int ti_moe_route_gate(int dtype, const void* h, const float* router, const float
                       const float* gate_row, float* gate_out, hipStream_t stream);
 // y f32 [M, W] = sum_k down[e_k] relu(up[e_k] (s_k h))^2 (scale_input) or sum_k s_k down[e_k] relu(up[e_k] h)^2;
 // up [E][F][W], down [E][W][F] in the dtype of h; act: scratch of that dtype, [M top][F]; part: f32 [M top][W].  A wavefront
-// per expert and a few outputs walks its weights once for every eight pairs that chose the expert: steps of few tokens, and float32.
+// per expert and a few outputs walks its weights once for every four pairs that chose the expert: steps of few tokens, and float32.
 // A token's rows of part are added in ascending order into y where y is given, else left to the caller.  identity: ids from E on
 // are identity experts, their row of part is s_k h
 int ti_moe_experts_rows(int dtype, const void* h, const int* ids, const float* wts, const void* up, const void* down, void* act,
@@ -396,7 +396,15 @@ int ti_moe_experts_rows_gated(int dtype, const void* h, const int* ids, const fl
                               void* act, float* part, float* y, int M, int W, int F, int E, int top, int act_kind, float limit,
                               float alpha, int identity, hipStream_t stream);
 
-// ---- libti_moe_bf16: the experts for steps of many tokens, on the matrix cores: the (token, expert) pairs are laid out expert
+// y[m] = the sum of a token's rows of part f32 [M top][W], in ascending order
+int ti_moe_sum_pairs(const float* part, float* y, int M, int W, int top, hipStream_t stream);
+
+// ---- libti_moe_bf16: steps of few tokens on the matrix cores, straight from memory: as ti_moe_experts_rows (act_kind < 0: relu^2) /
+// ti_moe_experts_rows_gated with y null, bfloat16.  3: sizes not served (W, F multiples of 32)
+int ti_moe_experts_few_bf16(const void* h, const int* ids, const float* wts, const void* up, const void* down, void* act, float* part,
+                            int M, int W, int F, int E, int top, int scale_input, int act_kind, float limit, float alpha, int identity,
+                            hipStream_t stream);
+// the experts for steps of many tokens, on the matrix cores: the (token, expert) pairs are laid out expert
 // by expert in tiles of 128 rows and both products run over the tiles.  Scratch: meta int32 [ti_moe_grouped_meta_ints(M top, E)],
 // where int32 [M top] (the row of every pair), rows bf16 [M top][W], act bf16 [M top][F], out f32 [M top][W].  y (may be
 // null): the tokens' sums; without it the caller adds the rows out[where[m top + k]] in ascending k.  The weights multiply the

@@ -1746,21 +1746,36 @@ void Ops::experts_of(const char* name, const Tensor& h, const Tensor& ids, const
     }
     if (rc != 3) check("moe_bf16", rc, (what + "(grouped)").c_str());
   }
-  took(rows && top > 1 ? "[rows, sums left]" : "[rows]");
   Tensor act = ws.tensor("moe.act", h.dtype, {pairs, F});
   // one expert a token: its row is the result; else the pairs' rows, added by this call or left to the norm that reads them
   Tensor part = top == 1 ? y : ws.tensor("moe.out", DType::F32, {pairs, W});
   const bool left = rows && top > 1;
   float* sums = (top == 1 || left) ? nullptr : (float*)y.data;
-  int rc;
-  if (gated)
-    rc = KERNEL("moe", ti_moe_experts_rows_gated)(code(h.dtype, name), h.data, (const int*)ids.data, (const float*)wts.data, up.data,
-                                                  down.data, act.data, (float*)part.data, sums, (int)M, (int)W, (int)F, experts, top,
-                                                  (int)kind, limit, alpha, identity > 0 ? 1 : 0, (hipStream_t)launch_stream());
-  else
-    rc = KERNEL("moe", ti_moe_experts_rows)(code(h.dtype, name), h.data, (const int*)ids.data, (const float*)wts.data, up.data, down.data,
-                                            act.data, (float*)part.data, sums, (int)M, (int)W, (int)F, experts, top, scale_input ? 1 : 0,
-                                            identity > 0 ? 1 : 0, (hipStream_t)launch_stream());
+  int rc = 3;
+  if (h.dtype == DType::BF16 && use.fast_gemm && kernel_library_available("moe_bf16")) {
+    rc = KERNEL("moe_bf16", ti_moe_experts_few_bf16)(h.data, (const int*)ids.data, (const float*)wts.data, up.data, down.data, act.data,
+                                                     (float*)part.data, (int)M, (int)W, (int)F, experts, top, scale_input ? 1 : 0,
+                                                     gated ? (int)kind : -1, limit, alpha, identity > 0 ? 1 : 0, (hipStream_t)launch_stream());
+    if (rc != 3) check("moe_bf16", rc, (what + "(few)").c_str());
+    if (rc == 0) {
+      took(left ? "[mfma, rows, sums left]" : "[mfma, rows]");
+      if (sums) {
+        rc = KERNEL("moe", ti_moe_sum_pairs)((const float*)part.data, sums, (int)M, (int)W, top, (hipStream_t)launch_stream());
+        check("moe", rc, (what + "(sum)").c_str());
+      }
+    }
+  }
+  if (rc == 3) {
+    took(left ? "[rows, sums left]" : "[rows]");
+    if (gated)
+      rc = KERNEL("moe", ti_moe_experts_rows_gated)(code(h.dtype, name), h.data, (const int*)ids.data, (const float*)wts.data, up.data,
+                                                    down.data, act.data, (float*)part.data, sums, (int)M, (int)W, (int)F, experts, top,
+                                                    (int)kind, limit, alpha, identity > 0 ? 1 : 0, (hipStream_t)launch_stream());
+    else
+      rc = KERNEL("moe", ti_moe_experts_rows)(code(h.dtype, name), h.data, (const int*)ids.data, (const float*)wts.data, up.data, down.data,
+                                              act.data, (float*)part.data, sums, (int)M, (int)W, (int)F, experts, top, scale_input ? 1 : 0,
+                                              identity > 0 ? 1 : 0, (hipStream_t)launch_stream());
+  }
   check("moe", rc, name);
   if (left) {
     rows->t = part;
