@@ -63,7 +63,8 @@ scan_tokens_kernel(const ti_scan_inputs in, float* __restrict__ state, long slot
                    float* __restrict__ o, int heads, int dk, int dv, int dvs, int dvp) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int h = blockIdx.y, hq = h / (heads / in.qk_heads);
-  const int row0 = entry_meta[4 * blockIdx.x], n = entry_meta[4 * blockIdx.x + 1], slot = entry_meta[4 * blockIdx.x + 3];
+  const int* entry = entry_meta + 4 * blockIdx.x;
+  const int row0 = entry[0], n = entry[1], start = entry[2], slot = entry[3];
   const int RG = NT / dvp;
   const int dkp = RPT * RG;
   const int j = threadIdx.x % dvp, rg = threadIdx.x / dvp;
@@ -89,11 +90,10 @@ scan_tokens_kernel(const ti_scan_inputs in, float* __restrict__ state, long slot
     for (int x = threadIdx.x; x < nt * width; x += NT) {
       const int tt = x / width, c = x % width, m = row0 + t0 + tt;
       const float* row = in.proj + (size_t)m * in.ld;
-      const int p = FORM == SCAN_ROTATED && in.rot_dims ? in.pos[m] : 0;
       if (c < 2 * dkp) {
         const bool is_q = c < dkp;
         const int i = is_q ? c : c - dkp;
-        const float e = i < dk ? scan_entry<FORM>(in, row + (is_q ? in.off_q : in.off_k) + hq * dk, i, p) : 0.f;
+        const float e = i < dk ? scan_entry<FORM>(in, row + (is_q ? in.off_q : in.off_k) + hq * dk, i, start + t0 + tt) : 0.f;
         (is_q ? s_q : s_k)[tt * dkp + i] = is_q ? e : e * in.k_scale;
       } else {
         const int i = c - 2 * dkp;
@@ -497,11 +497,11 @@ static int launch_scan(int rpt, dim3 grid, size_t lds, hipStream_t stream, const
   return 1;
 }
 
-// wide states are cut into slices of 64 columns, a workgroup each: more workgroups, and fewer rows a thread
+// wide states are cut into slices of 32 columns, a workgroup each: more workgroups, and fewer rows a thread
 struct ScanShape { int dvs, slices, dvp, rpt; size_t lds; };
 static ScanShape scan_shape(int dk, int dv) {
   ScanShape s;
-  s.dvs = dv > 64 ? 64 : dv;
+  s.dvs = dv > 32 ? 32 : dv;
   s.slices = (dv + s.dvs - 1) / s.dvs;
   s.dvp = 1;
   while (s.dvp < s.dvs) s.dvp *= 2;

@@ -170,15 +170,11 @@ moe_route_kernel(const T* __restrict__ h, const float* __restrict__ router, int*
         at = e;
       }
     }
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ob = __shfl_xor(best, o, 64);
-      const int oa = __shfl_xor(at, o, 64);
-      if (ob > best || (ob == best && oa < at)) {
-        best = ob;
-        at = oa;
-      }
-    }
+    // the largest of all lanes, then the lowest index among those that hold it (indices are exact in 32-bit floats)
+    const float largest = group_max<64>(best);
+    const float low = -group_max<64>(best == largest && at < E ? -(float)at : -2048.f);
+    best = largest;
+    at = low < 2048.f ? (int)low : 0x7fffffff;
     if (at >= E) at = k;      // no score compares as larger (not a number): an expert that exists all the same
     if (corrected) best = s_plain[at];
     if (lane == 0) {
