@@ -802,6 +802,12 @@ class MixerPart : public Part { public: using Part::Part; const char* family() c
   virtual bool can_store() const { return false; }
   virtual void forward_store(StepContext& ctx, const Rows& h, const Tensor& y);
   virtual bool takes_lazy_norm() const { return false; }         // h goes into exactly one Ops::linear
+  // a mixer that begins with one product of h and a stacked weight of so many rows (0: it does not) can take that product's result
+  // instead of h: columns col .. of proj f32 [M, N] (a mixer of several then does the products of all as one).  The weight's rows
+  // are then part of another tensor, handed over before load()
+  virtual int64_t input_rows() const { return 0; }
+  virtual void adopt_input(const Tensor& rows) {}
+  virtual void forward_projected(StepContext& ctx, const Tensor& proj, int col, const Tensor& y);
   // a mixer whose output is f1 y1 + f2 y2 may leave the two apart for a reader that adds them on its way (an arrangement that
   // scales or mixes outputs anyway): y1, y2 f32 [M, H]
   virtual bool leaves_pair() const { return false; }

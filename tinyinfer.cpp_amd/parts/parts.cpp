@@ -138,6 +138,9 @@ Rows NormPart::forward_mixed(StepContext&, const Tensor&, const Tensor&) {
 void MixerPart::forward_pair(StepContext&, const Rows&, const Tensor&, const Tensor&, float&, float&) {
   throw EngineError(std::string("the mixer '") + kind_name() + "' does not leave its output as a pair");
 }
+void MixerPart::forward_projected(StepContext&, const Tensor&, int, const Tensor&) {
+  throw EngineError(std::string("the mixer '") + kind_name() + "' does not begin with a product that can be taken out of it");
+}
 void MixerPart::forward_store(StepContext&, const Rows&, const Tensor&) {
   throw EngineError(std::string("the mixer '") + kind_name() + "' cannot write its output apart from the residual");
 }
@@ -545,6 +548,7 @@ class SwiGLU final : public FeedForwardPart {
 };
 
 void put_floats(const Tensor& dst, const std::vector<float>& values, bool on_host);      // dst (device or host memory) = values
+void put_zeros(const Tensor& dst, bool on_host);
 
 const int PREFILL_TILE_Q = 128;      // query rows per work item of the tiled attention kernels
 const int PREFILL_TILE_SMALL = 64;   // and of the kernel that pairs a tile of many keys with one of few
@@ -719,7 +723,7 @@ class Attention final : public MixerPart {
     }
     // q, k and v go straight into the fused matrix (the reference builds its fused copy beside the
     // originals and keeps both: /root/reference/src/inference.cu:154-169)
-    w_qkv = src.alloc(src.matrix_dtype, {nq + nk + nv + ng, hidden});      // the gate's rows behind q, k and v: one product
+    w_qkv = adopted.defined() ? adopted : src.alloc(src.matrix_dtype, {nq + nk + nv + ng, hidden});      // the gate's rows behind q, k and v: one product
     src.fill(n_q, w_qkv.rows(0, nq));
     if (!shares_kv) {
       src.fill(n_k, w_qkv.rows(nq, nk));
@@ -858,9 +862,12 @@ class Attention final : public MixerPart {
   // [q; k; v; gate] (32-bit sums), the preparation (per-head norms, rotation, the values' mixing, q out, k and v into the
   // pages), attention with the sink in the denominator and the gate on its output, then the output projection.
   void run_gated(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
-    const int64_t M = h.t.shape[0];
-    Tensor proj = ctx.buf("attn.qkv", DType::F32, {M, nq + nk + nv + ng});
+    Tensor proj = ctx.buf("attn.qkv", DType::F32, {h.t.shape[0], nq + nk + nv + ng});
     ctx.ops.linear(h, w_qkv, proj, Ops::Store);
+    run_gated(ctx, proj, 0, out, epi);
+  }
+  void run_gated(StepContext& ctx, const Tensor& proj, int col, const Tensor& out, Ops::Epilogue epi) {
+    const int64_t M = proj.shape[0];
     const auto bound = ctx.binding(this);
     const Tensor pool = ctx.kv_pool(bound.first, bound.second);
     const Ops::CacheView view = ctx.cache_view(bound.first);
@@ -868,9 +875,9 @@ class Attention final : public MixerPart {
     Ops::Rotation rot;
     if (pos && !pos->fused(rot)) throw EngineError("attention: the position encoding '" + std::string(pos->kind_name()) + "' has no fused form");
     Ops::QkvColumns cols;
-    cols.q = 0;
-    cols.k = (int)nq;
-    cols.v = values_from_keys ? -1 : (int)(nq + nk);
+    cols.q = col;
+    cols.k = col + (int)nq;
+    cols.v = values_from_keys ? -1 : col + (int)(nq + nk);
     Ops::ValueMix mix;
     mix.mode = mix_mode;
     if (mix_mode) {
@@ -883,11 +890,17 @@ class Attention final : public MixerPart {
     Ops::AttentionGate gate;
     gate.mode = gate_mode;
     gate.proj = proj;
-    gate.col = (int)(nq + nk + nv);
+    gate.col = col + (int)(nq + nk + nv);
     const AttentionWork w = work(ctx);
     ctx.ops.gated_attention(q, pool, view, ctx.positions, ctx.slots, sink, gate, a, heads, kv_heads, head_dim, v_dim, scale, window,
                             ctx.plan ? &w : nullptr, &ctx.ws);
     ctx.ops.linear(a, w_o, out, epi, epi == Ops::Add);
+  }
+  int64_t input_rows() const override { return gated ? nq + nk + nv + ng : 0; }
+  void adopt_input(const Tensor& rows) override { adopted = rows; }
+  void forward_projected(StepContext& ctx, const Tensor& proj, int col, const Tensor& y) override {
+    if (!gated) return MixerPart::forward_projected(ctx, proj, col, y);
+    run_gated(ctx, proj, col, y, Ops::Store);
   }
   void forward_store(StepContext& ctx, const Rows& h, const Tensor& y) override {
     if (!general) return MixerPart::forward_store(ctx, h, y);
@@ -974,7 +987,7 @@ class Attention final : public MixerPart {
   float eps = 1e-6f, scale = 1.f, softcap = 0.f, temp_coef = 0.f;
   std::string n_q, n_k, n_v, n_o;
   std::shared_ptr<PositionPart> pos;
-  Tensor w_qkv, w_o, q_norm_w, k_norm_w;
+  Tensor w_qkv, w_o, q_norm_w, k_norm_w, adopted;
 };
 
 // x += mixer(norm1(x)); x += ffn(norm2(x)).  The mixer and the feed-forward add into x
@@ -2748,7 +2761,7 @@ class DecayAttention final : public MixerPart {
     return t;
   }
   void load(WeightSource& src) override {
-    w_in = src.alloc(src.matrix_dtype, {width, hidden});
+    w_in = adopted.defined() ? adopted : src.alloc(src.matrix_dtype, {width, hidden});
     src.fill(name("q"), w_in.rows(0, nq));
     src.fill(name("k"), w_in.rows(nq, nq));
     src.fill(name("v"), w_in.rows(2 * nq, nv));
@@ -2778,14 +2791,18 @@ class DecayAttention final : public MixerPart {
                         ctx.planned("scan.chunks"), (int)(ctx.planned_size("scan.chunks") / 4), ctx.planned("scan.spans"), &ctx.ws);
   }
   void run(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
-    const int64_t M = h.t.shape[0];
-    Tensor proj = ctx.buf("decay.proj", DType::F32, {M, width});
+    Tensor proj = ctx.buf("decay.proj", DType::F32, {h.t.shape[0], width});
     ctx.ops.linear(h, w_in, proj, Ops::Store);
+    run(ctx, proj, 0, out, epi);
+  }
+  void run(StepContext& ctx, const Tensor& proj, int col, const Tensor& out, Ops::Epilogue epi) {
+    const int64_t M = proj.shape[0];
     Tensor o = ctx.buf("decay.o", DType::F32, {M, nv});
     Ops::LinearScan in;
     in.rows = proj;
-    in.cols.k = (int)nq;
-    in.cols.v = (int)(2 * nq);
+    in.cols.q = col;
+    in.cols.k = col + (int)nq;
+    in.cols.v = col + (int)(2 * nq);
     in.silu = silu;
     in.k_scale = k_scale;
     in.decay = w_decay;
@@ -2793,9 +2810,12 @@ class DecayAttention final : public MixerPart {
     in.positions = ctx.positions;
     scan(ctx, this, in, o, heads, dk, dv);
     Tensor a = ctx.buf("decay.gated", ctx.act_dtype, {M, nv});
-    ctx.ops.gated_group_norm(o, proj, (int)(2 * nq + nv), norm_w, eps, a, form);
+    ctx.ops.gated_group_norm(o, proj, col + (int)(2 * nq + nv), norm_w, eps, a, form);
     ctx.ops.linear(a, w_o, out, epi, epi == Ops::Add);
   }
+  int64_t input_rows() const override { return width; }
+  void adopt_input(const Tensor& rows) override { adopted = rows; }
+  void forward_projected(StepContext& ctx, const Tensor& proj, int col, const Tensor& y) override { run(ctx, proj, col, y, Ops::Store); }
   void forward(StepContext& ctx, const Rows& h, const Tensor& x) override { run(ctx, h, x, Ops::Add); }
   void forward_store(StepContext& ctx, const Rows& h, const Tensor& y) override { run(ctx, h, y, Ops::Store); }
   std::vector<std::pair<std::string, Tensor>> held() const override {
@@ -2808,7 +2828,7 @@ class DecayAttention final : public MixerPart {
   Ops::GroupNorm form;
   std::shared_ptr<PositionPart> pos;
   std::vector<float> decay;
-  Tensor w_in, w_o, norm_w, w_decay;
+  Tensor w_in, w_o, norm_w, w_decay, adopted;
 };
 
 // A Mamba-2 layer (state-space duality).  W_in h = [z: inner | x: inner | B: groups state | C: groups state | dt: heads], inner =
@@ -2879,7 +2899,11 @@ class Mamba2 final : public MixerPart {
   void load(WeightSource& src) override {
     const auto t = tensors();
     Tensor* const to[] = {&w_in, &w_o, &dt_bias, &a_log, &skip, &norm_w};
-    for (size_t i = 0; i < t.size(); ++i) *to[i] = src.fetch(t[i].first, t[i].second);
+    for (size_t i = adopted.defined() ? 1 : 0; i < t.size(); ++i) *to[i] = src.fetch(t[i].first, t[i].second);
+    if (adopted.defined()) {
+      w_in = adopted;
+      src.fill(t[0].first, w_in);
+    }
   }
   bool has_cache() const override { return true; }
   CacheNeed cache_need() const override {
@@ -2890,11 +2914,14 @@ class Mamba2 final : public MixerPart {
   }
   void plan(StepPlan& plan) const override { plan_chunks(plan, "scan", DecayAttention::CHUNK, DecayAttention::CHUNK_FROM); }
   void run(StepContext& ctx, const Rows& h, const Tensor& out, Ops::Epilogue epi) {
-    const int64_t M = h.t.shape[0], GN = (int64_t)groups * state;
-    Tensor proj = ctx.buf("mamba2.proj", DType::F32, {M, width});
+    Tensor proj = ctx.buf("mamba2.proj", DType::F32, {h.t.shape[0], width});
     ctx.ops.linear(h, w_in, proj, Ops::Store);
+    run(ctx, proj, 0, out, epi);
+  }
+  void run(StepContext& ctx, const Tensor& proj, int col, const Tensor& out, Ops::Epilogue epi) {
+    const int64_t M = proj.shape[0], GN = (int64_t)groups * state;
     Tensor xbc = ctx.buf("mamba2.xbc", DType::F32, {M, channels});
-    conv->forward(ctx, proj.cols(inner, channels), xbc);
+    conv->forward(ctx, proj.cols(col + inner, channels), xbc);
     Tensor y = ctx.buf("mamba2.y", DType::F32, {M, inner});
     Ops::LinearScan in;
     in.rows = xbc;
@@ -2903,15 +2930,18 @@ class Mamba2 final : public MixerPart {
     in.cols.v = 0;
     in.qk_heads = groups;
     in.dt = proj;
-    in.dt_col = (int)(inner + channels);
+    in.dt_col = col + (int)(inner + channels);
     in.dt_bias = dt_bias;
     in.a_log = a_log;
     in.skip = skip;
     DecayAttention::scan(ctx, this, in, y, heads, state, dv);
     Tensor a = ctx.buf("mamba2.gated", ctx.act_dtype, {M, inner});
-    ctx.ops.gated_group_norm(y, proj, 0, norm_w, eps, a, form);
+    ctx.ops.gated_group_norm(y, proj, col, norm_w, eps, a, form);
     ctx.ops.linear(a, w_o, out, epi, epi == Ops::Add);
   }
+  int64_t input_rows() const override { return width; }
+  void adopt_input(const Tensor& rows) override { adopted = rows; }
+  void forward_projected(StepContext& ctx, const Tensor& proj, int col, const Tensor& y) override { run(ctx, proj, col, y, Ops::Store); }
   void forward(StepContext& ctx, const Rows& h, const Tensor& x) override { run(ctx, h, x, Ops::Add); }
   void forward_store(StepContext& ctx, const Rows& h, const Tensor& y) override { run(ctx, h, y, Ops::Store); }
   std::vector<std::pair<std::string, Tensor>> held() const override {
@@ -2922,7 +2952,7 @@ class Mamba2 final : public MixerPart {
   float eps = 1e-6f;
   Ops::GroupNorm form;
   std::shared_ptr<FilterPart> conv;
-  Tensor w_in, w_o, dt_bias, a_log, skip, norm_w;
+  Tensor w_in, w_o, dt_bias, a_log, skip, norm_w, adopted;
 };
 
 // A minimal GRU: an element-wise recurrence over `width` channels whose gate and candidate read the current token only.
@@ -3140,7 +3170,8 @@ class SandwichBlock final : public BlockPart {
 
 // Two mixers side by side on the same input: y = left_scale * left(h) + right_scale * right(h), added in 32-bit.  `left`,
 // `right`: the two mixers as parts ({"kind", "params", "name"}; the name follows this part's prefix); each keeps its own cache
-// or state.
+// or state.  Where both begin with a product of h, the two products are one, with a weight that holds the rows of both (the right
+// mixer's from a multiple of 16 columns on, so that its rows keep their alignment).
 class SumMixer final : public MixerPart {
  public:
   SumMixer(const std::string& prefix, const Json& p, const PartChildren& children) : MixerPart(prefix) {
@@ -3170,12 +3201,32 @@ class SumMixer final : public MixerPart {
     s_right = src.alloc(DType::F32, {dim});
     put_floats(s_left, std::vector<float>((size_t)dim, left_scale), src.to_host);
     put_floats(s_right, std::vector<float>((size_t)dim, right_scale), src.to_host);
+    const int64_t nl = left->input_rows(), nr = right->input_rows();
+    if (nl > 0 && nr > 0) {      // (this part is loaded in front of its children)
+      right_col = (nl + 15) / 16 * 16;
+      width = (right_col + nr + 3) / 4 * 4;      // rows of proj keep their alignment too
+      w_in = src.alloc(src.matrix_dtype, {width, dim});
+      put_zeros(w_in.rows(nl, right_col - nl), src.to_host);
+      put_zeros(w_in.rows(right_col + nr, width - right_col - nr), src.to_host);
+      left->adopt_input(w_in.rows(0, nl));
+      right->adopt_input(w_in.rows(right_col, nr));
+    }
+  }
+  void run_pair(StepContext& ctx, const Rows& h, const Tensor& y1, const Tensor& y2) {
+    if (!w_in.defined()) {
+      left->forward_store(ctx, h, y1);
+      right->forward_store(ctx, h, y2);
+      return;
+    }
+    Tensor proj = ctx.buf("sum.proj", DType::F32, {h.t.shape[0], width});
+    ctx.ops.linear(h, w_in, proj, Ops::Store);
+    left->forward_projected(ctx, proj, 0, y1);
+    right->forward_projected(ctx, proj, (int)right_col, y2);
   }
   void run(StepContext& ctx, const Rows& h, const Tensor& x) {
     const int64_t M = h.t.shape[0];
     Tensor y1 = ctx.buf("sum.left", DType::F32, {M, dim}), y2 = ctx.buf("sum.right", DType::F32, {M, dim});
-    left->forward_store(ctx, h, y1);
-    right->forward_store(ctx, h, y2);
+    run_pair(ctx, h, y1, y2);
     ctx.ops.scaled_add(x, y1, s_left, y2, s_right);
   }
   void forward(StepContext& ctx, const Rows& h, const Tensor& x) override { run(ctx, h, x); }
@@ -3185,14 +3236,15 @@ class SumMixer final : public MixerPart {
   }
   bool leaves_pair() const override { return true; }
   void forward_pair(StepContext& ctx, const Rows& h, const Tensor& y1, const Tensor& y2, float& f1, float& f2) override {
-    left->forward_store(ctx, h, y1);
-    right->forward_store(ctx, h, y2);
+    run_pair(ctx, h, y1, y2);
     f1 = left_scale;
     f2 = right_scale;
   }
   std::shared_ptr<MixerPart> left, right;
   int64_t dim = 0;
   float left_scale = 1.f, right_scale = 1.f;
+  int64_t right_col = 0, width = 0;
+  Tensor w_in;                 // both mixers' input weights
   Tensor s_left, s_right;      // the factors spread over a row: what the kernel that adds two scaled branches takes
 };
 
@@ -3489,6 +3541,13 @@ float DiffAttention::lambda_of(const Tensor l[4], int dk, double diff, bool on_h
     s2 = std::fmaf(host[(size_t)2 * dk + d], host[(size_t)3 * dk + d], s2);
   }
   return std::exp(s1) - std::exp(s2) + (float)diff;
+}
+void put_zeros(const Tensor& dst, bool on_host) {
+  if (dst.numel() == 0) return;
+  const std::vector<char> zeros(dst.bytes(), 0);
+  if (on_host) memcpy(dst.data, zeros.data(), zeros.size());
+  else if (hipMemcpy(dst.data, zeros.data(), zeros.size(), hipMemcpyHostToDevice) != hipSuccess)
+    throw KernelError("copying a part's constants to the device failed");
 }
 void put_floats(const Tensor& dst, const std::vector<float>& values, bool on_host) {
   if (on_host) {

@@ -612,6 +612,95 @@ def case_sandwich_norms_gru_and_paired_rotation(ops, rng) -> int:
     return fails
 
 
+def case_layer_norm_pairs_scans_and_identities(ops, rng) -> int:
+    """Layer norms on either side of a sublayer of two branches, a short convolution with its bias and silu, the selective and the
+    rotated scan whole and in chunks, a gate in front of a norm in parts, experts beside identities."""
+    fails = 0
+    D = lambda a, dt=None: _dev(np.asarray(a), dt or (torch.int32 if np.asarray(a).dtype == np.int32 else torch.float32))      # noqa: E731
+    f32 = lambda a: np.asarray(a, dtype=np.float32).astype(np.float64)      # noqa: E731
+    silu = lambda z: z / (1.0 + np.exp(-z))      # noqa: E731
+
+    def ln(z, eps):
+        d = z - z.mean(-1, keepdims=True)
+        return d / np.sqrt((d * d).mean(-1, keepdims=True) + eps)
+    M, W = 7, 1028
+    x, y, plus = rng.normal(2, 1, size=(M, W)), rng.normal(1, 1, size=(M, W)), rng.normal(size=(M, W))
+    g, ng = rng.normal(1, 0.2, size=W), rng.normal(1, 0.2, size=W)
+    want = f32(x) + 0.7 * ln(0.8 * f32(y) + 1.1 * f32(plus), 1e-5) * f32(g)
+    xd, out = D(x), torch.empty(M, W, device="cuda")
+    ops.norm_residual_next(xd, D(y), D(g), 1e-5, None, 0, D(plus), None, D(ng), 1e-6, out, True, True, 0.7, 0.8, 1.1)
+    fails += _say("layer norm of two branches, onto the residual", float(np.abs(_f64(xd) - want).max()), 5e-5)
+    fails += _say("  the layer norm in front of the next", float(np.abs(_f64(out) - ln(want, 1e-6) * f32(ng)).max()), 5e-5)
+    # a Mamba-2 layer's convolution and scan, 150 tokens
+    T, H, P, N, K = 150, 4, 24, 20, 4
+    C = H * P + 2 * N
+    u, taps, bias = rng.normal(size=(T, C)), rng.normal(size=(C, K)) / 2, rng.normal(size=C)
+    padded = np.concatenate([np.zeros((K - 1, C)), f32(u)])
+    xbc = silu(sum(padded[j:j + T] * f32(taps)[:, j] for j in range(K)) + f32(bias))
+    entries, rows = D(np.array([[0, T, 0, 0]], dtype=np.int32)), torch.empty(T, C, device="cuda")
+    ops.short_conv(D(u), D(taps), torch.zeros(1, K - 1, C, device="cuda"), entries, D(np.zeros(T, dtype=np.int32)), D(np.arange(T, dtype=np.int32)), rows,
+                   D(bias), True)
+    fails += _say("short convolution with bias and silu", float(np.abs(_f64(rows) - xbc).max()), 5e-5)
+    dt, db, al, sk = rng.normal(-1, 1, size=(T, H)), rng.normal(size=H), rng.uniform(-2, 1, size=H), rng.normal(size=H)
+    d = np.logaddexp(0, f32(dt) + f32(db))
+    o_want, S = np.zeros((T, H, P)), np.zeros((H, N, P))
+    for t in range(T):
+        for h in range(H):
+            v, b, c = xbc[t, h * P:(h + 1) * P], xbc[t, H * P:H * P + N], xbc[t, H * P + N:]
+            S[h] = np.exp(-np.exp(f32(al)[h]) * d[t, h]) * S[h] + d[t, h] * np.outer(b, v)
+            o_want[t, h] = S[h].T @ c + f32(sk)[h] * v
+    lists = (None, None), (D(np.array([[0, 0, 64, 1], [0, 64, 64, 0], [0, 128, 22, 2]], dtype=np.int32)), D(np.array([[0, 3]], dtype=np.int32)))
+    for name, (chunks, spans) in zip(("whole", "in chunks"), lists):
+        state, o = torch.zeros(1, H, N * P, device="cuda"), torch.empty(T, H * P, device="cuda")
+        ops.linear_scan(D(xbc), state, entries, o, H, N, P, (H * P + N, H * P, 0), chunks=chunks, spans=spans, qk_heads=1, dt=D(dt), dt_bias=D(db),
+                        a_log=D(al), skip=D(sk))
+        fails += _say(f"selective scan, {name}", float(np.abs(_f64(o).reshape(T, H, P) - o_want).max()), 5e-5 * float(np.abs(o_want).max()))
+    # retention: heads of 32, the first 16 entries rotated
+    H, dk, dv, dims = 2, 32, 40, 16
+    proj, decay = rng.normal(size=(T, 2 * H * dk + H * dv)), np.array([0.99, 0.7])
+    f = np.array([50.0 ** (-2.0 * i / dims) for i in range(dims // 2)])
+    ang = (np.arange(T)[:, None] * f)[:, None]
+
+    def turn(z):
+        a, b = z[..., :dims // 2], z[..., dims // 2:dims]
+        return np.concatenate([a * np.cos(ang) - b * np.sin(ang), b * np.cos(ang) + a * np.sin(ang), z[..., dims:]], -1)
+    q, k = turn(f32(proj)[:, :H * dk].reshape(T, H, dk)), turn(f32(proj)[:, H * dk:2 * H * dk].reshape(T, H, dk)) * dk ** -0.5
+    v = f32(proj)[:, 2 * H * dk:].reshape(T, H, dv)
+    o_want, S = np.zeros((T, H, dv)), np.zeros((H, dk, dv))
+    for t in range(T):
+        for h in range(H):
+            S[h] = f32(decay)[h] * S[h] + np.outer(k[t, h], v[t, h])
+            o_want[t, h] = S[h].T @ q[t, h]
+    for name, (chunks, spans) in zip(("whole", "in chunks"), lists):
+        state, o = torch.zeros(1, H, dk * dv, device="cuda"), torch.empty(T, H * dv, device="cuda")
+        ops.linear_scan(D(proj), state, entries, o, H, dk, dv, (0, H * dk, 2 * H * dk), decay=D(decay), chunks=chunks, spans=spans, k_scale=dk ** -0.5,
+                        inv_freq=D(f), positions=D(np.arange(T, dtype=np.int32)), rot_dims=dims)
+        fails += _say(f"retention, {name}", float(np.abs(_f64(o).reshape(T, H, dv) - o_want).max()), 5e-5 * float(np.abs(o_want).max()))
+    y, z = o_want.reshape(T, H * dv), f32(rng.normal(size=(T, H * dv)))
+    p = (f32(y) * silu(z)).reshape(T, 4, -1)
+    out = torch.empty(T, H * dv, device="cuda")
+    ops.gated_group_norm(D(y), D(z), 0, None, 1e-5, out, 4, True, True)
+    fails += _say("a gate in front of a norm in parts", float(np.abs(_f64(out) - (p / np.sqrt((p * p).mean(-1, keepdims=True) + 1e-5)).reshape(T, -1)).max()), 5e-5)
+    # gated experts beside identities, few tokens and many
+    E, I, top, W, F = 5, 2, 3, 64, 96
+    router, corr = rng.normal(size=(E + I, W)) / 4, rng.normal(size=E + I) / 20
+    gu, down = _bf16(rng.normal(size=(E * 2 * F, W)) / 6), _bf16(rng.normal(size=(E * W, F)) / 8)
+    for M in (5, 200):
+        h = _bf16(rng.normal(size=(M, W)))
+        ids, wts, hd = torch.empty(M, top, device="cuda", dtype=torch.int32), torch.empty(M, top, device="cuda"), D(h, torch.bfloat16)
+        ops.moe_route_grouped(hd, D(router), ids, wts, D(corr), top, renormalize=False, score="softmax")
+        y = torch.empty(M, W, device="cuda")
+        ops.moe_experts_gated(hd, ids, wts, D(gu, torch.bfloat16), D(down, torch.bfloat16), y, E, "silu", identity=I)
+        sc = np.exp(h @ f32(router).T)
+        sc /= sc.sum(1, keepdims=True)
+        want, g4, d4 = np.zeros((M, W)), gu.reshape(E, 2, F, W), down.reshape(E, W, F)
+        for t in range(M):
+            for e in ids.cpu().numpy()[t]:
+                want[t] += sc[t, e] * (h[t] if e >= E else d4[e] @ (silu(g4[e, 0] @ h[t]) * (g4[e, 1] @ h[t])))
+        fails += _say(f"gated experts beside identities, {M} tokens", float(np.abs(_f64(y) - want).max()), 1.5e-2 * float(np.abs(want).max()))
+    return fails
+
+
 def run_selftest() -> int:
     if not torch.cuda.is_available():
         print("[selftest] no GPU: the kernels of this framework run on an AMD GPU (gfx950) only", flush=True)
@@ -641,6 +730,7 @@ def run_selftest() -> int:
     fails += case_diff_attention(ops, rng, nh=8, nkv=1, dk=64, dv=128, T=130, block=64, taps=2, rot=16, dtype=torch.bfloat16)
     fails += case_streams_gates_and_decay(ops, rng)
     fails += case_sandwich_norms_gru_and_paired_rotation(ops, rng)
+    fails += case_layer_norm_pairs_scans_and_identities(ops, rng)
     fails += case_embed_argmax_sample(ops, rng)
     fails += case_model_shapes(ops, rng)
     fails += case_head_bandwidth(ops, rng)
