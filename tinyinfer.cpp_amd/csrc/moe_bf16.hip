@@ -414,7 +414,7 @@ moe_few_kernel(const bf16_t* __restrict__ in, const int* __restrict__ ids, const
   }
 }
 
-// the same contract as ti_moe_experts_rows (act_kind < 0: relu^2) / ti_moe_experts_rows_gated for bfloat16 and W, F multiples of 32
+// what ti_moe_experts_rows (act_kind < 0: relu^2) / ti_moe_experts_rows_gated do, for bfloat16 and W, F multiples of 32
 // (3: sizes not served); part f32 [M top][W], a token's rows to be added by the caller
 extern "C" int ti_moe_experts_few_bf16(const void* h, const int* ids, const float* wts, const void* up, const void* down, void* act, float* part,
                                        int M, int W, int F, int E, int top, int scale_input, int act_kind, float limit, float alpha, int identity,
